@@ -1,0 +1,81 @@
+"""ctypes binding of libpoptransformer_hybrid.so (include/poptransformer_hybrid.h): the counterpart of `_lib` for the
+kernels of decoders with recurrent layers and a 32-bit residual.  A missing library is an error, there is no fallback.
+"""
+import ctypes
+import os
+from ctypes import POINTER, c_char_p, c_float, c_int, c_size_t, c_void_p
+
+from ._lib import PTA_EINVAL, PTA_EUNSUPPORTED, PTA_OK, PtaError
+
+LIB_PATH = os.path.join(os.path.dirname(os.path.abspath(__file__)), "libpoptransformer_hybrid.so")
+
+BF16, FP32 = 0, 1
+PAIR_NONE, PAIR_SWIGLU, PAIR_CLAMPED = 0, 1, 2
+WINDOW_TILE = 128
+MLSTM_SLICE = 32
+
+
+def _struct(name, fields):
+    return type(name, (ctypes.Structure,), {"_fields_": fields})
+
+
+_P, _I, _F = c_void_p, c_int, c_float
+WideLinearArgs = _struct("WideLinearArgs", [
+    ("dtype", _I), ("X", _P), ("M", _I), ("K", _I), ("N", _I), ("W", _P), ("W2", _P), ("pair", _I), ("limit", _F), ("slope", _F),
+    ("cap", _F), ("Y", _P), ("ld", _I), ("n_main", _I), ("out_f32", _I), ("tail", _P), ("tail_count", _I), ("tail_bias", _P),
+    ("workspace", _P), ("workspace_bytes", c_size_t)])
+StreamsArgs = _struct("StreamsArgs", [
+    ("dtype", _I), ("rows", _I), ("width", _I), ("S", _I), ("streams", _P), ("table", _P), ("vocab", _I), ("embed_scale", _F),
+    ("ids", _P), ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("y", _P), ("out", _P), ("mix", _P), ("mult", _F),
+    ("write_streams", _I), ("gather", _P), ("next_in", _P), ("weight", _P), ("eps", _F), ("h", _P), ("h_ld", _I), ("sum_out", _P)])
+WindowArgs = _struct("WindowArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("G", _I), ("D", _I), ("q", _P), ("k", _P), ("gate", _P), ("ld", _I), ("q_norm", _P),
+    ("k_norm", _P), ("eps", _F), ("scale", _F), ("slopes", _P), ("window", _I), ("ring", _P), ("rinv", _P), ("ring_len", _I),
+    ("slot", _P), ("pos", _P), ("q_scale", _P), ("tile_row", _P), ("tile_count", _P), ("tiles", _I), ("splits", _I),
+    ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P), ("out_ld", _I)])
+MlstmArgs = _struct("MlstmArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("E", _I), ("q", _P), ("k", _P), ("v", _P), ("ld", _I), ("gates", _P),
+    ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("chunked", _I), ("o", _P)])
+
+SIGNATURES = {
+    "pta_hybrid_last_error": (c_char_p, []),
+    "pta_bf16_tiled_bytes": (c_size_t, [_I, _I]),
+    "pta_bf16_tile": (_I, [_P, _P, _I, _I, _P]),
+    "pta_wide_linear_workspace_bytes": (c_size_t, [_I, _I]),
+    "pta_wide_linear": (_I, [POINTER(WideLinearArgs), _P]),
+    "pta_streams_norm": (_I, [POINTER(StreamsArgs), _P]),
+    "pta_window_attention_workspace_bytes": (c_size_t, [_I, _I, _I, _I]),
+    "pta_window_append": (_I, [POINTER(WindowArgs), _P]),
+    "pta_window_attention": (_I, [POINTER(WindowArgs), _P]),
+    "pta_window_decode": (_I, [POINTER(WindowArgs), _P]),
+    "pta_mlstm_state_floats": (c_size_t, [_I, _I, _I]),
+    "pta_mlstm": (_I, [POINTER(MlstmArgs), _P]),
+    "pta_head_norm_gate": (_I, [_I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P]),
+    "pta_argmax_f32": (_I, [_P, _P, _P, _I, _I, _P]),
+    "pta_topk_f32": (_I, [_P, _P, _P, _I, _I, _I, _P]),
+}
+
+_lib = None
+
+
+def load():
+    """Load the shared library and declare every prototype. Raises if it has not been built."""
+    global _lib
+    if _lib is None:
+        if not os.path.exists(LIB_PATH):
+            raise PtaError(f"{LIB_PATH} is missing: build it with `python -m poptransformer_amd.build` "
+                           "(there is no CPU fallback for the HIP kernels)")
+        lib = ctypes.CDLL(LIB_PATH)
+        for name, (res, args) in SIGNATURES.items():
+            fn = getattr(lib, name)
+            fn.restype, fn.argtypes = res, args
+        _lib = lib
+    return _lib
+
+
+def check(rc):
+    """Status code -> the exception `_lib.check` raises for it."""
+    if rc == PTA_OK:
+        return
+    msg = load().pta_hybrid_last_error().decode()
+    raise {PTA_EINVAL: ValueError, PTA_EUNSUPPORTED: NotImplementedError}.get(rc, PtaError)(msg)

@@ -44,7 +44,15 @@ __device__ __forceinline__ f16x8 dequant_step(u32x4 w, int m, f16x2 s2) {
 }
 
 
-struct FmtW4 {
+// The product of the formats that become fp16 operands; their epilogue rounds to fp16 step by step.
+struct F16Product {
+  static constexpr bool kWide = false;
+  static __device__ __forceinline__ f32x4 mma(f16x8 a, f16x8 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
+  }
+};
+
+struct FmtW4 : F16Product {
   static constexpr int kVec = 1;
   typedef f16x2 Scale;
   static __device__ __forceinline__ Scale load_scale(const void* scale, const int32_t*, int row, int N) {
@@ -62,7 +70,7 @@ struct FmtW4 {
 // Tile = 16 output channels x 128 input features = 4 vectors of 1 KiB; in vector j lane l holds
 // the 8 consecutive features  kt*128 + j*32 + (l/16)*8 + 0..7  of channel l%16, which is the
 // A operand of one 16x16x32 MFMA as it stands.
-struct FmtF16 {
+struct FmtF16 : F16Product {
   static constexpr int kVec = 4;
   struct Scale {};
   static __device__ __forceinline__ Scale load_scale(const void*, const int32_t*, int, int) { return Scale{}; }
@@ -124,7 +132,7 @@ __device__ __forceinline__ f16x8 f152_decode8(uint32_t lo, uint32_t hi) {
 struct F8Scale { float mul; };
 
 template <int FMT>
-struct FmtF8 {
+struct FmtF8 : F16Product {
   static constexpr int kVec = 2;
   typedef F8Scale Scale;
   static __device__ __forceinline__ Scale load_scale(const void* scale, const int32_t* x_scale, int, int) {
@@ -138,3 +146,17 @@ struct FmtF8 {
   static __device__ __forceinline__ float finish(float acc, Scale s) { return acc * s.mul; }
 };
 
+
+// bf16 weights and activations: the tiles of FmtF16 with bf16 elements (an operand travels through the core as the
+// sixteen bytes it is), and the fp32 epilogue.
+struct FmtBF16 {
+  static constexpr int kVec = 4;
+  static constexpr bool kWide = true;
+  struct Scale {};
+  static __device__ __forceinline__ Scale load_scale(const void*, const int32_t*, int, int) { return Scale{}; }
+  static __device__ __forceinline__ f16x8 a_operand(const u32x4 (&raw)[4], int j, Scale) { return bitcast<f16x8>(raw[j]); }
+  static __device__ __forceinline__ float finish(float acc, Scale) { return acc; }
+  static __device__ __forceinline__ f32x4 mma(f16x8 a, f16x8 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(bitcast<bf16x8>(a), bitcast<bf16x8>(b), c, 0, 0, 0);
+  }
+};

@@ -8,6 +8,19 @@
 #include "common.h"
 #include "f8codec.h"
 
+// Where and how a product of a "wide" format goes: one fp32 value per output, rounded once where it is stored.
+struct WideOut {
+  int ld;                   // elements between rows of Y
+  int n_main;               // channels [0, n_main) go to Y; channels past n_main + tail_count are padding of the weight
+  int out_f32;              // Y holds fp32 (else the format's own type)
+  float* tail;              // channels [n_main, n_main + tail_count) go here, fp32 [M, tail_count], plus tail_bias
+  int tail_count;
+  const float* tail_bias;
+  float cap;                // > 0: y = cap * tanh(y / cap)
+  int clamped;              // pairs: 0 = SwiGLU, 1 = min(g, limit) sigmoid(slope g) (clamp(u, -limit, limit) + 1)
+  float limit, slope;
+};
+
 struct GemmEpilogue {
   const f16* bias;
   const f16* residual;
@@ -22,6 +35,7 @@ struct GemmEpilogue {
   int out_fp8_format;
   f16* mix_state;                 // [2][M, K] or null: the previous token's rows for the token-shift mixes (gemv_lds_kernel)
   const int32_t* mix_step;
+  WideOut wide;                   // of the formats whose epilogue works in fp32 (Fmt::kWide)
 };
 
 __device__ __forceinline__ f16 sigmoid_f16(f16 x) {
@@ -68,7 +82,7 @@ __device__ __forceinline__ f16 swiglu_out(const GemmEpilogue& e, f16 gate, f16 u
 }
 
 static inline int make_epilogue(const pta_fusion* in, GemmEpilogue* out, const char* name) {
-  *out = GemmEpilogue{nullptr, nullptr, PTA_ACT_NONE, nullptr, 0.f, PTA_NORM_NONE, nullptr, nullptr, 0.f, nullptr, PTA_F143, nullptr, nullptr};
+  *out = GemmEpilogue{nullptr, nullptr, PTA_ACT_NONE, nullptr, 0.f, PTA_NORM_NONE, nullptr, nullptr, 0.f, nullptr, PTA_F143, nullptr, nullptr, WideOut{}};
   if (!in) return PTA_OK;
   PTA_REQUIRE(in->act >= PTA_ACT_NONE && in->act <= PTA_ACT_SIGMOID, "%s: unknown activation %d", name, in->act);
   PTA_REQUIRE(in->norm >= PTA_NORM_NONE && in->norm <= PTA_NORM_LAYER, "%s: unknown norm %d", name, in->norm);
@@ -109,6 +123,72 @@ struct GemmMat {
   int nb_begin;        // first 16-channel block of this matrix in the launch grid
 };
 
+// The fp32 epilogue of the wide formats (Y is a bf16 or fp32 buffer behind the f16* of GemmMat).
+__device__ __forceinline__ float wide_value(const WideOut& w, float v) { return w.cap > 0.f ? w.cap * tanhf(v / w.cap) : v; }
+
+__device__ __forceinline__ float wide_pair_value(const WideOut& w, float g, float u) {
+  if (!w.clamped) return u * g / (1.0f + expf(-g));
+  g = fminf(g, w.limit);
+  u = fminf(fmaxf(u, -w.limit), w.limit);
+  return g / (1.0f + expf(-w.slope * g)) * (u + 1.0f);
+}
+
+__device__ __forceinline__ void wide_store(const WideOut& w, const GemmMat& mat, int m, int n, float v) {
+  if (w.out_f32) reinterpret_cast<float*>(mat.Y)[(size_t)m * w.ld + n] = v;
+  else reinterpret_cast<bf16*>(mat.Y)[(size_t)m * w.ld + n] = (bf16)v;
+}
+
+__device__ __forceinline__ void wide_put(const WideOut& w, const GemmMat& mat, int m, int n, float v) {
+  if (n < w.n_main) {
+    wide_store(w, mat, m, n, wide_value(w, v));
+  } else if (n - w.n_main < w.tail_count) {
+    const int c = n - w.n_main;
+    w.tail[(size_t)m * w.tail_count + c] = w.tail_bias ? v + w.tail_bias[c] : v;
+  }
+}
+
+__device__ __forceinline__ void wide_put_pair(const WideOut& w, const GemmMat& mat, int m, int n, float gate, float up) {
+  if (n < w.n_main) wide_store(w, mat, m, n, wide_pair_value(w, gate, up));
+}
+
+// four consecutive channels of a row, n a multiple of four
+__device__ __forceinline__ void wide_store4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 v) {
+  if (w.out_f32) {
+    *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(mat.Y) + (size_t)m * w.ld + n) = v;
+  } else {
+    bf16x4 b;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) b[r] = (bf16)v[r];
+    *reinterpret_cast<bf16x4*>(reinterpret_cast<bf16*>(mat.Y) + (size_t)m * w.ld + n) = b;
+  }
+}
+
+__device__ __forceinline__ void wide_put4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 v) {
+  if (n + 4 <= w.n_main && (w.ld & 3) == 0) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = wide_value(w, v[r]);
+    wide_store4(w, mat, m, n, v);
+  } else {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) wide_put(w, mat, m, n + r, v[r]);
+  }
+}
+
+__device__ __forceinline__ void wide_put_pair4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 gate, f32x4 up) {
+  if (n + 4 <= w.n_main && (w.ld & 3) == 0) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) gate[r] = wide_pair_value(w, gate[r], up[r]);
+    wide_store4(w, mat, m, n, gate);
+  } else {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) wide_put_pair(w, mat, m, n + r, gate[r], up[r]);
+  }
+}
+
+static inline f16* wide_rows_from(const WideOut& w, f16* Y, int m0) {
+  return reinterpret_cast<f16*>(reinterpret_cast<unsigned char*>(Y) + (size_t)m0 * w.ld * (w.out_f32 ? 4 : 2));
+}
+
 struct GemmArgs {
   GemmMat mat[4];
   int count;
@@ -124,6 +204,25 @@ struct GemmArgs {
   int ksplit;          // 0 or 1: no split
   int prefer_stream;   // host side: up to 16 rows go to gemv_stream_kernel wherever it fits
 };
+// One finished fp32 sum of a matrix, or of a gate / up pair, on its way out.
+template <class Fmt>
+__device__ __forceinline__ void gemm_put(const GemmArgs& a, const GemmMat& mat, int m, int n, int N, float sum) {
+  if constexpr (Fmt::kWide) {
+    wide_put(a.epi.wide, mat, m, n, sum);
+  } else {
+    f16 y0 = (f16)sum;
+    if (mat.bias) y0 = y0 + mat.bias[n];
+    y0 = apply_act(mat.act, y0);
+    mat.Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+  }
+}
+
+template <class Fmt>
+__device__ __forceinline__ void gemm_put_pair(const GemmArgs& a, int m, int n, int N, float gate, float up) {
+  if constexpr (Fmt::kWide) wide_put_pair(a.epi.wide, a.mat[0], m, n, gate, up);
+  else a.mat[0].Y[(size_t)m * N + n] = swiglu_out(a.epi, (f16)gate, (f16)up);
+}
+
 static inline int device_compute_units();
 constexpr int GEMM_MAX_KSPLIT = 4;
 constexpr int GEMM_MAX_ROWS = 4096;
@@ -195,7 +294,7 @@ __global__ __launch_bounds__(NW * 64) void gemv_mfma_kernel(GemmArgs a) {
         const f16x8 av = Fmt::a_operand(w[g], j, sc[g]);
 #pragma unroll
         for (int mt = 0; mt < MT; ++mt)
-          acc[g][mt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av, xb[j][mt], acc[g][mt], 0, 0, 0);
+          acc[g][mt] = Fmt::mma(av, xb[j][mt], acc[g][mt]);
       }
     }
   }
@@ -225,14 +324,9 @@ __global__ __launch_bounds__(NW * 64) void gemv_mfma_kernel(GemmArgs a) {
       sum[g] = Fmt::finish(t, sc[g]);
     }
     if (PAIR) {
-      const f16 gate = (f16)sum[0];
-      const f16 up = (f16)sum[1];
-      a.mat[0].Y[(size_t)m * N + n] = swiglu_out(a.epi, gate, up);
+      gemm_put_pair<Fmt>(a, m, n, N, sum[0], sum[1]);
     } else {
-      f16 y0 = (f16)sum[0];
-      if (a.mat[mi].bias) y0 = y0 + a.mat[mi].bias[n];
-      y0 = apply_act(a.mat[mi].act, y0);
-      a.mat[mi].Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+      gemm_put<Fmt>(a, a.mat[mi], m, n, N, sum[0]);
     }
   }
 }
@@ -384,7 +478,7 @@ __global__ __launch_bounds__(NW * 64) void gemv_lds_kernel(GemmArgs a) {
 #pragma unroll
       for (int g = 0; g < NACC; ++g) {
         const f16x8 av = Fmt::a_operand(wcur[g], j, sc[g]);
-        acc[g] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av, xb, acc[g], 0, 0, 0);
+        acc[g] = Fmt::mma(av, xb, acc[g]);
       }
     }
     if (ktn < KT) {
@@ -415,14 +509,9 @@ __global__ __launch_bounds__(NW * 64) void gemv_lds_kernel(GemmArgs a) {
       sum[g] = Fmt::finish(t, sc[g]);
     }
     if (PAIR) {
-      const f16 gate = (f16)sum[0];
-      const f16 up = (f16)sum[1];
-      a.mat[0].Y[(size_t)m * N + n] = swiglu_out(a.epi, gate, up);
+      gemm_put_pair<Fmt>(a, m, n, N, sum[0], sum[1]);
     } else {
-      f16 y0 = (f16)sum[0];
-      if (a.mat[mi].bias) y0 = y0 + a.mat[mi].bias[n];
-      y0 = apply_act(a.mat[mi].act, y0);
-      a.mat[mi].Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+      gemm_put<Fmt>(a, a.mat[mi], m, n, N, sum[0]);
     }
   }
 }
@@ -579,8 +668,8 @@ __global__ __launch_bounds__(WIDE_WAVES * 64) void gemv_wide_kernel(GemmArgs a, 
           for (int b = 0; b < NB; ++b)
 #pragma unroll
             for (int g = 0; g < NACC; ++g)
-              acc[b][g][0] = __builtin_amdgcn_mfma_f32_16x16x32_f16(Fmt::a_operand(w[u][b][g], j, sc[b][g]), xb[u][j],
-                                                                    acc[b][g][0], 0, 0, 0);
+              acc[b][g][0] = Fmt::mma(Fmt::a_operand(w[u][b][g], j, sc[b][g]), xb[u][j],
+                                                                    acc[b][g][0]);
     };
     int kt0 = wave;
     if constexpr (NORM) {
@@ -628,7 +717,7 @@ __global__ __launch_bounds__(WIDE_WAVES * 64) void gemv_wide_kernel(GemmArgs a, 
             const f16x8 av = Fmt::a_operand(w[b][g], j, sc[b][g]);
 #pragma unroll
             for (int mt = 0; mt < MT; ++mt)
-              acc[b][g][mt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av, xb[mt], acc[b][g][mt], 0, 0, 0);
+              acc[b][g][mt] = Fmt::mma(av, xb[mt], acc[b][g][mt]);
           }
       }
     }
@@ -667,14 +756,9 @@ __global__ __launch_bounds__(WIDE_WAVES * 64) void gemv_wide_kernel(GemmArgs a, 
         sum[g] = Fmt::finish(t, sc[b][g]);      // no format's finish uses the per-channel part of the scale
       }
       if (PAIR) {
-        const f16 gate = (f16)sum[0];
-        const f16 up = (f16)sum[1];
-        mat.Y[(size_t)m * N + n] = swiglu_out(a.epi, gate, up);
+        gemm_put_pair<Fmt>(a, m, n, N, sum[0], sum[1]);
       } else {
-        f16 y0 = (f16)sum[0];
-        if (mat.bias) y0 = y0 + mat.bias[n];
-        y0 = apply_act(mat.act, y0);
-        mat.Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+        gemm_put<Fmt>(a, mat, m, n, N, sum[0]);
       }
     }
   }
@@ -855,7 +939,7 @@ void gemv_stream_kernel(GemmArgs a, int total_nb) {
       for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int g = 0; g < NACC; ++g)
-          acc[g] = __builtin_amdgcn_mfma_f32_16x16x32_f16(Fmt::a_operand(st.w[u][g], j, sc[g]), xs[u][j], acc[g], 0, 0, 0);
+          acc[g] = Fmt::mma(Fmt::a_operand(st.w[u][g], j, sc[g]), xs[u][j], acc[g]);
     if (++cs < spb) return;
     // the block is complete: lane l holds channels (l/16)*4 + r, r = 0..3, for activation row l%16
 #pragma unroll
@@ -882,7 +966,9 @@ void gemv_stream_kernel(GemmArgs a, int total_nb) {
           sum[g] = Fmt::finish(t, sc[g]);        // no format's finish uses the per-channel part of the scale
         }
         if (PAIR) {
-          mat.Y[(size_t)m * N + n] = swiglu_out(a.epi, (f16)sum[0], (f16)sum[1]);
+          gemm_put_pair<Fmt>(a, m, n, N, sum[0], sum[1]);
+        } else if constexpr (Fmt::kWide) {
+          gemm_put<Fmt>(a, mat, m, n, N, sum[0]);
         } else {
           // as apply_epilogue, with the operands that came with the weights
           f16 y0 = (f16)sum[0];
@@ -1047,7 +1133,7 @@ __global__ __launch_bounds__(NWV * 64) void gemm_tile_kernel(GemmArgs a) {
           for (int st = 0; st < 2; ++st) {
             const f16x8 av = Fmt::a_operand(w_cur[st], m, sc[st]);
 #pragma unroll
-            for (int mt = 0; mt < MT; ++mt) acc[st][mt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av, xb[mt], acc[st][mt], 0, 0, 0);
+            for (int mt = 0; mt < MT; ++mt) acc[st][mt] = Fmt::mma(av, xb[mt], acc[st][mt]);
           }
         } else {
           // many row groups: both weight fragments decoded once, then one activation fragment at a time feeds both
@@ -1055,8 +1141,8 @@ __global__ __launch_bounds__(NWV * 64) void gemm_tile_kernel(GemmArgs a) {
 #pragma unroll
           for (int mt = 0; mt < MT; ++mt) {
             const f16x8 xb = *reinterpret_cast<const f16x8*>(cur + mt * 16 * TILE_XSTRIDE + m * 32);
-            acc[0][mt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av0, xb, acc[0][mt], 0, 0, 0);
-            acc[1][mt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av1, xb, acc[1][mt], 0, 0, 0);
+            acc[0][mt] = Fmt::mma(av0, xb, acc[0][mt]);
+            acc[1][mt] = Fmt::mma(av1, xb, acc[1][mt]);
           }
         }
       }
@@ -1085,18 +1171,14 @@ __global__ __launch_bounds__(NWV * 64) void gemm_tile_kernel(GemmArgs a) {
         if (PAIR) {
           const int n = nb[0] * 16 + (lane >> 4) * 4 + r;
           if (n >= N) continue;
-          const f16 gate = (f16)Fmt::finish(acc[0][mt][r], sc[0]), up = (f16)Fmt::finish(acc[1][mt][r], sc[1]);
-          mat.Y[(size_t)m * N + n] = swiglu_out(a.epi, gate, up);
+          gemm_put_pair<Fmt>(a, m, n, N, Fmt::finish(acc[0][mt][r], sc[0]), Fmt::finish(acc[1][mt][r], sc[1]));
         } else {
 #pragma unroll
           for (int st = 0; st < 2; ++st) {
             const int n = nb[st] * 16 + (lane >> 4) * 4 + r;
             if (n >= N) continue;
             if (nsl > 1) { a.part[((size_t)blockIdx.y * M + m) * N + n] = acc[st][mt][r]; continue; }
-            f16 y0 = (f16)Fmt::finish(acc[st][mt][r], sc[st]);
-            if (mat.bias) y0 = y0 + mat.bias[n];
-            y0 = apply_act(mat.act, y0);
-            mat.Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+            gemm_put<Fmt>(a, mat, m, n, N, Fmt::finish(acc[st][mt][r], sc[st]));
           }
         }
       }
@@ -1141,14 +1223,9 @@ __global__ __launch_bounds__(NWV * 64) void gemm_tile_kernel(GemmArgs a) {
 #pragma unroll
     for (int g = 0; g < (PAIR ? 2 : 1); ++g) sum[g] = Fmt::finish(sum[g], sc[0]);   // no format's finish uses the per-channel part
     if (PAIR) {
-      const f16 gate = (f16)sum[0];
-      const f16 up = (f16)sum[1];
-      mat.Y[(size_t)m * N + n] = swiglu_out(a.epi, gate, up);
+      gemm_put_pair<Fmt>(a, m, n, N, sum[0], sum[1]);
     } else {
-      f16 y0 = (f16)sum[0];
-      if (mat.bias) y0 = y0 + mat.bias[n];
-      y0 = apply_act(mat.act, y0);
-      mat.Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+      gemm_put<Fmt>(a, mat, m, n, N, sum[0]);
     }
   }
 }
@@ -1165,10 +1242,7 @@ __global__ __launch_bounds__(256) void splitk_finish_kernel(GemmArgs a) {
   const int m = (int)(i / N), n = (int)(i % N);
   float t = 0.f;
   for (int sl = 0; sl < a.ksplit; ++sl) t += a.part[(size_t)sl * total + i];
-  f16 y0 = (f16)Fmt::finish(t, Fmt::load_scale(mat.scale, a.x_scale, n, N));
-  if (mat.bias) y0 = y0 + mat.bias[n];
-  y0 = apply_act(mat.act, y0);
-  mat.Y[i] = apply_epilogue(a.epi, y0, m, n, N);
+  gemm_put<Fmt>(a, mat, m, n, N, Fmt::finish(t, Fmt::load_scale(mat.scale, a.x_scale, n, N)));
 }
 
 template <class Fmt, int MT, int KQ, bool PAIR, int NWV = TILE_WAVES>
@@ -1314,7 +1388,7 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
 #pragma unroll
       for (int m = 0; m < 4; ++m)
 #pragma unroll
-        for (int rg = 0; rg < RG; ++rg) acc[rg][st] = __builtin_amdgcn_mfma_f32_16x16x32_f16(av[m], xf[rg][m], acc[rg][st], 0, 0, 0);
+        for (int rg = 0; rg < RG; ++rg) acc[rg][st] = Fmt::mma(av[m], xf[rg][m], acc[rg][st]);
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
       for (int m = 0; m < 4; ++m) av[m] = avn[m];
@@ -1343,11 +1417,15 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const int rg = i / (ROWS_CB / 2), st = i % (ROWS_CB / 2);
       const int m = row0 + rg * 16 + (lane & 15);
       const f32x4 g4 = sums[(rg * ROWS_CB + st) * 64 + lane], u4 = sums[(rg * ROWS_CB + st + ROWS_CB / 2) * 64 + lane];
+      if constexpr (Fmt::kWide) {
+        if (m < M) wide_put_pair4(a.epi.wide, mat, m, (first_blk + st) * 16 + (lane >> 4) * 4, g4, u4);
+        continue;
+      }
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int n = (first_blk + st) * 16 + (lane >> 4) * 4 + r;
         if (m >= M || n >= mat.N) continue;
-        mat.Y[(size_t)m * mat.N + n] = swiglu_out(a.epi, (f16)Fmt::finish(g4[r], sg), (f16)Fmt::finish(u4[r], su));
+        gemm_put_pair<Fmt>(a, m, n, mat.N, Fmt::finish(g4[r], sg), Fmt::finish(u4[r], su));
       }
     }
   } else {
@@ -1359,15 +1437,18 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const int rg = i / ROWS_CB, st = i % ROWS_CB;
       const int m = row0 + rg * 16 + (lane & 15);
       const f32x4 v4 = sums[i * 64 + lane];
+      if constexpr (Fmt::kWide) {
+        if (nsl == 1) {
+          if (m < M) wide_put4(a.epi.wide, mat, m, stream_blk(st) * 16 + (lane >> 4) * 4, v4);
+          continue;
+        }
+      }
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int n = stream_blk(st) * 16 + (lane >> 4) * 4 + r;
         if (m >= M || n >= N) continue;
         if (nsl > 1) { a.part[((size_t)blockIdx.y * M + m) * N + n] = v4[r]; continue; }
-        f16 y0 = (f16)Fmt::finish(v4[r], s1);
-        if (mat.bias) y0 = y0 + mat.bias[n];
-        y0 = apply_act(mat.act, y0);
-        mat.Y[(size_t)m * N + n] = apply_epilogue(a.epi, y0, m, n, N);
+        gemm_put<Fmt>(a, mat, m, n, N, Fmt::finish(v4[r], s1));
       }
     }
   }
@@ -1661,7 +1742,7 @@ __global__ __launch_bounds__(PANEL_WAVES * 64) __attribute__((amdgpu_waves_per_e
         else if (more) avn = Fmt::a_operand(wn[0], 0, sc[0]);
 #pragma unroll
         for (int rg = 0; rg < RG; ++rg) {
-          acc[rg][st] = __builtin_amdgcn_mfma_f32_16x16x32_f16(avc, xf[rg], acc[rg][st], 0, 0, 0);
+          acc[rg][st] = Fmt::mma(avc, xf[rg], acc[rg][st]);
           if (st == NST - 1) {
             if (m < 3) xf[rg] = *reinterpret_cast<const f16x8*>(xc + rg * 16 * 128 + b_piece(m + 1));
             else if (more) xf[rg] = *reinterpret_cast<const f16x8*>(xn + rg * 16 * 128 + b_piece(0));
@@ -1863,8 +1944,10 @@ static int dispatch_many_rows(const GemmArgs& a, int total_nb, hipStream_t s, co
     if (b.X) b.X += (size_t)m0 * a.K;
     for (int i = 0; i < a.count; ++i) {
       if (b.mat[i].X) b.mat[i].X += (size_t)m0 * a.K;
-      if (!PAIR || i == 0) b.mat[i].Y += (size_t)m0 * a.mat[i].N;
+      if constexpr (Fmt::kWide) b.mat[i].Y = wide_rows_from(a.epi.wide, a.mat[i].Y, m0);
+      else if (!PAIR || i == 0) b.mat[i].Y += (size_t)m0 * a.mat[i].N;
     }
+    if (b.epi.wide.tail) b.epi.wide.tail += (size_t)m0 * b.epi.wide.tail_count;
     if (PAIR) b.mat[1].Y = b.mat[0].Y;
     if (b.epi.residual) b.epi.residual += (size_t)m0 * a.mat[0].N;
     if (b.epi.mul) b.epi.mul += (size_t)m0 * a.mat[0].N;

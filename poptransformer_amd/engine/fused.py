@@ -14,11 +14,12 @@ shapes: GPT-2 (models/gpt2), Llama 2 (models/llama2), ChatGLM2 (models/chatglm2)
 from dataclasses import dataclass, field
 from typing import List, Optional
 
-import numpy as np
 import torch
 
 from .. import _lib
+from .. import hybrid_kernels as HK
 from .. import kernels as K
+from .loop import DecodeLoop
 
 
 @dataclass
@@ -247,12 +248,12 @@ class LayerOps:
 class NextToken:
     """LMHead's selection (layers/lm_head.py:52-56) over the logits of one iteration: top-1, or with topk > 1
     ops.random_sample (ops/popart.py:25-29): the top-k ids, then the column chosen by the argmax of k normal
-    draws, one draw per iteration for the whole batch."""
+    draws, one draw per iteration for the whole batch.  The logits are fp16, or fp32 with `f32_logits`."""
 
-    def __init__(self, batch, vocab, topk, device):
+    def __init__(self, batch, vocab, topk, device, f32_logits=False):
         if topk < 1 or topk > vocab:
             raise ValueError(f"topk = {topk} outside [1, vocabulary size {vocab}]")
-        self.topk = topk
+        self.topk, self.f32_logits = topk, f32_logits
         if topk > 1:
             i32, f16 = torch.int32, torch.float16
             self.ids = torch.zeros((batch, topk), dtype=i32, device=device)
@@ -262,15 +263,18 @@ class NextToken:
 
     def __call__(self, logits, next_ids):
         if self.topk == 1:
-            K.argmax(logits, next_ids)
+            (HK if self.f32_logits else K).argmax(logits, next_ids)
             return
-        K.topk(logits, self.topk, self.ids, self.vals)
+        if self.f32_logits:
+            HK.topk(logits, self.topk, self.ids)
+        else:
+            K.topk(logits, self.topk, self.ids, self.vals)
         self.draws.normal_()
         K.argmax(self.draws, self.pick)
         K.take_column(self.ids, self.pick, next_ids)
 
 
-class FusedDecoder(LayerOps):
+class FusedDecoder(DecodeLoop, LayerOps):
     def __init__(self, spec: DecoderSpec, weights: ModelWeights, device="cuda"):
         super().__init__(spec, weights, device, spec.batch)
         s, buf = spec, self._buf
@@ -369,30 +373,13 @@ class FusedDecoder(LayerOps):
     # ------------------------------------------------------------------ loop
     def reset(self, input_ids):
         """Initial loop state of build_model_graph_inputs (models/base_model.py:255-269)."""
-        s = self.spec
-        ids = torch.as_tensor(np.asarray(input_ids, np.int32))
-        if tuple(ids.shape) != (s.batch, s.max_len):
-            raise ValueError(f"input_ids must be [{s.batch}, {s.max_len}], got {tuple(ids.shape)}")
-        self._host_ids = ids.numpy().copy()
+        ids = self.checked_ids(input_ids)
         self.container.copy_(ids)
         self.mask.fill_(-10000.0)
         self.mask[:, 0] = 0
         self.stop_mask.zero_()
         self.step.zero_()
         self.keep_going.fill_(1)
-
-    def prompt_positions(self):
-        """How many leading loop iterations only read the prompt: their `next_ids` are dropped because the
-        container already holds a token at the next position (models/base_model.py:313-318), and no
-        sequence meets its end token there.  These are the positions `consume_prompt` may take at once."""
-        s, ids = self.spec, self._host_ids
-        n = s.max_len - 1
-        for row in ids:
-            later = row[1:]
-            pads = np.nonzero(later == s.pad_id)[0]
-            ends = np.nonzero(later == s.eos_id)[0]
-            n = min(n, int(pads[0]) if len(pads) else s.max_len - 1, int(ends[0]) if len(ends) else s.max_len - 1)
-        return max(n, 0)
 
     def consume_prompt(self, n=None, rows_per_pass=None):
         """Runs the first `n` loop iterations (default: `prompt_positions()`) as passes over up to
@@ -402,12 +389,7 @@ class FusedDecoder(LayerOps):
         (the loop would discard their tokens).  Call after `reset`.  Returns n."""
         from .prompt import PromptPass
         s = self.spec
-        limit = self.prompt_positions()
-        n = limit if n is None else int(n)
-        if n < 0 or n > limit:
-            raise ValueError(f"consume_prompt: n = {n} outside [0, {limit}] (the prompt's own positions before any end token)")
-        if int(self.step.item()) != 0:
-            raise RuntimeError("consume_prompt must follow reset()")
+        n = self.checked_prompt_count(n)
         if n == 0:
             return 0
         # by default passes of up to 1024 rows: from a few hundred rows on the projections run on the kernel whose
@@ -431,46 +413,8 @@ class FusedDecoder(LayerOps):
         self._stream.synchronize()
         return n
 
-    def capture(self):
-        """Record one loop iteration into a HIP graph (after an eager iteration has warmed up
-        every code path).  The iteration depends on device state only, so it can be replayed."""
-        self.reset(np.zeros((self.spec.batch, self.spec.max_len), np.int32))
-        with torch.cuda.stream(self._stream):
-            self.step_fn()
-            torch.cuda.synchronize()
-            self.graph = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(self.graph, stream=self._stream):
-                self.step_fn()
-        torch.cuda.synchronize()
-        return self.graph
-
-    def run_steps(self, n):
-        if self.graph is None:
-            for _ in range(n):
-                self.step_fn()
-        else:
-            for _ in range(n):
-                self.graph.replay()
-
-    def run(self, input_ids, max_loop, check_every=16, prompt_passes=False):
-        """The whole generation (one `session.run` of the reference, poptransformer/sessions.py:47-49).
-        Returns (container, step) like the anchors 'Loop:0' and 'Loop:1'.  prompt_passes: the leading
-        iterations that only read the prompt run as passes over several positions (consume_prompt)."""
-        self.reset(input_ids)
-        done = 0
-        if prompt_passes:
-            n = min(self.prompt_positions(), max_loop)
-            if n > 0:
-                done = self.consume_prompt(n)
-        while done < max_loop:
-            n = min(check_every, max_loop - done) if self.spec.early_stop else max_loop - done
-            self.run_steps(n)
-            done += n
-            if self.spec.early_stop and int(self.keep_going.item()) == 0:
-                break
-        torch.cuda.synchronize()
+    def check_finished(self):
         if self.persistent is not None and self.persistent.failed():
             raise RuntimeError("persistent decode step: a workgroup gave up waiting (the kernel needs every compute unit "
                                "of the device for itself while it runs); the loop state was not advanced past the failing "
                                "iteration.  The failure word is sticky: persistent.clear_failure() re-arms the decoder")
-        return self.container.cpu().numpy(), int(self.step.item())

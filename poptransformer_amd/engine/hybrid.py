@@ -1,0 +1,386 @@
+"""Executor of decoders that mix windowed attention with recurrent (matrix memory) layers over fp32 residual streams.
+
+The model is a list of layers, each described by its mixer, its feed-forward (or none) and the layer whose tensors it
+uses.  One forward function serves everything: it takes the ROWS of a pass (row = one token of the sequence in a slot, at
+a position) through all layers.  A decode iteration is a pass with one row per sequence and depends on device state only
+(it is recorded into a HIP graph); a prompt, or a batch of prompts of unequal lengths, is cut into passes of up to
+`pass_rows` rows.  Both leave the same cache and state behind.
+
+Per layer with a feed-forward the launches of a decode iteration are: projections, mixer (attention, with the parts of its
+window merged by a second launch; or recurrence and head norm), output projection, stream update + norm, gate / up pair,
+down projection, stream update + norm.
+"""
+from dataclasses import dataclass, field
+from typing import List, Optional
+
+import numpy as np
+import torch
+
+from .. import _hybrid_lib as H
+from .. import hybrid_kernels as HK
+from .fused import NextToken
+from .loop import DecodeLoop
+from .sequences import SequenceStore
+
+F32, I32 = torch.float32, torch.int32
+
+
+@dataclass
+class WindowMixer:
+    """Attention over the last `window` positions (None: all), key heads shared by groups of query heads, values that are
+    the raw keys, a distance bias of slope_h per position, and an output gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    window: Optional[int]
+    kind = "attention"
+
+    @property
+    def out_channels(self):
+        return self.heads * self.dim
+
+    @property
+    def gate_at(self):
+        return (self.heads + self.kv_heads) * self.dim
+
+    def slopes(self):
+        return 2.0 ** (-8.0 * (np.arange(self.heads) + 1) / self.heads)
+
+
+@dataclass
+class MemoryMixer:
+    """mLSTM: a matrix memory of dim x vdim per head."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+    kind = "mlstm"
+
+    @property
+    def out_channels(self):
+        return self.heads * self.vdim
+
+    @property
+    def gate_at(self):
+        return self.heads * (2 * self.dim + self.vdim)
+
+
+@dataclass
+class ClampedGLU:
+    """min(g, limit) sigmoid(slope g) (clamp(u, -limit, limit) + 1) between the gate / up pair and the down projection."""
+    ff: int
+    limit: float
+    slope: float = 1.702
+
+
+@dataclass
+class HybridLayer:
+    mixer: object
+    mlp: Optional[ClampedGLU]
+    source: int                      # the layer whose tensors this one uses (itself, or an earlier one)
+
+
+@dataclass
+class HybridSpec:
+    family: str
+    layers: List[HybridLayer]
+    width: int
+    vocab: int
+    streams: int
+    eps: float
+    residual_mult: float
+    embed_scale: float
+    logit_cap: float                 # 0: none
+    max_len: int
+    batch: int
+    pad_id: int = 0
+    eos_id: int = -1
+    early_stop: bool = False
+    topk: int = 1
+    dtype: str = "bfloat16"          # or float32: everything in true 32-bit
+
+
+@dataclass
+class HybridLayerWeights:
+    norm1: torch.Tensor
+    connect1: tuple                  # (in [S], out [S], mix [S, S] from -> to), fp32
+    proj: HK.WideWeight              # attention: q | k | gate; mlstm: q | k | v | gate, tail: input and forget gates
+    out: HK.WideWeight
+    q_norm: Optional[torch.Tensor] = None
+    k_norm: Optional[torch.Tensor] = None
+    slopes: Optional[torch.Tensor] = None
+    head_norm: Optional[torch.Tensor] = None
+    norm2: Optional[torch.Tensor] = None
+    connect2: Optional[tuple] = None
+    gate: Optional[HK.WideWeight] = None
+    up: Optional[HK.WideWeight] = None
+    down: Optional[HK.WideWeight] = None
+
+    def linears(self):
+        return [w for w in (self.proj, self.out, self.gate, self.up, self.down) if w is not None]
+
+
+@dataclass
+class HybridWeights:
+    embed: torch.Tensor
+    layers: List[Optional[HybridLayerWeights]]      # None where a layer uses another one's
+    final_norm: torch.Tensor
+    head: HK.WideWeight
+
+    def nbytes(self):
+        """Bytes of weights one iteration reads (a layer counts as often as it is run by its users: see step_bytes)."""
+        return self.head.nbytes + sum(w.nbytes for lay in self.layers if lay is not None for w in lay.linears())
+
+
+class RowBuffers:
+    """Activations of up to `rows` rows."""
+
+    def __init__(self, spec, weights, rows, dtype, device):
+        def buf(*shape, dtype=dtype):
+            return torch.zeros(shape, dtype=dtype, device=device)
+        mixers = [lay.mixer for lay in spec.layers]
+        self.rows = rows
+        self.streams = buf(rows, spec.streams, spec.width, dtype=F32)
+        self.h = buf(rows, HK.pad8(spec.width))
+        self.y = buf(rows, spec.width, dtype=F32)
+        self.ctx = {n: buf(rows, n) for n in {HK.pad8(m.out_channels) for m in mixers}}
+        used = [lw for lw in weights.layers if lw is not None]
+        self.proj = {n: buf(rows, n) for n in {HK.pad8(lw.proj.n_main) for lw in used}}
+        self.act = {n: buf(rows, n) for n in {lw.gate.n_main for lw in used if lw.gate is not None}}
+        memory = [m for m in mixers if m.kind == "mlstm"]
+        self.gates = buf(rows * 2 * max((m.heads for m in memory), default=0), dtype=F32)
+        self.o = buf(rows * max((m.out_channels for m in memory), default=0), dtype=F32)
+        self.q_scale = buf(rows, dtype=F32)
+        self.workspace = HK.linear_workspace(rows, max((lw.out.N for lw in used), default=1), device) if rows > 16 else None
+
+
+@dataclass
+class Rows:
+    """The rows of one pass, as device tensors: slot and position of every row; the sequences (first row, rows); the tiles
+    the attention works on (first row, rows).  `single`: one row per sequence."""
+    n: int
+    slot: torch.Tensor
+    pos: torch.Tensor
+    seqs: tuple
+    single: bool
+    tiles: tuple = ()
+    ids: Optional[torch.Tensor] = None
+    ids_index: Optional[torch.Tensor] = None
+    longest: int = 1
+
+
+class HybridDecoder(DecodeLoop):
+    """Two ways in, one set of layers, caches and kernels behind both:
+      * the decode loop of the other executors (reset / run_steps / consume_prompt / run): `spec.batch` sequences in step;
+      * `open` / `advance` / `close`: sequences that come, bring their next tokens in batches of any lengths, and go."""
+
+    pass_rows = 2048                 # rows of a pass, at most
+
+    def __init__(self, spec, weights, device="cuda", slots=None):
+        self.spec, self.w, self.dev = spec, weights, device
+        self.dtype = HK.DTYPES[spec.dtype]
+        self.store = SequenceStore(spec, self.dtype, slots or max(spec.batch, 1), spec.max_len, self.pass_rows, device)
+        self.probe = None            # callable(layer index, fp32 [rows, width]): the summed streams after every layer
+        self._buffers = {}
+        self._stream = torch.cuda.Stream()
+        self._splits_for = {}
+
+    # ------------------------------------------------------------------ layers
+    def _layer_weights(self, i):
+        return self.w.layers[self.spec.layers[i].source]
+
+    def _rows_buffers(self, rows):
+        size = rows if rows <= 16 else max(64, 1 << (rows - 1).bit_length())
+        if size not in self._buffers:
+            self._buffers[size] = RowBuffers(self.spec, self.w, size, self.dtype, self.dev)
+        return self._buffers[size]
+
+    def _splits(self, rows, mixer):
+        """Parts of the window per (row, key head) of a decode pass, and the scratch they meet in.  Fixed per shape (the
+        launch is replayed while the context grows): enough workgroups to fill the machine, at least 64 keys per part."""
+        key = (rows, mixer.heads, mixer.kv_heads, mixer.dim, mixer.window)
+        if key not in self._splits_for:
+            group = mixer.heads // mixer.kv_heads
+            wgs = rows * mixer.kv_heads * -(-group // (group if group <= 2 else 4))
+            keys = min(mixer.window or self.store.max_len, self.store.max_len)
+            splits = max(1, min(1024 // wgs if wgs else 1, -(-keys // 64), 64))
+            splits = 1 if keys <= 256 else splits
+            self._splits_for[key] = (splits, HK.window_workspace(rows, mixer.heads, mixer.dim, splits, self.dev) if splits > 1 else None)
+        return self._splits_for[key]
+
+    def _mixer(self, i, b, rows):
+        spec, m, lw, store = self.spec, self.spec.layers[i].mixer, self._layer_weights(i), self.store.stores[i]
+        n = rows.n
+        proj, ctx = b.proj[HK.pad8(lw.proj.n_main)], b.ctx[HK.pad8(m.out_channels)]
+        HK.linear(b.h, lw.proj, proj, n, ld=proj.shape[1], tail=b.gates if lw.proj.tail else None)
+        if m.kind == "attention":
+            att = HK.WindowAttention(m.heads, m.kv_heads, m.dim, m.scale, m.window, spec.eps, lw.q_norm, lw.k_norm, lw.slopes, *store)
+            if rows.single:
+                splits, ws = self._splits(n, m)
+                att.decode(proj, n, rows.slot, rows.pos, ctx, splits, ws)
+            else:
+                att.prompt(proj, n, rows.slot, rows.pos, ctx, b.q_scale, rows.tiles)
+        else:
+            HK.mlstm(proj, n, m.heads, m.dim, m.vdim, b.gates, m.gate_cap, store[0], rows.slot, rows.seqs, b.o, rows.longest > 8)
+            HK.head_norm_gate(b.o, lw.head_norm, proj, m.gate_at, ctx, n, m.heads, m.vdim, spec.eps)
+        HK.linear(ctx, lw.out, b.y, n, ld=spec.width, workspace=b.workspace)
+
+    def _feed_forward(self, i, b, rows):
+        mlp, lw = self.spec.layers[i].mlp, self._layer_weights(i)
+        act = b.act[lw.gate.n_main]
+        HK.linear(b.h, lw.gate, act, rows.n, up=lw.up, pair=H.PAIR_CLAMPED, limit=mlp.limit, slope=mlp.slope)
+        HK.linear(act, lw.down, b.y, rows.n, ld=self.spec.width, workspace=b.workspace)
+
+    def _layers(self, rows, pos_out=None):
+        """All layers over the rows.  Returns the buffers with the last sublayer's result still to be added, and that
+        sublayer's connections (`_logits` does both at once)."""
+        spec, b = self.spec, self._rows_buffers(rows.n)
+        norm = dict(eps=spec.eps, mult=spec.residual_mult, h=b.h)
+        first = self._layer_weights(0)
+        HK.streams_norm(b.streams, rows.n, table=self.w.embed, embed_scale=spec.embed_scale, ids=rows.ids, ids_index=rows.ids_index,
+                        pos_out=pos_out, next_in=first.connect1[0], weight=first.norm1, **norm)
+        done = None
+        for i, layer in enumerate(spec.layers):
+            lw = self._layer_weights(i)
+            if i:
+                HK.streams_norm(b.streams, rows.n, y=b.y, connect=done, next_in=lw.connect1[0], weight=lw.norm1, **norm)
+            self._mixer(i, b, rows)
+            done = lw.connect1[1:]
+            if layer.mlp is not None:
+                HK.streams_norm(b.streams, rows.n, y=b.y, connect=done, next_in=lw.connect2[0], weight=lw.norm2, **norm)
+                self._feed_forward(i, b, rows)
+                done = lw.connect2[1:]
+            if self.probe is not None:
+                total = torch.empty((rows.n, spec.width), dtype=F32, device=self.dev)
+                HK.streams_norm(b.streams, rows.n, spec.eps, y=b.y, connect=done, mult=spec.residual_mult, write=False, sum_out=total,
+                                dtype=self.dtype)
+                self.probe(i, total)
+        return b, done
+
+    def _logits(self, b, done, count, out, gather=None):
+        """Final norm and head of `count` rows (all, or those listed in `gather`)."""
+        spec = self.spec
+        HK.streams_norm(b.streams, count, spec.eps, y=b.y, connect=done, mult=spec.residual_mult, write=False, gather=gather,
+                        weight=self.w.final_norm, h=b.h)
+        HK.linear(b.h, self.w.head, out, count, ld=spec.vocab, cap=spec.logit_cap)
+
+    # ------------------------------------------------------------------ sequences that come and go
+    def open(self):
+        return self.store.open()
+
+    def close(self, slot):
+        self.store.close(slot)
+
+    def _pass(self, portions):
+        """portions [(slot, token ids)]: device description of their rows."""
+        ids = np.concatenate([np.asarray(t, np.int32) for _, t in portions])
+        counts = np.array([len(t) for _, t in portions], np.int32)
+        starts = np.concatenate([[0], np.cumsum(counts)[:-1]]).astype(np.int32)
+        slots = np.repeat(np.array([s for s, _ in portions], np.int32), counts)
+        pos = np.concatenate([self.store.length[s] + np.arange(len(t), dtype=np.int32) for s, t in portions]).astype(np.int32)
+        tiles = [(a + k, min(H.WINDOW_TILE, c - k)) for a, c in zip(starts, counts) for k in range(0, c, H.WINDOW_TILE)]
+        tr, tc = (np.array([t[j] for t in tiles], np.int32) for j in (0, 1))
+        flat = torch.from_numpy(np.concatenate([ids, slots, pos, starts, counts, tr, tc])).to(self.dev)
+        parts = torch.split(flat, [len(ids)] * 3 + [len(counts)] * 2 + [len(tiles)] * 2)
+        return Rows(len(ids), parts[1], parts[2], (parts[3], parts[4], len(counts)), bool((counts == 1).all()),
+                    (parts[5], parts[6], len(tiles)), ids=parts[0], longest=int(counts.max()))
+
+    def advance(self, entries):
+        """entries [(slot, token ids, wanted places)]: the sequences' next tokens, as one batch, cut into passes where they
+        are many.  Returns the logits fp32 [sum of wanted, vocab] at the wanted places, in their order."""
+        spec, store = self.spec, self.store
+        if len({e[0] for e in entries}) != len(entries):
+            raise ValueError("advance: a sequence appears twice in one batch")
+        for slot, tokens, want in entries:
+            if store.length[slot] < 0:
+                raise ValueError(f"advance: slot {slot} is not in use")
+            if len(tokens) == 0 or store.length[slot] + len(tokens) > store.max_len:
+                raise ValueError(f"advance: {len(tokens)} tokens after {store.length[slot]} (max_len {store.max_len})")
+            if min(tokens) < 0 or max(tokens) >= spec.vocab:
+                raise ValueError(f"advance: a token id outside [0, {spec.vocab})")
+            if any(not 0 <= w < len(tokens) for w in want):
+                raise ValueError("advance: a wanted place outside the tokens of its entry")
+        out_at, total = {}, 0
+        for e, (_, _, want) in enumerate(entries):
+            for w in want:
+                out_at.setdefault((e, w), []).append(total)
+                total += 1
+        logits = torch.empty((total, spec.vocab), dtype=F32, device=self.dev)
+        at = [0] * len(entries)
+        while any(a < len(e[1]) for a, e in zip(at, entries)):
+            portions, rows_of, n = [], [], 0
+            for e, (slot, tokens, _) in enumerate(entries):
+                take = min(len(tokens) - at[e], store.portion, self.pass_rows - n)
+                if take <= 0:
+                    continue
+                portions.append((slot, tokens[at[e]:at[e] + take]))
+                rows_of += [(e, at[e] + k) for k in range(take)]
+                at[e] += take
+                n += take
+            rows = self._pass(portions)
+            b, done = self._layers(rows)
+            picks = [(r, o) for r, key in enumerate(rows_of) for o in out_at.get(key, ())]
+            for c in range(0, len(picks), 256):
+                part = picks[c:c + 256]
+                gather = torch.tensor([r for r, _ in part], dtype=I32, device=self.dev)
+                got = torch.empty((len(part), spec.vocab), dtype=F32, device=self.dev)
+                self._logits(b, done, len(part), got, gather)
+                logits[torch.tensor([o for _, o in part], device=self.dev)] = got
+            for slot, tokens in portions:
+                store.length[slot] += len(tokens)
+        return logits
+
+    # ------------------------------------------------------------------ decode loop
+    def _prepare_loop(self):
+        s = self.spec
+        if hasattr(self, "container"):
+            return
+        if self.store.capacity < s.batch:
+            self.store._grow(s.batch)
+        B = s.batch
+
+        def zeros(*shape, dtype=I32):
+            return torch.zeros(shape, dtype=dtype, device=self.dev)
+        self.container, self.stop_mask, self.next_ids = zeros(B, s.max_len), zeros(B), zeros(B)
+        self.step, self.keep_going = zeros(), zeros() + 1
+        self.logits = zeros(B, s.vocab, dtype=F32)
+        self.select = NextToken(B, s.vocab, s.topk, self.dev, f32_logits=True)
+        lanes = torch.arange(B, dtype=I32, device=self.dev)
+        self._loop_rows = Rows(B, lanes, zeros(B), (lanes, zeros(B) + 1, B), True, ids=self.container, ids_index=self.step)
+
+    def reset(self, input_ids):
+        ids = self.checked_ids(input_ids)
+        self._prepare_loop()
+        self.container.copy_(ids)
+        self.stop_mask.zero_()
+        self.step.zero_()
+        self.keep_going.fill_(1)
+        self.store.restart(range(self.spec.batch))
+
+    def step_fn(self):
+        from .. import kernels as K
+        s, rows = self.spec, self._loop_rows
+        b, done = self._layers(rows, pos_out=rows.pos)
+        self._logits(b, done, rows.n, self.logits)
+        self.select(self.logits, self.next_ids)
+        K.step_update(self.container, None, self.stop_mask, self.step, self.next_ids, None, self.keep_going, s.pad_id, s.eos_id,
+                      s.early_stop)
+
+    def consume_prompt(self, n=None, rows_per_pass=None):
+        """The first n loop iterations (default: all that only read the prompt) as passes over several positions of every
+        sequence.  Cache, state and loop state end up as n iterations leave them.  Call after `reset`.  Returns n."""
+        n = self.checked_prompt_count(n)
+        B = self.spec.batch
+        R = min(rows_per_pass or max(1, self.pass_rows // B), self.store.portion)
+        if R < 1 or R * B > 4096:
+            raise ValueError(f"consume_prompt: rows_per_pass * batch must lie in [1, 4096], got {R} * {B}")
+        with torch.cuda.stream(self._stream):
+            for p0 in range(0, n, R):
+                ids = self._host_ids[:, p0:min(p0 + R, n)]
+                self._layers(self._pass([(b, ids[b]) for b in range(B)]))
+                for b in range(B):
+                    self.store.length[b] += ids.shape[1]
+            self.step.fill_(n)
+        self._stream.synchronize()
+        return n

@@ -151,3 +151,91 @@ def rwkv_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False):
     return RWKVSpec(cfg["num_hidden_layers"], cfg["hidden_size"], cfg["attention_hidden_size"], cfg["intermediate_size"],
                     cfg["vocab_size"], max_len, batch, cfg["layer_norm_epsilon"], cfg["rescale_every"], pad_id, eos_id,
                     early_stop)
+
+
+def hybrid_layers(layers):
+    """The `layers` list of a hybrid configuration -> [HybridLayer].  `weights_of` may point to a layer that itself
+    uses another one's tensors."""
+    from .hybrid import ClampedGLU, HybridLayer, MemoryMixer, WindowMixer
+    out = []
+    for i, c in enumerate(layers):
+        m, kind = c["mixer"], c["type"]
+        if kind == "attention":
+            if m.get("vdim", m["dim"]) != m["dim"]:
+                raise ValueError(f"layer {i}: the values are the keys, so vdim ({m['vdim']}) must equal dim ({m['dim']})")
+            mixer = WindowMixer(m["heads"], m["kv_heads"], m["dim"], float(m["scale"]), (m.get("mask") or {}).get("size"))
+        elif kind == "mlstm":
+            mixer = MemoryMixer(m["heads"], m["dim"], m["vdim"], float(m["gate_cap"]))
+        else:
+            raise NotImplementedError(f"layer {i}: mixer {kind}")
+        f = c.get("mlp")
+        if f is not None and f.get("kind", "dense") != "dense":
+            raise NotImplementedError(f"layer {i}: feed-forward {f['kind']}")
+        source = i
+        while layers[source].get("weights_of") is not None:
+            source = layers[source]["weights_of"]
+        out.append(HybridLayer(mixer, ClampedGLU(f["ff"], float(f["limit"])) if f is not None else None, source))
+    return out
+
+
+def zekilix_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
+    from .hybrid import HybridSpec
+    return HybridSpec("zekilix", hybrid_layers(cfg["layers"]), cfg["width"], cfg["vocab"], cfg["streams"], cfg["norm"]["eps"],
+                      cfg["residual_mult"], cfg["embedding"]["scale"], cfg["logit_softcap"], max_len, batch, pad_id, eos_id,
+                      early_stop, topk, dtype)
+
+
+def hybrid_weights(tensors, spec, device="cuda"):
+    """tensors: name -> tensor or array (names as in a checkpoint of the design).  Concatenates the projections of a mixer,
+    pads, and lays the weights out for the device; layers that use another one's tensors have no entry of their own."""
+    from .. import hybrid_kernels as HK
+    from .hybrid import HybridLayerWeights, HybridWeights
+    dtype = HK.DTYPES[spec.dtype]
+
+    def get(name, shape):
+        if name not in tensors:
+            raise KeyError(f"tensor {name} is missing")
+        t = tensors[name]
+        t = (t if torch.is_tensor(t) else torch.from_numpy(np.ascontiguousarray(t))).to(device)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"tensor {name} is {tuple(t.shape)}, expected {tuple(shape)}")
+        return t
+
+    def vec(name, n):
+        return get(name, (n,)).float().contiguous()
+
+    d, S = spec.width, spec.streams
+    layers = []
+    for i, lay in enumerate(spec.layers):
+        if lay.source != i:
+            layers.append(None)
+            continue
+        p, m = f"l{i}.", lay.mixer
+        mix = p + "mix."
+
+        def connect(q):
+            hc = p + f"hc{q}."
+            return (vec(hc + "in", S), vec(hc + "out", S), get(hc + "mix", (S, S)).float().contiguous())
+
+        N = m.out_channels
+        lw = dict(norm1=vec(p + "norm1", d), connect1=connect(1), out=HK.WideWeight(get(mix + "o", (d, N)), dtype))
+        if m.kind == "attention":
+            KD = m.kv_heads * m.dim
+            parts = [get(mix + "q", (N, d)), get(mix + "k", (KD, d)), get(mix + "g", (N, d))]
+            lw.update(proj=HK.WideWeight(torch.cat(parts), dtype), q_norm=vec(mix + "q.norm", N), k_norm=vec(mix + "k.norm", KD),
+                      slopes=torch.tensor(m.slopes(), dtype=torch.float32, device=device))
+        else:
+            QD = m.heads * m.dim
+            parts = [get(mix + "q", (QD, d)), get(mix + "k", (QD, d)), get(mix + "v", (N, d)), get(mix + "g", (N, d)),
+                     get(mix + "i", (m.heads, d)), get(mix + "f", (m.heads, d))]
+            bias = torch.cat([vec(mix + "i.b", m.heads), vec(mix + "f.b", m.heads)])
+            lw.update(proj=HK.WideWeight(torch.cat(parts), dtype, tail=2 * m.heads, tail_bias=bias), head_norm=vec(mix + "norm", N))
+        if lay.mlp is not None:
+            ff, mlp = lay.mlp.ff, p + "mlp."
+            lw.update(norm2=vec(p + "norm2", d), connect2=connect(2),
+                      gate=HK.WideWeight(get(mlp + "gate", (ff, d)), dtype, main_to=HK.pad8(ff)),
+                      up=HK.WideWeight(get(mlp + "up", (ff, d)), dtype, main_to=HK.pad8(ff)),
+                      down=HK.WideWeight(get(mlp + "down", (d, ff)), dtype))
+        layers.append(HybridLayerWeights(**lw))
+    return HybridWeights(get("embed", (spec.vocab, d)).to(dtype).contiguous(), layers, vec("final.norm", d),
+                         HK.WideWeight(get("head", (spec.vocab, d)), dtype))

@@ -8,12 +8,12 @@ into a HIP graph like the transformer executor (engine/fused.py).
 from dataclasses import dataclass
 from typing import List, Optional
 
-import numpy as np
 import torch
 
 from .. import _lib
 from .. import kernels as K
 from .fused import LinearWeights, NextToken
+from .loop import DecodeLoop
 
 
 @dataclass
@@ -66,7 +66,7 @@ class RWKVWeights:
         return n
 
 
-class RWKVDecoder:
+class RWKVDecoder(DecodeLoop):
     def __init__(self, spec: RWKVSpec, weights: RWKVWeights, device="cuda"):
         self.spec, self.w, self.dev = spec, weights, device
         s = spec
@@ -159,10 +159,7 @@ class RWKVDecoder:
                       s.pad_id, s.eos_id, s.early_stop)
 
     def reset(self, input_ids):
-        s = self.spec
-        ids = torch.as_tensor(np.asarray(input_ids, np.int32))
-        if tuple(ids.shape) != (s.batch, s.max_len):
-            raise ValueError(f"input_ids must be [{s.batch}, {s.max_len}], got {tuple(ids.shape)}")
+        ids = self.checked_ids(input_ids)
         self.container.copy_(ids)
         self.stop_mask.zero_()
         self.step.zero_()
@@ -171,35 +168,3 @@ class RWKVDecoder:
             t.zero_()
         for t in self.st_max:
             t.fill_(-1e30)
-
-    def capture(self):
-        self.reset(np.zeros((self.spec.batch, self.spec.max_len), np.int32))
-        with torch.cuda.stream(self._stream):
-            self.step_fn()
-            torch.cuda.synchronize()
-            self.graph = torch.cuda.CUDAGraph()
-            with torch.cuda.graph(self.graph, stream=self._stream):
-                self.step_fn()
-        torch.cuda.synchronize()
-        return self.graph
-
-    def run_steps(self, n):
-        for _ in range(n):
-            if self.graph is None:
-                self.step_fn()
-            else:
-                self.graph.replay()
-
-    def run(self, input_ids, max_loop, check_every=16, prompt_passes=False):
-        """prompt_passes is accepted for symmetry with the transformer executor; a recurrent model reads its
-        prompt one position per iteration."""
-        self.reset(input_ids)
-        done = 0
-        while done < max_loop:
-            n = min(check_every, max_loop - done) if self.spec.early_stop else max_loop - done
-            self.run_steps(n)
-            done += n
-            if self.spec.early_stop and int(self.keep_going.item()) == 0:
-                break
-        torch.cuda.synchronize()
-        return self.container.cpu().numpy(), int(self.step.item())

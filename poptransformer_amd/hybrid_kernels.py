@@ -1,0 +1,203 @@
+"""Torch-tensor front end of poptransformer_hybrid.h, as `kernels` is of poptransformer_hip.h: operands are checked on the
+host, raw pointers go to the library on torch's current stream, nothing is computed on the CPU.
+"""
+import ctypes
+
+import torch
+
+from . import _hybrid_lib as H
+
+F32, I32 = torch.float32, torch.int32
+DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
+_CODE = {torch.bfloat16: H.BF16, torch.float32: H.FP32}
+
+
+def _stream():
+    return ctypes.c_void_p(torch.cuda.current_stream().cuda_stream)
+
+
+def _p(t):
+    return t.data_ptr() if t is not None else None
+
+
+def _need(t, dtype, what, numel=None):
+    if not t.is_cuda or t.dtype != dtype or not t.is_contiguous():
+        raise ValueError(f"{what} must be a contiguous {dtype} device tensor")
+    if numel is not None and t.numel() < numel:
+        raise ValueError(f"{what} holds {t.numel()} elements, {numel} needed")
+
+
+def pad8(n):
+    return (n + 7) // 8 * 8
+
+
+class WideWeight:
+    """A Linear weight [N, K] in bf16 (tiled for the matrix unit) or fp32 (as it is).  K is padded with zeros to a multiple
+    of 8.  The last `tail` channels may go to an fp32 buffer of their own, with a bias.  `main_to`: further zero channels
+    after the main ones (results 0) up to that count, so that the result can be the padded input of another Linear."""
+
+    def __init__(self, w, dtype, tail=0, tail_bias=None, main_to=None):
+        n, k = w.shape
+        main = n - tail
+        self.n_main = main if main_to is None else main_to
+        self.tail, self.K, self.dtype = tail, pad8(k), dtype
+        if self.n_main != main and tail:
+            raise ValueError("a weight with a tail takes no further channels")
+        total = self.n_main + tail
+        # many channels: whole workgroup tiles of 128 (the padding goes nowhere)
+        self.N = (total + 127) // 128 * 128 if dtype == torch.bfloat16 and total >= 1024 else total
+        full = torch.zeros((self.N, self.K), dtype=dtype, device=w.device)
+        full[:n, :k] = w.to(dtype)
+        self.tail_bias = tail_bias.to(F32).contiguous() if tail_bias is not None else None
+        if dtype == torch.bfloat16:
+            lib = H.load()
+            self.data = torch.empty(lib.pta_bf16_tiled_bytes(self.N, self.K), dtype=torch.uint8, device=w.device)
+            H.check(lib.pta_bf16_tile(full.data_ptr(), self.data.data_ptr(), self.N, self.K, _stream()))
+            torch.cuda.current_stream().synchronize()      # `full` goes back to the allocator here
+        else:
+            self.data = full
+
+    @property
+    def nbytes(self):
+        return (self.n_main + self.tail) * self.K * (2 if self.dtype == torch.bfloat16 else 4)
+
+
+def linear_workspace(rows, channels, device):
+    return torch.empty(H.load().pta_wide_linear_workspace_bytes(rows, channels), dtype=torch.uint8, device=device)
+
+
+def linear(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.PAIR_NONE, limit=0.0, slope=0.0, workspace=None):
+    """out[:rows] = x[:rows] @ w^T with the fused epilogues of pta_wide_linear; `up`: the second weight of a pair."""
+    _need(x, w.dtype, "x", rows * w.K)
+    ld = w.n_main if ld is None else ld
+    if out.dtype not in (w.dtype, F32):
+        raise ValueError(f"out must be {w.dtype} or float32")
+    _need(out, out.dtype, "out", rows * ld)
+    if x.shape[-1] != w.K:
+        raise ValueError(f"matmul: contracting dimensions differ ({x.shape[-1]} vs {w.K})")
+    if up is not None and (up.N, up.K, up.dtype) != (w.N, w.K, w.dtype):
+        raise ValueError("the weights of a pair must be alike")
+    if w.tail:
+        _need(tail, F32, "tail", rows * w.tail)
+    a = H.WideLinearArgs(_CODE[w.dtype], _p(x), rows, w.K, w.N, _p(w.data), _p(up.data) if up is not None else None, pair, limit, slope,
+                         cap, _p(out), ld, w.n_main, int(out.dtype == F32), _p(tail) if w.tail else None, w.tail, _p(w.tail_bias),
+                         _p(workspace), workspace.numel() if workspace is not None else 0)
+    H.check(H.load().pta_wide_linear(ctypes.byref(a), _stream()))
+    return out
+
+
+def streams_norm(streams, rows, eps, weight=None, h=None, table=None, embed_scale=1.0, ids=None, ids_index=None, pos_out=None, y=None,
+                 connect=None, mult=1.0, write=True, gather=None, next_in=None, sum_out=None, dtype=None):
+    """One sublayer boundary (pta_streams_norm).  streams [R, S, width]; connect = (out [S], mix [S, S]) of the finished
+    sublayer whose result is y; next_in [S] of the sublayer that follows (None: the plain sum)."""
+    _, S, width = streams.shape
+    _need(streams, F32, "streams", 0 if gather is not None else rows * S * width)
+    code = _CODE[h.dtype if h is not None else dtype]
+    if table is not None:
+        _need(table, h.dtype if h is not None else dtype, "table")
+        _need(ids, I32, "ids")
+    if h is not None:
+        _need(h, h.dtype, "h", rows * h.shape[-1])
+        _need(weight, F32, "weight", width)
+    if y is not None:
+        _need(y, F32, "y")
+    stride = ids.shape[-1] if ids is not None and ids.dim() == 2 else 1
+    a = H.StreamsArgs(code, rows, width, S, _p(streams), _p(table), table.shape[0] if table is not None else 0, embed_scale, _p(ids),
+                      stride, _p(ids_index), _p(pos_out), _p(y), _p(connect[0]) if connect is not None else None,
+                      _p(connect[1]) if connect is not None else None, mult, int(write), _p(gather), _p(next_in), _p(weight), eps,
+                      _p(h), h.shape[-1] if h is not None else 0, _p(sum_out))
+    H.check(H.load().pta_streams_norm(ctypes.byref(a), _stream()))
+    return h
+
+
+def window_workspace(rows, heads, dim, splits, device):
+    n = H.load().pta_window_attention_workspace_bytes(rows, heads, dim, splits)
+    return torch.empty(max(n, 16), dtype=torch.uint8, device=device)
+
+
+class WindowAttention:
+    """The arguments of the windowed-attention calls over one set of row buffers and one layer's cache."""
+
+    def __init__(self, heads, kv_heads, dim, scale, window, eps, q_norm, k_norm, slopes, ring, rinv):
+        _need(q_norm, F32, "q_norm", heads * dim)
+        _need(k_norm, F32, "k_norm", kv_heads * dim)
+        _need(slopes, F32, "slopes", heads)
+        if ring.dim() != 4 or ring.shape[1] != kv_heads or ring.shape[3] != pad8(dim):
+            raise ValueError(f"ring must be [slots, {kv_heads}, length, {pad8(dim)}], got {tuple(ring.shape)}")
+        self.H, self.G, self.D = heads, kv_heads, dim
+        self.scale, self.window, self.eps = scale, window, eps
+        self.q_norm, self.k_norm, self.slopes, self.ring, self.rinv = q_norm, k_norm, slopes, ring, rinv
+
+    def _args(self, proj, rows, slot, pos, out, q_scale=None, tiles=None, splits=1, workspace=None):
+        es, HD = proj.element_size(), self.H * self.D
+        ring_len = self.ring.shape[2]
+        _need(proj, self.ring.dtype, "projection", rows * proj.shape[-1])
+        _need(slot, I32, "slot", rows)
+        _need(pos, I32, "pos", rows)
+        _need(out, proj.dtype, "out", rows * out.shape[-1])
+        if proj.shape[-1] < 2 * HD + self.G * self.D:
+            raise ValueError("the projection rows must hold q | k | gate")
+        base = proj.data_ptr()
+        tr, tc, nt = tiles if tiles is not None else (None, None, 0)
+        return H.WindowArgs(_CODE[proj.dtype], rows, self.H, self.G, self.D, base, base + HD * es, base + (HD + self.G * self.D) * es,
+                            proj.shape[-1], _p(self.q_norm), _p(self.k_norm), self.eps, self.scale, _p(self.slopes),
+                            self.window or (1 << 30), _p(self.ring), _p(self.rinv), ring_len, _p(slot), _p(pos), _p(q_scale), _p(tr),
+                            _p(tc), nt, splits, _p(workspace), workspace.numel() if workspace is not None else 0, _p(out), out.shape[-1])
+
+    def decode(self, proj, rows, slot, pos, out, splits, workspace):
+        """One row per sequence: norms, append and attention."""
+        a = self._args(proj, rows, slot, pos, out, splits=splits, workspace=workspace)
+        H.check(H.load().pta_window_decode(ctypes.byref(a), _stream()))
+
+    def prompt(self, proj, rows, slot, pos, out, q_scale, tiles):
+        """Rows of a pass with several rows per sequence; tiles = (first rows, row counts, how many)."""
+        a = self._args(proj, rows, slot, pos, out, q_scale=q_scale, tiles=tiles)
+        lib = H.load()
+        H.check(lib.pta_window_append(ctypes.byref(a), _stream()))
+        H.check(lib.pta_window_attention(ctypes.byref(a), _stream()))
+
+
+def mlstm_state(slots, heads, dim, vdim, device):
+    return torch.zeros((slots, H.load().pta_mlstm_state_floats(heads, dim, vdim)), dtype=F32, device=device)
+
+
+def mlstm(proj, rows, heads, dim, vdim, gates, cap, state, slot, seqs, o, chunked):
+    """proj rows hold q | k | v | ...; seqs = (first rows, row counts, how many); o [rows, heads * vdim] fp32."""
+    es, HD, HE = proj.element_size(), heads * dim, heads * vdim
+    seq_row, seq_count, n = seqs
+    _need(proj, proj.dtype, "projection", rows * proj.shape[-1])
+    _need(gates, F32, "gates", rows * 2 * heads)
+    _need(state, F32, "state")
+    _need(o, F32, "o", rows * HE)
+    if state.shape[1] != H.load().pta_mlstm_state_floats(heads, dim, vdim) or proj.shape[-1] < 2 * HD + 2 * HE:
+        raise ValueError("mlstm: the state or the projection does not fit the sizes")
+    base = proj.data_ptr()
+    a = H.MlstmArgs(_CODE[proj.dtype], rows, heads, dim, vdim, base, base + HD * es, base + 2 * HD * es, proj.shape[-1], _p(gates), cap,
+                    _p(state), _p(slot), _p(seq_row), _p(seq_count), n, int(chunked), _p(o))
+    H.check(H.load().pta_mlstm(ctypes.byref(a), _stream()))
+
+
+def head_norm_gate(o, weight, proj, gate_at, out, rows, heads, vdim, eps):
+    """out = per-head RMS norm of o, times weight, times sigmoid of the projection's channels from gate_at on."""
+    _need(o, F32, "o", rows * heads * vdim)
+    _need(weight, F32, "weight", heads * vdim)
+    _need(out, proj.dtype, "out", rows * out.shape[-1])
+    if proj.shape[-1] < gate_at + heads * vdim:
+        raise ValueError("the projection does not hold the gate")
+    H.check(H.load().pta_head_norm_gate(_CODE[proj.dtype], _p(o), _p(weight), proj.data_ptr() + gate_at * proj.element_size(),
+                                        proj.shape[-1], _p(out), out.shape[-1], rows, heads, vdim, eps, _stream()))
+
+
+def argmax(logits, ids):
+    _need(logits, F32, "logits")
+    _need(ids, I32, "ids")
+    n = logits.shape[-1]
+    H.check(H.load().pta_argmax_f32(_p(logits), _p(ids), None, logits.numel() // n, n, _stream()))
+    return ids
+
+
+def topk(logits, k, ids, values=None):
+    _need(logits, F32, "logits")
+    n = logits.shape[-1]
+    H.check(H.load().pta_topk_f32(_p(logits), _p(ids), _p(values), logits.numel() // n, n, k, _stream()))
+    return ids

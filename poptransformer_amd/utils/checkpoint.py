@@ -9,7 +9,8 @@ fetched: a checkpoint is a directory or a file on the local disk.
 Formats read: `*.safetensors` (one file, or the shards listed in `*.safetensors.index.json`), and
 torch `*.bin` / `*.pt` / `*.pth` state dicts, which are opened with `weights_only=True` (nothing in
 the file is executed).  Floating-point tensors come back as fp16, which is what the reference's
-graphs hold; integer tensors (packed INT4 weights, FP8 bytes) are left as they are.
+graphs hold - or, with `floats="fp32"`, as fp32, which holds bf16 checkpoints exactly; integer tensors (packed INT4
+weights, FP8 bytes) are left as they are.
 
 INT4 checkpoints follow the layout of the reference's int4 path
 (utils/param_handler/precision_strategy.py:24-42, examples/chatglm/conf/int4_sharding.yaml:20):
@@ -30,42 +31,42 @@ import numpy as np
 _TORCH_SUFFIXES = (".bin", ".pt", ".pth")
 
 
-def _to_numpy(t):
-    """torch tensor -> numpy; floating point becomes fp16."""
+def _to_numpy(t, floats="fp16"):
+    """torch tensor -> numpy; floating point becomes fp16, or fp32."""
     import torch
     if t.is_floating_point():
-        return t.to(torch.float16).contiguous().numpy()
+        return t.to({"fp16": torch.float16, "fp32": torch.float32}[floats]).contiguous().numpy()
     return t.contiguous().numpy()
 
 
-def _read_safetensors(path):
+def _read_safetensors(path, floats):
     # through torch, so that bf16 tensors (which numpy cannot hold) are read too
     from safetensors import safe_open
     out = {}
     with safe_open(path, framework="pt", device="cpu") as f:
         for key in f.keys():
-            out[key] = _to_numpy(f.get_tensor(key))
+            out[key] = _to_numpy(f.get_tensor(key), floats)
     return out
 
 
-def _read_torch(path):
+def _read_torch(path, floats):
     import torch
     sd = torch.load(path, map_location="cpu", weights_only=True)
     if isinstance(sd, dict) and "state_dict" in sd and isinstance(sd["state_dict"], dict):
         sd = sd["state_dict"]
     if not isinstance(sd, dict):
         raise ValueError(f"{path} does not hold a state dict")
-    return {k: _to_numpy(v) for k, v in sd.items() if hasattr(v, "is_floating_point")}
+    return {k: _to_numpy(v, floats) for k, v in sd.items() if hasattr(v, "is_floating_point")}
 
 
-def load_state_dict(path):
+def load_state_dict(path, floats="fp16"):
     """path: a .safetensors / .bin / .pt / .pth file, a *.index.json shard index, or a directory
     holding any of these (Hugging Face layout).  Returns {key: numpy array}."""
     if os.path.isdir(path):
         for pattern in ("*.safetensors.index.json", "*.bin.index.json"):
             index = sorted(glob.glob(os.path.join(path, pattern)))
             if index:
-                return load_state_dict(index[0])
+                return load_state_dict(index[0], floats)
         files = sorted(glob.glob(os.path.join(path, "*.safetensors")))
         if not files:
             files = sorted(f for s in _TORCH_SUFFIXES for f in glob.glob(os.path.join(path, "*" + s)))
@@ -73,22 +74,22 @@ def load_state_dict(path):
             raise FileNotFoundError(f"no checkpoint files (*.safetensors, *.bin, *.pt, *.pth) in {path}")
         out = {}
         for f in files:
-            out.update(load_state_dict(f))
+            out.update(load_state_dict(f, floats))
         return out
     if path.endswith(".index.json"):
         with open(path) as f:
             weight_map = json.load(f)["weight_map"]
         out = {}
         for shard in sorted(set(weight_map.values())):
-            out.update(load_state_dict(os.path.join(os.path.dirname(path), shard)))
+            out.update(load_state_dict(os.path.join(os.path.dirname(path), shard), floats))
         missing = [k for k in weight_map if k not in out]
         if missing:
             raise KeyError(f"{path} lists tensors its shards do not hold: {missing[:3]} ...")
         return out
     if path.endswith(".safetensors"):
-        return _read_safetensors(path)
+        return _read_safetensors(path, floats)
     if path.endswith(_TORCH_SUFFIXES):
-        return _read_torch(path)
+        return _read_torch(path, floats)
     raise ValueError(f"unknown checkpoint format: {path}")
 
 
