@@ -3,6 +3,9 @@
 Test infrastructure only.  Arrays are [tokens, features] of ONE sequence, positions count from 0, `cfg` is the
 model's configuration (the dictionary of its config.json) and `sd` its tensors by name.  Nothing here is shared with the
 product path: a sequence is always evaluated as a whole and from scratch.
+
+`rnd` (default: nothing) is applied where a 16-bit evaluation rounds - what enters a matrix product and what a projection
+gives - so that tests can measure how much of a difference rounding alone explains.
 """
 import numpy as np
 
@@ -51,16 +54,20 @@ def windowed_attention(q, k, v, scale, slopes, window):
     return out
 
 
-def attention_mixer(sd, p, mixer, h, eps):
+def exact(a):
+    return a
+
+
+def attention_mixer(sd, p, mixer, h, eps, rnd=exact):
     H, G, D = mixer["heads"], mixer["kv_heads"], mixer["dim"]
     T = h.shape[0]
-    q, k = h @ sd[p + "q"].T, h @ sd[p + "k"].T
+    q, k = rnd(h @ sd[p + "q"].T), rnd(h @ sd[p + "k"].T)
     v = k.reshape(T, G, D)
     q = (rms_norm(q, eps) * sd[p + "q.norm"]).reshape(T, H, D)
     k = (rms_norm(k, eps) * sd[p + "k.norm"]).reshape(T, G, D)
     window = (mixer.get("mask") or {}).get("size")
     o = windowed_attention(q, k, v, mixer["scale"], head_slopes(H), window).reshape(T, H * D)
-    return (o * sigmoid(h @ sd[p + "g"].T)) @ sd[p + "o"].T
+    return rnd(o * sigmoid(rnd(h @ sd[p + "g"].T))) @ sd[p + "o"].T
 
 
 def mlstm_recurrence(q, k, v, i, f):
@@ -85,15 +92,15 @@ def mlstm_gates(sd, p, h, cap):
     return i, f
 
 
-def mlstm_mixer(sd, p, mixer, h, eps):
+def mlstm_mixer(sd, p, mixer, h, eps, rnd=exact):
     H, D, E = mixer["heads"], mixer["dim"], mixer["vdim"]
     T = h.shape[0]
-    q = (h @ sd[p + "q"].T).reshape(T, H, D) * D ** -0.5
-    k = (h @ sd[p + "k"].T).reshape(T, H, D)
-    v = (h @ sd[p + "v"].T).reshape(T, H, E)
+    q = rnd(h @ sd[p + "q"].T).reshape(T, H, D) * D ** -0.5
+    k = rnd(h @ sd[p + "k"].T).reshape(T, H, D)
+    v = rnd(h @ sd[p + "v"].T).reshape(T, H, E)
     i, f = mlstm_gates(sd, p, h, mixer["gate_cap"])
     o = rms_norm(mlstm_recurrence(q, k, v, i, f), eps).reshape(T, H * E)
-    return (o * sd[p + "norm"] * sigmoid(h @ sd[p + "g"].T)) @ sd[p + "o"].T
+    return rnd(o * sd[p + "norm"] * sigmoid(rnd(h @ sd[p + "g"].T))) @ sd[p + "o"].T
 
 
 MIXERS = {"attention": attention_mixer, "mlstm": mlstm_mixer}
@@ -104,12 +111,14 @@ def clamped_glu(gate, up, limit):
     return g * sigmoid(SIGMOID_SLOPE * g) * (u + 1.0)
 
 
-def feed_forward(sd, p, mlp, h):
-    return clamped_glu(h @ sd[p + "gate"].T, h @ sd[p + "up"].T, mlp["limit"]) @ sd[p + "down"].T
+def feed_forward(sd, p, mlp, h, rnd=exact):
+    return rnd(clamped_glu(h @ sd[p + "gate"].T, h @ sd[p + "up"].T, mlp["limit"])) @ sd[p + "down"].T
 
 
 def connect(streams, weights_in, weights_out, mix, mult, sublayer):
-    """One sublayer between `streams` [S, T, d]: read with weights_in, write with weights_out, mix from -> to."""
+    """One sublayer between `streams` [S, T, d] (weights None: a single plain residual): read with weights_in, write with weights_out, mix from -> to."""
+    if weights_in is None:
+        return streams + mult * sublayer(streams[0])[None]
     y = sublayer(np.tensordot(weights_in, streams, axes=1))
     return np.einsum("st,sxd->txd", mix, streams) + mult * weights_out[:, None, None] * y[None]
 
@@ -120,23 +129,24 @@ def owner(cfg, i):
     return i
 
 
-def forward(sd, cfg, ids, collect=None):
+def forward(sd, cfg, ids, collect=None, rnd=exact):
     """Logits [T, vocab] of one sequence.  `collect` (a list) receives the sum of the streams after every layer."""
     sd = {k: np.asarray(v, np.float64) for k, v in sd.items()}
     eps, mult = cfg["norm"]["eps"], cfg["residual_mult"]
     x = sd["embed"][np.asarray(ids)] * cfg["embedding"]["scale"]
-    streams = np.stack([x] * cfg["streams"])
+    streams = np.stack([x] * (cfg.get("streams") or 1))
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{owner(cfg, i)}."
 
         def run(q, norm, fn):
             hc = p + f"hc{q}."
-            return connect(streams, sd[hc + "in"], sd[hc + "out"], sd[hc + "mix"], mult,
-                           lambda u: fn(layer_norm(u, sd[p + norm], eps)))
+            return connect(streams, *(sd.get(hc + n) for n in ("in", "out", "mix")), mult,
+                           lambda u: fn(rnd(layer_norm(u, sd[p + norm], eps))))
 
-        streams = run(1, "norm1", lambda h: MIXERS[layer["type"]](sd, p + "mix.", layer["mixer"], h, eps))
+        streams = run(1, "norm1", lambda h: MIXERS[layer["type"]](sd, p + "mix.", layer["mixer"], h, eps, rnd))
         if layer.get("mlp") is not None:
-            streams = run(2, "norm2", lambda h: feed_forward(sd, p + "mlp.", layer["mlp"], h))
+            streams = run(2, "norm2", lambda h: feed_forward(sd, p + "mlp.", layer["mlp"], h, rnd))
         if collect is not None:
             collect.append(streams.sum(0))
-    return softcap(layer_norm(streams.sum(0), sd["final.norm"], eps) @ sd["head"].T, cfg["logit_softcap"])
+    logits = rnd(layer_norm(streams.sum(0), sd["final.norm"], eps)) @ sd["head"].T
+    return softcap(logits, cfg["logit_softcap"]) if cfg.get("logit_softcap") else logits

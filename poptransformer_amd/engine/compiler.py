@@ -1,7 +1,7 @@
 """From a recorded graph to something that runs: `Session.compile` ends here.
 
 Every graph can run op by op (engine/interpreter.py).  A graph that is one of the decoder loops
-this package knows - GPT-2, Llama 2, ChatGLM2, RWKV as the models build them through the operator
+this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix as the models build them through the operator
 API - is additionally mapped onto the fused executor for its family: the family is read off the
 state-dict keys the layers registered as initializer names, the shapes off a one-iteration probe of
 the interpreter, and the weights off the initializers.  The fused executor is then VALIDATED: it
@@ -250,6 +250,48 @@ def _build_rwkv(facts, shapes, topk=1):
     return RWKVDecoder(spec, w)
 
 
+def _build_hybrid(facts, topk=1):
+    """The hybrid executor of a graph whose layers are tensors `l<i>.*`: sizes from the tensors, constants from the named
+    constants the layers recorded, the arithmetic ('bf16' or 'fp32') from the precision the graph was built with."""
+    from ..utils import REGISTRY
+    from .hybrid import ClampedGLU, HybridDecoder, HybridLayer, HybridSpec, MemoryMixer, WindowMixer
+    from .loader import hybrid_weights
+
+    def const(name, required=True):
+        v = _named_const(facts.body, name)
+        if v is None and required:
+            raise ValueError(f"constant {name} not found")
+        return v
+
+    layers = []
+    while const(f"l{len(layers)}.source", False) is not None:
+        i = len(layers)
+        source = int(const(f"l{i}.source"))
+        mix = f"l{source}.mix."
+        q = _need(facts, mix + "q").shape[0]
+        if facts.has(mix + "i"):
+            heads = int(const(f"l{i}.heads"))
+            mixer = MemoryMixer(heads, q // heads, _need(facts, mix + "v").shape[0] // heads, float(const(f"l{i}.gate_cap")))
+        else:
+            H, G = int(const(f"l{i}.heads")), int(const(f"l{i}.kv_heads"))
+            window = int(const(f"l{i}.window"))
+            mixer = WindowMixer(H, G, q // H, float(const(f"l{i}.scale")), window or None)
+        mlp = None
+        if facts.has(f"l{source}.mlp.gate"):
+            mlp = ClampedGLU(_need(facts, f"l{source}.mlp.gate").shape[0], float(const(f"l{i}.limit")), float(const("gate_slope")))
+        layers.append(HybridLayer(mixer, mlp, source))
+    if not layers:
+        raise ValueError("no layers found among the graph's constants")
+    vocab, width = _need(facts, "embed").shape
+    cap = const("logit_softcap", False)
+    precision = REGISTRY.get("tensor_type").precision
+    spec = HybridSpec("zekilix", layers, width, vocab, facts.init["l0.hc1.in"].shape[0] if facts.has("l0.hc1.in") else 1,
+                      float(const("norm_eps")), float(const("residual_mult")), float(const("embedding_scale")),
+                      float(cap) if cap is not None else 0.0, facts.max_len, facts.batch, facts.pad_id, facts.eos_id,
+                      facts.early_stop, topk, {"bf16": "bfloat16", "fp32": "float32"}[precision])
+    return HybridDecoder(spec, hybrid_weights(facts.init, spec))
+
+
 def _family(facts):
     if facts.has("model.layers.0.self_attn.q_proj.weight"):
         return "llama2"
@@ -259,6 +301,8 @@ def _family(facts):
         return "gpt2"
     if facts.has("rwkv.blocks.0.attention.key.weight"):
         return "rwkv"
+    if facts.has("l0.mix.q") and facts.has("l0.norm1"):
+        return "zekilix"
     return None
 
 
@@ -347,7 +391,8 @@ def _validate_greedy(decoder, prog, facts, steps, prompt_passes, what, seeds=(0,
     Otherwise the graph's logits of every iteration (the inputs of its top-1 selection) are recorded for each probe
     of a fixed list, and the executor is run iteration by iteration beside them, its container following the
     graph's tokens: every iteration's logits must agree within 2 % of the iteration's largest magnitude (10 % where
-    the graph casts activations to FP8: one code of an activation is an eighth of its value), and the selected token
+    the graph casts activations to FP8 - one code of an activation is an eighth of its value - or the executor multiplies
+    in bf16 what the graph multiplies in fp32), and the selected token
     must be the graph's wherever the graph's two best logits are further apart than twice that tolerance.  With
     prompt_passes the probe's leading positions go through the passes first, so those are part of what is checked."""
     interp = prog.interp
@@ -356,7 +401,8 @@ def _validate_greedy(decoder, prog, facts, steps, prompt_passes, what, seeds=(0,
     got, _ = decoder.run(ids, steps, prompt_passes=prompt_passes)
     if np.array_equal(got, want):
         return
-    tol = 0.1 if any("CastToUint8" in n.op for n in facts.body.nodes) else 0.02
+    coarse = any("CastToUint8" in n.op for n in facts.body.nodes) or getattr(decoder.spec, "dtype", None) == "bfloat16"
+    tol = 0.1 if coarse else 0.02
     for seed in seeds:
         ids = _probe_ids(facts, seed, n=3)
         interp.input_trace = {"aiOnnx.topk": []}
@@ -406,6 +452,7 @@ def _validate_sampling(decoder, prog, facts, ids, steps, k):
     try:
         prog._run_once({facts.ids_name: ids})
         want = [np.asarray(o[1]).reshape(facts.batch, k) for o in interp.value_trace["aiOnnx.topk"]]
+        values = [np.asarray(o[0], np.float32).reshape(facts.batch, k) for o in interp.value_trace["aiOnnx.topk"]]
     finally:
         interp.value_trace = None
     if len(want) != steps:
@@ -414,6 +461,12 @@ def _validate_sampling(decoder, prog, facts, ids, steps, k):
     for it in range(steps):
         decoder.step_fn()
         torch.cuda.synchronize()
+        if getattr(decoder.spec, "dtype", None) == "bfloat16":
+            # the graph multiplies in fp32: near ties may be ordered differently, the candidates' logits must agree
+            mine = np.take_along_axis(decoder.logits.cpu().numpy(), want[it], axis=1)
+            if not np.abs(mine - values[it]).max() <= 0.1 * np.abs(values[it]).max():
+                raise ValueError(f"the fused executor's logits of the graph's top-{k} candidates differ at probe iteration {it}")
+            continue
         if not np.array_equal(decoder.select.ids.cpu().numpy(), want[it]):
             raise ValueError(f"the fused executor's top-{k} candidates differ from the graph's at probe iteration {it}")
 
@@ -445,8 +498,8 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
         prog.interp_outputs = list(graph.outputs)
         k = _sampling_k(facts)
         use_fp8_cache = _fp8_cache_of(facts, fp8_cache)
-        if use_fp8_cache and family == "rwkv":
-            raise ValueError("fp8_cache: a recurrent model has no KV cache")
+        if use_fp8_cache and family in ("rwkv", "zekilix"):
+            raise ValueError(f"fp8_cache: the {family} executor has no FP8 KV cache")
         steps = min(PROBE_STEPS, facts.max_loop)
         # one-iteration probe: operand shapes of the native operators
         interp.shape_trace = {}
@@ -456,6 +509,8 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
         shapes, interp.shape_trace = interp.shape_trace, None
         if family == "rwkv":
             decoder = _build_rwkv(facts, shapes, k)
+        elif family == "zekilix":
+            decoder = _build_hybrid(facts, k)
         else:
             spec, weights = _build_transformer(facts, shapes, family, k, use_fp8_cache)
             decoder = fused.FusedDecoder(spec, weights)

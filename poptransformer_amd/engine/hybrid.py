@@ -176,6 +176,7 @@ class HybridDecoder(DecodeLoop):
       * `open` / `advance` / `close`: sequences that come, bring their next tokens in batches of any lengths, and go."""
 
     pass_rows = 2048                 # rows of a pass, at most
+    head_rows = 256                  # rows whose logits are made at once
 
     def __init__(self, spec, weights, device="cuda", slots=None):
         self.spec, self.w, self.dev = spec, weights, device
@@ -185,6 +186,7 @@ class HybridDecoder(DecodeLoop):
         self._buffers = {}
         self._stream = torch.cuda.Stream()
         self._splits_for = {}
+        self._head_h = None
 
     # ------------------------------------------------------------------ layers
     def _layer_weights(self, i):
@@ -259,11 +261,15 @@ class HybridDecoder(DecodeLoop):
         return b, done
 
     def _logits(self, b, done, count, out, gather=None):
-        """Final norm and head of `count` rows (all, or those listed in `gather`)."""
-        spec = self.spec
+        """Final norm and head of `count` rows: the pass's own, or those listed in `gather` (up to head_rows, repeats allowed)."""
+        spec, h = self.spec, b.h
+        if gather is not None:
+            if self._head_h is None:
+                self._head_h = torch.zeros((self.head_rows, h.shape[1]), dtype=self.dtype, device=self.dev)
+            h = self._head_h
         HK.streams_norm(b.streams, count, spec.eps, y=b.y, connect=done, mult=spec.residual_mult, write=False, gather=gather,
-                        weight=self.w.final_norm, h=b.h)
-        HK.linear(b.h, self.w.head, out, count, ld=spec.vocab, cap=spec.logit_cap)
+                        weight=self.w.final_norm, h=h)
+        HK.linear(h, self.w.head, out, count, ld=spec.vocab, cap=spec.logit_cap)
 
     # ------------------------------------------------------------------ sequences that come and go
     def open(self):
@@ -321,8 +327,8 @@ class HybridDecoder(DecodeLoop):
             rows = self._pass(portions)
             b, done = self._layers(rows)
             picks = [(r, o) for r, key in enumerate(rows_of) for o in out_at.get(key, ())]
-            for c in range(0, len(picks), 256):
-                part = picks[c:c + 256]
+            for c in range(0, len(picks), self.head_rows):
+                part = picks[c:c + self.head_rows]
                 gather = torch.tensor([r for r, _ in part], dtype=I32, device=self.dev)
                 got = torch.empty((len(part), spec.vocab), dtype=F32, device=self.dev)
                 self._logits(b, done, len(part), got, gather)

@@ -180,8 +180,8 @@ def hybrid_layers(layers):
 
 def zekilix_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
     from .hybrid import HybridSpec
-    return HybridSpec("zekilix", hybrid_layers(cfg["layers"]), cfg["width"], cfg["vocab"], cfg["streams"], cfg["norm"]["eps"],
-                      cfg["residual_mult"], cfg["embedding"]["scale"], cfg["logit_softcap"], max_len, batch, pad_id, eos_id,
+    return HybridSpec("zekilix", hybrid_layers(cfg["layers"]), cfg["width"], cfg["vocab"], cfg.get("streams") or 1,
+                      cfg["norm"]["eps"], cfg["residual_mult"], cfg["embedding"]["scale"], cfg.get("logit_softcap") or 0.0, max_len, batch, pad_id, eos_id,
                       early_stop, topk, dtype)
 
 
@@ -215,6 +215,9 @@ def hybrid_weights(tensors, spec, device="cuda"):
 
         def connect(q):
             hc = p + f"hc{q}."
+            if S == 1 and hc + "in" not in tensors:            # a plain residual
+                one = torch.ones(1, dtype=torch.float32, device=device)
+                return (one, one, one)
             return (vec(hc + "in", S), vec(hc + "out", S), get(hc + "mix", (S, S)).float().contiguous())
 
         N = m.out_channels

@@ -8,5 +8,7 @@ from .rms_layer_norm import RMSLayerNorm
 from .embedding import Embedding
 from .mlp import MLP
 from .lm_head import LMHead
+from .streams import NamedLinear, StreamConnection, WeightNorm
 
-__all__ = ["BaseLayer", "Linear", "LayerNorm", "RMSLayerNorm", "Embedding", "MLP", "LMHead"]
+__all__ = ["BaseLayer", "Linear", "LayerNorm", "RMSLayerNorm", "Embedding", "MLP", "LMHead", "NamedLinear", "StreamConnection",
+           "WeightNorm"]

@@ -49,8 +49,9 @@ REGISTRY.reset()
 
 class TensorType:
     """Activation dtype per precision (reference: utils/tensor_type.py:17-33): the INT4 and FP8 modes
-    compute on fp16 activations."""
-    all_precision = ["fp32", "fp16", "int4", "fp8", "fp8_weight"]
+    compute on fp16 activations.  'bf16' graphs are recorded in fp32 (numpy has no bf16, and fp32 holds bf16 weights
+    exactly); the executor multiplies in bf16."""
+    all_precision = ["fp32", "fp16", "int4", "fp8", "fp8_weight", "bf16"]
 
     def __init__(self, precision):
         assert precision in self.all_precision
@@ -58,11 +59,11 @@ class TensorType:
 
     @property
     def np_float_type(self):
-        return np.float32 if self.precision == "fp32" else np.float16
+        return np.float32 if self.precision in ("fp32", "bf16") else np.float16
 
     @property
     def popart_float_type(self):
-        return "FLOAT" if self.precision == "fp32" else "FLOAT16"
+        return "FLOAT" if self.precision in ("fp32", "bf16") else "FLOAT16"
 
 
 class DeviceScope:

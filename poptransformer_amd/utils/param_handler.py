@@ -84,7 +84,7 @@ class _Fp8Weight(_Fp8):
     cast_activations = False
 
 
-PrecisionStrategyMap = {"fp16": _Float(), "fp32": _Float(), "int4": _Int4(), "fp8": _Fp8(), "fp8_weight": _Fp8Weight()}
+PrecisionStrategyMap = {"fp16": _Float(), "fp32": _Float(), "bf16": _Float(), "int4": _Int4(), "fp8": _Fp8(), "fp8_weight": _Fp8Weight()}
 
 
 class ParamHandler:

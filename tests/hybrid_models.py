@@ -1,0 +1,94 @@
+"""Small configurations and random tensors of hybrid decoders for the tests."""
+import numpy as np
+
+
+def attention(heads=4, kv_heads=2, dim=16, window=12, scale=None, mlp=None, of=None):
+    c = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+                                        "scale": dim ** -0.5 if scale is None else scale}, "mlp": mlp}
+    if window is not None:
+        c["mixer"]["mask"] = {"size": window}
+    if of is not None:
+        c["weights_of"] = of
+    return c
+
+
+def mlstm(heads=3, dim=24, vdim=40, cap=7.0, mlp=None, of=None):
+    c = {"type": "mlstm", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": cap}, "mlp": mlp}
+    if of is not None:
+        c["weights_of"] = of
+    return c
+
+
+def dense(ff=56, limit=0.9):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def config(layers, width=80, vocab=112, streams=3, eps=1e-5, mult=0.35, embed=3.0, cap=9.0):
+    c = {"architecture": "Zekilix", "embedding": {"scale": embed}, "layers": layers, "logit_softcap": cap, "norm": {"eps": eps},
+         "residual_mult": mult, "vocab": vocab, "width": width}
+    if streams is not None:
+        c["streams"] = streams
+    return c
+
+
+def small_config(**kw):
+    """Both mixers, a layer without a feed-forward, and both kinds used a second time."""
+    return config([mlstm(mlp=dense()), attention(mlp=dense(ff=64, limit=1.3)), mlstm(heads=2, dim=16, vdim=32, mlp=None),
+                   attention(mlp=dense(ff=64, limit=1.3), of=1), mlstm(mlp=dense(), of=0)], **kw)
+
+
+def bf16(a):
+    """fp32 values that bf16 holds exactly (round to nearest even)."""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32).view(np.float32)
+
+
+def random_tensors(cfg, seed, forget_bias=2.0):
+    rng = np.random.default_rng(seed)
+    d, V, S = cfg["width"], cfg["vocab"], cfg.get("streams")
+    sd = {}
+
+    def lin(name, n, k, gain=1.0):
+        sd[name] = bf16(rng.standard_normal((n, k)) * gain / np.sqrt(k))
+
+    def vec(name, n, mean=1.0, spread=0.2):
+        sd[name] = bf16(mean + spread * rng.standard_normal(n))
+
+    def connect(name):
+        vec(name + ".in", S, 0.6, 0.2)
+        vec(name + ".out", S, 0.8, 0.2)
+        sd[name + ".mix"] = bf16(np.eye(S) * 0.8 + 0.15 * rng.standard_normal((S, S)))
+
+    sd["embed"] = bf16(rng.standard_normal((V, d)))
+    for i, lay in enumerate(cfg["layers"]):
+        if lay.get("weights_of") is not None:
+            continue
+        p, m = f"l{i}.", lay["mixer"]
+        vec(p + "norm1", d)
+        if S is not None:
+            connect(p + "hc1")
+        if lay["type"] == "attention":
+            N, KD = m["heads"] * m["dim"], m["kv_heads"] * m["dim"]
+            for n, c in (("q", N), ("k", KD), ("g", N)):
+                lin(p + "mix." + n, c, d)
+            vec(p + "mix.q.norm", N, 1.3)
+            vec(p + "mix.k.norm", KD, 1.3)
+        else:
+            N, QD = m["heads"] * m["vdim"], m["heads"] * m["dim"]
+            for n, c in (("q", QD), ("k", QD), ("v", N), ("g", N), ("i", m["heads"]), ("f", m["heads"])):
+                lin(p + "mix." + n, c, d)
+            vec(p + "mix.i.b", m["heads"], -0.5, 0.5)
+            vec(p + "mix.f.b", m["heads"], forget_bias, 0.5)
+            vec(p + "mix.norm", N)
+        lin(p + "mix.o", d, N)
+        if lay.get("mlp") is not None:
+            ff = lay["mlp"]["ff"]
+            vec(p + "norm2", d)
+            if S is not None:
+                connect(p + "hc2")
+            lin(p + "mlp.gate", ff, d)
+            lin(p + "mlp.up", ff, d)
+            lin(p + "mlp.down", d, ff)
+    vec("final.norm", d)
+    lin("head", V, d, 2.0)
+    return sd

@@ -1,0 +1,307 @@
+"""Whole hybrid decoders against the plain evaluation of oracle/zekilix.py: prompts, decoding, portions, batches, slots that
+are used again, generation through the session, and the trace runner."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+from oracle import zekilix as Z
+from tests.hybrid_models import attention, bf16, config, dense, mlstm, random_tensors, small_config
+
+pytestmark = pytest.mark.gpu
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+ODD = config([attention(heads=3, kv_heads=1, dim=20, window=7, mlp=dense(ff=36, limit=2.0)), mlstm(heads=1, dim=12, vdim=20, cap=3.0),
+              mlstm(heads=5, dim=20, vdim=4, mlp=dense(ff=20)), attention(heads=1, kv_heads=1, dim=44, window=None),
+              attention(heads=5, kv_heads=5, dim=9, window=1, mlp=dense(ff=12)), mlstm(heads=5, dim=20, vdim=4, mlp=dense(ff=20), of=2)],
+             width=52, vocab=91, streams=2, embed=1.0)
+ALIKE = config([attention(heads=2, kv_heads=2, dim=32, window=64, mlp=dense(ff=64, limit=1.0)),
+                mlstm(heads=2, dim=32, vdim=32, cap=1.0, mlp=dense(ff=64, limit=1.0)),
+                attention(heads=2, kv_heads=2, dim=32, window=64, mlp=dense(ff=64, limit=1.0), of=0)],
+               width=64, vocab=64, streams=1, mult=1.0, embed=1.0, cap=1.0)
+PLAIN = config([mlstm(mlp=dense()), attention(window=5)], streams=None)
+WIDE = config([attention(heads=8, kv_heads=2, dim=136, window=90, mlp=dense(ff=1100)), mlstm(heads=2, dim=130, vdim=200, mlp=dense(ff=1100)),
+               mlstm(heads=1, dim=300, vdim=64)], width=1032, vocab=300, streams=4)
+CONFIGS = {"small": small_config(), "odd": ODD, "alike": ALIKE, "plain": PLAIN, "wide": WIDE}
+
+
+def _decoder(cfg, sd, dtype, max_len=400, slots=2, pass_rows=None, batch=1, **kw):
+    from poptransformer_amd.engine import hybrid, loader
+    spec = loader.zekilix_spec(cfg, max_len, batch, dtype=dtype, **kw)
+
+    class Decoder(hybrid.HybridDecoder):
+        pass
+    if pass_rows:
+        Decoder.pass_rows = pass_rows
+    return Decoder(spec, loader.hybrid_weights(sd, spec), slots=slots)
+
+
+def _ids(seed, n, cfg):
+    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
+
+
+class Expected:
+    """The oracle's logits of one sequence, and per number format how far from them a result may be: the rms of the
+    difference over the rms of all logits is compared with what rounding alone does to this very sequence (fp32 accumulates
+    in another order: a floor)."""
+
+    def __init__(self, sd, cfg, ids, dtype):
+        self.logits = Z.forward(sd, cfg, ids)
+        self.scale = np.sqrt((self.logits ** 2).mean())
+        if dtype == "float32":
+            self.limit = 1e-4
+        else:
+            # (three roundings: one sample of what rounding does says little about a single position)
+            draws = [self.error(Z.forward(sd, cfg, ids, rnd=lambda a, k=k: bf16(a * (1 + k)) / (1 + k))).max() for k in (0, 0.13, 0.31)]
+            self.limit = 2.0 * max(draws) + 0.01
+
+    def error(self, got, at=slice(None)):
+        return np.sqrt(((got - self.logits[at]) ** 2).mean(-1)) / self.scale
+
+    def check(self, got, at=slice(None)):
+        got = got.float().cpu().numpy() if torch.is_tensor(got) else got
+        err = self.error(got, at)
+        assert err.max() < self.limit, f"place {int(err.argmax())}: {err.max():.2e}, limit {self.limit:.2e}"
+
+
+def _feed(dec, slot, ids, cuts):
+    """The tokens in portions of the given sizes (the rest one by one); logits of all positions."""
+    out, p, cuts = [], 0, list(cuts)
+    while p < len(ids):
+        c = min(cuts.pop(0) if cuts else 1, len(ids) - p)
+        out.append(dec.advance([(slot, ids[p:p + c], list(range(c)))]).cpu().numpy())
+        p += c
+    return np.concatenate(out)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_prompts_portions_and_decoding(name, dtype):
+    cfg = CONFIGS[name]
+    sd = random_tensors(cfg, 5)
+    T = 150
+    ids = _ids(1, T, cfg)
+    want = Expected(sd, cfg, ids, dtype)
+    dec = _decoder(cfg, sd, dtype)
+    for cuts in ((T,), (2, 2, 3, 64, 65), (1, 70, 2, 63), (100,), (1,)):
+        print(f"{name} {dtype} cuts {cuts}", flush=True)
+        s = dec.open()                       # the slot of the sequence before
+        want.check(_feed(dec, s, ids, cuts))
+        dec.close(s)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_a_short_sequence_from_its_first_token(dtype):
+    cfg = small_config()
+    sd = random_tensors(cfg, 6)
+    dec = _decoder(cfg, sd, dtype)
+    for n in (1, 2, 3):
+        ids = _ids(n, n, cfg)
+        for cuts in ((n,), (1,)):
+            s = dec.open()
+            Expected(sd, cfg, ids, dtype).check(_feed(dec, s, ids, cuts))
+            dec.close(s)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_unequal_batches_against_each_alone_and_slots_used_again(dtype):
+    """Prompts of very different lengths in one batch, decoded together while the shorter ones end; then other sequences in
+    the slots that were given back, and more sequences than there were slots."""
+    cfg = small_config()
+    sd = random_tensors(cfg, 7)
+    dec = _decoder(cfg, sd, dtype, slots=1)
+    for round_, lens in enumerate(((1, 90, 33, 140), (130, 2, 64), (65, 17, 1, 3, 80, 129))):
+        seqs = [_ids(10 * round_ + i, n + 12, cfg) for i, n in enumerate(lens)]
+        want = [Expected(sd, cfg, q, dtype) for q in seqs]
+        slots = [dec.open() for _ in seqs]
+        got = dec.advance([(s, q[:n], list(range(n))) for s, q, n in zip(slots, seqs, lens)]).cpu().numpy()
+        at = 0
+        for n, w in zip(lens, want):
+            w.check(got[at:at + n], slice(0, n))
+            at += n
+        live = list(range(len(seqs)))
+        for t in range(12):
+            got = dec.advance([(slots[i], [seqs[i][lens[i] + t]], [0]) for i in live]).cpu().numpy()
+            for r, i in enumerate(live):
+                want[i].check(got[r:r + 1], [lens[i] + t])
+            if t % 3 == 2 and len(live) > 1:
+                dec.close(slots[live.pop(0)])
+        for i in live:
+            dec.close(slots[i])
+    assert dec.store.capacity >= 6
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_mixed_batches_and_passes_smaller_than_a_prompt(dtype):
+    """Sequences that decode beside sequences that bring portions, and prompts cut into passes by the row limit (the cut
+    falls inside sequences, the windowed rings wrap several times)."""
+    cfg = small_config()
+    sd = random_tensors(cfg, 8)
+    dec = _decoder(cfg, sd, dtype, slots=3, pass_rows=48)
+    seqs = [_ids(30 + i, 170, cfg) for i in range(3)]
+    want = [Expected(sd, cfg, q, dtype) for q in seqs]
+    slots = [dec.open() for _ in seqs]
+    at = [0, 0, 0]
+    for counts in ((100, 1, 20), (1, 60, 2), (2, 1, 1), (1, 1, 1), (50, 50, 50), (3, 2, 90)):
+        entries, rows = [], []
+        for i, c in enumerate(counts):
+            entries.append((slots[i], seqs[i][at[i]:at[i] + c], [c - 1, 0]))       # wanted places in any order
+            rows += [(i, at[i] + c - 1), (i, at[i])]
+            at[i] += c
+        got = dec.advance(entries).cpu().numpy()
+        for r, (i, p) in enumerate(rows):
+            want[i].check(got[r:r + 1], [p])
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_decoding(dtype):
+    """Several windows and ring lengths of decoded tokens (the ring of a decoder whose passes are short wraps often)."""
+    cfg = small_config()
+    sd = random_tensors(cfg, 9, forget_bias=5.0)
+    dec = _decoder(cfg, sd, dtype, max_len=700, pass_rows=16)
+    ids = _ids(2, 600, cfg)
+    s = dec.open()
+    Expected(sd, cfg, ids, dtype).check(_feed(dec, s, ids, (16,)))
+
+
+def test_requests_that_do_not_fit_are_refused():
+    cfg = small_config()
+    dec = _decoder(cfg, random_tensors(cfg, 1), "float32", max_len=20)
+    s = dec.open()
+    for bad in ([(s, [], [])], [(s, list(range(21)), [])], [(s, [cfg["vocab"]], [])], [(s, [1], [1])], [(s, [1], []), (s, [2], [])],
+                [(1 - s, [1], [])]):
+        with pytest.raises(ValueError):
+            dec.advance(bad)
+    dec.close(s)
+    with pytest.raises(ValueError):
+        dec.close(s)
+
+
+# ------------------------------------------------------------------------------------------- generation
+def _greedy(cfg, sd, ids, steps, pad, tie):
+    """The loop by the oracle: container after `steps` iterations, and per row the number of comparable columns (up to the
+    first place where two logits are closer than `tie` of the largest)."""
+    out = ids.copy()
+    B, L = ids.shape
+    cols = np.full(B, min(steps + 1, L))
+    for b in range(B):
+        for t in range(min(steps, L - 1)):
+            if out[b, t + 1] != pad:
+                continue
+            logits = Z.forward(sd, cfg, out[b, :t + 1])[-1]
+            top = np.sort(logits)[-2:]
+            if top[1] - top[0] < tie * np.abs(logits).max():
+                cols[b] = min(cols[b], t + 1)
+            out[b, t + 1] = int(logits.argmax())
+    return out, cols
+
+
+def _session(cfg, sd, precision, B, L, steps, allow_fused=True, **kw):
+    from poptransformer_amd.models.zekilix import ZekilixDecModel
+    from poptransformer_amd.utils import prepare_model_session
+    extra = {k: kw.pop(k) for k in ("topk", "early_stop") if k in kw}
+    model = dict(hf_config=cfg, state_dict=sd, pad_token_id=0, eos_token_id=1, max_length=L, max_loop=steps, **extra)
+    return prepare_model_session({"global_args": {"batch_size": B, "precision": precision}, "model": model,
+                                  "session": dict(kw, allow_fused=allow_fused)}, ZekilixDecModel)
+
+
+@pytest.mark.parametrize("precision,allow_fused", [("fp32", False), ("fp32", True), ("bf16", True)])
+@pytest.mark.parametrize("name", ["small", "odd", "plain"])
+def test_generation_through_the_session(name, precision, allow_fused):
+    cfg = CONFIGS[name]
+    sd = random_tensors(cfg, 11)
+    B, L, steps = 3, 48, 40
+    rng = np.random.default_rng(4)
+    ids = np.zeros((B, L), np.int32)
+    for b, n in enumerate((9, 4, 20)):                       # unequal prompts
+        ids[b, :n] = rng.integers(2, cfg["vocab"], n)
+    session, model = _session(cfg, sd, precision, B, L, steps, allow_fused, **({"strict": True} if allow_fused else {}))
+    assert session.executor_kind == ("fused:zekilix" if allow_fused else "interpreter"), session.fallback_reason
+    want, cols = _greedy(cfg, sd, ids, steps, 0, 1e-4 if precision == "fp32" else 0.05)
+    for _ in range(2):                                       # the second run starts from a used cache
+        session.run(model.build_input_dict(input_ids=[list(r[r != 0]) for r in ids]))
+        got = session.anchor_arrays["Loop:0"]
+        for b in range(B):
+            assert np.array_equal(got[b, :cols[b]], want[b, :cols[b]]), f"row {b}"
+    lens = (ids != 0).sum(1)
+    assert (cols - lens).clip(0).sum() >= (30 if precision == "fp32" else 3)         # generated tokens were compared
+
+
+def test_generation_ends_early_and_draws_from_the_top_k():
+    cfg = small_config()
+    sd = random_tensors(cfg, 12)
+    session, model = _session(cfg, sd, "fp32", 2, 40, 30, topk=4, strict=True)
+    session.run(model.build_input_dict(input_ids=[[5, 6, 7], [8, 9, 10, 11]]))
+    got = session.anchor_arrays["Loop:0"]
+    assert session.executor_kind == "fused:zekilix"
+    for b in range(2):
+        n = 4 + 20
+        logits = Z.forward(sd, cfg, got[b, :n])
+        for t in range(4, n - 1):
+            assert got[b, t + 1] in np.argsort(-logits[t])[:5]
+    session, model = _session(cfg, sd, "fp32", 1, 40, 39, early_stop=True, strict=True)
+    session.run(model.build_input_dict(input_ids=[[5, 1, 7]]))          # the end token is in the prompt
+    assert int(np.asarray(session.anchor_arrays["Loop:1"]).reshape(-1)[0]) < 39
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_prompt_passes_leave_what_the_loop_leaves(dtype):
+    cfg = small_config()
+    sd = random_tensors(cfg, 13)
+    B, L, n = 3, 120, 90
+    ids = np.zeros((B, L), np.int32)
+    ids[:, :n] = np.random.default_rng(0).integers(2, cfg["vocab"], (B, n))
+    want = [Expected(sd, cfg, ids[b, :n], dtype) for b in range(B)]
+
+    def check():
+        for b in range(B):
+            want[b].check(dec.logits[b:b + 1], [n - 1])
+    dec = _decoder(cfg, sd, dtype, max_len=L, batch=B)
+    dec.capture()
+    for passes in (None, 7, 64):
+        dec.reset(ids)
+        done = dec.consume_prompt(n - 1, rows_per_pass=passes) if passes else 0
+        dec.run_steps(n - done)                              # replays, the last one on the prompt's last token
+        torch.cuda.synchronize()
+        assert int(dec.step.item()) == n
+        check()
+    for _ in range(3):                                       # replays between eager work give what eager iterations give
+        dec.reset(ids)
+        dec.run_steps(n)
+        torch.cuda.synchronize()
+        check()
+
+
+# ------------------------------------------------------------------------------------------- trace runner
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_runner(tmp_path, dtype):
+    from safetensors.torch import save_file
+    cfg = small_config()
+    sd = random_tensors(cfg, 14)
+    model, out = tmp_path / "model", tmp_path / "out"
+    model.mkdir()
+    out.mkdir()
+    (model / "config.json").write_text(json.dumps(cfg))
+    save_file({k: torch.from_numpy(v).to(torch.bfloat16) for k, v in sd.items()}, str(model / "model.safetensors"))
+    a, b = _ids(1, 40, cfg), _ids(2, 7, cfg)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:30], "want": [29, 0]}, {"id": "b", "tokens": b[:5], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "b", "tokens": b[5:6], "want": [0]}, {"id": "a", "tokens": a[30:31], "want": [0]}], "end": ["b"]},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[31:32], "want": []}], "end": ["a"]},
+             {"step": 3, "entries": [{"id": "c", "tokens": b, "want": [6]}], "end": ["c"]}]
+    run = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(model), "--dtype", dtype, "--out",
+                          str(out), "--max-tokens", "64"], input="".join(json.dumps(s) + "\n" for s in steps), text=True,
+                         capture_output=True, timeout=100)
+    assert run.returncode == 0, run.stderr[-2000:]
+    assert [x for x in run.stdout.splitlines() if x.startswith("done ")] == ["done 0", "done 1", "done 2", "done 3"]
+    wa, wb = Expected(sd, cfg, a, dtype), Expected(sd, cfg, b, dtype)
+    want = {0: [(wa, 29), (wa, 0)], 1: [(wb, 5), (wa, 30)], 3: [(wb, 6)]}
+    assert sorted(os.listdir(out)) == [f"{k}.f32" for k in want]
+    for k, rows in want.items():
+        got = np.fromfile(out / f"{k}.f32", "<f4").reshape(len(rows), -1)
+        for r, (w, p) in enumerate(rows):
+            w.check(got[r:r + 1], [p])
