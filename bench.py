@@ -26,7 +26,9 @@ bytes; or, with the per-operator executor, the fused INT4 gate/up projection), a
 Other workloads (``--workload``), each printing one line of the same form: ``gemm`` = the single INT4
 weight-only operator X[M, 4096] by W[4096, 11008] at M = ``--batch``; ``chatglm2`` = ChatGLM2-6B-shape FP8
 decode; ``rwkv`` = RWKV-4-7B-shape INT4 recurrent decode; ``prompt`` = the prompt of the headline model taken in
-passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration.  ``--copy-calibration`` and ``--summarize-pmc``
+passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix`` = the
+Zekilix design (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights at the same sizes: decode at batch
+1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
 serve the hardware-counter measurement of the HBM traffic (see their help).
 """
 import argparse
@@ -420,6 +422,118 @@ def prompt_workload(args):
     }
 
 
+def zekilix_config(width, ff, layers):
+    """Half windowed-attention, half matrix-memory layers of one size (heads of 128; memories of 256 x 512)."""
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    attention = {"type": "attention", "mlp": dense, "mixer": {"heads": width // 128, "kv_heads": width // 512, "dim": 128, "vdim": 128,
+                                                            "scale": 128 ** -0.5, "mask": {"size": 1024}}}
+    memory = {"type": "mlstm", "mlp": dense, "mixer": {"heads": width // 512, "dim": 256, "vdim": 512, "gate_cap": 15.0}}
+    return {"architecture": "Zekilix", "embedding": {"scale": 1.0}, "layers": [attention, memory] * (layers // 2), "logit_softcap": 30.0,
+            "norm": {"eps": 1e-5}, "residual_mult": 1.0, "streams": 2, "vocab": 32000, "width": width}
+
+
+def hybrid_step_bytes(spec, weights, B, t):
+    """Bytes one decode iteration of a hybrid decoder must move at context t: the weights of every layer run, the key rows
+    of the windows, the memories (read and written), the head."""
+    n = weights.head.nbytes
+    for lay in spec.layers:
+        n += sum(w.nbytes for w in weights.layers[lay.source].linears())
+        m = lay.mixer
+        if m.kind == "attention":
+            n += B * m.kv_heads * (2 * m.dim + 4 / m.kv_heads) * min(t + 1, m.window or t + 1)
+        else:
+            n += B * 2 * 4 * m.heads * m.dim * (m.vdim + 1)
+    return n
+
+
+def zekilix_workload(args):
+    """Decode iterations (contexts 1024 .. 1024 + steps - 1, replayed from a HIP graph, one launch per operator) and prompt
+    passes of the Zekilix design, and of the Llama-2 executor with fp16 weights at equal width, feed-forward size, layer
+    count, vocabulary and head size.  --layers shortens both models (for profiles)."""
+    import torch
+    from poptransformer_amd.engine import fused, hybrid, loader, synthetic
+    rng = np.random.Generator(np.random.PCG64(1234))
+    first, steps, max_len = 1024, args.steps, 2048
+    results = []
+
+    def timed(fn):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        fn()
+        torch.cuda.synchronize()
+        return time.perf_counter() - t0
+
+    for width, ff, layers in ((2048, 5632, 8), (4096, 11008, 8)):
+        if args.width and args.width != width:
+            continue
+        layers = args.layers or layers
+        cfg = zekilix_config(width, ff, layers)
+        lcfg = dict(LLAMA2_7B, hidden_size=width, intermediate_size=ff, num_attention_heads=width // 128, num_hidden_layers=layers)
+        makers = {}
+        if args.only != "llama2":
+            spec = loader.zekilix_spec(cfg, max_len, 1)
+            hw = loader.hybrid_weights(synthetic.HybridTensors(cfg), spec)
+            makers["zekilix"] = (lambda B: hybrid.HybridDecoder(loader.zekilix_spec(cfg, max_len, B), hw),
+                                 lambda B, t: hybrid_step_bytes(spec, hw, B, t), sum(w.n_main * w.K for lay in spec.layers for w in
+                                                                                    hw.layers[lay.source].linears()))
+        if args.only != "zekilix":
+            lw = synthetic.llama2_f16_synthetic_weights(lcfg)
+            makers["llama2_fp16"] = (lambda B: fused.FusedDecoder(loader.llama2_spec(lcfg, max_len, B), lw),
+                                     lambda B, t: lw.nbytes() + B * layers * 4 * width * (t + 1), layers * (4 * width * width + 3 * width * ff))
+        row = {"width": width, "ff": ff, "layers": layers}
+        for name, (make, step_bytes, params) in makers.items():
+            r = row[name] = {"linear_parameters": params}
+            for B in (1, 16):
+                if args.rows_only:
+                    break
+                dec = make(B)
+                dec.capture()
+                ids = np.zeros((B, max_len), np.int32)
+                ids[:, :first] = rng.integers(3, 32000, (B, first))
+                dec.reset(ids)
+                n = dec.consume_prompt(dec.prompt_positions())
+                dec.run_steps(first - n + args.warmup + 8)
+                dt = timed(lambda: dec.run_steps(steps))
+                t = first + args.warmup + 8
+                nbytes = float(np.mean([step_bytes(B, c) for c in range(t, t + steps)]))
+                r[f"decode_b{B}"] = {"ms_per_step": dt / steps * 1e3, "tokens_per_s": B * steps / dt,
+                                     "hbm_frac": nbytes / (dt / steps) / (HBM_PEAK_GBS * 1e9)}
+                note(f"{name} width {width} batch {B}: {dt / steps * 1e3:.4f} ms per step")
+                del dec
+                torch.cuda.empty_cache()
+            for rows in (512, 2048):
+                if args.decode_only:
+                    break
+                L = rows + 2
+                spec_L = (lambda B: hybrid.HybridDecoder(loader.zekilix_spec(cfg, L, B), hw)) if name == "zekilix" else \
+                    (lambda B: fused.FusedDecoder(loader.llama2_spec(lcfg, L, B), lw))
+                dec = spec_L(1)
+                ids = np.zeros((1, L), np.int32)
+                ids[:, :rows + 1] = rng.integers(3, 32000, (1, rows + 1))
+
+                def one():
+                    dec.reset(ids)
+                    dec.consume_prompt(rows, rows_per_pass=rows)
+                for _ in range(3):
+                    one()
+                best = min(timed(one) for _ in range(5))
+                r[f"prompt_{rows}"] = {"ms": best * 1e3, "tokens_per_s": rows / best, "linear_tflops": 2e-12 * rows * params / best}
+                note(f"{name} width {width} prompt {rows}: {best * 1e3:.3f} ms")
+                del dec
+                torch.cuda.empty_cache()
+        results.append(row)
+        makers.clear()
+        hw = lw = None
+        torch.cuda.empty_cache()
+    last = results[-1].get("zekilix") or results[-1]["llama2_fp16"]
+    head = last.get("decode_b1") or {"tokens_per_s": last["prompt_2048"]["tokens_per_s"], "ms_per_step": last["prompt_2048"]["ms"]}
+    return {"metric": "decode tokens/s", "value": head["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": args.warmup,
+            "ms_per_step": head["ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16 weights and activations, f32 accumulation, residual and state", "data": "synthetic",
+            "config": {"workload": "Zekilix-shaped decode at batch 1 beside Llama-2 with fp16 weights at equal size", "executor": "operators"},
+            "sizes": results}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -430,11 +544,17 @@ def main():
     ap.add_argument("--batch", type=int, default=1)
     ap.add_argument("--executor", choices=["persistent", "operators"], default=None,
                     help="default: persistent when the batch fits it (<= 16, fp16 cache), else operators")
-    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix"], default="decode",
                     help="decode: the Llama2-7B-shape INT4 decode loop (the headline); gemm: the single INT4 "
                          "weight-only operator at M = --batch rows; chatglm2: ChatGLM2-6B-shape FP8 decode; "
                          "rwkv: RWKV-4-7B-shape INT4 recurrent decode; prompt: the headline model's prompt in passes "
-                         "of --rows-per-pass rows (--steps passes)")
+                         "of --rows-per-pass rows (--steps passes); zekilix: the Zekilix design beside Llama-2 with fp16 weights at "
+                         "equal sizes, decode and prompts")
+    ap.add_argument("--width", type=int, default=0, help="zekilix workload: only this width")
+    ap.add_argument("--layers", type=int, default=0, help="zekilix workload: layers of both models (even)")
+    ap.add_argument("--only", choices=["zekilix", "llama2"], default=None, help="zekilix workload: one of the two models")
+    ap.add_argument("--decode-only", action="store_true", help="zekilix workload: no prompts")
+    ap.add_argument("--rows-only", action="store_true", help="zekilix workload: prompts only")
     ap.add_argument("--rows-per-pass", type=int, default=64,
                     help="prompt workload: rows (batch x positions) per pass, up to 2048")
     ap.add_argument("--fp8-cache", action="store_true",
@@ -482,6 +602,9 @@ def main():
         return
     if args.workload == "prompt":
         print(json.dumps(prompt_workload(args)))
+        return
+    if args.workload == "zekilix":
+        print(json.dumps(zekilix_workload(args)))
         return
     B, cfg = args.batch, LLAMA2_7B
     executor = args.executor or ("persistent" if B <= 16 else "operators")

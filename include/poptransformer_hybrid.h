@@ -145,7 +145,7 @@ int pta_window_decode(const pta_window_attention_args* host_args, pta_stream_t s
  * Per head, with log gates i = cap tanh(z_i / cap), f = log sigmoid(cap tanh(z_f / cap)) from the fp32 pre-activations:
  *   m' = max(f + m, i);  S = exp(f + m - m') S + exp(i - m') k v^T;  n likewise with k alone;
  *   o = S^T q / (max(|n . q|, exp(-m')) + 1e-6),  q scaled by D^-1/2.
- * State of a layer, fp32: [slots][H][slices][D * PTA_MLSTM_SLICE + D + 1]: a head's columns of S (E of them, in slices of
+ * State of a layer, fp32: [slots][H][slices][D * PTA_MLSTM_SLICE + D + 2, up to a multiple of 4]: a head's columns of S (E of them, in slices of
  * PTA_MLSTM_SLICE, each [D][PTA_MLSTM_SLICE]), followed by that slice's own copy of n and m. */
 enum { PTA_MLSTM_SLICE = 32 };
 
@@ -163,11 +163,15 @@ typedef struct pta_mlstm_args {
   const int32_t* seq_row; /* [seqs] first row of each sequence of the pass, seq_count its rows                     */
   const int32_t* seq_count;
   int seqs;
+  int longest;            /* rows of the longest sequence of the pass                                              */
   int chunked;            /* bf16: work through the rows in chunks on the matrix unit where D <= 256 (else: one by one) */
   float* o;               /* fp32 [rows, H * E]                                                                    */
+  void* workspace;        /* chunked: pta_mlstm_workspace_bytes (0 where the pass is not cut into segments)        */
+  size_t workspace_bytes;
 } pta_mlstm_args;
 
 size_t pta_mlstm_state_floats(int H, int D, int E);   /* per slot */
+size_t pta_mlstm_workspace_bytes(const pta_mlstm_args* host_args);   /* reads the sizes only */
 int pta_mlstm(const pta_mlstm_args* host_args, pta_stream_t stream);
 
 /* out = (o of each head / its root mean square) * weight * sigmoid(gate); out [rows, out_ld], the rest of a row zero */

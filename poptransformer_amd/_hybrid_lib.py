@@ -35,7 +35,8 @@ WindowArgs = _struct("WindowArgs", [
     ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P), ("out_ld", _I)])
 MlstmArgs = _struct("MlstmArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("E", _I), ("q", _P), ("k", _P), ("v", _P), ("ld", _I), ("gates", _P),
-    ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("chunked", _I), ("o", _P)])
+    ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("longest", _I), ("chunked", _I),
+    ("o", _P), ("workspace", _P), ("workspace_bytes", c_size_t)])
 
 SIGNATURES = {
     "pta_hybrid_last_error": (c_char_p, []),
@@ -49,6 +50,7 @@ SIGNATURES = {
     "pta_window_attention": (_I, [POINTER(WindowArgs), _P]),
     "pta_window_decode": (_I, [POINTER(WindowArgs), _P]),
     "pta_mlstm_state_floats": (c_size_t, [_I, _I, _I]),
+    "pta_mlstm_workspace_bytes": (c_size_t, [POINTER(MlstmArgs)]),
     "pta_mlstm": (_I, [POINTER(MlstmArgs), _P]),
     "pta_head_norm_gate": (_I, [_I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P]),
     "pta_argmax_f32": (_I, [_P, _P, _P, _I, _I, _P]),

@@ -7,10 +7,10 @@ constexpr int SL = PTA_MLSTM_SLICE;
 
 extern "C" size_t pta_mlstm_state_floats(int H, int D, int E) {
   if (H <= 0 || D <= 0 || E <= 0) return 0;
-  const size_t slice = ((size_t)D * SL + D + 1 + 3) / 4 * 4;             // slices start on 16-byte boundaries
+  const size_t slice = ((size_t)D * SL + D + 2 + 3) / 4 * 4;             // slices start on 16-byte boundaries
   return (size_t)H * ((E + SL - 1) / SL) * slice;
 }
-__device__ __forceinline__ size_t slice_floats(int D) { return ((size_t)D * SL + D + 1 + 3) / 4 * 4; }
+__device__ __forceinline__ size_t slice_floats(int D) { return ((size_t)D * SL + D + 2 + 3) / 4 * 4; }
 
 // log input gate and log forget gate from their pre-activations
 __device__ __forceinline__ float log_input_gate(float z, float cap) { return cap * tanhf(z / cap); }
@@ -33,7 +33,8 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(MA a) {
   const int slice = b % slices; b /= slices;
   const int head = b % a.H, seq = b / a.H;
   const int x = threadIdx.x & 7, y = threadIdx.x >> 3, wave = threadIdx.x >> 6;
-  const int D = a.D, row0 = a.seq_row[seq], count = a.seq_count[seq];
+  const bool single = a.rows == a.seqs;                  // one row per sequence: row = sequence
+  const int D = a.D, row0 = single ? seq : a.seq_row[seq], count = single ? 1 : a.seq_count[seq];
   const size_t per = slice_floats(D);
   float* st = a.state + (((size_t)a.slot[row0] * a.H + head) * slices + slice) * per;
   float *st_n = st + (size_t)D * SL, *st_m = st_n + D;
@@ -109,32 +110,45 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(MA a) {
 
 // ------------------------------------------------------------------------------------------
 // In chunks of CT tokens on the matrix unit (bf16, D <= 32 * DT): a workgroup of four waves per (sequence, head, CE value
-// columns = two slices).  With b_t the running sum of the chunk's log forget gates, a_s = i_s - b_s and
+// columns = two slices, segment).  With b_t the running sum of the chunk's log forget gates, a_s = i_s - b_s and
 // M_t = max(m_prev, max_{s <= t} a_s), unrolling the recurrence gives m_t = b_t + M_t and
 //   o_t ~ sum_{s <= t} exp(a_s - M_t) (q_t . k_s) v_s + exp(m_prev - M_t) S_prev^T q_t      (n . q likewise)
 //   S  <- exp(m_prev - M_C) S_prev + sum_s exp(a_s - M_C) k_s v_s^T
 // Everything but the projections is held in fp32; where such a value has to enter the bf16 matrix unit (the weighted
 // products, the weighted values, S) it goes in as the sum of two bf16 numbers, i.e. with 16 bits.
 //
+// Long sequences are cut into segments that run side by side.  A first launch (OUTPUTS = false) leaves in `parts` what each
+// segment but the last adds to the state (from an empty one; the first segment from the sequence's own), its m and the sum
+// of its log forget gates; in the second launch a segment puts the ones before it together,
+//   m' = max(m + B_i, m_i),  S' = exp(m + B_i - m') S + exp(m_i - m') S_i,
+// and goes on from there.  Place 0 of `parts` keeps the state the sequence came with: the last segment overwrites it.
+//
 // Wave w computes the outputs of tokens 16 w .. 16 w + 15 (as columns: P^T = K Q^T, O^T = V^T P^T + S^T Q^T) and owns rows
-// d = w * DW .. of S (DW = 8 DT) in its accumulators.  The transposed values hold their tokens in the order in which a
-// lane of the product P^T holds them (see window_tile_kernel); the transposed keys, and the weighted values beside them,
-// in plain order.
+// d = w * DW .. of S in its accumulators.  The transposed values hold their tokens in the order in which a lane of the
+// product P^T holds them (key 4 x + e of the first sixteen of 32 in place 8 x + e, of the second in 8 x + 4 + e); the
+// transposed keys, and the weighted values beside them, in plain order.  The next chunk's rows are requested while a chunk
+// is worked on.
 // ------------------------------------------------------------------------------------------
 constexpr int CT = 64, CE = 2 * SL;
 constexpr int CS = CT + 8;
 
-template <int DT>
-__global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
-  constexpr int DM = DT * 32, KS = DM + 8, CH = DM / 8, TD = DT;      // TD 16-row tiles of S per two waves' share: DM / 64 = DT / 2
-  constexpr int ST = (DM / 4 + 15) / 16;                              // 16-row tiles of S per wave
-  constexpr int DW = ST * 16;
-  constexpr int DS = DW * 4;                                          // rows of S the waves cover (>= DM)
-  constexpr int SS = DS + 8;
+template <int DT> struct ChunkShape {
+  static constexpr int DM = DT * 32, KS = DM + 8, CH = DM / 8;
+  static constexpr int ST = (DM / 4 + 15) / 16;                       // 16-row tiles of S per wave
+  static constexpr int DW = ST * 16, DS = DW * 4, SS = DS + 8;        // DS >= DM rows of S in all
+  static constexpr int KT = DS * CS + DS;                             // transposed keys: row d starts at d * CS + (d / 8) * 8
+  static constexpr size_t lds = 2 * ((size_t)CT * KS + KT + CE * CS + 2 * CE * (size_t)(SS > CS ? SS : CS));
+};
+
+template <int DT, bool OUTPUTS>
+__global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int segment, int segments, float* parts) {
+  typedef ChunkShape<DT> C;
+  constexpr int DM = C::DM, KS = C::KS, CH = C::CH, ST = C::ST, DW = C::DW, DS = C::DS, SS = C::SS;
+  constexpr int IPT = (CT / 2 * CH + 255) / 256;                      // (pair of keys, 16-byte piece) items per thread
   extern __shared__ __align__(16) unsigned char smem[];
   bf16* sk = reinterpret_cast<bf16*>(smem);                           // [CT][KS] keys
-  bf16* skt = sk + CT * KS;                                           // [DS][CS] keys transposed
-  bf16* svt = skt + DS * CS;                                          // [CE][CS] values transposed, permuted
+  bf16* skt = sk + CT * KS;                                           // keys transposed
+  bf16* svt = skt + C::KT;                                            // [CE][CS] values transposed, permuted
   bf16* big = svt + CE * CS;
   bf16* ss_hi = big;                                                  // [CE][SS] S transposed, two parts
   bf16* ss_lo = big + CE * SS;
@@ -142,107 +156,164 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
   bf16* sw_lo = big + CE * CS;
   __shared__ float s_n[DM], s_a[CT], s_M[CT], s_b[CT], s_w[CT];
   __shared__ float s_m;
-  (void)TD;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15;
   const int slices = (a.E + SL - 1) / SL, groups = (slices + 1) / 2;
   int blk = blockIdx.x;
   const int grp = blk % groups; blk /= groups;
-  const int head = blk % a.H, seq = blk / a.H;
-  const int D = a.D, E = a.E, row0 = a.seq_row[seq], count = a.seq_count[seq];
+  const int head = blk % a.H; blk /= a.H;
+  const int seg = blk % segments, seq = blk / segments;
+  const int total = a.seq_count[seq], first = seg * segment;
+  const bool final_seg = first + segment >= total;                    // ... of its sequence
+  if (first >= total || (!OUTPUTS && final_seg)) return;
+  const int D = a.D, E = a.E, count = total - first < segment ? total - first : segment;
+  const int row_s = a.seq_row[seq], row0 = row_s + first;
   const int e0 = grp * CE, ecols = E - e0 < CE ? E - e0 : CE;
   const size_t per = slice_floats(D);
-  float* st = a.state + (((size_t)a.slot[row0] * a.H + head) * slices + grp * 2) * per;
-  const bool second = grp * 2 + 1 < slices;
+  const size_t pair_at = ((size_t)head * slices + grp * 2) * per, whole = (size_t)a.H * slices * per;
+  float* st = a.state + (size_t)a.slot[row_s] * whole + pair_at;
+  float* part = parts + (size_t)seq * segments * whole + pair_at;     // place j: what segment j starts from (j = 0), or segment j - 1 left
+  const bool second = grp * 2 + 1 < slices, several = total > segment;
   const float qscale = 1.0f / sqrtf((float)D);
 
-  // S: lane holds rows d = wave * DW + 16 i + 4 lg + 0..3 of column e = 16 j + lc
+  // ---- the chunk's rows on their way to LDS (keys, values), to registers (queries) and the gates
+  u32x4 kr[IPT][2], vr[2], qr[DT];
+  float gi, gf;
+  auto row8 = [&](const void* base, size_t r, size_t at, bool whole8, int left) {
+    const bf16* src = reinterpret_cast<const bf16*>(base) + r * a.ld + at;
+    if (left <= 0) return u32x4{0, 0, 0, 0};
+    if (whole8) return *reinterpret_cast<const u32x4*>(src);
+    bf16x8 z;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) z[e] = e < left ? src[e] : (bf16)0.0f;
+    return bitcast<u32x4>(z);
+  };
+  auto fetch = [&](int t0) {
+    const int cnt = count - t0 < CT ? count - t0 : CT;
+    const size_t rb = (size_t)row0 + t0;
+#pragma unroll
+    for (int it = 0; it < IPT; ++it) {
+      const int idx = threadIdx.x + it * 256, c = idx % CH, kp = idx / CH, left = D - c * 8;
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        const int s = kp * 2 + t;
+        kr[it][t] = row8(a.k, rb + s, (size_t)head * D + c * 8, vec && left >= 8, s < cnt ? left : 0);
+      }
+    }
+    {
+      const int s = threadIdx.x & 63, c0 = (threadIdx.x >> 6) * 16;
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        const int left = s < cnt ? ecols - c0 - h * 8 : 0;
+        vr[h] = row8(a.v, rb + s, (size_t)head * E + e0 + c0 + h * 8, vec && left >= 8 && (E & 7) == 0, left);
+      }
+    }
+    if (OUTPUTS) {
+      const int t = wave * 16 + lc;
+#pragma unroll
+      for (int c = 0; c < DT; ++c) {
+        const int left = D - c * 32 - lg * 8;
+        qr[c] = row8(a.q, rb + (t < cnt ? t : cnt - 1), (size_t)head * D + c * 32 + lg * 8, vec && left >= 8, left);
+      }
+    }
+    gi = -INFINITY;
+    gf = 0.f;
+    if (wave == 0 && lane < cnt) {
+      const float* z = a.gates + (rb + lane) * 2 * a.H + head;
+      gi = log_input_gate(z[0], a.cap);
+      gf = log_forget_gate(z[a.H], a.cap);
+    }
+  };
+  fetch(0);
+
+  // ---- the state at the start.  Lane holds rows d = wave * DW + 16 i + 4 lg + 0..3 of column e = 16 j + lc
   f32x4 S[ST][4];
-  auto state_at = [&](int d, int e) -> float* { return st + (e >= SL ? per : 0) + (size_t)d * SL + (e & (SL - 1)); };
+  float m_prev;
+  const int lane_d = wave * DW + lg * 4, lane_at = lane_d * SL + lc, iper = (int)per;
+  auto each = [&](auto fn) {
+    int base = lane_at;
+    asm volatile("" : "+v"(base));       // the 64 offsets are made anew at every use instead of being kept in registers
 #pragma unroll
-  for (int i = 0; i < ST; ++i)
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
+    for (int i = 0; i < ST; ++i)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int d = wave * DW + i * 16 + lg * 4 + r, e = j * 16 + lc;
-        S[i][j][r] = d < D && (e < SL || second) ? *state_at(d, e) : 0.f;
+        const bool row = lane_d + i * 16 + r < D;
+        const int at = base + (i * 16 + r) * SL;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          S[i][j][r] = fn(S[i][j][r], at + (j & 1) * 16 + (j >> 1) * iper, row && (j < 2 || second));
       }
-  for (int d = threadIdx.x; d < DM; d += 256) s_n[d] = d < D ? st[(size_t)D * SL + d] : 0.f;
-  float m_prev = st[(size_t)D * SL + D];
+  };
+  {
+    const bool empty = !OUTPUTS && seg > 0;
+    // a segment of several starts from what the first launch kept: the state itself is overwritten by the last segment
+    const float* from = OUTPUTS && several ? part + (seg > 0 ? whole : 0) : st;
+    each([&](float, int at, bool there) { return there && !empty ? from[at] : 0.f; });
+    for (int d = threadIdx.x; d < DM; d += 256) s_n[d] = d < D && !empty ? from[(size_t)D * SL + d] : 0.f;
+    m_prev = empty ? -INFINITY : from[(size_t)D * SL + D];
+    if (!OUTPUTS && seg == 0) {                               // keep what the sequence came with
+      each([&](float x, int at, bool there) { if (there) part[at] = x; return x; });
+      for (int d = threadIdx.x; d < D; d += 256) part[(size_t)D * SL + d] = s_n[d];
+      if (threadIdx.x == 0) part[(size_t)D * SL + D] = m_prev;
+    }
+    if (OUTPUTS)
+      for (int j = 2; j <= seg; ++j) {
+        const float* add = part + (size_t)j * whole;
+        const float mi = add[(size_t)D * SL + D], carried = m_prev + add[(size_t)D * SL + D + 1];
+        const float mn = fmaxf(carried, mi), keep = expf(carried - mn), take = expf(mi - mn);
+        each([&](float x, int at, bool there) { return __builtin_fmaf(keep, x, there ? take * add[at] : 0.f); });
+        for (int d = threadIdx.x; d < D; d += 256) s_n[d] = __builtin_fmaf(keep, s_n[d], take * add[(size_t)D * SL + d]);
+        m_prev = mn;
+      }
+  }
+  if (DS > DM)
+    for (int idx = threadIdx.x; idx < (DS - DM) * (CS + 1); idx += 256) skt[DM * (CS + 1) + idx] = (bf16)0.0f;
 
+  float b_total = 0.f;
   for (int t0 = 0; t0 < count; t0 += CT) {
     const int cnt = count - t0 < CT ? count - t0 : CT;
     const size_t rb = (size_t)row0 + t0;
     // ---- S in two bf16 parts, keys and values into LDS, gates
+    if (OUTPUTS) {
 #pragma unroll
-    for (int i = 0; i < ST; ++i)
+      for (int i = 0; i < ST; ++i)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        bf16x4 hi, lo;
+        for (int j = 0; j < 4; ++j) {
+          bf16x4 hi, lo;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          hi[r] = (bf16)S[i][j][r];
-          lo[r] = (bf16)(S[i][j][r] - (float)hi[r]);
-        }
-        const int at = (j * 16 + lc) * SS + wave * DW + i * 16 + lg * 4;
-        *reinterpret_cast<bf16x4*>(ss_hi + at) = hi;
-        *reinterpret_cast<bf16x4*>(ss_lo + at) = lo;
-      }
-    for (int idx = threadIdx.x; idx < CT / 2 * CH; idx += 256) {
-      const int c = idx % CH, kp = idx / CH;
-      u32x4 w[2];
-#pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        const int s = kp * 2 + t, left = D - c * 8;
-        w[t] = u32x4{0, 0, 0, 0};
-        if (s < cnt && left > 0) {
-          const bf16* src = reinterpret_cast<const bf16*>(a.k) + (rb + s) * a.ld + (size_t)head * D + c * 8;
-          if (vec && left >= 8) {
-            w[t] = *reinterpret_cast<const u32x4*>(src);
-          } else {
-            bf16x8 z;
-#pragma unroll
-            for (int e = 0; e < 8; ++e) z[e] = e < left ? src[e] : (bf16)0.0f;
-            w[t] = bitcast<u32x4>(z);
+          for (int r = 0; r < 4; ++r) {
+            hi[r] = (bf16)S[i][j][r];
+            lo[r] = (bf16)(S[i][j][r] - (float)hi[r]);
           }
+          const int at = (j * 16 + lc) * SS + wave * DW + i * 16 + lg * 4;
+          *reinterpret_cast<bf16x4*>(ss_hi + at) = hi;
+          *reinterpret_cast<bf16x4*>(ss_lo + at) = lo;
         }
-        *reinterpret_cast<u32x4*>(sk + s * KS + c * 8) = w[t];
+    }
+#pragma unroll
+    for (int it = 0; it < IPT; ++it) {
+      const int idx = threadIdx.x + it * 256, c = idx % CH, kp = idx / CH;
+      if (idx >= CT / 2 * CH) break;
+      if (OUTPUTS) {
+        *reinterpret_cast<u32x4*>(sk + (kp * 2) * KS + c * 8) = kr[it][0];
+        *reinterpret_cast<u32x4*>(sk + (kp * 2 + 1) * KS + c * 8) = kr[it][1];
       }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        bf16* base = skt + (c * 8 + 2 * e) * CS + kp * 2;
-        *reinterpret_cast<uint32_t*>(base) = (w[0][e] & 0xffffu) | (w[1][e] << 16);
-        *reinterpret_cast<uint32_t*>(base + CS) = (w[0][e] >> 16) | (w[1][e] & 0xffff0000u);
+        bf16* base = skt + (c * 8 + 2 * e) * CS + c * 8 + kp * 2;
+        *reinterpret_cast<uint32_t*>(base) = (kr[it][0][e] & 0xffffu) | (kr[it][1][e] << 16);
+        *reinterpret_cast<uint32_t*>(base + CS) = (kr[it][0][e] >> 16) | (kr[it][1][e] & 0xffff0000u);
       }
     }
-    if (DS > DM)
-      for (int idx = threadIdx.x; idx < (DS - DM) * CS; idx += 256) skt[DM * CS + idx] = (bf16)0.0f;
     // values: thread (token s = tid % 64, columns 16 * (tid / 64) ..): kept in registers for the weighted copy
-    float vv[16];
-    {
+    const bf16x8 v0 = bitcast<bf16x8>(vr[0]), v1 = bitcast<bf16x8>(vr[1]);
+    if (OUTPUTS) {
       const int s = threadIdx.x & 63, c0 = (threadIdx.x >> 6) * 16;
-      const bf16* src = reinterpret_cast<const bf16*>(a.v) + (rb + s) * a.ld + (size_t)head * E + e0 + c0;
       const int k32 = s & 31, place = (s & 32) + ((k32 & 15) >> 2) * 8 + (k32 >> 4) * 4 + (k32 & 3);
 #pragma unroll
-      for (int h = 0; h < 2; ++h) {
-        float t8[8] = {};
-        const int left = s < cnt ? ecols - c0 - h * 8 : 0;
-        if (left > 0) load8(src + h * 8, vec && left >= 8 && ((E | e0) & 7) == 0, left, t8);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          vv[h * 8 + e] = t8[e];
-          svt[(c0 + h * 8 + e) * CS + place] = (bf16)t8[e];
-        }
-      }
+      for (int e = 0; e < 16; ++e) svt[(c0 + e) * CS + place] = e < 8 ? v0[e & 7] : v1[e & 7];
     }
     // gates of the chunk: running sums and maxima over the 64 lanes of the first wave
     if (wave == 0) {
-      float gi = -INFINITY, gf = 0.f;
-      if (lane < cnt) {
-        const float* z = a.gates + (rb + lane) * 2 * a.H + head;
-        gi = log_input_gate(z[0], a.cap);
-        gf = log_forget_gate(z[a.H], a.cap);
-      }
       float bsum = gf;
 #pragma unroll
       for (int o = 1; o < 64; o <<= 1) {
@@ -264,40 +335,41 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
       s_w[lane] = expf(av - last);
       if (lane == 63) s_m = bsum + last;
     }
+    bf16x8 qf[DT];
+    if (OUTPUTS) {
+#pragma unroll
+      for (int c = 0; c < DT; ++c) qf[c] = bitcast<bf16x8>(qr[c]);
+    }
     __syncthreads();
+    if (t0 + CT < count) fetch(t0 + CT);
 
-    // ---- outputs of this wave's sixteen tokens
     const float m_chunk = s_m, M_last = s_M[CT - 1];
-    {
+    b_total += s_b[CT - 1];
+    // ---- outputs of this wave's sixteen tokens
+    if (OUTPUTS) {
       const int t = wave * 16 + lc;
-      const bf16* q = reinterpret_cast<const bf16*>(a.q) + (rb + (t < cnt ? t : cnt - 1)) * a.ld + (size_t)head * D;
-      bf16x8 qf[DT];
       float nq = 0.f;
 #pragma unroll
-      for (int c = 0; c < DT; ++c) {
-        const int d = c * 32 + lg * 8, left = D - d;
-        float v[8];
-        load8(q + (left > 0 ? d : 0), vec && left >= 8, left, v);
+      for (int c = 0; c < DT; ++c)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          qf[c][e] = (bf16)v[e];
-          nq = __builtin_fmaf(v[e], s_n[d + e], nq);
-        }
-      }
+        for (int e = 0; e < 8; ++e) nq = __builtin_fmaf((float)qf[c][e], s_n[c * 32 + lg * 8 + e], nq);
       nq += __shfl_xor(nq, 16, 64);
       nq += __shfl_xor(nq, 32, 64);
       const float Mt = s_M[t], bt = s_b[t], inter = expf(m_prev - Mt);
       f32x4 o[4];
 #pragma unroll
       for (int j = 0; j < 4; ++j) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+      // (two 32-row steps at a time: left to itself the scheduler requests every operand at once and spills)
 #pragma unroll
-      for (int c = 0; c < DT; ++c)
+      for (int c = 0; c < DT; ++c) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int at = (j * 16 + lc) * SS + c * 32 + lg * 8;
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ss_hi + at), qf[c], o[j], 0, 0, 0);
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ss_lo + at), qf[c], o[j], 0, 0, 0);
         }
+        if (c & 1) __builtin_amdgcn_sched_barrier(0);
+      }
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -323,6 +395,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
             hi[h * 4 + r] = (bf16)x;
             lo[h * 4 + r] = (bf16)(x - (float)hi[h * 4 + r]);
           }
+          __builtin_amdgcn_sched_barrier(0);
         }
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
@@ -330,6 +403,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi, o[j], 0, 0, 0);
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo, o[j], 0, 0, 0);
         }
+        __builtin_amdgcn_sched_barrier(0);
       }
       psum += __shfl_xor(psum, 16, 64);
       psum += __shfl_xor(psum, 32, 64);
@@ -349,8 +423,8 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
           }
         }
       }
+      __syncthreads();                                        // S, the keys as they are and n have been read
     }
-    __syncthreads();                                          // S, the keys as they are and n have been read
 
     // ---- the state at the end of the chunk
     {
@@ -358,7 +432,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
       const float w = s < cnt ? s_w[s] : 0.f;
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
-        const float x = vv[e] * w;
+        const float x = (float)(e < 8 ? v0[e & 7] : v1[e & 7]) * w;
         const bf16 hi = (bf16)x;
         sw_hi[(c0 + e) * CS + s] = hi;
         sw_lo[(c0 + e) * CS + s] = (bf16)(x - (float)hi);
@@ -369,7 +443,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
       float n = s_n[d] * decay;
 #pragma unroll
       for (int s = 0; s < CT; s += 8) {
-        const bf16x8 kv = *reinterpret_cast<const bf16x8*>(skt + d * CS + s);
+        const bf16x8 kv = *reinterpret_cast<const bf16x8*>(skt + d * CS + (d >> 3) * 8 + s);
 #pragma unroll
         for (int e = 0; e < 8; ++e) n = __builtin_fmaf(s_w[s + e], (float)kv[e], n);
       }
@@ -393,45 +467,70 @@ __global__ __launch_bounds__(256) void mlstm_chunk_kernel(MA a, bool vec) {
       }
 #pragma unroll
       for (int i = 0; i < ST; ++i) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(skt + (wave * DW + i * 16 + lc) * CS + kg * 32 + lg * 8);
+        const int d = wave * DW + i * 16 + lc;
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(skt + d * CS + (d >> 3) * 8 + kg * 32 + lg * 8);
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           S[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, wh[j], S[i][j], 0, 0, 0);
           S[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, wl[j], S[i][j], 0, 0, 0);
         }
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
     m_prev = m_chunk;
     __syncthreads();                                          // before the next chunk's data replaces this one's
   }
-#pragma unroll
-  for (int i = 0; i < ST; ++i)
-#pragma unroll
-    for (int j = 0; j < 4; ++j)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = wave * DW + i * 16 + lg * 4 + r, e = j * 16 + lc;
-        if (d < D && (e < SL || second)) *state_at(d, e) = S[i][j][r];
+  if (!OUTPUTS || final_seg) {
+    float* to = OUTPUTS ? st : part + (size_t)(seg + 1) * whole;
+    each([&](float x, int at, bool there) { if (there) to[at] = x; return x; });
+    for (int h = 0; h < (second ? 2 : 1); ++h) {
+      for (int d = threadIdx.x; d < D; d += 256) to[h * per + (size_t)D * SL + d] = s_n[d];
+      if (threadIdx.x == 0) {
+        to[h * per + (size_t)D * SL + D] = m_prev;
+        if (!OUTPUTS) to[h * per + (size_t)D * SL + D + 1] = b_total;
       }
-  for (int h = 0; h < (second ? 2 : 1); ++h) {
-    for (int d = threadIdx.x; d < D; d += 256) st[h * per + (size_t)D * SL + d] = s_n[d];
-    if (threadIdx.x == 0) st[h * per + (size_t)D * SL + D] = m_prev;
+    }
   }
+}
+
+// Segments of a pass: as many as fill the machine with workgroups, of at least two chunks each.
+static int chunk_segments(const MA& a, int* length) {
+  const int base = a.seqs * a.H * (((a.E + SL - 1) / SL + 1) / 2);
+  int n = (256 + base - 1) / base;
+  n = n > 16 ? 16 : n;
+  int len = (a.longest + n - 1) / n;
+  len = (len + CT - 1) / CT * CT;
+  if (len < 2 * CT) len = 2 * CT;
+  *length = len;
+  return (a.longest + len - 1) / len;
+}
+
+extern "C" size_t pta_mlstm_workspace_bytes(const MA* args) {
+  if (!args || args->dtype != PTA_BF16 || !args->chunked || args->D > 256 || args->seqs <= 0 || args->longest <= 0 || args->H <= 0 || args->E <= 0) return 0;
+  int len;
+  const int n = chunk_segments(*args, &len);
+  return n > 1 ? (size_t)args->seqs * n * pta_mlstm_state_floats(args->H, args->D, args->E) * sizeof(float) : 0;
 }
 
 template <int DT>
 static int launch_chunk(const MA& a, bool vec, hipStream_t s) {
   static bool ready = false;
-  constexpr int DM = DT * 32, DS = ((DM / 4 + 15) / 16) * 64;
-  constexpr size_t smem = 2 * ((size_t)CT * (DM + 8) + (size_t)DS * CS + CE * CS + 2 * CE * (size_t)(DS + 8 > CS ? DS + 8 : CS));
-  static_assert(smem + 8192 <= 160 * 1024, "LDS");
+  constexpr size_t smem = ChunkShape<DT>::lds;
+  static_assert(smem + 4096 <= 160 * 1024, "LDS");
   if (!ready) {
-    PTA_REQUIRE(hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess,
+    PTA_REQUIRE(hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DT, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess &&
+                hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DT, false>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess,
                 "pta_mlstm: cannot reserve %zu bytes of LDS", smem);
     ready = true;
   }
+  int length;
+  const int segments = chunk_segments(a, &length);
+  const size_t need = pta_mlstm_workspace_bytes(&a);
+  PTA_REQUIRE(segments == 1 || (a.workspace && a.workspace_bytes >= need), "pta_mlstm: the workspace needs %zu bytes", need);
   const int slices = (a.E + SL - 1) / SL;
-  hipLaunchKernelGGL((mlstm_chunk_kernel<DT>), dim3(a.seqs * a.H * ((slices + 1) / 2)), dim3(256), smem, s, a, vec);
+  const dim3 grid(a.seqs * a.H * ((slices + 1) / 2) * segments);
+  if (segments > 1) hipLaunchKernelGGL((mlstm_chunk_kernel<DT, false>), grid, dim3(256), smem, s, a, vec, length, segments, (float*)a.workspace);
+  hipLaunchKernelGGL((mlstm_chunk_kernel<DT, true>), grid, dim3(256), smem, s, a, vec, length, segments, (float*)a.workspace);
   return PTA_OK;
 }
 
@@ -458,6 +557,7 @@ extern "C" int pta_mlstm(const MA* args, pta_stream_t stream) {
   if (a.dtype == PTA_FP32) {
     launch_scan<float>(a, s);
   } else if (a.chunked && a.D <= 256) {
+    PTA_REQUIRE(a.longest >= 1 && a.longest <= a.rows, "pta_mlstm: longest sequence %d of %d rows", a.longest, a.rows);
     const bool vec = a.D % 8 == 0 && a.ld % 8 == 0 && pta_aligned(a.q, 16) && pta_aligned(a.k, 16) && pta_aligned(a.v, 16);
     int rc;
     if (a.D <= 32) rc = launch_chunk<1>(a, vec, s);
@@ -478,7 +578,8 @@ extern "C" int pta_mlstm(const MA* args, pta_stream_t stream) {
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ weight,
                                                              const T* __restrict__ gate, int gate_ld, T* __restrict__ out,
-                                                             int out_ld, int rows, int H, int E, float eps) {
+                                                             int out_ld, int rows, int H, int E, float eps, bool vec) {
+  constexpr int KEEP = 2;                                    // 8-element pieces of a head a lane keeps in registers
   const int lane = threadIdx.x & 63;
   const int idx = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (idx >= rows * H) return;
@@ -488,9 +589,31 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   const float* w = weight + (size_t)head * E;
   T* y = out + (size_t)r * out_ld + (size_t)head * E;
   float sq = 0.f;
-  for (int e = lane; e < E; e += 64) sq = __builtin_fmaf(x[e], x[e], sq);
-  const float inv = 1.0f / sqrtf(wave_total_dpp(sq) / (float)E + eps);
-  for (int e = lane; e < E; e += 64) y[e] = (T)(x[e] * inv * w[e] * sigmoid_f32((float)g[e]));
+  if (vec && E <= KEEP * 512) {
+    float xv[KEEP][8], gv[KEEP][8], wv[KEEP][8];
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int e = (k * 64 + lane) * 8, left = E - e;
+      load8(x + (left > 0 ? e : 0), left > 0, 0, xv[k]);
+      load8(g + (left > 0 ? e : 0), left > 0, 0, gv[k]);
+      load8(w + (left > 0 ? e : 0), left > 0, 0, wv[k]);
+#pragma unroll
+      for (int c = 0; c < 8; ++c) sq = __builtin_fmaf(xv[k][c], xv[k][c], sq);
+    }
+    const float inv = 1.0f / sqrtf(wave_total_dpp(sq) / (float)E + eps);
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+      const int e = (k * 64 + lane) * 8;
+      if (e >= E) break;
+#pragma unroll
+      for (int c = 0; c < 8; ++c) xv[k][c] = xv[k][c] * inv * wv[k][c] * sigmoid_f32(gv[k][c]);
+      store8(y + e, xv[k]);
+    }
+  } else {
+    for (int e = lane; e < E; e += 64) sq = __builtin_fmaf(x[e], x[e], sq);
+    const float inv = 1.0f / sqrtf(wave_total_dpp(sq) / (float)E + eps);
+    for (int e = lane; e < E; e += 64) y[e] = (T)(x[e] * inv * w[e] * sigmoid_f32((float)g[e]));
+  }
   if (head == 0)
     for (int c = H * E + lane; c < out_ld; c += 64) out[(size_t)r * out_ld + c] = (T)0.0f;
 }
@@ -502,12 +625,15 @@ extern "C" int pta_head_norm_gate(int dtype, const float* o, const float* weight
   PTA_REQUIRE(rows > 0 && H > 0 && E > 0 && gate_ld >= H * E && out_ld >= H * E, "pta_head_norm_gate: rows %d, heads %d, size %d, strides %d and %d",
               rows, H, E, gate_ld, out_ld);
   const dim3 grid((rows * H + 3) / 4);
+  const int es = dtype == PTA_BF16 ? 2 : 4;
+  const bool vec = E % 8 == 0 && (gate_ld * es) % 16 == 0 && (out_ld * es) % 16 == 0 && pta_aligned(o, 16) && pta_aligned(weight, 16) &&
+                   pta_aligned(gate, 16) && pta_aligned(out, 16);
   if (dtype == PTA_BF16)
     hipLaunchKernelGGL((head_norm_gate_kernel<bf16>), grid, dim3(256), 0, (hipStream_t)stream, o, weight, (const bf16*)gate, gate_ld,
-                       (bf16*)out, out_ld, rows, H, E, eps);
+                       (bf16*)out, out_ld, rows, H, E, eps, vec);
   else
     hipLaunchKernelGGL((head_norm_gate_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, o, weight, (const float*)gate, gate_ld,
-                       (float*)out, out_ld, rows, H, E, eps);
+                       (float*)out, out_ld, rows, H, E, eps, vec);
   PTA_CHECK_LAUNCH("pta_head_norm_gate");
   return PTA_OK;
 }

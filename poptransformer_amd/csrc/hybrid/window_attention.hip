@@ -73,6 +73,34 @@ __global__ __launch_bounds__(256) void window_append_kernel(WA a, bool vec) {
 // ------------------------------------------------------------------------------------------
 constexpr int WR_KEYS = 4;               // keys a lane group takes per step
 
+// eight elements on their way from memory
+template <typename T> struct Raw8;
+template <> struct Raw8<bf16> {
+  u32x4 w;
+  __device__ __forceinline__ void load(const bf16* p, bool vec, int valid) {
+    if (vec) {
+      w = *reinterpret_cast<const u32x4*>(p);
+    } else {
+      bf16x8 z;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) z[e] = e < valid ? p[e] : (bf16)0.0f;
+      w = bitcast<u32x4>(z);
+    }
+  }
+  __device__ __forceinline__ void unpack(float (&v)[8]) const {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { v[2 * e] = bitcast<float>(w[e] << 16); v[2 * e + 1] = bitcast<float>(w[e] & 0xffff0000u); }
+  }
+};
+template <> struct Raw8<float> {
+  float w[8];
+  __device__ __forceinline__ void load(const float* p, bool vec, int valid) { load8(p, vec, valid, w); }
+  __device__ __forceinline__ void unpack(float (&v)[8]) const {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = w[e];
+  }
+};
+
 template <typename T, int RG, int LPK>
 __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fused, int groups, float* part_o, float* part_ml) {
   constexpr int NG = 4 * 64 / LPK;       // lane groups of the workgroup, each with a softmax state of its own
@@ -94,11 +122,50 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fu
 
   const T* q = reinterpret_cast<const T*>(a.q) + (size_t)r * a.ld;
   const T* kp = reinterpret_cast<const T*>(a.k) + (size_t)r * a.ld;
+  const int sub = lane % LPK, d0 = sub * 8, grp = wave * (64 / LPK) + lane / LPK;
+  const int left = D - d0;               // elements of a row from d0 on
+  const T* ring = reinterpret_cast<const T*>(a.ring) + ((size_t)slot * a.G + g) * a.ring_len * Dp;
+  const float* rinv = a.rinv + (size_t)slot * a.ring_len;
+
+  // a step's keys, as they lie in memory; the row's own key comes from the projection
+  Raw8<T> kr[WR_KEYS];
+  float ri[WR_KEYS];
+  auto fetch = [&](int jb) {
+#pragma unroll
+    for (int u = 0; u < WR_KEYS; ++u) {
+      const int j = jb + u * NG + grp;
+      const int jc = j < j1 ? j : j1 - 1;
+      const bool self = fused && jc == i;
+      const int at = jc % a.ring_len;
+      ri[u] = rinv[at];                                                   // (not used for the own key)
+      const T* src = self ? kp + g * D + (left > 0 ? d0 : 0) : ring + (size_t)at * Dp + (left > 0 ? d0 : 0);
+      kr[u].load(src, left > 0 && (!self || (vec && left >= 8)), left);
+    }
+  };
+  // everything that does not depend on the sums below is requested before them
+  if (j0 < j1) fetch(j0);
+  float qv[RG][8], slope[RG];
+  {
+    float wk[8];
+    load8(a.k_norm + g * D + (left > 0 ? d0 : 0), vec && left >= 8, left, wk);
+#pragma unroll
+    for (int h = 0; h < RG; ++h) {
+      const int hr = hg * RG + h < R ? hg * RG + h : R - 1;              // a duplicate that is not stored
+      const int head = g * R + hr;
+      float wq[8];
+      load8(q + head * D + (left > 0 ? d0 : 0), vec && left >= 8, left, qv[h]);
+      load8(a.q_norm + head * D + (left > 0 ? d0 : 0), vec && left >= 8, left, wq);
+      slope[h] = a.slopes[head];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) qv[h][e] = qv[h][e] * wq[e] * (wk[e] * a.scale);
+    }
+  }
   float rq, rk = 0.f;
   if (fused) {
-    rq = 1.0f / sqrtf(workgroup_sum<4>(squares(q, a.H * D, vec), red[0]) / (float)(a.H * D) + a.eps);
+    const float qs = squares(q, a.H * D, vec), ks = own ? squares(kp, a.G * D, vec) : 0.f;
+    rq = 1.0f / sqrtf(workgroup_sum<4>(qs, red[0]) / (float)(a.H * D) + a.eps);
     if (own) {
-      rk = 1.0f / sqrtf(workgroup_sum<4>(squares(kp, a.G * D, vec), red[1]) / (float)(a.G * D) + a.eps);
+      rk = 1.0f / sqrtf(workgroup_sum<4>(ks, red[1]) / (float)(a.G * D) + a.eps);
       if (hg == 0) {
         put_ring_row(a, kp, g, slot, i);
         if (g == 0 && threadIdx.x == 0) a.rinv[(size_t)slot * a.ring_len + i % a.ring_len] = rk;
@@ -107,27 +174,6 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fu
   } else {
     rq = a.q_scale[r];
   }
-
-  const int sub = lane % LPK, d0 = sub * 8, grp = wave * (64 / LPK) + lane / LPK;
-  const int left = D - d0;               // elements of a row from d0 on
-  float qv[RG][8], slope[RG];
-  {
-    float wk[8];
-    load8(a.k_norm + g * D + (left > 0 ? d0 : 0), false, left, wk);
-#pragma unroll
-    for (int h = 0; h < RG; ++h) {
-      const int hr = hg * RG + h < R ? hg * RG + h : R - 1;              // a duplicate that is not stored
-      const int head = g * R + hr;
-      float wq[8];
-      load8(q + head * D + (left > 0 ? d0 : 0), vec && left >= 8, left, qv[h]);
-      load8(a.q_norm + head * D + (left > 0 ? d0 : 0), false, left, wq);
-      slope[h] = a.slopes[head];
-#pragma unroll
-      for (int e = 0; e < 8; ++e) qv[h][e] = qv[h][e] * rq * wq[e] * (wk[e] * a.scale);
-    }
-  }
-  const T* ring = reinterpret_cast<const T*>(a.ring) + ((size_t)slot * a.G + g) * a.ring_len * Dp;
-  const float* rinv = a.rinv + (size_t)slot * a.ring_len;
 
   float m[RG], l[RG], o[RG][8];
 #pragma unroll
@@ -138,19 +184,16 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fu
     for (int e = 0; e < 8; ++e) o[h][e] = 0.f;
   }
   for (int jb = j0; jb < j1; jb += NG * WR_KEYS) {
-    float kv[WR_KEYS][8], s[WR_KEYS][RG], ri[WR_KEYS];
+    float kv[WR_KEYS][8], s[WR_KEYS][RG], rj[WR_KEYS];
     int dist[WR_KEYS];
 #pragma unroll
     for (int u = 0; u < WR_KEYS; ++u) {
       const int j = jb + u * NG + grp;
-      const int jc = j < j1 ? j : j1 - 1;
       dist[u] = j < j1 ? i - j : -1;
-      const bool self = fused && jc == i;
-      const int at = jc % a.ring_len;
-      ri[u] = self ? rk : rinv[at];
-      const T* src = self ? kp + g * D + (left > 0 ? d0 : 0) : ring + (size_t)at * Dp + (left > 0 ? d0 : 0);
-      load8(src, left > 0 && (!self || (vec && left >= 8)), left, kv[u]);
+      rj[u] = rq * (fused && dist[u] == 0 ? rk : ri[u]);
+      kr[u].unpack(kv[u]);
     }
+    if (jb + NG * WR_KEYS < j1) fetch(jb + NG * WR_KEYS);
 #pragma unroll
     for (int h = 0; h < RG; ++h) {
       float top = m[h];
@@ -160,7 +203,7 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fu
 #pragma unroll
         for (int e = 0; e < 8; ++e) t = __builtin_fmaf(qv[h][e], kv[u][e], t);
         t = group_sum<LPK>(t);
-        s[u][h] = dist[u] >= 0 ? t * ri[u] - slope[h] * (float)dist[u] : -INFINITY;
+        s[u][h] = dist[u] >= 0 ? t * rj[u] - slope[h] * (float)dist[u] : -INFINITY;
         top = fmaxf(top, s[u][h]);
       }
       const float keep = exp_of<T>(m[h] - top);
@@ -219,25 +262,40 @@ __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fu
     for (int c = a.H * D + threadIdx.x; c < a.out_ld; c += 256) (reinterpret_cast<T*>(a.out) + (size_t)r * a.out_ld)[c] = (T)0.0f;
 }
 
-// the parts of a row's window meet, and the gate is applied
+// the parts of a row's window (at most 64) meet, and the gate is applied: one wave per (row, head)
 template <typename T>
 __global__ __launch_bounds__(64) void window_merge_kernel(WA a, const float* part_o, const float* part_ml) {
-  const int r = blockIdx.x / a.H, head = blockIdx.x % a.H, D = a.D;
-  const float* ml = part_ml + ((size_t)r * a.H + head) * a.splits * 2;
-  float top = -1e30f;
-  for (int s = 0; s < a.splits; ++s) top = fmaxf(top, ml[2 * s]);
-  float tot = 0.f;
-  for (int s = 0; s < a.splits; ++s) tot = __builtin_fmaf(exp_of<T>(ml[2 * s] - top), ml[2 * s + 1], tot);
+  __shared__ float weight[64];
+  const int r = blockIdx.x / a.H, head = blockIdx.x % a.H, D = a.D, lane = threadIdx.x, n = a.splits;
+  const size_t at = ((size_t)r * a.H + head) * n;
+  const float* po = part_o + at * D;
+  const T* gate = reinterpret_cast<const T*>(a.gate) + (size_t)r * a.ld + head * D;
   T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.out_ld;
-  const T* gate = reinterpret_cast<const T*>(a.gate) + (size_t)r * a.ld;
-  for (int d = threadIdx.x; d < D; d += 64) {
+  float m = -1e30f, l = 0.f;
+  if (lane < n) { m = part_ml[(at + lane) * 2]; l = part_ml[(at + lane) * 2 + 1]; }
+  // the first eight parts of this lane's first feature are requested before the weights are known
+  float v[8];
+#pragma unroll
+  for (int u = 0; u < 8; ++u) v[u] = u < n && lane < D ? po[(size_t)u * D + lane] : 0.f;
+  const float top = wave_max(m);
+  const float w = lane < n ? exp_of<T>(m - top) : 0.f;
+  weight[lane] = w;
+  const float inv = 1.0f / wave_sum(w * l);
+  __syncthreads();
+  for (int d = lane; d < D; d += 64) {
     float t = 0.f;
-    for (int s = 0; s < a.splits; ++s)
-      t = __builtin_fmaf(exp_of<T>(ml[2 * s] - top), part_o[(((size_t)r * a.H + head) * a.splits + s) * D + d], t);
-    out[head * D + d] = (T)(t / tot * sigmoid_f32((float)gate[head * D + d]));
+    for (int s = 0; s < n; s += 8) {
+      if (s > 0 || d != lane) {
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v[u] = s + u < n ? po[(size_t)(s + u) * D + d] : 0.f;
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) t = __builtin_fmaf(s + u < n ? weight[s + u] : 0.f, v[u], t);
+    }
+    out[head * D + d] = (T)(t * inv * sigmoid_f32((float)gate[d]));
   }
   if (head == 0)
-    for (int c = a.H * D + threadIdx.x; c < a.out_ld; c += 64) out[c] = (T)0.0f;
+    for (int c = a.H * D + lane; c < a.out_ld; c += 64) out[c] = (T)0.0f;
 }
 
 // ------------------------------------------------------------------------------------------
@@ -288,8 +346,8 @@ __global__ __launch_bounds__(256) void window_tile_kernel(WA a, bool vec) {
       const int d = m * 32 + lg * 8, left = D - d;
       float v[8], wq[8], wk[8];
       load8(q + (left > 0 ? d : 0), vec && left >= 8, left, v);
-      load8(a.q_norm + head * D + (left > 0 ? d : 0), false, left, wq);
-      load8(a.k_norm + g * D + (left > 0 ? d : 0), false, left, wk);
+      load8(a.q_norm + head * D + (left > 0 ? d : 0), vec && left >= 8, left, wq);
+      load8(a.k_norm + g * D + (left > 0 ? d : 0), vec && left >= 8, left, wk);
 #pragma unroll
       for (int e = 0; e < 8; ++e) qf[w][m][e] = (bf16)(v[e] * rq * wq[e] * wk[e]);
     }
@@ -455,7 +513,7 @@ static int check_window(const WA& a, const char* name) {
 static bool vectors_fit(const WA& a) {
   const size_t es = a.dtype == PTA_BF16 ? 2 : 4;
   return a.D % 8 == 0 && (size_t)a.ld * es % 16 == 0 && pta_aligned(a.q, 16) && pta_aligned(a.k, 16) && pta_aligned(a.gate, 16) &&
-         (size_t)a.out_ld * es % 8 == 0 && pta_aligned(a.out, 8);
+         (size_t)a.out_ld * es % 8 == 0 && pta_aligned(a.out, 8) && pta_aligned(a.q_norm, 16) && pta_aligned(a.k_norm, 16);
 }
 
 template <typename T, int RG>
@@ -526,7 +584,7 @@ extern "C" int pta_window_decode(const WA* args, pta_stream_t stream) {
   const WA& a = *args;
   const int rc = check_window(a, "pta_window_decode");
   if (rc) return rc;
-  PTA_REQUIRE(a.out && a.out_ld >= a.H * a.D && a.splits >= 1, "pta_window_decode: output or splits");
+  PTA_REQUIRE(a.out && a.out_ld >= a.H * a.D && a.splits >= 1 && a.splits <= 64, "pta_window_decode: output, or splits %d (1 .. 64)", a.splits);
   const size_t need = pta_window_attention_workspace_bytes(a.rows, a.H, a.D, a.splits);
   PTA_REQUIRE(a.splits == 1 || (a.workspace && a.workspace_bytes >= need), "pta_window_decode: the workspace needs %zu bytes", need);
   hipStream_t s = (hipStream_t)stream;

@@ -186,7 +186,7 @@ class HybridDecoder(DecodeLoop):
         self._buffers = {}
         self._stream = torch.cuda.Stream()
         self._splits_for = {}
-        self._head_h = None
+        self._head_h = self._scratch_buf = None
 
     # ------------------------------------------------------------------ layers
     def _layer_weights(self, i):
@@ -206,10 +206,15 @@ class HybridDecoder(DecodeLoop):
             group = mixer.heads // mixer.kv_heads
             wgs = rows * mixer.kv_heads * -(-group // (group if group <= 2 else 4))
             keys = min(mixer.window or self.store.max_len, self.store.max_len)
-            splits = max(1, min(1024 // wgs if wgs else 1, -(-keys // 64), 64))
-            splits = 1 if keys <= 256 else splits
+            splits = max(1, min(768 // wgs, -(-keys // 64), 64)) if keys > 256 else 1
             self._splits_for[key] = (splits, HK.window_workspace(rows, mixer.heads, mixer.dim, splits, self.dev) if splits > 1 else None)
         return self._splits_for[key]
+
+    def _scratch(self, nbytes):
+        """Memory that the launches of a pass use one after the other."""
+        if self._scratch_buf is None or self._scratch_buf.numel() < nbytes:
+            self._scratch_buf = torch.empty(nbytes, dtype=torch.uint8, device=self.dev)
+        return self._scratch_buf
 
     def _mixer(self, i, b, rows):
         spec, m, lw, store = self.spec, self.spec.layers[i].mixer, self._layer_weights(i), self.store.stores[i]
@@ -224,7 +229,8 @@ class HybridDecoder(DecodeLoop):
             else:
                 att.prompt(proj, n, rows.slot, rows.pos, ctx, b.q_scale, rows.tiles)
         else:
-            HK.mlstm(proj, n, m.heads, m.dim, m.vdim, b.gates, m.gate_cap, store[0], rows.slot, rows.seqs, b.o, rows.longest > 8)
+            HK.mlstm(proj, n, m.heads, m.dim, m.vdim, b.gates, m.gate_cap, store[0], rows.slot, rows.seqs, rows.longest, b.o,
+                     rows.longest > 8, self._scratch)
             HK.head_norm_gate(b.o, lw.head_norm, proj, m.gate_at, ctx, n, m.heads, m.vdim, spec.eps)
         HK.linear(ctx, lw.out, b.y, n, ld=spec.width, workspace=b.workspace)
 

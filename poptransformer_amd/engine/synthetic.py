@@ -161,3 +161,64 @@ def gpt2_synthetic_state_dict(cfg, seed=0):
     sd["transformer.ln_f.weight"] = np.ones(d, np.float16)
     sd["transformer.ln_f.bias"] = np.zeros(d, np.float16)
     return sd
+
+
+def llama2_f16_synthetic_weights(cfg, seed=0, device="cuda"):
+    """The shape of llama2_synthetic_weights with fp16 Linears."""
+    gen = torch.Generator(device=device)
+    gen.manual_seed(seed)
+    d, f, v = cfg["hidden_size"], cfg["intermediate_size"], cfg["vocab_size"]
+    hd = d // cfg["num_attention_heads"]
+    ones = torch.ones(d, dtype=torch.float16, device=device)
+
+    def f16w(rows, cols):
+        return (torch.randn((rows, cols), generator=gen, device=device, dtype=torch.float32) * 0.02).half()
+
+    def lin(rows, cols):
+        return LinearWeights(K.F16Weight(f16w(rows, cols)))
+
+    blocks = [BlockWeights(norm1=(ones.clone(), None), norm2=(ones.clone(), None), qkv=[lin(d, d) for _ in range(3)], out=lin(d, d),
+                           mlp_in=[lin(f, d) for _ in range(2)], mlp_out=lin(d, f)) for _ in range(cfg["num_hidden_layers"])]
+    inv_freq = torch.from_numpy(np.array([1.0 / (10000 ** (i / hd)) for i in range(0, hd, 2)]).astype(np.float16)).to(device)
+    torch.cuda.synchronize()
+    return ModelWeights(embed=f16w(v, d), pos_embed=None, blocks=blocks, final_norm=(ones.clone(), None), head=lin(v, d), inv_freq=inv_freq)
+
+
+class HybridTensors(dict):
+    """Random tensors of a hybrid configuration by name, drawn on the device when they are asked for (one layer's worth at a
+    time is held by the loader)."""
+
+    def __init__(self, cfg, seed=0, device="cuda"):
+        super().__init__()
+        self.gen = torch.Generator(device=device)
+        self.gen.manual_seed(seed)
+        self.dev, S, d, V = device, cfg["streams"], cfg["width"], cfg["vocab"]
+        self.shapes = {"embed": (V, d), "head": (V, d), "final.norm": (d,)}
+        for i, lay in enumerate(cfg["layers"]):
+            if lay.get("weights_of") is not None:
+                continue
+            p, m = f"l{i}.", lay["mixer"]
+            H, D = m["heads"], m["dim"]
+            if lay["type"] == "attention":
+                N, G = H * D, m["kv_heads"] * D
+                mix = {"q": (N, d), "k": (G, d), "g": (N, d), "q.norm": (N,), "k.norm": (G,)}
+            else:
+                N = H * m["vdim"]
+                mix = {"q": (H * D, d), "k": (H * D, d), "v": (N, d), "g": (N, d), "i": (H, d), "f": (H, d), "i.b": (H,), "f.b": (H,), "norm": (N,)}
+            self.shapes.update({p + "mix." + k: s for k, s in dict(mix, o=(d, N)).items()})
+            ff = lay["mlp"]["ff"]
+            self.shapes.update({p + "mlp.gate": (ff, d), p + "mlp.up": (ff, d), p + "mlp.down": (d, ff)})
+            for q in "12":
+                self.shapes.update({p + "norm" + q: (d,), p + f"hc{q}.in": (S,), p + f"hc{q}.out": (S,), p + f"hc{q}.mix": (S, S)})
+
+    def __contains__(self, name):
+        return name in self.shapes
+
+    def __getitem__(self, name):
+        shape = self.shapes[name]
+        if name.endswith(".mix") and len(shape) == 2 and ".hc" in name:
+            return torch.eye(shape[0], device=self.dev)
+        if len(shape) == 1:
+            return torch.full(shape, 3.0 if name.endswith("f.b") else 1.0 / shape[0] if ".hc" in name and name.endswith(".in") else 1.0,
+                              device=self.dev)
+        return torch.randn(shape, generator=self.gen, device=self.dev, dtype=torch.float32).mul_(0.02).to(torch.bfloat16)

@@ -161,8 +161,9 @@ def mlstm_state(slots, heads, dim, vdim, device):
     return torch.zeros((slots, H.load().pta_mlstm_state_floats(heads, dim, vdim)), dtype=F32, device=device)
 
 
-def mlstm(proj, rows, heads, dim, vdim, gates, cap, state, slot, seqs, o, chunked):
-    """proj rows hold q | k | v | ...; seqs = (first rows, row counts, how many); o [rows, heads * vdim] fp32."""
+def mlstm(proj, rows, heads, dim, vdim, gates, cap, state, slot, seqs, longest, o, chunked, scratch=None):
+    """proj rows hold q | k | v | ...; seqs = (first rows, row counts, how many), longest: the largest count; o [rows, heads *
+    vdim] fp32.  scratch(bytes) -> uint8 tensor: memory for passes that are cut into segments (default: allocated here)."""
     es, HD, HE = proj.element_size(), heads * dim, heads * vdim
     seq_row, seq_count, n = seqs
     _need(proj, proj.dtype, "projection", rows * proj.shape[-1])
@@ -173,7 +174,11 @@ def mlstm(proj, rows, heads, dim, vdim, gates, cap, state, slot, seqs, o, chunke
         raise ValueError("mlstm: the state or the projection does not fit the sizes")
     base = proj.data_ptr()
     a = H.MlstmArgs(_CODE[proj.dtype], rows, heads, dim, vdim, base, base + HD * es, base + 2 * HD * es, proj.shape[-1], _p(gates), cap,
-                    _p(state), _p(slot), _p(seq_row), _p(seq_count), n, int(chunked), _p(o))
+                    _p(state), _p(slot), _p(seq_row), _p(seq_count), n, longest, int(chunked), _p(o), None, 0)
+    need = H.load().pta_mlstm_workspace_bytes(ctypes.byref(a))
+    if need:
+        ws = scratch(need) if scratch is not None else torch.empty(need, dtype=torch.uint8, device=proj.device)
+        a.workspace, a.workspace_bytes = _p(ws), ws.numel()
     H.check(H.load().pta_mlstm(ctypes.byref(a), _stream()))
 
 

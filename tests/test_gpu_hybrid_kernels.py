@@ -181,7 +181,7 @@ class Attention:
         return o.reshape(T, H * D) * Z.sigmoid(gate)
 
     def tol(self):
-        return 5e-6 if self.dtype == torch.float32 else 2e-2        # bf16: queries, weights and results are rounded
+        return 2e-5 if self.dtype == torch.float32 else 2e-2        # bf16: queries, weights and results are rounded
 
 
 SHAPES = [(4, 2, 8, 5), (6, 2, 20, 33), (2, 2, 48, 64), (8, 1, 64, 65), (5, 1, 72, 63), (4, 1, 128, 100), (3, 3, 136, 40),
@@ -288,7 +288,7 @@ class Memory:
         starts = np.concatenate([[0], np.cumsum(counts)[:-1]])
         o = torch.full((n, self.H * self.E), 7.0, device="cuda")
         self.HK.mlstm(proj, n, self.H, self.D, self.E, _dev(gates), self.cap, self.state, _dev(slot, i32),
-                      (_dev(starts, i32), _dev(counts, i32), len(spans)), o, chunked)
+                      (_dev(starts, i32), _dev(counts, i32), len(spans)), int(counts.max()), o, chunked)
         return _np(o).reshape(n, self.H, self.E)
 
     def want(self, proj, gates):
@@ -318,7 +318,7 @@ def test_mlstm(dtype, H, D, E, kind):
     """Whole, in portions (down to two tokens, at and around multiples of the chunk), token by token, and a batch of
     unequal sequences; the state carried from one to the next."""
     rng = np.random.default_rng(D + E)
-    T = 200
+    T = 330                                  # chunked: three segments of up to 128 tokens
     m = Memory(dtype, H, D, E, 7.0, 4)
     proj = m.project(*(rng.standard_normal((T, c)) for c in (H * D, H * D, H * E)))
     gates = _gates(rng, T, H, kind)
@@ -332,7 +332,7 @@ def test_mlstm(dtype, H, D, E, kind):
         print(f"mlstm {dtype} H {H} D {D} E {E} {kind} chunked {chunked}", flush=True)
         m.state.zero_()
         assert close(m.run(proj, gates, [(1, T)], chunked), want)
-        for cuts in ((64, 64, 72), (2, 63, 65, 2, 68), (199, 1)):
+        for cuts in ((64, 64, 202), (2, 63, 65, 2, 198), (129, 127, 74), (329, 1)):
             m.state.zero_()
             parts, p = [], 0
             for c in cuts:
@@ -344,7 +344,7 @@ def test_mlstm(dtype, H, D, E, kind):
         got += [m.run(proj[t:t + 1].contiguous(), gates[t:t + 1], [(3, 1)], False) for t in range(130, T)]
         assert close(np.concatenate(got), want)
         m.state.zero_()
-        lens, slots = [70, 1, 200, 64], [3, 0, 2, 1]
+        lens, slots = [70, 1, 330, 129], [3, 0, 2, 1]
         got = m.run(torch.cat([proj[:n] for n in lens]), np.concatenate([gates[:n] for n in lens]), list(zip(slots, lens)), chunked)
         assert close(got, np.concatenate([want[:n] for n in lens]))
 
@@ -374,6 +374,9 @@ def test_selection_over_fp32_logits():
     HK.argmax(_dev(x), ids)
     clean = np.where(np.isnan(x), -np.inf, x)
     assert ids.cpu().tolist() == [int(r.argmax()) for r in clean[:2]] + [0] + [int(r.argmax()) for r in clean[3:]]
+    y = rng.integers(-20, 20, (3, 40000)).astype(np.float32)              # whole vectors, several per thread
+    HK.argmax(_dev(y), ids)
+    assert ids[:3].cpu().tolist() == [int(r.argmax()) for r in y]
     top = torch.zeros((5, 7), dtype=torch.int32, device="cuda")
     HK.topk(_dev(x), 7, top)
     for r in (0, 1, 3, 4):
