@@ -109,7 +109,7 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(MA a) {
 }
 
 // ------------------------------------------------------------------------------------------
-// In chunks of CT tokens on the matrix unit (bf16, D <= 32 * DT): a workgroup of four waves per (sequence, head, CE value
+// In chunks of CT tokens on the matrix unit (bf16, D <= 32 * DT): a workgroup per (sequence, head, CE value
 // columns = two slices, segment).  With b_t the running sum of the chunk's log forget gates, a_s = i_s - b_s and
 // M_t = max(m_prev, max_{s <= t} a_s), unrolling the recurrence gives m_t = b_t + M_t and
 //   o_t ~ sum_{s <= t} exp(a_s - M_t) (q_t . k_s) v_s + exp(m_prev - M_t) S_prev^T q_t      (n . q likewise)
@@ -123,8 +123,8 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(MA a) {
 //   m' = max(m + B_i, m_i),  S' = exp(m + B_i - m') S + exp(m_i - m') S_i,
 // and goes on from there.  Place 0 of `parts` keeps the state the sequence came with: the last segment overwrites it.
 //
-// Wave w computes the outputs of tokens 16 w .. 16 w + 15 (as columns: P^T = K Q^T, O^T = V^T P^T + S^T Q^T) and owns rows
-// d = w * DW .. of S in its accumulators.  The transposed values hold their tokens in the order in which a lane of the
+// Wave w computes outputs of tokens 16 (w % 4) .. + 15 (as columns: P^T = K Q^T, O^T = V^T P^T + S^T Q^T; with eight waves two
+// share the tokens and halve the value columns) and owns rows d = w * DW .. of S in its accumulators.  The transposed values hold their tokens in the order in which a lane of the
 // product P^T holds them (key 4 x + e of the first sixteen of 32 in place 8 x + e, of the second in 8 x + 4 + e); the
 // transposed keys, and the weighted values beside them, in plain order.  The next chunk's rows are requested while a chunk
 // is worked on.
@@ -134,17 +134,24 @@ constexpr int CS = CT + 8;
 
 template <int DT> struct ChunkShape {
   static constexpr int DM = DT * 32, KS = DM + 8, CH = DM / 8;
-  static constexpr int ST = (DM / 4 + 15) / 16;                       // 16-row tiles of S per wave
-  static constexpr int DW = ST * 16, DS = DW * 4, SS = DS + 8;        // DS >= DM rows of S in all
+  static constexpr int NW = DT >= 4 ? 8 : 4, THREADS = NW * 64;       // waves
+  static constexpr int JT = 16 / NW;                                  // 16-column tiles of the outputs per wave
+  static constexpr int ST = (DM / NW + 15) / 16;                      // 16-row tiles of S per wave
+  static constexpr int DW = ST * 16, DS = DW * NW, SS = DS + 8;       // DS >= DM rows of S in all
   static constexpr int KT = DS * CS + DS;                             // transposed keys: row d starts at d * CS + (d / 8) * 8
   static constexpr size_t lds = 2 * ((size_t)CT * KS + KT + CE * CS + 2 * CE * (size_t)(SS > CS ? SS : CS));
 };
 
-template <int DT, bool OUTPUTS>
-__global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int segment, int segments, float* parts) {
+// VEC: D and E multiples of 8 and everything 16-byte aligned - whole pieces, requested without a branch (a load in a branch
+// is waited for at its end): rows past the chunk and columns past the sizes repeat others.  That is harmless in keys and
+// values of rows (their weights are zero) and in key columns (they only reach rows of S that are never read); queries and
+// value columns are zeroed.
+template <int DT, bool OUTPUTS, bool VEC>
+__global__ __launch_bounds__(ChunkShape<DT>::THREADS) void mlstm_chunk_kernel(MA a, int segment, int segments, float* parts) {
   typedef ChunkShape<DT> C;
-  constexpr int DM = C::DM, KS = C::KS, CH = C::CH, ST = C::ST, DW = C::DW, DS = C::DS, SS = C::SS;
-  constexpr int IPT = (CT / 2 * CH + 255) / 256;                      // (pair of keys, 16-byte piece) items per thread
+  constexpr int DM = C::DM, KS = C::KS, CH = C::CH, ST = C::ST, DW = C::DW, DS = C::DS, SS = C::SS, THREADS = C::THREADS, JT = C::JT;
+  constexpr int VV = 8 / C::NW, VC = VV * 8;                          // 8-column pieces and columns of the values a thread stages
+  constexpr int IPT = (CT / 2 * CH + THREADS - 1) / THREADS;                      // (pair of keys, 16-byte piece) items per thread
   extern __shared__ __align__(16) unsigned char smem[];
   bf16* sk = reinterpret_cast<bf16*>(smem);                           // [CT][KS] keys
   bf16* skt = sk + CT * KS;                                           // keys transposed
@@ -154,9 +161,10 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
   bf16* ss_lo = big + CE * SS;
   bf16* sw_hi = big;                                                  // [CE][CS] weighted values, over S once that is read
   bf16* sw_lo = big + CE * CS;
-  __shared__ float s_n[DM], s_a[CT], s_M[CT], s_b[CT], s_w[CT];
+  __shared__ __align__(16) float s_n[DM], s_a[CT], s_M[CT], s_b[CT], s_w[CT];
   __shared__ float s_m;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  int lane = threadIdx.x & 63, lg = lane >> 4, lc = lane & 15;
   const int slices = (a.E + SL - 1) / SL, groups = (slices + 1) / 2;
   int blk = blockIdx.x;
   const int grp = blk % groups; blk /= groups;
@@ -176,51 +184,52 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
   const float qscale = 1.0f / sqrtf((float)D);
 
   // ---- the chunk's rows on their way to LDS (keys, values), to registers (queries) and the gates
-  u32x4 kr[IPT][2], vr[2], qr[DT];
-  float gi, gf;
-  auto row8 = [&](const void* base, size_t r, size_t at, bool whole8, int left) {
-    const bf16* src = reinterpret_cast<const bf16*>(base) + r * a.ld + at;
-    if (left <= 0) return u32x4{0, 0, 0, 0};
-    if (whole8) return *reinterpret_cast<const u32x4*>(src);
+  u32x4 kr[IPT][2], vr[VV], qr[DT];
+  float zi, zf;
+  // (a uniform base per chunk and a 32-bit offset per lane)
+  auto row8 = [&](const bf16* base, int r, int at, int left) {
+    const bf16* src = base + (unsigned)(r * a.ld + at);
+    if constexpr (VEC) return *reinterpret_cast<const u32x4*>(src);
     bf16x8 z;
 #pragma unroll
     for (int e = 0; e < 8; ++e) z[e] = e < left ? src[e] : (bf16)0.0f;
     return bitcast<u32x4>(z);
   };
+  const u32x4 none = {0, 0, 0, 0};
   auto fetch = [&](int t0) {
     const int cnt = count - t0 < CT ? count - t0 : CT;
     const size_t rb = (size_t)row0 + t0;
+    const bf16 *kb = reinterpret_cast<const bf16*>(a.k) + rb * a.ld + head * D, *qb = reinterpret_cast<const bf16*>(a.q) + rb * a.ld + head * D,
+               *vb = reinterpret_cast<const bf16*>(a.v) + rb * a.ld + head * E + e0;
+    {
+      const float* z = a.gates + rb * 2 * a.H + head + (unsigned)((lane < cnt ? lane : cnt - 1) * 2 * a.H);
+      zi = z[0];
+      zf = z[a.H];
+    }
 #pragma unroll
     for (int it = 0; it < IPT; ++it) {
-      const int idx = threadIdx.x + it * 256, c = idx % CH, kp = idx / CH, left = D - c * 8;
+      const int idx = threadIdx.x + it * THREADS, c = idx % CH, kp = idx / CH, left = D - c * 8;
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
         const int s = kp * 2 + t;
-        kr[it][t] = row8(a.k, rb + s, (size_t)head * D + c * 8, vec && left >= 8, s < cnt ? left : 0);
+        kr[it][t] = row8(kb, s < cnt ? s : cnt - 1, left > 0 ? c * 8 : 0, left);
       }
     }
     {
-      const int s = threadIdx.x & 63, c0 = (threadIdx.x >> 6) * 16;
+      const int s = threadIdx.x & 63, c0 = wave * VC;
 #pragma unroll
-      for (int h = 0; h < 2; ++h) {
-        const int left = s < cnt ? ecols - c0 - h * 8 : 0;
-        vr[h] = row8(a.v, rb + s, (size_t)head * E + e0 + c0 + h * 8, vec && left >= 8 && (E & 7) == 0, left);
+      for (int h = 0; h < VV; ++h) {
+        const int left = ecols - c0 - h * 8;
+        vr[h] = row8(vb, s < cnt ? s : cnt - 1, left > 0 ? c0 + h * 8 : 0, left);
       }
     }
     if (OUTPUTS) {
-      const int t = wave * 16 + lc;
+      const int t = (wave & 3) * 16 + lc;
 #pragma unroll
       for (int c = 0; c < DT; ++c) {
         const int left = D - c * 32 - lg * 8;
-        qr[c] = row8(a.q, rb + (t < cnt ? t : cnt - 1), (size_t)head * D + c * 32 + lg * 8, vec && left >= 8, left);
+        qr[c] = row8(qb, t < cnt ? t : cnt - 1, left > 0 ? c * 32 + lg * 8 : 0, left);
       }
-    }
-    gi = -INFINITY;
-    gf = 0.f;
-    if (wave == 0 && lane < cnt) {
-      const float* z = a.gates + (rb + lane) * 2 * a.H + head;
-      gi = log_input_gate(z[0], a.cap);
-      gf = log_forget_gate(z[a.H], a.cap);
     }
   };
   fetch(0);
@@ -247,12 +256,15 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
     const bool empty = !OUTPUTS && seg > 0;
     // a segment of several starts from what the first launch kept: the state itself is overwritten by the last segment
     const float* from = OUTPUTS && several ? part + (seg > 0 ? whole : 0) : st;
-    each([&](float, int at, bool there) { return there && !empty ? from[at] : 0.f; });
-    for (int d = threadIdx.x; d < DM; d += 256) s_n[d] = d < D && !empty ? from[(size_t)D * SL + d] : 0.f;
+    each([&](float, int at, bool there) {                     // (loads without a branch, as above)
+      const float x = from[there ? at : 0];
+      return there && !empty ? x : 0.f;
+    });
+    for (int d = threadIdx.x; d < DM; d += THREADS) s_n[d] = d < D && !empty ? from[(size_t)D * SL + d] : 0.f;
     m_prev = empty ? -INFINITY : from[(size_t)D * SL + D];
     if (!OUTPUTS && seg == 0) {                               // keep what the sequence came with
       each([&](float x, int at, bool there) { if (there) part[at] = x; return x; });
-      for (int d = threadIdx.x; d < D; d += 256) part[(size_t)D * SL + d] = s_n[d];
+      for (int d = threadIdx.x; d < D; d += THREADS) part[(size_t)D * SL + d] = s_n[d];
       if (threadIdx.x == 0) part[(size_t)D * SL + D] = m_prev;
     }
     if (OUTPUTS)
@@ -260,18 +272,26 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
         const float* add = part + (size_t)j * whole;
         const float mi = add[(size_t)D * SL + D], carried = m_prev + add[(size_t)D * SL + D + 1];
         const float mn = fmaxf(carried, mi), keep = expf(carried - mn), take = expf(mi - mn);
-        each([&](float x, int at, bool there) { return __builtin_fmaf(keep, x, there ? take * add[at] : 0.f); });
-        for (int d = threadIdx.x; d < D; d += 256) s_n[d] = __builtin_fmaf(keep, s_n[d], take * add[(size_t)D * SL + d]);
+        each([&](float x, int at, bool there) {
+          const float y = add[there ? at : 0];
+          return __builtin_fmaf(keep, x, (there ? take : 0.f) * y);
+        });
+        for (int d = threadIdx.x; d < D; d += THREADS) s_n[d] = __builtin_fmaf(keep, s_n[d], take * add[(size_t)D * SL + d]);
         m_prev = mn;
       }
   }
   if (DS > DM)
-    for (int idx = threadIdx.x; idx < (DS - DM) * (CS + 1); idx += 256) skt[DM * (CS + 1) + idx] = (bf16)0.0f;
+    for (int idx = threadIdx.x; idx < (DS - DM) * (CS + 1); idx += THREADS) skt[DM * (CS + 1) + idx] = (bf16)0.0f;
 
   float b_total = 0.f;
   for (int t0 = 0; t0 < count; t0 += CT) {
     const int cnt = count - t0 < CT ? count - t0 : CT;
     const size_t rb = (size_t)row0 + t0;
+    // (the many LDS addresses below are made anew in every chunk: kept in registers across chunks they spill)
+    asm volatile("" : "+v"(lane));
+    lg = lane >> 4;
+    lc = lane & 15;
+    const int tid = wave * 64 + lane;
     // ---- S in two bf16 parts, keys and values into LDS, gates
     if (OUTPUTS) {
 #pragma unroll
@@ -291,7 +311,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
     }
 #pragma unroll
     for (int it = 0; it < IPT; ++it) {
-      const int idx = threadIdx.x + it * 256, c = idx % CH, kp = idx / CH;
+      const int idx = tid + it * THREADS, c = idx % CH, kp = idx / CH;
       if (idx >= CT / 2 * CH) break;
       if (OUTPUTS) {
         *reinterpret_cast<u32x4*>(sk + (kp * 2) * KS + c * 8) = kr[it][0];
@@ -304,16 +324,18 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
         *reinterpret_cast<uint32_t*>(base + CS) = (kr[it][0][e] >> 16) | (kr[it][1][e] & 0xffff0000u);
       }
     }
-    // values: thread (token s = tid % 64, columns 16 * (tid / 64) ..): kept in registers for the weighted copy
-    const bf16x8 v0 = bitcast<bf16x8>(vr[0]), v1 = bitcast<bf16x8>(vr[1]);
-    if (OUTPUTS) {
-      const int s = threadIdx.x & 63, c0 = (threadIdx.x >> 6) * 16;
-      const int k32 = s & 31, place = (s & 32) + ((k32 & 15) >> 2) * 8 + (k32 >> 4) * 4 + (k32 & 3);
+    // values: thread (token s = tid % 64, columns VC * (tid / 64) ..): kept in registers for the weighted copy
+    bf16x8 v8[VV];
 #pragma unroll
-      for (int e = 0; e < 16; ++e) svt[(c0 + e) * CS + place] = e < 8 ? v0[e & 7] : v1[e & 7];
+    for (int h = 0; h < VV; ++h) v8[h] = bitcast<bf16x8>(ecols - wave * VC - h * 8 > 0 ? vr[h] : none);
+    if (OUTPUTS) {
+      const int s = lane, k32 = s & 31, place = (s & 32) + ((k32 & 15) >> 2) * 8 + (k32 >> 4) * 4 + (k32 & 3);
+#pragma unroll
+      for (int e = 0; e < VC; ++e) svt[(wave * VC + e) * CS + place] = v8[e >> 3][e & 7];
     }
     // gates of the chunk: running sums and maxima over the 64 lanes of the first wave
     if (wave == 0) {
+      const float gi = lane < cnt ? log_input_gate(zi, a.cap) : -INFINITY, gf = lane < cnt ? log_forget_gate(zf, a.cap) : 0.f;
       float bsum = gf;
 #pragma unroll
       for (int o = 1; o < 64; o <<= 1) {
@@ -338,7 +360,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
     bf16x8 qf[DT];
     if (OUTPUTS) {
 #pragma unroll
-      for (int c = 0; c < DT; ++c) qf[c] = bitcast<bf16x8>(qr[c]);
+      for (int c = 0; c < DT; ++c) qf[c] = bitcast<bf16x8>(D - c * 32 - lg * 8 > 0 ? qr[c] : none);
     }
     __syncthreads();
     if (t0 + CT < count) fetch(t0 + CT);
@@ -347,7 +369,8 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
     b_total += s_b[CT - 1];
     // ---- outputs of this wave's sixteen tokens
     if (OUTPUTS) {
-      const int t = wave * 16 + lc;
+      const int t = (wave & 3) * 16 + lc;
+      const int j0 = (wave >> 2) * JT;                        // first column tile of this wave's outputs
       float nq = 0.f;
 #pragma unroll
       for (int c = 0; c < DT; ++c)
@@ -356,33 +379,32 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
       nq += __shfl_xor(nq, 16, 64);
       nq += __shfl_xor(nq, 32, 64);
       const float Mt = s_M[t], bt = s_b[t], inter = expf(m_prev - Mt);
-      f32x4 o[4];
+      f32x4 o[JT];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-      // (two 32-row steps at a time: left to itself the scheduler requests every operand at once and spills)
+      for (int j = 0; j < JT; ++j) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int c = 0; c < DT; ++c) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int at = (j * 16 + lc) * SS + c * 32 + lg * 8;
+        for (int j = 0; j < JT; ++j) {
+          const int at = ((j0 + j) * 16 + lc) * SS + c * 32 + lg * 8;
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ss_hi + at), qf[c], o[j], 0, 0, 0);
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(ss_lo + at), qf[c], o[j], 0, 0, 0);
         }
-        if (c & 1) __builtin_amdgcn_sched_barrier(0);
       }
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < JT; ++j)
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[j][r] *= inter;
       nq *= inter;
       float psum = 0.f;
 #pragma unroll
       for (int kg = 0; kg < 2; ++kg) {
-        if (kg * 32 > wave * 16 + 15) continue;              // all of these keys come after this wave's tokens
+        if (kg * 32 > (wave & 3) * 16 + 15) continue;              // all of these keys come after this wave's tokens
         bf16x8 hi, lo;
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
           f32x4 p = {0.f, 0.f, 0.f, 0.f};
+          const f32x4 as = *reinterpret_cast<const f32x4*>(s_a + kg * 32 + h * 16 + lg * 4);
 #pragma unroll
           for (int c = 0; c < DT; ++c)
             p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
@@ -390,20 +412,18 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int s = kg * 32 + h * 16 + lg * 4 + r;
-            const float x = s <= t ? p[r] * expf(s_a[s] - Mt) : 0.f;
+            const float x = p[r] * __expf(s <= t ? as[r] - Mt : -INFINITY);
             psum += x;
             hi[h * 4 + r] = (bf16)x;
             lo[h * 4 + r] = (bf16)(x - (float)hi[h * 4 + r]);
           }
-          __builtin_amdgcn_sched_barrier(0);
         }
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(svt + (j * 16 + lc) * CS + kg * 32 + lg * 8);
+        for (int j = 0; j < JT; ++j) {
+          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(svt + ((j0 + j) * 16 + lc) * CS + kg * 32 + lg * 8);
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi, o[j], 0, 0, 0);
           o[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo, o[j], 0, 0, 0);
         }
-        __builtin_amdgcn_sched_barrier(0);
       }
       psum += __shfl_xor(psum, 16, 64);
       psum += __shfl_xor(psum, 32, 64);
@@ -412,8 +432,8 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
       if (t < cnt) {
         float* dst = a.o + (rb + t) * a.H * E + (size_t)head * E + e0;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int e = j * 16 + lg * 4;
+        for (int j = 0; j < JT; ++j) {
+          const int e = (j0 + j) * 16 + lg * 4;
           if (e + 4 <= ecols && (E & 3) == 0) {
             *reinterpret_cast<f32x4*>(dst + e) = f32x4{o[j][0] * f, o[j][1] * f, o[j][2] * f, o[j][3] * f};
           } else {
@@ -428,18 +448,18 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
 
     // ---- the state at the end of the chunk
     {
-      const int s = threadIdx.x & 63, c0 = (threadIdx.x >> 6) * 16;
+      const int s = lane;
       const float w = s < cnt ? s_w[s] : 0.f;
 #pragma unroll
-      for (int e = 0; e < 16; ++e) {
-        const float x = (float)(e < 8 ? v0[e & 7] : v1[e & 7]) * w;
+      for (int e = 0; e < VC; ++e) {
+        const float x = (float)v8[e >> 3][e & 7] * w;
         const bf16 hi = (bf16)x;
-        sw_hi[(c0 + e) * CS + s] = hi;
-        sw_lo[(c0 + e) * CS + s] = (bf16)(x - (float)hi);
+        sw_hi[(wave * VC + e) * CS + s] = hi;
+        sw_lo[(wave * VC + e) * CS + s] = (bf16)(x - (float)hi);
       }
     }
     const float decay = expf(m_prev - M_last);
-    for (int d = threadIdx.x; d < DM; d += 256) {
+    for (int d = tid; d < DM; d += THREADS) {
       float n = s_n[d] * decay;
 #pragma unroll
       for (int s = 0; s < CT; s += 8) {
@@ -475,7 +495,6 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
           S[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, wl[j], S[i][j], 0, 0, 0);
         }
       }
-      __builtin_amdgcn_sched_barrier(0);
     }
     m_prev = m_chunk;
     __syncthreads();                                          // before the next chunk's data replaces this one's
@@ -484,7 +503,7 @@ __global__ __launch_bounds__(256, 1) void mlstm_chunk_kernel(MA a, bool vec, int
     float* to = OUTPUTS ? st : part + (size_t)(seg + 1) * whole;
     each([&](float x, int at, bool there) { if (there) to[at] = x; return x; });
     for (int h = 0; h < (second ? 2 : 1); ++h) {
-      for (int d = threadIdx.x; d < D; d += 256) to[h * per + (size_t)D * SL + d] = s_n[d];
+      for (int d = threadIdx.x; d < D; d += THREADS) to[h * per + (size_t)D * SL + d] = s_n[d];
       if (threadIdx.x == 0) {
         to[h * per + (size_t)D * SL + D] = m_prev;
         if (!OUTPUTS) to[h * per + (size_t)D * SL + D + 1] = b_total;
@@ -512,14 +531,15 @@ extern "C" size_t pta_mlstm_workspace_bytes(const MA* args) {
   return n > 1 ? (size_t)args->seqs * n * pta_mlstm_state_floats(args->H, args->D, args->E) * sizeof(float) : 0;
 }
 
-template <int DT>
-static int launch_chunk(const MA& a, bool vec, hipStream_t s) {
+template <int DT, bool VEC>
+static int launch_chunk(const MA& a, hipStream_t s) {
   static bool ready = false;
   constexpr size_t smem = ChunkShape<DT>::lds;
   static_assert(smem + 4096 <= 160 * 1024, "LDS");
+  const void *outs = (const void*)mlstm_chunk_kernel<DT, true, VEC>, *sums = (const void*)mlstm_chunk_kernel<DT, false, VEC>;
   if (!ready) {
-    PTA_REQUIRE(hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DT, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess &&
-                hipFuncSetAttribute((const void*)mlstm_chunk_kernel<DT, false>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess,
+    PTA_REQUIRE(hipFuncSetAttribute(outs, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess &&
+                hipFuncSetAttribute(sums, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) == hipSuccess,
                 "pta_mlstm: cannot reserve %zu bytes of LDS", smem);
     ready = true;
   }
@@ -529,9 +549,15 @@ static int launch_chunk(const MA& a, bool vec, hipStream_t s) {
   PTA_REQUIRE(segments == 1 || (a.workspace && a.workspace_bytes >= need), "pta_mlstm: the workspace needs %zu bytes", need);
   const int slices = (a.E + SL - 1) / SL;
   const dim3 grid(a.seqs * a.H * ((slices + 1) / 2) * segments);
-  if (segments > 1) hipLaunchKernelGGL((mlstm_chunk_kernel<DT, false>), grid, dim3(256), smem, s, a, vec, length, segments, (float*)a.workspace);
-  hipLaunchKernelGGL((mlstm_chunk_kernel<DT, true>), grid, dim3(256), smem, s, a, vec, length, segments, (float*)a.workspace);
+  if (segments > 1)
+    hipLaunchKernelGGL((mlstm_chunk_kernel<DT, false, VEC>), grid, dim3(ChunkShape<DT>::THREADS), smem, s, a, length, segments, (float*)a.workspace);
+  hipLaunchKernelGGL((mlstm_chunk_kernel<DT, true, VEC>), grid, dim3(ChunkShape<DT>::THREADS), smem, s, a, length, segments, (float*)a.workspace);
   return PTA_OK;
+}
+
+template <int DT>
+static int launch_chunk(const MA& a, bool vec, hipStream_t s) {
+  return vec ? launch_chunk<DT, true>(a, s) : launch_chunk<DT, false>(a, s);
 }
 
 template <typename T>
@@ -558,7 +584,7 @@ extern "C" int pta_mlstm(const MA* args, pta_stream_t stream) {
     launch_scan<float>(a, s);
   } else if (a.chunked && a.D <= 256) {
     PTA_REQUIRE(a.longest >= 1 && a.longest <= a.rows, "pta_mlstm: longest sequence %d of %d rows", a.longest, a.rows);
-    const bool vec = a.D % 8 == 0 && a.ld % 8 == 0 && pta_aligned(a.q, 16) && pta_aligned(a.k, 16) && pta_aligned(a.v, 16);
+    const bool vec = a.D % 8 == 0 && a.E % 8 == 0 && a.ld % 8 == 0 && pta_aligned(a.q, 16) && pta_aligned(a.k, 16) && pta_aligned(a.v, 16);
     int rc;
     if (a.D <= 32) rc = launch_chunk<1>(a, vec, s);
     else if (a.D <= 64) rc = launch_chunk<2>(a, vec, s);
