@@ -10,7 +10,7 @@ Per layer with a feed-forward the launches of a decode iteration are: projection
 window merged by a second launch; or recurrence and head norm), output projection, stream update + norm, gate / up pair,
 down projection, stream update + norm.
 """
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 from typing import List, Optional
 
 import numpy as np
@@ -129,7 +129,7 @@ class HybridWeights:
     head: HK.WideWeight
 
     def nbytes(self):
-        """Bytes of weights one iteration reads (a layer counts as often as it is run by its users: see step_bytes)."""
+        """Bytes of the weights, each counted once (a layer that uses another one's reads them again)."""
         return self.head.nbytes + sum(w.nbytes for lay in self.layers if lay is not None for w in lay.linears())
 
 
@@ -279,7 +279,11 @@ class HybridDecoder(DecodeLoop):
 
     # ------------------------------------------------------------------ sequences that come and go
     def open(self):
-        return self.store.open()
+        capacity = self.store.capacity
+        slot = self.store.open()
+        if self.store.capacity != capacity:
+            self.graph = None            # the recorded iteration addresses the memory the store has left
+        return slot
 
     def close(self, slot):
         self.store.close(slot)
