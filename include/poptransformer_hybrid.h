@@ -56,10 +56,18 @@ typedef struct pta_wide_linear_args {
   void* workspace;        /* NULL, or scratch of pta_wide_linear_workspace_bytes(M, N): lets bf16 launches with few
                              channels split K across workgroups                                                    */
   size_t workspace_bytes;
+  /* main channels, in this order: sum + bias, cap, sigmoid, * mul, += Y */
+  const float* bias;      /* [n_main] or NULL (of a pair: the gate's)                                              */
+  const float* bias2;     /* [n_main] or NULL: the up weight's of a pair                                           */
+  int sigmoid;            /* y = sigmoid(y)                                                                        */
+  const void* mul;        /* NULL, or [M, ld] of the type of X: y = y * mul                                        */
+  int accumulate;         /* Y += y (fp32 Y only)                                                                  */
 } pta_wide_linear_args;
 
 size_t pta_wide_linear_workspace_bytes(int M, int N);
 int pta_wide_linear(const pta_wide_linear_args* host_args, pta_stream_t stream);
+/* up to four single weights over inputs of the same shape, each with its own input and result: one launch for up to 16 rows */
+int pta_wide_linear_group(const pta_wide_linear_args* host_list, int count, pta_stream_t stream);
 
 /* ---- Residual streams (hyper-connections) and layer norm ---------------------------------------------------------
  * streams fp32 [rows][S][width].  One launch per sublayer boundary, one workgroup per row:
@@ -94,6 +102,41 @@ typedef struct pta_streams_args {
 } pta_streams_args;
 
 int pta_streams_norm(const pta_streams_args* host_args, pta_stream_t stream);
+
+/* ---- One fp32 residual, sublayers in parallel: grouped RMS norm and token shift -----------------------------------
+ * x fp32 [rows][width].  With n(x) = every one of `groups` equal parts of x over its own sqrt(mean square + eps):
+ *   h1 = n(x) w1,  h2 = n(x) w2,  hm_t = h1_t + (h1_{t-1} - h1_t) * shift   (h1 in fp32; zeros before position 0).
+ * With `table` the row is made first: x = table[id] * embed_scale + pos_table[position].
+ * state fp32 [slots][width] holds h1 of a sequence's newest token.  last[r]: for the first row of a sequence in the pass
+ * the row of its last token, else -1 (NULL: every row is a sequence of its own).  Positions are clamped to positions - 1. */
+typedef struct pta_shift_norm_args {
+  int dtype;              /* type of h1, h2, hm and of the tables                                                  */
+  int rows, width, groups;
+  float* x;
+  const void* table;      /* [vocab, width] or NULL                                                                */
+  const void* pos_table;  /* [positions, width] or NULL                                                            */
+  int vocab, positions;
+  float embed_scale;
+  const int32_t* ids;     /* id of row r: ids[r * ids_stride + (ids_index ? *ids_index : 0)]                       */
+  int ids_stride;
+  const int32_t* ids_index;
+  const int32_t* pos;     /* [rows]; with ids_index every row's position is *ids_index                             */
+  int32_t* pos_out;       /* [rows] or NULL                                                                        */
+  const int32_t* gather;  /* NULL, or: output row r is made from row gather[r]                                     */
+  float eps;
+  const float* w1;        /* [width]                                                                               */
+  const float* w2;        /* [width], with h2                                                                      */
+  const float* shift;     /* [width] or NULL                                                                       */
+  float* state;
+  const int32_t* slot;    /* [rows]                                                                                */
+  const int32_t* last;
+  void* h1;               /* [rows, h_ld], columns past width zero; h2 and hm likewise                             */
+  void* h2;
+  void* hm;
+  int h_ld;
+} pta_shift_norm_args;
+
+int pta_shift_norm(const pta_shift_norm_args* host_args, pta_stream_t stream);
 
 /* ---- Windowed attention with a distance bias ---------------------------------------------------------------------
  * score(i, j) = scale * (q_i . k_j) - slope_h * (i - j) for 0 <= i - j < window, ordinary softmax, and the concatenated
@@ -140,6 +183,73 @@ int pta_window_append(const pta_window_attention_args* host_args, pta_stream_t s
 int pta_window_attention(const pta_window_attention_args* host_args, pta_stream_t stream);
 /* one row per sequence: norm, append and attention in one launch (two with splits > 1) */
 int pta_window_decode(const pta_window_attention_args* host_args, pta_stream_t stream);
+
+/* ---- Attention over latents ---------------------------------------------------------------------------------------
+ * A token leaves one row in the cache: its normed latent c and one rotated key part that all heads share.  Head h has the
+ * key (W_uk,h c | rotated part), the value W_uv,h c, and score(i, j) = scale * (q_i . k_j) for 0 <= i - j < window, an
+ * ordinary softmax, and its result times sigmoid(gate_h).  Two ways to the same numbers:
+ *   absorbed (decode, short portions, fp32): q'_h = W_uk,h^T q_h meets the cached rows themselves, and W_uv,h is applied
+ *     to the weighted sum of latents;
+ *   over heads (prompts): keys and values of all heads are made from the cached rows (a Linear over pta_latent_gather's
+ *     result) and a tile of rows works through them on the matrix unit.
+ * Sizes as stored: D, P and R are the head's unrotated and rotated dimensions and the latent, each rounded up to 32 with
+ * zeros, E the value size rounded up to 16.  A query head is [D | P].  Rotated features come in pairs: 2 i and 2 i + 1 are
+ * turned by cos_sin[position][i], which pairs any layout's partners after a permutation of the weights' rows.
+ * Cache of a layer: ring [slots][ring_len][R + P]; position p is row p % ring_len, and ring_len >= window - 1 + (most rows
+ * a sequence has in one pass).  Several layers may read one cache. */
+typedef struct pta_latent_args {
+  int dtype;
+  int rows, H, D, P, E, R;
+  int q_rank, kv_rank;    /* true sizes of the two norms                                                           */
+  const void* proj;       /* [rows, ld]: query latent (q_rank rounded up to 8) | latent (R) | rotated part (P)     */
+  int ld;
+  const float* q_norm;    /* [q_rank]                                                                              */
+  const float* kv_norm;   /* [kv_rank]; NULL: the layer reads another one's cache, proj holds the query latent only */
+  float eps;
+  void* cq;               /* [rows, q_rank rounded up to 8]: the normed query latent                               */
+  const float* cos_sin;   /* [positions][P / 2][2]                                                                 */
+  int positions;
+  void* ring;
+  int ring_len;
+  const int32_t* slot;    /* [rows]                                                                                */
+  const int32_t* pos;     /* [rows]                                                                                */
+  const void* q;          /* [rows, H, D + P], not rotated yet                                                     */
+  const void* uk_t;       /* [H, R, D]                                                                             */
+  void* q_latent;         /* [rows, H, R + P]                                                                      */
+  float scale;
+  int window;             /* > 0                                                                                   */
+  int splits;             /* absorbed: parts a row's window is cut into, 1 .. 64                                   */
+  float* part_o;          /* [rows, H, splits, R]: sums of weighted latents                                        */
+  float* part_ml;         /* [rows, H, splits, 2]: their largest score and sum of weights                          */
+  const void* uv;         /* [H, E, R]                                                                             */
+  const float* gate;      /* [rows, H], before the sigmoid                                                         */
+  void* out;              /* [rows, H * E]                                                                         */
+  /* over heads */
+  int keys;               /* rows of the key buffers                                                               */
+  const int32_t* key_slot;   /* [keys] the cache rows of pta_latent_gather                                         */
+  const int32_t* key_pos;
+  void* key_latent;       /* [keys, R]                                                                             */
+  void* key_rot;          /* [keys, P]                                                                             */
+  const void* kv;         /* [keys, H * D | H * E]                                                                 */
+  const int32_t* tile_row;   /* [tiles] first row of a tile: rows of one sequence, at most PTA_LATENT_TILE          */
+  const int32_t* tile_count; /* [tiles]                                                                            */
+  const int32_t* tile_key;   /* [tiles] key row of the sequence's position 0 (negative where the buffer starts later) */
+  int tiles;
+} pta_latent_args;
+
+enum { PTA_LATENT_TILE = 128 };
+
+/* normed query latents; the rows' cache entries where the layer has a cache of its own */
+int pta_latent_append(const pta_latent_args* host_args, pta_stream_t stream);
+int pta_latent_absorb(const pta_latent_args* host_args, pta_stream_t stream);
+/* every row over its part of the cache: bf16 on the matrix unit where R <= 1024 and P <= 128, else on the vector unit */
+int pta_latent_rows(const pta_latent_args* host_args, pta_stream_t stream);
+/* parts put together, W_uv, gate */
+int pta_latent_values(const pta_latent_args* host_args, pta_stream_t stream);
+int pta_latent_gather(const pta_latent_args* host_args, pta_stream_t stream);
+/* whether pta_latent_tiles takes these sizes */
+int pta_latent_tiles_fit(int dtype, int D, int P, int E);
+int pta_latent_tiles(const pta_latent_args* host_args, pta_stream_t stream);
 
 /* ---- Matrix memory (mLSTM) ---------------------------------------------------------------------------------------
  * Per head, with log gates i = cap tanh(z_i / cap), f = log sigmoid(cap tanh(z_f / cap)) from the fp32 pre-activations:

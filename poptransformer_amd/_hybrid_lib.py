@@ -13,6 +13,7 @@ BF16, FP32 = 0, 1
 PAIR_NONE, PAIR_SWIGLU, PAIR_CLAMPED = 0, 1, 2
 WINDOW_TILE = 128
 MLSTM_SLICE = 32
+LATENT_TILE = 128
 
 
 def _struct(name, fields):
@@ -23,7 +24,7 @@ _P, _I, _F = c_void_p, c_int, c_float
 WideLinearArgs = _struct("WideLinearArgs", [
     ("dtype", _I), ("X", _P), ("M", _I), ("K", _I), ("N", _I), ("W", _P), ("W2", _P), ("pair", _I), ("limit", _F), ("slope", _F),
     ("cap", _F), ("Y", _P), ("ld", _I), ("n_main", _I), ("out_f32", _I), ("tail", _P), ("tail_count", _I), ("tail_bias", _P),
-    ("workspace", _P), ("workspace_bytes", c_size_t)])
+    ("workspace", _P), ("workspace_bytes", c_size_t), ("bias", _P), ("bias2", _P), ("sigmoid", _I), ("mul", _P), ("accumulate", _I)])
 StreamsArgs = _struct("StreamsArgs", [
     ("dtype", _I), ("rows", _I), ("width", _I), ("S", _I), ("streams", _P), ("table", _P), ("vocab", _I), ("embed_scale", _F),
     ("ids", _P), ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("y", _P), ("out", _P), ("mix", _P), ("mult", _F),
@@ -33,6 +34,18 @@ WindowArgs = _struct("WindowArgs", [
     ("k_norm", _P), ("eps", _F), ("scale", _F), ("slopes", _P), ("window", _I), ("ring", _P), ("rinv", _P), ("ring_len", _I),
     ("slot", _P), ("pos", _P), ("q_scale", _P), ("tile_row", _P), ("tile_count", _P), ("tiles", _I), ("splits", _I),
     ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P), ("out_ld", _I)])
+ShiftNormArgs = _struct("ShiftNormArgs", [
+    ("dtype", _I), ("rows", _I), ("width", _I), ("groups", _I), ("x", _P), ("table", _P), ("pos_table", _P), ("vocab", _I),
+    ("positions", _I), ("embed_scale", _F), ("ids", _P), ("ids_stride", _I), ("ids_index", _P), ("pos", _P), ("pos_out", _P),
+    ("gather", _P), ("eps", _F), ("w1", _P), ("w2", _P), ("shift", _P), ("state", _P), ("slot", _P), ("last", _P), ("h1", _P),
+    ("h2", _P), ("hm", _P), ("h_ld", _I)])
+LatentArgs = _struct("LatentArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("P", _I), ("E", _I), ("R", _I), ("q_rank", _I), ("kv_rank", _I), ("proj", _P),
+    ("ld", _I), ("q_norm", _P), ("kv_norm", _P), ("eps", _F), ("cq", _P), ("cos_sin", _P), ("positions", _I), ("ring", _P),
+    ("ring_len", _I), ("slot", _P), ("pos", _P), ("q", _P), ("uk_t", _P), ("q_latent", _P), ("scale", _F), ("window", _I),
+    ("splits", _I), ("part_o", _P), ("part_ml", _P), ("uv", _P), ("gate", _P), ("out", _P), ("keys", _I), ("key_slot", _P),
+    ("key_pos", _P), ("key_latent", _P), ("key_rot", _P), ("kv", _P), ("tile_row", _P), ("tile_count", _P), ("tile_key", _P),
+    ("tiles", _I)])
 MlstmArgs = _struct("MlstmArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("E", _I), ("q", _P), ("k", _P), ("v", _P), ("ld", _I), ("gates", _P),
     ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("longest", _I), ("chunked", _I),
@@ -44,6 +57,10 @@ SIGNATURES = {
     "pta_bf16_tile": (_I, [_P, _P, _I, _I, _P]),
     "pta_wide_linear_workspace_bytes": (c_size_t, [_I, _I]),
     "pta_wide_linear": (_I, [POINTER(WideLinearArgs), _P]),
+    "pta_wide_linear_group": (_I, [POINTER(WideLinearArgs), _I, _P]),
+    "pta_shift_norm": (_I, [POINTER(ShiftNormArgs), _P]),
+    **{f"pta_latent_{n}": (_I, [POINTER(LatentArgs), _P]) for n in ("append", "absorb", "rows", "values", "gather", "tiles")},
+    "pta_latent_tiles_fit": (_I, [_I, _I, _I, _I]),
     "pta_streams_norm": (_I, [POINTER(StreamsArgs), _P]),
     "pta_window_attention_workspace_bytes": (c_size_t, [_I, _I, _I, _I]),
     "pta_window_append": (_I, [POINTER(WindowArgs), _P]),

@@ -19,6 +19,12 @@ struct WideOut {
   float cap;                // > 0: y = cap * tanh(y / cap)
   int clamped;              // pairs: 0 = SwiGLU, 1 = min(g, limit) sigmoid(slope g) (clamp(u, -limit, limit) + 1)
   float limit, slope;
+  const float* bias;        // [n_main] or null, added to the sum (of a pair: to the gate's)
+  const float* bias2;       // [n_main] or null, added to the sum of a pair's second weight
+  int sigmoid;              // y = sigmoid(y)
+  const void* mul;          // [M, ld] or null, fp32 (mul_f32) or bf16: y = y * mul
+  int mul_f32;
+  int accumulate;           // Y (fp32) += y
 };
 
 struct GemmEpilogue {
@@ -35,7 +41,6 @@ struct GemmEpilogue {
   int out_fp8_format;
   f16* mix_state;                 // [2][M, K] or null: the previous token's rows for the token-shift mixes (gemv_lds_kernel)
   const int32_t* mix_step;
-  WideOut wide;                   // of the formats whose epilogue works in fp32 (Fmt::kWide)
 };
 
 __device__ __forceinline__ f16 sigmoid_f16(f16 x) {
@@ -82,7 +87,7 @@ __device__ __forceinline__ f16 swiglu_out(const GemmEpilogue& e, f16 gate, f16 u
 }
 
 static inline int make_epilogue(const pta_fusion* in, GemmEpilogue* out, const char* name) {
-  *out = GemmEpilogue{nullptr, nullptr, PTA_ACT_NONE, nullptr, 0.f, PTA_NORM_NONE, nullptr, nullptr, 0.f, nullptr, PTA_F143, nullptr, nullptr, WideOut{}};
+  *out = GemmEpilogue{nullptr, nullptr, PTA_ACT_NONE, nullptr, 0.f, PTA_NORM_NONE, nullptr, nullptr, 0.f, nullptr, PTA_F143, nullptr, nullptr};
   if (!in) return PTA_OK;
   PTA_REQUIRE(in->act >= PTA_ACT_NONE && in->act <= PTA_ACT_SIGMOID, "%s: unknown activation %d", name, in->act);
   PTA_REQUIRE(in->norm >= PTA_NORM_NONE && in->norm <= PTA_NORM_LAYER, "%s: unknown norm %d", name, in->norm);
@@ -121,12 +126,19 @@ struct GemmMat {
   f16* Y;
   int N;
   int nb_begin;        // first 16-channel block of this matrix in the launch grid
+  WideOut wide;        // of the formats whose epilogue works in fp32 (Fmt::kWide)
 };
 
 // The fp32 epilogue of the wide formats (Y is a bf16 or fp32 buffer behind the f16* of GemmMat).
-__device__ __forceinline__ float wide_value(const WideOut& w, float v) { return w.cap > 0.f ? w.cap * tanhf(v / w.cap) : v; }
+__device__ __forceinline__ float wide_value(const WideOut& w, int n, float v) {
+  if (w.bias) v += w.bias[n];
+  if (w.cap > 0.f) v = w.cap * tanhf(v / w.cap);
+  return w.sigmoid ? 1.0f / (1.0f + expf(-v)) : v;
+}
 
-__device__ __forceinline__ float wide_pair_value(const WideOut& w, float g, float u) {
+__device__ __forceinline__ float wide_pair_value(const WideOut& w, int n, float g, float u) {
+  if (w.bias) g += w.bias[n];
+  if (w.bias2) u += w.bias2[n];
   if (!w.clamped) return u * g / (1.0f + expf(-g));
   g = fminf(g, w.limit);
   u = fminf(fmaxf(u, -w.limit), w.limit);
@@ -134,59 +146,88 @@ __device__ __forceinline__ float wide_pair_value(const WideOut& w, float g, floa
 }
 
 __device__ __forceinline__ void wide_store(const WideOut& w, const GemmMat& mat, int m, int n, float v) {
-  if (w.out_f32) reinterpret_cast<float*>(mat.Y)[(size_t)m * w.ld + n] = v;
-  else reinterpret_cast<bf16*>(mat.Y)[(size_t)m * w.ld + n] = (bf16)v;
+  const size_t at = (size_t)m * w.ld + n;
+  if (w.mul) v *= w.mul_f32 ? reinterpret_cast<const float*>(w.mul)[at] : (float)reinterpret_cast<const bf16*>(w.mul)[at];
+  if (w.accumulate) v += reinterpret_cast<const float*>(mat.Y)[at];
+  if (w.out_f32) reinterpret_cast<float*>(mat.Y)[at] = v;
+  else reinterpret_cast<bf16*>(mat.Y)[at] = (bf16)v;
 }
 
-__device__ __forceinline__ void wide_put(const WideOut& w, const GemmMat& mat, int m, int n, float v) {
+__device__ __forceinline__ void wide_put(const GemmMat& mat, int m, int n, float v) {
+  const WideOut& w = mat.wide;
   if (n < w.n_main) {
-    wide_store(w, mat, m, n, wide_value(w, v));
+    wide_store(w, mat, m, n, wide_value(w, n, v));
   } else if (n - w.n_main < w.tail_count) {
     const int c = n - w.n_main;
     w.tail[(size_t)m * w.tail_count + c] = w.tail_bias ? v + w.tail_bias[c] : v;
   }
 }
 
-__device__ __forceinline__ void wide_put_pair(const WideOut& w, const GemmMat& mat, int m, int n, float gate, float up) {
-  if (n < w.n_main) wide_store(w, mat, m, n, wide_pair_value(w, gate, up));
+__device__ __forceinline__ void wide_put_pair(const GemmMat& mat, int m, int n, float gate, float up) {
+  const WideOut& w = mat.wide;
+  if (n < w.n_main) wide_store(w, mat, m, n, wide_pair_value(w, n, gate, up));
 }
 
 // four consecutive channels of a row, n a multiple of four
 __device__ __forceinline__ void wide_store4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 v) {
+  const size_t at = (size_t)m * w.ld + n;
+  if (w.mul) {
+    f32x4 g;
+    if (w.mul_f32) {
+      g = *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(w.mul) + at);
+    } else {
+      const bf16x4 b = *reinterpret_cast<const bf16x4*>(reinterpret_cast<const bf16*>(w.mul) + at);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) g[r] = (float)b[r];
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] *= g[r];
+  }
+  if (w.accumulate) {
+    const f32x4 y = *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(mat.Y) + at);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] += y[r];
+  }
   if (w.out_f32) {
-    *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(mat.Y) + (size_t)m * w.ld + n) = v;
+    *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(mat.Y) + at) = v;
   } else {
     bf16x4 b;
 #pragma unroll
     for (int r = 0; r < 4; ++r) b[r] = (bf16)v[r];
-    *reinterpret_cast<bf16x4*>(reinterpret_cast<bf16*>(mat.Y) + (size_t)m * w.ld + n) = b;
+    *reinterpret_cast<bf16x4*>(reinterpret_cast<bf16*>(mat.Y) + at) = b;
   }
 }
 
-__device__ __forceinline__ void wide_put4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 v) {
+__device__ __forceinline__ void wide_put4(const GemmMat& mat, int m, int n, f32x4 v) {
+  const WideOut& w = mat.wide;
   if (n + 4 <= w.n_main && (w.ld & 3) == 0) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = wide_value(w, v[r]);
+    for (int r = 0; r < 4; ++r) v[r] = wide_value(w, n + r, v[r]);
     wide_store4(w, mat, m, n, v);
   } else {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) wide_put(w, mat, m, n + r, v[r]);
+    for (int r = 0; r < 4; ++r) wide_put(mat, m, n + r, v[r]);
   }
 }
 
-__device__ __forceinline__ void wide_put_pair4(const WideOut& w, const GemmMat& mat, int m, int n, f32x4 gate, f32x4 up) {
+__device__ __forceinline__ void wide_put_pair4(const GemmMat& mat, int m, int n, f32x4 gate, f32x4 up) {
+  const WideOut& w = mat.wide;
   if (n + 4 <= w.n_main && (w.ld & 3) == 0) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) gate[r] = wide_pair_value(w, gate[r], up[r]);
+    for (int r = 0; r < 4; ++r) gate[r] = wide_pair_value(w, n + r, gate[r], up[r]);
     wide_store4(w, mat, m, n, gate);
   } else {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) wide_put_pair(w, mat, m, n + r, gate[r], up[r]);
+    for (int r = 0; r < 4; ++r) wide_put_pair(mat, m, n + r, gate[r], up[r]);
   }
 }
 
-static inline f16* wide_rows_from(const WideOut& w, f16* Y, int m0) {
-  return reinterpret_cast<f16*>(reinterpret_cast<unsigned char*>(Y) + (size_t)m0 * w.ld * (w.out_f32 ? 4 : 2));
+// the rows from m0 on
+static inline void wide_skip_rows(GemmMat& mat, int m0) {
+  WideOut& w = mat.wide;
+  mat.Y = reinterpret_cast<f16*>(reinterpret_cast<unsigned char*>(mat.Y) + (size_t)m0 * w.ld * (w.out_f32 ? 4 : 2));
+  if (w.tail) w.tail += (size_t)m0 * w.tail_count;
+  if (w.mul) w.mul = reinterpret_cast<const unsigned char*>(w.mul) + (size_t)m0 * w.ld * (w.mul_f32 ? 4 : 2);
 }
 
 struct GemmArgs {
@@ -208,7 +249,7 @@ struct GemmArgs {
 template <class Fmt>
 __device__ __forceinline__ void gemm_put(const GemmArgs& a, const GemmMat& mat, int m, int n, int N, float sum) {
   if constexpr (Fmt::kWide) {
-    wide_put(a.epi.wide, mat, m, n, sum);
+    wide_put(mat, m, n, sum);
   } else {
     f16 y0 = (f16)sum;
     if (mat.bias) y0 = y0 + mat.bias[n];
@@ -219,7 +260,7 @@ __device__ __forceinline__ void gemm_put(const GemmArgs& a, const GemmMat& mat, 
 
 template <class Fmt>
 __device__ __forceinline__ void gemm_put_pair(const GemmArgs& a, int m, int n, int N, float gate, float up) {
-  if constexpr (Fmt::kWide) wide_put_pair(a.epi.wide, a.mat[0], m, n, gate, up);
+  if constexpr (Fmt::kWide) wide_put_pair(a.mat[0], m, n, gate, up);
   else a.mat[0].Y[(size_t)m * N + n] = swiglu_out(a.epi, (f16)gate, (f16)up);
 }
 
@@ -1418,7 +1459,7 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const int m = row0 + rg * 16 + (lane & 15);
       const f32x4 g4 = sums[(rg * ROWS_CB + st) * 64 + lane], u4 = sums[(rg * ROWS_CB + st + ROWS_CB / 2) * 64 + lane];
       if constexpr (Fmt::kWide) {
-        if (m < M) wide_put_pair4(a.epi.wide, mat, m, (first_blk + st) * 16 + (lane >> 4) * 4, g4, u4);
+        if (m < M) wide_put_pair4(mat, m, (first_blk + st) * 16 + (lane >> 4) * 4, g4, u4);
         continue;
       }
 #pragma unroll
@@ -1439,7 +1480,7 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const f32x4 v4 = sums[i * 64 + lane];
       if constexpr (Fmt::kWide) {
         if (nsl == 1) {
-          if (m < M) wide_put4(a.epi.wide, mat, m, stream_blk(st) * 16 + (lane >> 4) * 4, v4);
+          if (m < M) wide_put4(mat, m, stream_blk(st) * 16 + (lane >> 4) * 4, v4);
           continue;
         }
       }
@@ -1944,10 +1985,9 @@ static int dispatch_many_rows(const GemmArgs& a, int total_nb, hipStream_t s, co
     if (b.X) b.X += (size_t)m0 * a.K;
     for (int i = 0; i < a.count; ++i) {
       if (b.mat[i].X) b.mat[i].X += (size_t)m0 * a.K;
-      if constexpr (Fmt::kWide) b.mat[i].Y = wide_rows_from(a.epi.wide, a.mat[i].Y, m0);
+      if constexpr (Fmt::kWide) wide_skip_rows(b.mat[i], m0);
       else if (!PAIR || i == 0) b.mat[i].Y += (size_t)m0 * a.mat[i].N;
     }
-    if (b.epi.wide.tail) b.epi.wide.tail += (size_t)m0 * b.epi.wide.tail_count;
     if (PAIR) b.mat[1].Y = b.mat[0].Y;
     if (b.epi.residual) b.epi.residual += (size_t)m0 * a.mat[0].N;
     if (b.epi.mul) b.epi.mul += (size_t)m0 * a.mat[0].N;

@@ -41,7 +41,7 @@ constexpr int F32_ROWS = 8;
 
 template <bool PAIR>
 __global__ __launch_bounds__(256) void f32_gemv_kernel(const float* __restrict__ X, const float* __restrict__ W,
-                                                       const float* __restrict__ W2, int M, int K, int N, WideOut out, GemmMat mat) {
+                                                       const float* __restrict__ W2, int M, int K, int N, GemmMat mat) {
   const int lane = threadIdx.x & 63;
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (n >= N) return;
@@ -66,8 +66,8 @@ __global__ __launch_bounds__(256) void f32_gemv_kernel(const float* __restrict__
     const float s = wave_sum(acc[m]);
     const float s2 = PAIR ? wave_sum(acc2[m]) : 0.f;
     if (lane == 0 && m < M) {
-      if (PAIR) wide_put_pair(out, mat, m, n, s, s2);
-      else wide_put(out, mat, m, n, s);
+      if (PAIR) wide_put_pair(mat, m, n, s, s2);
+      else wide_put(mat, m, n, s);
     }
   }
 }
@@ -75,7 +75,7 @@ __global__ __launch_bounds__(256) void f32_gemv_kernel(const float* __restrict__
 // many rows: 64 x 64 outputs per workgroup, 4 x 4 per thread, 16 features at a time through LDS
 template <bool PAIR>
 __global__ __launch_bounds__(256) void f32_gemm_kernel(const float* __restrict__ X, const float* __restrict__ W,
-                                                       const float* __restrict__ W2, int M, int K, int N, WideOut out, GemmMat mat) {
+                                                       const float* __restrict__ W2, int M, int K, int N, GemmMat mat) {
   constexpr int T = 64, KS = 16, NW = PAIR ? 2 : 1;
   __shared__ float xs[KS][T + 4], ws[NW][KS][T + 4];
   const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
@@ -117,19 +117,19 @@ __global__ __launch_bounds__(256) void f32_gemm_kernel(const float* __restrict__
     for (int j = 0; j < 4; ++j) {
       const int m = m0 + ty * 4 + i, n = n0 + tx * 4 + j;
       if (m >= M || n >= N) continue;
-      if (PAIR) wide_put_pair(out, mat, m, n, acc[0][i][j], acc[NW - 1][i][j]);
-      else wide_put(out, mat, m, n, acc[0][i][j]);
+      if (PAIR) wide_put_pair(mat, m, n, acc[0][i][j], acc[NW - 1][i][j]);
+      else wide_put(mat, m, n, acc[0][i][j]);
     }
 }
 
 template <bool PAIR>
-static void launch_f32(const pta_wide_linear_args& a, const WideOut& out, const GemmMat& mat, hipStream_t s) {
+static void launch_f32(const pta_wide_linear_args& a, const GemmMat& mat, hipStream_t s) {
   const float *X = (const float*)a.X, *W = (const float*)a.W, *W2 = (const float*)a.W2;
   if (a.M <= F32_ROWS)
-    hipLaunchKernelGGL((f32_gemv_kernel<PAIR>), dim3((a.N + 3) / 4), dim3(256), 0, s, X, W, W2, a.M, a.K, a.N, out, mat);
+    hipLaunchKernelGGL((f32_gemv_kernel<PAIR>), dim3((a.N + 3) / 4), dim3(256), 0, s, X, W, W2, a.M, a.K, a.N, mat);
   else
     hipLaunchKernelGGL((f32_gemm_kernel<PAIR>), dim3((a.N + 63) / 64, (a.M + 63) / 64), dim3(256), 0, s, X, W, W2, a.M, a.K,
-                       a.N, out, mat);
+                       a.N, mat);
 }
 
 extern "C" size_t pta_wide_linear_workspace_bytes(int M, int N) {
@@ -137,29 +137,58 @@ extern "C" size_t pta_wide_linear_workspace_bytes(int M, int N) {
   return (size_t)GEMM_MAX_KSPLIT * M * N * sizeof(float);
 }
 
-extern "C" int pta_wide_linear(const pta_wide_linear_args* args, pta_stream_t stream) {
-  PTA_REQUIRE(args, "pta_wide_linear: null arguments");
-  const pta_wide_linear_args& a = *args;
+static int check_wide(const pta_wide_linear_args& a, const char* name) {
   const bool pair = a.pair != PTA_PAIR_NONE;
-  PTA_REQUIRE(a.dtype == PTA_BF16 || a.dtype == PTA_FP32, "pta_wide_linear: unknown type %d", a.dtype);
-  PTA_REQUIRE(a.pair >= PTA_PAIR_NONE && a.pair <= PTA_PAIR_CLAMPED, "pta_wide_linear: unknown pair %d", a.pair);
-  const int rc = check_gemv_common("pta_wide_linear", a.X, a.M, a.K);
+  PTA_REQUIRE(a.dtype == PTA_BF16 || a.dtype == PTA_FP32, "%s: unknown type %d", name, a.dtype);
+  PTA_REQUIRE(a.pair >= PTA_PAIR_NONE && a.pair <= PTA_PAIR_CLAMPED, "%s: unknown pair %d", name, a.pair);
+  const int rc = check_gemv_common(name, a.X, a.M, a.K);
   if (rc) return rc;
-  PTA_REQUIRE(a.W && a.Y && a.N > 0 && pta_aligned(a.W, 16) && pta_aligned(a.Y, 16), "pta_wide_linear: null or unaligned operand");
-  PTA_REQUIRE(!pair || (a.W2 && pta_aligned(a.W2, 16)), "pta_wide_linear: a pair needs its second weight");
+  PTA_REQUIRE(a.W && a.Y && a.N > 0 && pta_aligned(a.W, 16) && pta_aligned(a.Y, 16), "%s: null or unaligned operand", name);
+  PTA_REQUIRE(!pair || (a.W2 && pta_aligned(a.W2, 16)), "%s: a pair needs its second weight", name);
   PTA_REQUIRE(a.n_main >= 1 && a.n_main <= a.ld && a.tail_count >= 0 && a.n_main + a.tail_count <= a.N,
-              "pta_wide_linear: n_main %d (ld %d) and tail %d do not fit %d channels", a.n_main, a.ld, a.tail_count, a.N);
-  PTA_REQUIRE(a.tail_count == 0 || (a.tail && !pair), "pta_wide_linear: a tail needs its buffer, and a single weight");
-  PTA_REQUIRE(a.pair != PTA_PAIR_CLAMPED || a.limit > 0.f, "pta_wide_linear: the clamped pair needs a positive limit");
-  WideOut out{a.ld, a.n_main, a.dtype == PTA_FP32 ? 1 : a.out_f32, a.tail, a.tail_count, a.tail_bias, a.cap,
-              a.pair == PTA_PAIR_CLAMPED ? 1 : 0, a.limit, a.slope};
-  hipStream_t s = (hipStream_t)stream;
+              "%s: n_main %d (ld %d) and tail %d do not fit %d channels", name, a.n_main, a.ld, a.tail_count, a.N);
+  PTA_REQUIRE(a.tail_count == 0 || (a.tail && !pair), "%s: a tail needs its buffer, and a single weight", name);
+  PTA_REQUIRE(a.pair != PTA_PAIR_CLAMPED || a.limit > 0.f, "%s: the clamped pair needs a positive limit", name);
+  PTA_REQUIRE(pair || !a.bias2, "%s: a second bias belongs to a pair", name);
+  PTA_REQUIRE(!a.accumulate || a.out_f32 || a.dtype == PTA_FP32, "%s: only fp32 results accumulate", name);
+  PTA_REQUIRE(!a.mul || pta_aligned(a.mul, 16), "%s: the multiplier must be 16-byte aligned", name);
+  PTA_REQUIRE(!a.workspace || pta_aligned(a.workspace, 16), "%s: the workspace must be 16-byte aligned", name);
+  return PTA_OK;
+}
+
+static GemmMat wide_matrix(const pta_wide_linear_args& a, const void* W) {
+  GemmMat mat{};
+  mat.tiled = W;
+  mat.act = PTA_ACT_NONE;
+  mat.Y = (f16*)a.Y;
+  mat.N = a.N;
+  WideOut& w = mat.wide;
+  w.ld = a.ld;
+  w.n_main = a.n_main;
+  w.out_f32 = a.dtype == PTA_FP32 ? 1 : a.out_f32;
+  w.tail = a.tail;
+  w.tail_count = a.tail_count;
+  w.tail_bias = a.tail_bias;
+  w.cap = a.cap;
+  w.clamped = a.pair == PTA_PAIR_CLAMPED;
+  w.limit = a.limit;
+  w.slope = a.slope;
+  w.bias = a.bias;
+  w.bias2 = a.bias2;
+  w.sigmoid = a.sigmoid;
+  w.mul = a.mul;
+  w.mul_f32 = a.dtype == PTA_FP32;
+  w.accumulate = a.accumulate;
+  return mat;
+}
+
+static int wide_linear(const pta_wide_linear_args& a, hipStream_t s, const char* name) {
+  const bool pair = a.pair != PTA_PAIR_NONE;
   if (a.dtype == PTA_FP32) {
-    GemmMat mat{};
-    mat.Y = (f16*)a.Y;
-    if (pair) launch_f32<true>(a, out, mat, s);
-    else launch_f32<false>(a, out, mat, s);
-    PTA_CHECK_LAUNCH("pta_wide_linear");
+    const GemmMat mat = wide_matrix(a, a.W);
+    if (pair) launch_f32<true>(a, mat, s);
+    else launch_f32<false>(a, mat, s);
+    PTA_CHECK_LAUNCH(name);
     return PTA_OK;
   }
   GemmArgs g{};
@@ -168,15 +197,51 @@ extern "C" int pta_wide_linear(const pta_wide_linear_args* args, pta_stream_t st
   g.M = a.M;
   g.K = a.K;
   g.KT = (a.K + 127) / 128;
-  g.mat[0] = GemmMat{a.W, nullptr, nullptr, nullptr, nullptr, PTA_ACT_NONE, (f16*)a.Y, a.N, 0};
-  if (pair) g.mat[1] = GemmMat{a.W2, nullptr, nullptr, nullptr, nullptr, PTA_ACT_NONE, (f16*)a.Y, a.N, 0};
-  make_epilogue(nullptr, &g.epi, "pta_wide_linear");
-  g.epi.wide = out;
-  if (a.workspace) {
-    PTA_REQUIRE(pta_aligned(a.workspace, 16), "pta_wide_linear: the workspace must be 16-byte aligned");
-    g.part = (float*)a.workspace;
-    g.part_bytes = a.workspace_bytes;
-  }
+  g.mat[0] = wide_matrix(a, a.W);
+  if (pair) g.mat[1] = wide_matrix(a, a.W2);
+  make_epilogue(nullptr, &g.epi, name);
+  g.part = (float*)a.workspace;
+  g.part_bytes = a.workspace ? a.workspace_bytes : 0;
   const int nb = (a.N + 15) / 16;
-  return pair ? dispatch_gemv<FmtBF16, true>(g, nb, s, "pta_wide_linear") : dispatch_gemv<FmtBF16, false>(g, nb, s, "pta_wide_linear");
+  return pair ? dispatch_gemv<FmtBF16, true>(g, nb, s, name) : dispatch_gemv<FmtBF16, false>(g, nb, s, name);
+}
+
+extern "C" int pta_wide_linear(const pta_wide_linear_args* args, pta_stream_t stream) {
+  PTA_REQUIRE(args, "pta_wide_linear: null arguments");
+  const int rc = check_wide(*args, "pta_wide_linear");
+  return rc ? rc : wide_linear(*args, (hipStream_t)stream, "pta_wide_linear");
+}
+
+extern "C" int pta_wide_linear_group(const pta_wide_linear_args* list, int count, pta_stream_t stream) {
+  const char* name = "pta_wide_linear_group";
+  PTA_REQUIRE(list && count >= 1 && count <= 4, "%s: 1 to 4 matrices, got %d", name, count);
+  for (int i = 0; i < count; ++i) {
+    const int rc = check_wide(list[i], name);
+    if (rc) return rc;
+    PTA_REQUIRE(list[i].pair == PTA_PAIR_NONE && list[i].dtype == list[0].dtype && list[i].M == list[0].M && list[i].K == list[0].K,
+                "%s: single matrices with the same rows and features", name);
+  }
+  hipStream_t s = (hipStream_t)stream;
+  if (list[0].dtype == PTA_FP32 || list[0].M > 16) {         // many rows: each fills the machine by itself
+    for (int i = 0; i < count; ++i) {
+      const int rc = wide_linear(list[i], s, name);
+      if (rc) return rc;
+    }
+    return PTA_OK;
+  }
+  GemmArgs g{};
+  g.count = count;
+  g.X = (const f16*)list[0].X;
+  g.M = list[0].M;
+  g.K = list[0].K;
+  g.KT = (g.K + 127) / 128;
+  int nb = 0;
+  for (int i = 0; i < count; ++i) {
+    g.mat[i] = wide_matrix(list[i], list[i].W);
+    g.mat[i].X = list[i].X != list[0].X ? (const f16*)list[i].X : nullptr;
+    g.mat[i].nb_begin = nb;
+    nb += (list[i].N + 15) / 16;
+  }
+  make_epilogue(nullptr, &g.epi, name);
+  return dispatch_gemv<FmtBF16, false>(g, nb, s, name);
 }

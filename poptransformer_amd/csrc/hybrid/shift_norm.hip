@@ -1,0 +1,167 @@
+// The front of a layer whose sublayers all read the same fp32 residual: embedding (first layer), RMS norm in groups with
+// one weight per sublayer, and the token shift of what the mixer reads.
+#include "hybrid.h"
+#include <type_traits>
+
+typedef pta_shift_norm_args SN;
+
+constexpr int SN_ROWS = 4;               // rows a workgroup walks through where there are many (and the row before them)
+
+// A workgroup takes `rows_each` rows one after the other.  A thread owns the same columns of all of them, so the row before
+// (normed, fp32) waits for it in LDS; the row before the first comes from the sequence's state, or is made once more.
+// The workgroup that holds a sequence's first row of the pass reads its state, and is also the one that writes it: it
+// makes the sequence's last row a second time.
+template <typename T, int THREADS>
+__global__ __launch_bounds__(THREADS) void shift_norm_kernel(SN a, int rows_each) {
+  constexpr int WAVES = THREADS / 64;
+  extern __shared__ __align__(16) float smem[];
+  const int d = a.width, G = a.groups, gsz = d / G;
+  const int per = WAVES > G ? WAVES / G : 1, units = G * per;            // waves per group
+  float* u = smem;                                                       // [width] the row
+  float* before = u + d;                                                 // [width] the normed row before (with a shift)
+  float* part = a.shift ? before + d : before;                           // [units]
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const bool vec = (gsz & 3) == 0;
+  const int span = vec ? 4 : 1, step = THREADS * span, c_first = threadIdx.x * span;
+  const int piece = (gsz + per - 1) / per;
+
+  auto position = [&](int r) {
+    int p = a.ids_index ? *a.ids_index : a.pos[r];
+    return p < 0 ? 0 : (p >= a.positions ? a.positions - 1 : p);
+  };
+  // the row into u, the sums of squares of its groups into part
+  auto load = [&](int r, bool store) {
+    const int src = a.gather ? a.gather[r] : r;
+    float* x = a.x + (size_t)src * d;
+    if (a.table) {
+      const int p = position(src);
+      int col = a.ids_index ? *a.ids_index : 0;
+      col = col < 0 ? 0 : (col >= a.ids_stride ? a.ids_stride - 1 : col);
+      int id = a.ids[(size_t)src * a.ids_stride + col];
+      id = id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id);
+      const T* e = reinterpret_cast<const T*>(a.table) + (size_t)id * d;
+      const T* q = a.pos_table ? reinterpret_cast<const T*>(a.pos_table) + (size_t)p * d : nullptr;
+      for (int c = c_first; c < d; c += step)
+        for (int k = 0; k < span; ++k) {
+          float v = (float)e[c + k] * a.embed_scale;
+          if (q) v += (float)q[c + k];
+          u[c + k] = v;
+          if (store) x[c + k] = v;
+        }
+    } else if (vec) {
+      for (int c = c_first; c < d; c += step) *reinterpret_cast<f32x4*>(u + c) = *reinterpret_cast<const f32x4*>(x + c);
+    } else {
+      for (int c = c_first; c < d; c += step) u[c] = x[c];
+    }
+    __syncthreads();
+    for (int n = wave; n < units; n += WAVES) {
+      const int g = n / per, lo = g * gsz + (n % per) * piece, end = (g + 1) * gsz, hi = lo + piece < end ? lo + piece : end;
+      float s = 0.f;
+      for (int c = lo + lane; c < hi; c += 64) s = __builtin_fmaf(u[c], u[c], s);
+      s = wave_total_dpp(s);
+      if (lane == 0) part[n] = s;
+    }
+    __syncthreads();
+  };
+  auto inverse = [&](int c) {
+    const int g = c / gsz;
+    float s = 0.f;
+    for (int k = 0; k < per; ++k) s += part[g * per + k];
+    return 1.0f / sqrtf(s / (float)gsz + a.eps);
+  };
+
+  const int r0 = blockIdx.x * rows_each, r1 = r0 + rows_each < a.rows ? r0 + rows_each : a.rows;
+  for (int r = r0; r < r1; ++r) {
+    const int last = a.shift ? (a.last ? a.last[r] : r) : -1;            // >= 0: the first row of its sequence
+    float* state = last >= 0 ? a.state + (size_t)a.slot[r] * d : nullptr;
+    if (state) {
+      const bool start = position(r) == 0;
+      for (int c = c_first; c < d; c += step)
+        for (int k = 0; k < span; ++k) before[c + k] = start ? 0.f : state[c + k];
+    } else if (a.shift && r == r0) {
+      load(r - 1, false);
+      for (int c = c_first; c < d; c += step) {
+        const float inv = inverse(c);
+        for (int k = 0; k < span; ++k) before[c + k] = u[c + k] * inv * a.w1[c + k];
+      }
+    }
+    load(r, true);
+    T* h1 = reinterpret_cast<T*>(a.h1) + (size_t)r * a.h_ld;
+    T* h2 = a.h2 ? reinterpret_cast<T*>(a.h2) + (size_t)r * a.h_ld : nullptr;
+    T* hm = a.shift ? reinterpret_cast<T*>(a.hm) + (size_t)r * a.h_ld : nullptr;
+    auto column = [&](auto tag, int c) {
+      constexpr int V = decltype(tag)::value;
+      typedef T vecT __attribute__((ext_vector_type(V)));
+      vecT o1, o2, om;
+      const float inv = inverse(c);
+#pragma unroll
+      for (int k = 0; k < V; ++k) {
+        const float n = u[c + k] * inv, n1 = n * a.w1[c + k];
+        o1[k] = (T)n1;
+        if (h2) o2[k] = (T)(n * a.w2[c + k]);
+        if (hm) {
+          om[k] = (T)(n1 + (before[c + k] - n1) * a.shift[c + k]);
+          before[c + k] = n1;
+          if (last == r) state[c + k] = n1;
+        }
+      }
+      *reinterpret_cast<vecT*>(h1 + c) = o1;
+      if (h2) *reinterpret_cast<vecT*>(h2 + c) = o2;
+      if (hm) *reinterpret_cast<vecT*>(hm + c) = om;
+    };
+    if (vec) for (int c = c_first; c < d; c += step) column(std::integral_constant<int, 4>{}, c);
+    else for (int c = c_first; c < d; c += step) column(std::integral_constant<int, 1>{}, c);
+    for (int c = d + threadIdx.x; c < a.h_ld; c += THREADS) {
+      h1[c] = (T)0.0f;
+      if (h2) h2[c] = (T)0.0f;
+      if (hm) hm[c] = (T)0.0f;
+    }
+    if (a.pos_out && threadIdx.x == 0) a.pos_out[r] = position(r);
+    if (last > r) {
+      load(last, false);
+      for (int c = c_first; c < d; c += step) {
+        const float inv = inverse(c);
+        for (int k = 0; k < span; ++k) state[c + k] = u[c + k] * inv * a.w1[c + k];
+      }
+    }
+  }
+}
+
+template <typename T>
+static int launch_shift_norm(const SN& a, hipStream_t s) {
+  const bool wide = a.rows <= 64 && a.width >= 2048;       // few rows: a row of 1024 threads shortens the chain of a row
+  const int waves = wide ? 16 : 4, per = waves > a.groups ? waves / a.groups : 1;
+  const size_t smem = ((size_t)a.width * (a.shift ? 2 : 1) + (size_t)a.groups * per) * sizeof(float);
+  const int rows_each = a.rows <= 256 || !a.shift ? 1 : SN_ROWS;
+  const dim3 grid((a.rows + rows_each - 1) / rows_each);
+  auto launch = [&](auto tag) -> int {
+    constexpr int THREADS = decltype(tag)::value;
+    if (smem > 64 * 1024)
+      PTA_REQUIRE(hipFuncSetAttribute((const void*)shift_norm_kernel<T, THREADS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) ==
+                  hipSuccess, "pta_shift_norm: %zu bytes of LDS refused", smem);
+    hipLaunchKernelGGL((shift_norm_kernel<T, THREADS>), grid, dim3(THREADS), smem, s, a, rows_each);
+    return PTA_OK;
+  };
+  const int rc = wide ? launch(std::integral_constant<int, 1024>{}) : launch(std::integral_constant<int, 256>{});
+  if (rc) return rc;
+  PTA_CHECK_LAUNCH("pta_shift_norm");
+  return PTA_OK;
+}
+
+extern "C" int pta_shift_norm(const SN* args, pta_stream_t stream) {
+  PTA_REQUIRE(args, "pta_shift_norm: null arguments");
+  const SN& a = *args;
+  PTA_REQUIRE(a.dtype == PTA_BF16 || a.dtype == PTA_FP32, "pta_shift_norm: unknown type %d", a.dtype);
+  PTA_REQUIRE(a.rows > 0 && a.width > 0 && a.width <= 16000, "pta_shift_norm: rows %d, width %d (1 .. 16000)", a.rows, a.width);
+  PTA_REQUIRE(a.groups > 0 && a.groups <= 1024 && a.width % a.groups == 0, "pta_shift_norm: %d groups of a width of %d", a.groups, a.width);
+  PTA_REQUIRE(a.x && a.w1 && a.h1 && a.h_ld >= a.width && pta_aligned(a.x, 16), "pta_shift_norm: null or unaligned operand");
+  PTA_REQUIRE(!a.h2 || a.w2, "pta_shift_norm: the second result needs its weight");
+  PTA_REQUIRE(!a.shift || (a.hm && a.state && a.slot && (a.pos || a.ids_index) && a.positions > 0),
+              "pta_shift_norm: the token shift needs its result, the state, and the rows' slots and positions");
+  PTA_REQUIRE(!a.table || (a.ids && a.vocab > 0 && a.ids_stride > 0 && (a.pos || a.ids_index) && a.positions > 0),
+              "pta_shift_norm: the embedding needs ids and positions");
+  PTA_REQUIRE(!a.gather || (!a.shift && !a.table), "pta_shift_norm: gathered rows take neither a shift nor the embedding");
+  PTA_REQUIRE(a.h_ld % 8 == 0 && pta_aligned(a.h1, 16) && (!a.h2 || pta_aligned(a.h2, 16)) && (!a.shift || pta_aligned(a.hm, 16)),
+              "pta_shift_norm: results must be 16-byte aligned rows");
+  return a.dtype == PTA_BF16 ? launch_shift_norm<bf16>(a, (hipStream_t)stream) : launch_shift_norm<float>(a, (hipStream_t)stream);
+}

@@ -1,4 +1,5 @@
-"""Executor of decoders that mix windowed attention with recurrent (matrix memory) layers over fp32 residual streams.
+"""Executor of decoders that mix windowed attention with recurrent (matrix memory) layers over fp32 residual streams; the
+mixers, feed-forwards and the row handling that `parallel` uses for layers whose sublayers stand side by side.
 
 The model is a list of layers, each described by its mixer, its feed-forward (or none) and the layer whose tensors it
 uses.  One forward function serves everything: it takes the ROWS of a pass (row = one token of the sequence in a slot, at
@@ -67,6 +68,59 @@ class MemoryMixer:
 
 
 @dataclass
+class LatentMixer:
+    """Attention over the last `window` positions (None: all) whose keys and values are made from a cached latent of kv_rank
+    and one rotated key part shared by the heads; queries through a latent of q_rank, one output gate per head.  `source`: the
+    layer whose cache is read (None: the layer's own)."""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    window: Optional[int]
+    rot_base: float
+    rot_turned: int                  # rotated features of rot_dim; the rest of it passes as it is
+    source: Optional[int] = None
+    kind = "latent"
+
+    @property
+    def sizes(self):
+        """(heads, D, P, E, R, q_rank, kv_rank) with the head sizes as they are stored."""
+        return (self.heads, HK.pad32(self.dim), HK.pad32(self.rot_dim), (self.vdim + 15) // 16 * 16, HK.pad32(self.kv_rank),
+                self.q_rank, self.kv_rank)
+
+    @property
+    def out_channels(self):
+        return self.heads * self.sizes[3]
+
+    @property
+    def cache_row(self):
+        return self.sizes[4] + self.sizes[2]
+
+    def pairs(self):
+        """Order of the rotated features in which the two of a pair follow each other."""
+        half = self.rot_turned // 2
+        turned = np.arange(self.rot_turned).reshape(2, half).T.reshape(-1)
+        return np.concatenate([turned, np.arange(self.rot_turned, self.rot_dim)])
+
+    def angles(self, positions):
+        """[positions, P / 2, (cos, sin)] of those pairs."""
+        f = np.zeros(HK.pad32(self.rot_dim) // 2)
+        half = self.rot_turned // 2
+        f[:half] = float(self.rot_base) ** (-2.0 * np.arange(half) / self.rot_turned)
+        a = np.arange(positions)[:, None] * f
+        return np.stack([np.cos(a), np.sin(a)], -1).astype(np.float32)
+
+
+@dataclass
+class BiasedSwiGLU:
+    """silu(g) u between the gate / up pair and the down projection, all three with biases."""
+    ff: int
+
+
+@dataclass
 class ClampedGLU:
     """min(g, limit) sigmoid(slope g) (clamp(u, -limit, limit) + 1) between the gate / up pair and the down projection."""
     ff: int
@@ -77,8 +131,9 @@ class ClampedGLU:
 @dataclass
 class HybridLayer:
     mixer: object
-    mlp: Optional[ClampedGLU]
+    mlp: object                      # or None
     source: int                      # the layer whose tensors this one uses (itself, or an earlier one)
+    shift: bool = False              # parallel layers: the mixer reads a mixture with the token before
 
 
 @dataclass
@@ -99,6 +154,8 @@ class HybridSpec:
     early_stop: bool = False
     topk: int = 1
     dtype: str = "bfloat16"          # or float32: everything in true 32-bit
+    norm_groups: int = 1             # parallel layers: equal parts of the width with a norm of their own
+    positions: Optional[int] = None  # parallel layers: rows of the position table
 
 
 @dataclass
@@ -168,6 +225,8 @@ class Rows:
     ids: Optional[torch.Tensor] = None
     ids_index: Optional[torch.Tensor] = None
     longest: int = 1
+    last: Optional[torch.Tensor] = None      # of a sequence's first row: its last one, else -1 (None: one row each)
+    portions: tuple = ()                     # (slot, position of the first row, rows) on the host
 
 
 class HybridDecoder(DecodeLoop):
@@ -181,7 +240,8 @@ class HybridDecoder(DecodeLoop):
     def __init__(self, spec, weights, device="cuda", slots=None):
         self.spec, self.w, self.dev = spec, weights, device
         self.dtype = HK.DTYPES[spec.dtype]
-        self.store = SequenceStore(spec, self.dtype, slots or max(spec.batch, 1), spec.max_len, self.pass_rows, device)
+        self.store = SequenceStore(spec, self.dtype, slots or max(spec.batch, 1), min(spec.max_len, spec.positions or spec.max_len),
+                                   self.pass_rows, device)
         self.probe = None            # callable(layer index, fp32 [rows, width]): the summed streams after every layer
         self._buffers = {}
         self._stream = torch.cuda.Stream()
@@ -297,10 +357,13 @@ class HybridDecoder(DecodeLoop):
         pos = np.concatenate([self.store.length[s] + np.arange(len(t), dtype=np.int32) for s, t in portions]).astype(np.int32)
         tiles = [(a + k, min(H.WINDOW_TILE, c - k)) for a, c in zip(starts, counts) for k in range(0, c, H.WINDOW_TILE)]
         tr, tc = (np.array([t[j] for t in tiles], np.int32) for j in (0, 1))
-        flat = torch.from_numpy(np.concatenate([ids, slots, pos, starts, counts, tr, tc])).to(self.dev)
-        parts = torch.split(flat, [len(ids)] * 3 + [len(counts)] * 2 + [len(tiles)] * 2)
-        return Rows(len(ids), parts[1], parts[2], (parts[3], parts[4], len(counts)), bool((counts == 1).all()),
-                    (parts[5], parts[6], len(tiles)), ids=parts[0], longest=int(counts.max()))
+        last = np.full(len(ids), -1, np.int32)
+        last[starts] = starts + counts - 1
+        flat = torch.from_numpy(np.concatenate([ids, slots, pos, last, starts, counts, tr, tc])).to(self.dev)
+        parts = torch.split(flat, [len(ids)] * 4 + [len(counts)] * 2 + [len(tiles)] * 2)
+        return Rows(len(ids), parts[1], parts[2], (parts[4], parts[5], len(counts)), bool((counts == 1).all()),
+                    (parts[6], parts[7], len(tiles)), ids=parts[0], longest=int(counts.max()), last=parts[3],
+                    portions=tuple((s, self.store.length[s], len(t)) for s, t in portions))
 
     def advance(self, entries):
         """entries [(slot, token ids, wanted places)]: the sequences' next tokens, as one batch, cut into passes where they
@@ -352,6 +415,8 @@ class HybridDecoder(DecodeLoop):
         s = self.spec
         if hasattr(self, "container"):
             return
+        if self.store.max_len < s.max_len:
+            raise ValueError(f"sequences of {s.max_len} tokens: the model has {self.store.max_len} positions")
         if self.store.capacity < s.batch:
             self.store._grow(s.batch)
         B = s.batch

@@ -185,13 +185,8 @@ def zekilix_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dty
                       early_stop, topk, dtype)
 
 
-def hybrid_weights(tensors, spec, device="cuda"):
-    """tensors: name -> tensor or array (names as in a checkpoint of the design).  Concatenates the projections of a mixer,
-    pads, and lays the weights out for the device; layers that use another one's tensors have no entry of their own."""
-    from .. import hybrid_kernels as HK
-    from .hybrid import HybridLayerWeights, HybridWeights
-    dtype = HK.DTYPES[spec.dtype]
-
+def _lookup(tensors, device):
+    """(tensor of a name and shape on the device, fp32 vector of a name and length) over name -> tensor or array."""
     def get(name, shape):
         if name not in tensors:
             raise KeyError(f"tensor {name} is missing")
@@ -203,7 +198,16 @@ def hybrid_weights(tensors, spec, device="cuda"):
 
     def vec(name, n):
         return get(name, (n,)).float().contiguous()
+    return get, vec
 
+
+def hybrid_weights(tensors, spec, device="cuda"):
+    """tensors: name -> tensor or array (names as in a checkpoint of the design).  Concatenates the projections of a mixer,
+    pads, and lays the weights out for the device; layers that use another one's tensors have no entry of their own."""
+    from .. import hybrid_kernels as HK
+    from .hybrid import HybridLayerWeights, HybridWeights
+    dtype = HK.DTYPES[spec.dtype]
+    get, vec = _lookup(tensors, device)
     d, S = spec.width, spec.streams
     layers = []
     for i, lay in enumerate(spec.layers):
@@ -242,3 +246,89 @@ def hybrid_weights(tensors, spec, device="cuda"):
         layers.append(HybridLayerWeights(**lw))
     return HybridWeights(get("embed", (spec.vocab, d)).to(dtype).contiguous(), layers, vec("final.norm", d),
                          HK.WideWeight(get("head", (spec.vocab, d)), dtype))
+
+
+# ----------------------------------------------------------------------------------- layers with sublayers side by side
+def latent_layers(layers):
+    """The `layers` list of a configuration with latent attention -> [HybridLayer]."""
+    from .hybrid import BiasedSwiGLU, HybridLayer, LatentMixer
+    out = []
+    for i, c in enumerate(layers):
+        if c["type"] != "latent_attention":
+            raise NotImplementedError(f"layer {i}: mixer {c['type']}")
+        m, rot = c["mixer"], c["mixer"]["rot"]
+        if rot["dims"] % 2 or rot["dims"] > m["rot_dim"]:
+            raise ValueError(f"layer {i}: {rot['dims']} rotated features of {m['rot_dim']}")
+        source = m.get("kv_from")
+        mixer = LatentMixer(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["q_rank"], m["kv_rank"], float(m["scale"]),
+                            (m.get("mask") or {}).get("size"), float(rot["base"]), rot["dims"], source)
+        if source is not None:
+            if not 0 <= source < i or out[source].mixer.source is not None:
+                raise ValueError(f"layer {i}: kv_from {source} names no earlier layer with a cache of its own")
+            o = out[source].mixer
+            if (o.kv_rank, o.rot_dim, o.rot_base, o.rot_turned) != (mixer.kv_rank, mixer.rot_dim, mixer.rot_base, mixer.rot_turned):
+                raise ValueError(f"layer {i}: the latent or the rotation differs from layer {source}'s")
+        f = c.get("mlp")
+        if f is not None and f.get("kind", "dense") != "dense":
+            raise NotImplementedError(f"layer {i}: feed-forward {f['kind']}")
+        out.append(HybridLayer(mixer, BiasedSwiGLU(f["ff"]) if f is not None else None, i, shift=True))
+    return out
+
+
+def ruperax_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
+    from .hybrid import HybridSpec
+    return HybridSpec("ruperax", latent_layers(cfg["layers"]), cfg["width"], cfg["vocab"], 1, cfg["norm"]["eps"], 1.0,
+                      cfg["embedding"]["scale"], 0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype,
+                      norm_groups=cfg["norm"].get("groups") or 1, positions=cfg["max_positions"])
+
+
+def _padded(t, *shape):
+    """t in the corner of a zero tensor of the given shape."""
+    if tuple(t.shape) == shape:
+        return t
+    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
+    out[tuple(slice(n) for n in t.shape)] = t
+    return out
+
+
+def parallel_weights(tensors, spec, device="cuda"):
+    """As hybrid_weights, for layers with latent attention whose sublayers stand side by side.  Every head size is rounded up to
+    what the kernels take, with zeros; the two features of a rotated pair come to stand side by side, in queries and keys."""
+    from .. import hybrid_kernels as HK
+    from .parallel import ParallelLayerWeights, ParallelWeights
+    dtype = HK.DTYPES[spec.dtype]
+    get, vec = _lookup(tensors, device)
+    d = spec.width
+    layers = []
+    for i, lay in enumerate(spec.layers):
+        p, m = f"l{i}.", lay.mixer
+        mix = p + "mix."
+        heads, D, P, E, R, q_rank, kv_rank = m.sizes
+        Qp, pairs = HK.pad8(q_rank), torch.from_numpy(m.pairs()).to(device)
+        parts = [_padded(get(mix + "dq", (q_rank, d)), Qp, d)]
+        if m.source is None:
+            dkv = get(mix + "dkv", (kv_rank + m.rot_dim, d))
+            parts += [_padded(dkv[:kv_rank], R, d), _padded(dkv[kv_rank:][pairs], P, d)]
+        parts.append(get(mix + "g", (heads, d)))
+        uq = get(mix + "uq", (heads * (m.dim + m.rot_dim), q_rank)).view(heads, m.dim + m.rot_dim, q_rank)
+        uq = torch.cat([_padded(uq[:, :m.dim], heads, D, q_rank), _padded(uq[:, m.dim:][:, pairs], heads, P, q_rank)], 1)
+        uk = _padded(get(mix + "uk", (heads * m.dim, kv_rank)).view(heads, m.dim, kv_rank), heads, D, R)
+        uv = _padded(get(mix + "uv", (heads * m.vdim, kv_rank)).view(heads, m.vdim, kv_rank), heads, E, R)
+        o = _padded(get(mix + "o", (d, heads * m.vdim)).view(d, heads, m.vdim), d, heads, E)
+        lw = dict(norm1=vec(p + "norm1", d), shift=vec(p + "shift", d), gate1=HK.WideWeight(get(p + "rg1", (d, d)), dtype),
+                  gate1_bias=vec(p + "rg1.b", d), proj=HK.WideWeight(torch.cat(parts), dtype, tail=heads),
+                  q_norm=vec(mix + "dq.norm", q_rank), kv_norm=vec(mix + "dkv.norm", kv_rank) if m.source is None else None,
+                  uq=HK.WideWeight(uq.reshape(-1, q_rank), dtype), uk_t=uk.transpose(1, 2).to(dtype).contiguous(),
+                  uv=uv.to(dtype).contiguous(), kv=None, out=HK.WideWeight(o.reshape(d, -1), dtype))
+        if HK.latent_tiles_fit(dtype, D, P, E):
+            lw.update(kv=HK.WideWeight(torch.cat([uk.reshape(-1, R), uv.reshape(-1, R)]), dtype))
+        if lay.mlp is not None:
+            ff, mlp = lay.mlp.ff, p + "mlp."
+            n = HK.pad8(ff)
+            lw.update(norm2=vec(p + "norm2", d), gate2=HK.WideWeight(get(p + "rg2", (d, d)), dtype), gate2_bias=vec(p + "rg2.b", d),
+                      gate=HK.WideWeight(get(mlp + "gate", (ff, d)), dtype, main_to=n), gate_bias=_padded(vec(mlp + "gate.b", ff), n),
+                      up=HK.WideWeight(get(mlp + "up", (ff, d)), dtype, main_to=n), up_bias=_padded(vec(mlp + "up.b", ff), n),
+                      down=HK.WideWeight(get(mlp + "down", (d, ff)), dtype), down_bias=vec(mlp + "down.b", d))
+        layers.append(ParallelLayerWeights(**lw))
+    return ParallelWeights(get("embed", (spec.vocab, d)).to(dtype).contiguous(), get("pos", (spec.positions, d)).to(dtype).contiguous(),
+                           layers, vec("final.norm", d), HK.WideWeight(get("head", (spec.vocab, d)), dtype))

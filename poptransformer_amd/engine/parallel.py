@@ -1,0 +1,204 @@
+"""Executor of decoders whose layers run mixer and feed-forward side by side on one fp32 residual:
+
+    x <- x + gate1 * mixer(shift(n1(x))) + gate2 * ff(n2(x)),    gate = sigmoid(W n(x) + b)
+
+with a norm in groups, a token shift in front of the mixer and latent attention.  Rows, sequences, sampling and the decode
+loop are HybridDecoder's.
+
+Launches of a layer in a decode iteration: norms and token shift; both residual gates with the mixer's down-projections;
+latent norms and cache entry; queries; queries against the latent; attention over the cached rows; values; output projection
+(its epilogue gates and adds to the residual); gate / up pair; down projection (likewise).  Prompts take keys and values of
+every head instead of the middle three.
+"""
+from dataclasses import dataclass
+from typing import List, Optional
+
+import numpy as np
+import torch
+
+from .. import _hybrid_lib as H
+from .. import hybrid_kernels as HK
+from .hybrid import F32, I32, HybridDecoder
+
+
+@dataclass
+class ParallelLayerWeights:
+    norm1: torch.Tensor
+    shift: torch.Tensor
+    gate1: HK.WideWeight
+    gate1_bias: torch.Tensor
+    proj: HK.WideWeight              # query latent | cache entry (layers with a cache of their own), tail: the heads' gates
+    q_norm: torch.Tensor
+    kv_norm: Optional[torch.Tensor]
+    uq: HK.WideWeight
+    uk_t: torch.Tensor               # [heads, R, D]
+    uv: torch.Tensor                 # [heads, E, R]
+    kv: Optional[HK.WideWeight]      # keys of all heads | values of all heads, from the latent (None: the sizes are taken absorbed)
+    out: HK.WideWeight
+    norm2: Optional[torch.Tensor] = None
+    gate2: Optional[HK.WideWeight] = None
+    gate2_bias: Optional[torch.Tensor] = None
+    gate: Optional[HK.WideWeight] = None
+    gate_bias: Optional[torch.Tensor] = None
+    up: Optional[HK.WideWeight] = None
+    up_bias: Optional[torch.Tensor] = None
+    down: Optional[HK.WideWeight] = None
+    down_bias: Optional[torch.Tensor] = None
+
+    def linears(self):
+        """Every weight once, as a decode iteration reads them."""
+        return [w for w in (self.gate1, self.proj, self.uq, self.out, self.gate2, self.gate, self.up, self.down) if w is not None]
+
+
+@dataclass
+class ParallelWeights:
+    embed: torch.Tensor
+    pos: torch.Tensor
+    layers: List[ParallelLayerWeights]
+    final_norm: torch.Tensor
+    head: HK.WideWeight
+
+    def nbytes(self):
+        """Bytes of the weights, each counted once."""
+        return self.head.nbytes + sum(sum(w.nbytes for w in lay.linears()) + sum(t.numel() * t.element_size() for t in (lay.uk_t, lay.uv))
+                                      for lay in self.layers)
+
+
+class ParallelBuffers:
+    """Activations of up to `rows` rows."""
+
+    def __init__(self, spec, weights, rows, dtype, device):
+        def buf(*shape, dtype=dtype):
+            return torch.zeros(shape, dtype=dtype, device=device)
+        mixers, ld = [lay.mixer for lay in spec.layers], HK.pad8(spec.width)
+        self._buf = buf
+        self.rows = rows
+        self.x = buf(rows, spec.width, dtype=F32)
+        self.h1, self.h2, self.hm = buf(rows, ld), buf(rows, ld), buf(rows, ld)
+        self.gate1, self.gate2 = buf(rows, spec.width), buf(rows, spec.width)
+        self.proj = {n: buf(rows, n) for n in {lw.proj.n_main for lw in weights.layers}}
+        self.head_gates = {n: buf(rows, n, dtype=F32) for n in {m.heads for m in mixers}}
+        self.cq = {n: buf(rows, n) for n in {lw.uq.K for lw in weights.layers}}
+        self.q = {n: buf(rows, n) for n in {lw.uq.n_main for lw in weights.layers}}
+        self.ctx = {n: buf(rows, n) for n in {m.out_channels for m in mixers}}
+        self.act = {n: buf(rows, n) for n in {lw.gate.n_main for lw in weights.layers if lw.gate is not None}}
+        channels = max(w.N for lw in weights.layers for w in lw.linears())
+        self.workspace = HK.linear_workspace(rows, channels, device) if rows > 16 else None
+        self._absorbed = {}
+
+    def absorbed(self, heads, R, P, splits):
+        """(queries against the latent, the parts' sums, their softmax states)"""
+        key = (heads, R, P, splits)
+        if key not in self._absorbed:
+            n = self.rows * heads
+            self._absorbed[key] = (self._buf(n, R + P), self._buf(n * splits, R, dtype=F32), self._buf(n * splits, 2, dtype=F32))
+        return self._absorbed[key]
+
+
+class ParallelDecoder(HybridDecoder):
+    absorbed_rows = 16               # sequences with up to this many rows in a pass work on the cached rows themselves
+
+    def __init__(self, spec, weights, device="cuda", slots=None):
+        super().__init__(spec, weights, device, slots)
+        self._angles = {}
+        self._key_lists = None
+
+    def _rows_buffers(self, rows):
+        size = rows if rows <= 16 else max(64, 1 << (rows - 1).bit_length())
+        if size not in self._buffers:
+            self._buffers[size] = ParallelBuffers(self.spec, self.w, size, self.dtype, self.dev)
+        return self._buffers[size]
+
+    def _cos_sin(self, m):
+        key = (m.rot_base, m.rot_turned, m.rot_dim)
+        if key not in self._angles:
+            self._angles[key] = torch.from_numpy(m.angles(self.store.max_len)).to(self.dev)
+        return self._angles[key]
+
+    def _splits(self, rows, mixer):
+        """Parts of the window per row: enough workgroups to fill the machine, at least 64 keys per part.  Fixed per shape, since
+        the launch is replayed while the context grows."""
+        wgs = rows * (-(-mixer.heads // 16) if self.dtype == torch.bfloat16 else mixer.heads)
+        keys = min(mixer.window or self.store.max_len, self.store.max_len)
+        return max(1, min(256 // wgs, -(-keys // 64), 64))
+
+    def _keys(self, rows, window):
+        """Cache rows that a pass's rows look at, sequence after sequence: (slots, positions), and where position 0 of a tile's
+        sequence would lie among them.  One list per distinct window of a pass."""
+        if self._key_lists is None or self._key_lists[0] is not rows:
+            self._key_lists = (rows, {})
+        lists = self._key_lists[1]
+        if window not in lists:
+            slots, places, zero, at = [], [], [], 0
+            for slot, p0, count in rows.portions:
+                first = max(0, p0 - window + 1) if window is not None else 0
+                n = p0 + count - first
+                slots.append(np.full(n, slot, np.int32))
+                places.append(np.arange(first, first + n, dtype=np.int32))
+                zero += [at - first] * -(-count // H.LATENT_TILE)
+                at += n
+            flat = torch.from_numpy(np.concatenate(slots + places + [np.array(zero, np.int32)])).to(self.dev)
+            slot, pos, tile_key = torch.split(flat, [at, at, len(zero)])
+            lists[window] = ((slot, pos), (*rows.tiles[:2], tile_key))
+        return lists[window]
+
+    def _mixer(self, i, b, rows):
+        m, lw, n = self.spec.layers[i].mixer, self.w.layers[i], rows.n
+        heads, D, P, E, R = m.sizes[:5]
+        proj, cq, q = b.proj[lw.proj.n_main], b.cq[lw.uq.K], b.q[lw.uq.n_main]
+        gates, ctx = b.head_gates[heads], b.ctx[m.out_channels]
+        ring, = self.store.stores[i if m.source is None else m.source]
+        att = HK.LatentAttention(m.sizes, m.scale, m.window, self.spec.eps, lw.q_norm, lw.kv_norm, self._cos_sin(m), ring, n, rows.slot, rows.pos)
+        att.append(proj, cq)
+        HK.linear(cq, lw.uq, q, n, workspace=b.workspace)
+        if lw.kv is None or rows.single or rows.longest <= self.absorbed_rows:
+            splits = self._splits(b.rows, m)
+            q_latent, part_o, part_ml = b.absorbed(heads, R, P, splits)
+            att.absorbed(q, lw.uk_t, q_latent, splits, part_o, part_ml, lw.uv, gates, ctx)
+        else:
+            keys, tiles = self._keys(rows, m.window)
+            count = keys[0].numel()
+            # latents, rotated parts, then keys and values of all heads
+            sizes = [count * R, count * P, count * lw.kv.n_main]
+            flat = self._scratch(2 * sum(sizes))[:2 * sum(sizes)].view(self.dtype)
+            latent, rot, kv = torch.split(flat, sizes)
+            att.over_heads(q, keys, latent.view(count, R), rot.view(count, P), lw.kv, kv.view(count, -1), tiles, gates, ctx)
+        HK.linear(ctx, lw.out, b.x, n, ld=self.spec.width, mul=b.gate1, accumulate=True, workspace=b.workspace)
+
+    def _feed_forward(self, i, b, rows):
+        lw, n = self.w.layers[i], rows.n
+        act = b.act[lw.gate.n_main]
+        HK.linear(b.h2, lw.gate, act, n, up=lw.up, pair=H.PAIR_SWIGLU, bias=lw.gate_bias, bias2=lw.up_bias)
+        HK.linear(act, lw.down, b.x, n, ld=self.spec.width, bias=lw.down_bias, mul=b.gate2, accumulate=True, workspace=b.workspace)
+
+    def _layers(self, rows, pos_out=None):
+        """All layers over the rows; the residual is left in the buffers."""
+        spec, w, store, n = self.spec, self.w, self.store, rows.n
+        b = self._rows_buffers(n)
+        last = None if rows.single else rows.last
+        for i, layer in enumerate(spec.layers):
+            lw, ff = w.layers[i], layer.mlp is not None
+            first = dict(table=w.embed, pos_table=w.pos, embed_scale=spec.embed_scale, ids=rows.ids, ids_index=rows.ids_index,
+                         pos_out=pos_out) if i == 0 else {}
+            HK.shift_norm(b.x, n, spec.norm_groups, spec.eps, lw.norm1, b.h1, lw.norm2, b.h2 if ff else None, lw.shift, b.hm,
+                          store.shifted[i], rows.slot, last, rows.pos, store.max_len, **first)
+            calls = [(b.h1, lw.gate1, b.gate1, dict(ld=spec.width, bias=lw.gate1_bias, sigmoid=True, workspace=b.workspace)),
+                     (b.hm, lw.proj, b.proj[lw.proj.n_main], dict(tail=b.head_gates[layer.mixer.heads], workspace=b.workspace))]
+            if ff:
+                calls.append((b.h2, lw.gate2, b.gate2, dict(ld=spec.width, bias=lw.gate2_bias, sigmoid=True, workspace=b.workspace)))
+            HK.linear_group(n, *calls)
+            self._mixer(i, b, rows)
+            if ff:
+                self._feed_forward(i, b, rows)
+            if self.probe is not None:
+                self.probe(i, b.x[:n].clone())
+        return b, None
+
+    def _logits(self, b, done, count, out, gather=None):
+        spec, h = self.spec, b.h1
+        if gather is not None:
+            if self._head_h is None:
+                self._head_h = torch.zeros((self.head_rows, h.shape[1]), dtype=self.dtype, device=self.dev)
+            h = self._head_h
+        HK.shift_norm(b.x, count, spec.norm_groups, spec.eps, self.w.final_norm, h, gather=gather)
+        HK.linear(h, self.w.head, out, count, ld=spec.vocab)

@@ -12,6 +12,13 @@ def _zekilix(cfg, path, max_len, batch, dtype, slots):
     return HybridDecoder(spec, loader.hybrid_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
 
 
+def _ruperax(cfg, path, max_len, batch, dtype, slots):
+    from ..utils import checkpoint
+    from .parallel import ParallelDecoder
+    spec = loader.ruperax_spec(cfg, max_len, batch, dtype=dtype)
+    return ParallelDecoder(spec, loader.parallel_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
+
+
 def _fused(spec_of, weights_of):
     def make(cfg, path, max_len, batch, dtype, slots):
         from ..utils import checkpoint
@@ -36,6 +43,7 @@ def _only_fp16(dtype):
 # config.json's "architecture" (or the first of "architectures") -> (libraries it needs, maker)
 ARCHITECTURES = {
     "Zekilix": (("hybrid",), _zekilix),
+    "Ruperax": (("hybrid",), _ruperax),
     "GPT2LMHeadModel": (("hip", "hybrid"), _fused(loader.gpt2_spec, loader.gpt2_weights)),
     "LlamaForCausalLM": (("hip", "hybrid"), _fused(loader.llama2_spec, loader.llama2_weights)),
     "ChatGLMModel": (("hip", "hybrid"), _fused(loader.chatglm2_spec, loader.chatglm2_weights)),

@@ -3,8 +3,11 @@
 A sequence holds one SLOT while it lives.  Per layer run (a layer whose weights are another layer's has a cache of its
 own) a slot is
   * for windowed attention: a ring of key rows, position p in row p % ring_len, and one fp32 factor per position;
-  * for matrix memory: the fp32 state, zero before the first token.
-Ring rows need no clearing: a position is only looked at once its own sequence has written it.
+  * for latent attention: a ring of latents with their rotated key part - a layer that reads another one's cache has none;
+  * for matrix memory: the fp32 state, zero before the first token;
+and with a token shift per layer the normed fp32 row of the newest token.
+Ring rows need no clearing: a position is only looked at once its own sequence has written it; nor does the shift's row,
+which position 0 does not look at.
 """
 import torch
 
@@ -20,25 +23,42 @@ class SequenceStore:
         self.portion = min(pass_rows, max_len)
         self.capacity = 0
         self.stores = [None] * len(spec.layers)
+        self.shifted = [None] * len(spec.layers)      # fp32 [slots, width] per layer with a token shift
         self.length = []                      # tokens each slot holds, -1: free
         self._grow(slots)
 
-    def ring_len(self, mixer):
-        n = self.max_len if mixer.window is None else min(self.max_len, mixer.window - 1 + self.portion)
+    def cache_window(self, i):
+        """The widest window over the cache of layer i: its own, and those of the layers that read it (None: everything)."""
+        windows = [m.window for j, m in enumerate(lay.mixer for lay in self.spec.layers)
+                   if j == i or getattr(m, "source", None) == i]
+        return None if None in windows else max(windows)
+
+    def ring_len(self, i):
+        window = self.cache_window(i)
+        n = self.max_len if window is None else min(self.max_len, window - 1 + self.portion)
         return (n + 63) // 64 * 64
 
     def _grow(self, slots):
+        def zeros(*shape, dtype=self.dtype):
+            return torch.zeros(shape, dtype=dtype, device=self.dev)
+
+        def moved(old, new):
+            for o, t in zip(old or (), new):
+                t[:o.shape[0]].copy_(o)
+            return new
         for i, layer in enumerate(self.spec.layers):
             m = layer.mixer
             if m.kind == "attention":
-                n = self.ring_len(m)
-                new = (torch.zeros((slots, m.kv_heads, n, HK.pad8(m.dim)), dtype=self.dtype, device=self.dev),
-                       torch.zeros((slots, n), dtype=torch.float32, device=self.dev))
+                n = self.ring_len(i)
+                new = (zeros(slots, m.kv_heads, n, HK.pad8(m.dim)), zeros(slots, n, dtype=torch.float32))
+            elif m.kind == "latent":
+                new = (zeros(slots, self.ring_len(i), m.cache_row),) if m.source is None else ()
             else:
                 new = (HK.mlstm_state(slots, m.heads, m.dim, m.vdim, self.dev),)
-            for old, t in zip(self.stores[i] or (), new):
-                t[:old.shape[0]].copy_(old)
-            self.stores[i] = new
+            self.stores[i] = moved(self.stores[i], new)
+            if layer.shift:
+                old = self.shifted[i]
+                self.shifted[i], = moved(old if old is None else (old,), (zeros(slots, self.spec.width, dtype=torch.float32),))
         self.length += [-1] * (slots - self.capacity)
         self.capacity = slots
 
@@ -66,4 +86,4 @@ class SequenceStore:
 
     @property
     def nbytes(self):
-        return sum(t.numel() * t.element_size() for store in self.stores for t in store)
+        return sum(t.numel() * t.element_size() for store in self.stores + [[s] for s in self.shifted if s is not None] for t in store)

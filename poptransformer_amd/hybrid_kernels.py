@@ -66,8 +66,8 @@ def linear_workspace(rows, channels, device):
     return torch.empty(H.load().pta_wide_linear_workspace_bytes(rows, channels), dtype=torch.uint8, device=device)
 
 
-def linear(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.PAIR_NONE, limit=0.0, slope=0.0, workspace=None):
-    """out[:rows] = x[:rows] @ w^T with the fused epilogues of pta_wide_linear; `up`: the second weight of a pair."""
+def _linear_args(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.PAIR_NONE, limit=0.0, slope=0.0, workspace=None, bias=None,
+                 bias2=None, sigmoid=False, mul=None, accumulate=False):
     _need(x, w.dtype, "x", rows * w.K)
     ld = w.n_main if ld is None else ld
     if out.dtype not in (w.dtype, F32):
@@ -79,11 +79,28 @@ def linear(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.PAIR_NO
         raise ValueError("the weights of a pair must be alike")
     if w.tail:
         _need(tail, F32, "tail", rows * w.tail)
-    a = H.WideLinearArgs(_CODE[w.dtype], _p(x), rows, w.K, w.N, _p(w.data), _p(up.data) if up is not None else None, pair, limit, slope,
-                         cap, _p(out), ld, w.n_main, int(out.dtype == F32), _p(tail) if w.tail else None, w.tail, _p(w.tail_bias),
-                         _p(workspace), workspace.numel() if workspace is not None else 0)
+    for b in (bias, bias2):
+        if b is not None:
+            _need(b, F32, "bias", w.n_main)
+    if mul is not None:
+        _need(mul, w.dtype, "mul", rows * ld)
+    return H.WideLinearArgs(_CODE[w.dtype], _p(x), rows, w.K, w.N, _p(w.data), _p(up.data) if up is not None else None, pair, limit, slope,
+                            cap, _p(out), ld, w.n_main, int(out.dtype == F32), _p(tail) if w.tail else None, w.tail, _p(w.tail_bias),
+                            _p(workspace), workspace.numel() if workspace is not None else 0, _p(bias), _p(bias2), int(sigmoid), _p(mul),
+                            int(accumulate))
+
+
+def linear(x, w, out, rows, **kw):
+    """out[:rows] = x[:rows] @ w^T with the fused epilogues of pta_wide_linear; `up`: the second weight of a pair."""
+    a = _linear_args(x, w, out, rows, **kw)
     H.check(H.load().pta_wide_linear(ctypes.byref(a), _stream()))
     return out
+
+
+def linear_group(rows, *calls):
+    """Several `linear`s (x, w, out, keywords) over inputs of one shape, in one launch where there are few rows."""
+    a = (H.WideLinearArgs * len(calls))(*(_linear_args(x, w, out, rows, **kw) for x, w, out, kw in calls))
+    H.check(H.load().pta_wide_linear_group(a, len(calls), _stream()))
 
 
 def streams_norm(streams, rows, eps, weight=None, h=None, table=None, embed_scale=1.0, ids=None, ids_index=None, pos_out=None, y=None,
@@ -155,6 +172,118 @@ class WindowAttention:
         lib = H.load()
         H.check(lib.pta_window_append(ctypes.byref(a), _stream()))
         H.check(lib.pta_window_attention(ctypes.byref(a), _stream()))
+
+
+def shift_norm(x, rows, groups, eps, w1, h1, w2=None, h2=None, shift=None, hm=None, state=None, slot=None, last=None, pos=None,
+               positions=0, table=None, pos_table=None, embed_scale=1.0, ids=None, ids_index=None, pos_out=None, gather=None):
+    """Front of a layer with parallel sublayers (pta_shift_norm).  x [R, width] fp32; h1, h2, hm [R, ld]."""
+    width = x.shape[-1]
+    _need(x, F32, "x", 0 if gather is not None else rows * width)
+    _need(w1, F32, "w1", width)
+    _need(h1, h1.dtype, "h1", rows * h1.shape[-1])
+    for h, w in ((h2, w2), (hm, shift)):
+        if h is not None:
+            _need(h, h1.dtype, "result", rows * h1.shape[-1])
+            _need(w, F32, "weight", width)
+    if shift is not None:
+        _need(state, F32, "state")
+        _need(slot, I32, "slot", rows)
+    if last is not None:
+        _need(last, I32, "last", rows)
+    if table is not None:
+        _need(table, h1.dtype, "table")
+        _need(ids, I32, "ids")
+    if pos_table is not None:
+        _need(pos_table, h1.dtype, "pos_table", positions * width)
+    stride = ids.shape[-1] if ids is not None and ids.dim() == 2 else 1
+    a = H.ShiftNormArgs(_CODE[h1.dtype], rows, width, groups, _p(x), _p(table), _p(pos_table), table.shape[0] if table is not None else 0,
+                        positions, embed_scale, _p(ids), stride, _p(ids_index), _p(pos), _p(pos_out), _p(gather), eps, _p(w1), _p(w2),
+                        _p(shift), _p(state), _p(slot), _p(last), _p(h1), _p(h2), _p(hm), h1.shape[-1])
+    H.check(H.load().pta_shift_norm(ctypes.byref(a), _stream()))
+
+
+def pad32(n):
+    return (n + 31) // 32 * 32
+
+
+class LatentAttention:
+    """The latent-attention calls of one layer over one set of row buffers.  Sizes as stored; `proj` rows hold the query latent
+    and, where `kv_norm` is given (the layer has a cache of its own), the row's cache entry."""
+
+    def __init__(self, sizes, scale, window, eps, q_norm, kv_norm, cos_sin, ring, rows, slot, pos):
+        """sizes = (heads, D, P, E, R, q_rank, kv_rank)."""
+        self.H, self.D, self.P, self.E, self.R, self.q_rank, self.kv_rank = sizes
+        _need(q_norm, F32, "q_norm", self.q_rank)
+        if kv_norm is not None:
+            _need(kv_norm, F32, "kv_norm", self.kv_rank)
+        if ring.dim() != 3 or ring.shape[2] != self.R + self.P:
+            raise ValueError(f"ring must be [slots, length, {self.R + self.P}], got {tuple(ring.shape)}")
+        _need(ring, ring.dtype, "ring")
+        _need(cos_sin, F32, "cos_sin")
+        if cos_sin.shape[1:] != (self.P // 2, 2):
+            raise ValueError("cos_sin must be [positions, P / 2, 2]")
+        _need(slot, I32, "slot", rows)
+        _need(pos, I32, "pos", rows)
+        self.rows, self.dtype = rows, ring.dtype
+        self.a = H.LatentArgs(_CODE[ring.dtype], rows, *sizes)
+        a = self.a
+        a.q_norm, a.kv_norm, a.eps, a.scale, a.window = _p(q_norm), _p(kv_norm), eps, scale, window or (1 << 30)
+        a.cos_sin, a.positions, a.ring, a.ring_len, a.slot, a.pos = _p(cos_sin), cos_sin.shape[0], _p(ring), ring.shape[1], _p(slot), _p(pos)
+
+    def _call(self, name):
+        H.check(getattr(H.load(), "pta_latent_" + name)(ctypes.byref(self.a), _stream()))
+
+    def append(self, proj, cq):
+        """Normed query latents, and the rows' entries in the layer's own cache."""
+        _need(proj, self.dtype, "projection", self.rows * proj.shape[-1])
+        _need(cq, self.dtype, "cq", self.rows * pad8(self.q_rank))
+        self.a.proj, self.a.ld, self.a.cq = _p(proj), proj.shape[-1], _p(cq)
+        self._call("append")
+
+    def _result(self, q, gate, out):
+        _need(q, self.dtype, "q", self.rows * self.H * (self.D + self.P))
+        _need(gate, F32, "gate", self.rows * self.H)
+        _need(out, self.dtype, "out", self.rows * self.H * self.E)
+        self.a.q, self.a.gate, self.a.out = _p(q), _p(gate), _p(out)
+
+    def absorbed(self, q, uk_t, q_latent, splits, part_o, part_ml, uv, gate, out):
+        """Every row over the cache itself, its window in `splits` parts."""
+        n = self.rows * self.H
+        self._result(q, gate, out)
+        _need(uk_t, self.dtype, "uk_t", self.H * self.R * self.D)
+        _need(q_latent, self.dtype, "q_latent", n * (self.R + self.P))
+        _need(part_o, F32, "part_o", n * splits * self.R)
+        _need(part_ml, F32, "part_ml", n * splits * 2)
+        _need(uv, self.dtype, "uv", self.H * self.E * self.R)
+        a = self.a
+        a.uk_t, a.q_latent, a.splits, a.part_o, a.part_ml, a.uv = _p(uk_t), _p(q_latent), splits, _p(part_o), _p(part_ml), _p(uv)
+        for name in ("absorb", "rows", "values"):
+            self._call(name)
+
+    def over_heads(self, q, keys, key_latent, key_rot, kv_weight, kv, tiles, gate, out):
+        """Tiles of rows over keys and values of every head, which are made from the cache first.  keys = (slots, positions);
+        tiles = (first rows, row counts, key row of position 0)."""
+        n, (slot, pos), (tr, tc, tk) = keys[0].numel(), keys, tiles
+        self._result(q, gate, out)
+        for t, want in ((slot, n), (pos, n), (tr, len(tr)), (tc, len(tr)), (tk, len(tr))):
+            _need(t, I32, "keys and tiles", want)
+        _need(key_latent, self.dtype, "key_latent", n * self.R)
+        _need(key_rot, self.dtype, "key_rot", n * self.P)
+        _need(kv, self.dtype, "kv", n * kv_weight.n_main)
+        if kv_weight.n_main != self.H * (self.D + self.E) or kv_weight.K != self.R:
+            raise ValueError("kv_weight does not fit the sizes")
+        a = self.a
+        a.keys, a.key_slot, a.key_pos, a.key_latent, a.key_rot, a.kv = n, _p(slot), _p(pos), _p(key_latent), _p(key_rot), _p(kv)
+        a.tile_row, a.tile_count, a.tile_key, a.tiles = _p(tr), _p(tc), _p(tk), len(tr)
+        self._call("gather")
+        for k in range(0, n, 4096):
+            m = min(4096, n - k)
+            linear(key_latent[k:k + m], kv_weight, kv[k:k + m], m)
+        self._call("tiles")
+
+
+def latent_tiles_fit(dtype, D, P, E):
+    return bool(H.load().pta_latent_tiles_fit(_CODE[dtype], D, P, E))
 
 
 def mlstm_state(slots, heads, dim, vdim, device):
