@@ -52,14 +52,13 @@ def rotate_half(x, base, dims):
 
 def sliding_softmax_attention(q, k, v, scale, window):
     """q, k [T, H, D], v [T, H, E]: causal attention over the last `window` positions (None: all of them)."""
-    T, H, _ = q.shape
-    out = np.zeros((T, H, v.shape[2]))
+    T = q.shape[0]
+    out = np.zeros((T,) + v.shape[1:])
     for i in range(T):
         lo = 0 if window is None else max(0, i - window + 1)
-        for h in range(H):
-            s = k[lo:i + 1, h] @ q[i, h] * scale
-            p = np.exp(s - s.max())
-            out[i, h] = (p / p.sum()) @ v[lo:i + 1, h]
+        s = np.einsum("jhd,hd->hj", k[lo:i + 1], q[i]) * scale
+        p = np.exp(s - s.max(1, keepdims=True))
+        out[i] = np.einsum("hj,jhe->he", p / p.sum(1, keepdims=True), v[lo:i + 1])
     return out
 
 

@@ -1,7 +1,7 @@
 """From a recorded graph to something that runs: `Session.compile` ends here.
 
 Every graph can run op by op (engine/interpreter.py).  A graph that is one of the decoder loops
-this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix as the models build them through the operator
+this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix, Ruperax as the models build them through the operator
 API - is additionally mapped onto the fused executor for its family: the family is read off the
 state-dict keys the layers registered as initializer names, the shapes off a one-iteration probe of
 the interpreter, and the weights off the initializers.  The fused executor is then VALIDATED: it
@@ -250,19 +250,53 @@ def _build_rwkv(facts, shapes, topk=1):
     return RWKVDecoder(spec, w)
 
 
-def _build_hybrid(facts, topk=1):
-    """The hybrid executor of a graph whose layers are tensors `l<i>.*`: sizes from the tensors, constants from the named
-    constants the layers recorded, the arithmetic ('bf16' or 'fp32') from the precision the graph was built with."""
-    from ..utils import REGISTRY
-    from .hybrid import ClampedGLU, HybridDecoder, HybridLayer, HybridSpec, MemoryMixer, WindowMixer
-    from .loader import hybrid_weights
-
+def _const_reader(facts):
     def const(name, required=True):
         v = _named_const(facts.body, name)
         if v is None and required:
             raise ValueError(f"constant {name} not found")
         return v
+    return const
 
+
+def _executor_dtype():
+    from ..utils import REGISTRY
+    return {"bf16": "bfloat16", "fp32": "float32"}[REGISTRY.get("tensor_type").precision]
+
+
+def _build_parallel(facts, topk=1):
+    """As _build_hybrid, for layers with latent attention whose sublayers stand side by side."""
+    from .hybrid import BiasedSwiGLU, HybridLayer, HybridSpec, LatentMixer
+    from .loader import parallel_weights
+    from .parallel import ParallelDecoder
+    const = _const_reader(facts)
+    layers = []
+    while const(f"l{len(layers)}.cache_of", False) is not None:
+        i = len(layers)
+        mix = f"l{i}.mix."
+        heads, source = int(const(f"l{i}.heads")), int(const(f"l{i}.cache_of"))
+        uk, uv, uq = (_need(facts, mix + n) for n in ("uk", "uv", "uq"))
+        dim = uk.shape[0] // heads
+        mixer = LatentMixer(heads, dim, uq.shape[0] // heads - dim, uv.shape[0] // heads, uq.shape[1], uk.shape[1],
+                            float(const(f"l{i}.scale")), int(const(f"l{i}.window")) or None, float(const(f"l{i}.rot_base")),
+                            int(const(f"l{i}.rot_dims")), source if source != i else None)
+        ff = f"l{i}.mlp.gate"
+        layers.append(HybridLayer(mixer, BiasedSwiGLU(_need(facts, ff).shape[0]) if facts.has(ff) else None, i, shift=True))
+    if not layers:
+        raise ValueError("no layers found among the graph's constants")
+    vocab, width = _need(facts, "embed").shape
+    spec = HybridSpec("ruperax", layers, width, vocab, 1, float(const("norm_eps")), 1.0, float(const("embedding_scale")), 0.0,
+                      facts.max_len, facts.batch, facts.pad_id, facts.eos_id, facts.early_stop, topk, _executor_dtype(),
+                      norm_groups=int(const("norm_groups")), positions=_need(facts, "pos").shape[0])
+    return ParallelDecoder(spec, parallel_weights(facts.init, spec))
+
+
+def _build_hybrid(facts, topk=1):
+    """The hybrid executor of a graph whose layers are tensors `l<i>.*`: sizes from the tensors, constants from the named
+    constants the layers recorded, the arithmetic ('bf16' or 'fp32') from the precision the graph was built with."""
+    from .hybrid import ClampedGLU, HybridDecoder, HybridLayer, HybridSpec, MemoryMixer, WindowMixer
+    from .loader import hybrid_weights
+    const = _const_reader(facts)
     layers = []
     while const(f"l{len(layers)}.source", False) is not None:
         i = len(layers)
@@ -284,11 +318,10 @@ def _build_hybrid(facts, topk=1):
         raise ValueError("no layers found among the graph's constants")
     vocab, width = _need(facts, "embed").shape
     cap = const("logit_softcap", False)
-    precision = REGISTRY.get("tensor_type").precision
     spec = HybridSpec("zekilix", layers, width, vocab, facts.init["l0.hc1.in"].shape[0] if facts.has("l0.hc1.in") else 1,
                       float(const("norm_eps")), float(const("residual_mult")), float(const("embedding_scale")),
                       float(cap) if cap is not None else 0.0, facts.max_len, facts.batch, facts.pad_id, facts.eos_id,
-                      facts.early_stop, topk, {"bf16": "bfloat16", "fp32": "float32"}[precision])
+                      facts.early_stop, topk, _executor_dtype())
     return HybridDecoder(spec, hybrid_weights(facts.init, spec))
 
 
@@ -303,6 +336,8 @@ def _family(facts):
         return "rwkv"
     if facts.has("l0.mix.q") and facts.has("l0.norm1"):
         return "zekilix"
+    if facts.has("l0.mix.uk") and facts.has("l0.rg1"):
+        return "ruperax"
     return None
 
 
@@ -498,7 +533,7 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
         prog.interp_outputs = list(graph.outputs)
         k = _sampling_k(facts)
         use_fp8_cache = _fp8_cache_of(facts, fp8_cache)
-        if use_fp8_cache and family in ("rwkv", "zekilix"):
+        if use_fp8_cache and family in ("rwkv", "zekilix", "ruperax"):
             raise ValueError(f"fp8_cache: the {family} executor has no FP8 KV cache")
         steps = min(PROBE_STEPS, facts.max_loop)
         # one-iteration probe: operand shapes of the native operators
@@ -511,6 +546,8 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
             decoder = _build_rwkv(facts, shapes, k)
         elif family == "zekilix":
             decoder = _build_hybrid(facts, k)
+        elif family == "ruperax":
+            decoder = _build_parallel(facts, k)
         else:
             spec, weights = _build_transformer(facts, shapes, family, k, use_fp8_cache)
             decoder = fused.FusedDecoder(spec, weights)

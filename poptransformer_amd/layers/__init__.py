@@ -9,6 +9,7 @@ from .embedding import Embedding
 from .mlp import MLP
 from .lm_head import LMHead
 from .streams import NamedLinear, StreamConnection, WeightNorm
+from .parallel import BiasedSwiGLU, GroupedRMSNorm, ResultGate, RotaryTable, TokenShift
 
 __all__ = ["BaseLayer", "Linear", "LayerNorm", "RMSLayerNorm", "Embedding", "MLP", "LMHead", "NamedLinear", "StreamConnection",
-           "WeightNorm"]
+           "WeightNorm", "BiasedSwiGLU", "GroupedRMSNorm", "ResultGate", "RotaryTable", "TokenShift"]

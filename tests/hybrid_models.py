@@ -1,4 +1,4 @@
-"""Small configurations and random tensors of hybrid decoders for the tests."""
+"""Small configurations and random tensors of hybrid decoders for the tests, and what the tests of whole decoders share."""
 import numpy as np
 
 
@@ -92,3 +92,59 @@ def random_tensors(cfg, seed, forget_bias=2.0):
     vec("final.norm", d)
     lin("head", V, d, 2.0)
     return sd
+
+
+def token_ids(seed, n, cfg):
+    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
+
+
+class Reference:
+    """The oracle's logits of one sequence, and per number format how far from them a result may be: the rms of the
+    difference over the rms of all logits is compared with what rounding alone does to this very sequence (fp32 accumulates
+    in another order: a floor)."""
+
+    def __init__(self, forward, sd, cfg, ids, dtype):
+        self.logits = forward(sd, cfg, ids)
+        self.scale = np.sqrt((self.logits ** 2).mean())
+        if dtype == "float32":
+            self.limit = 1e-4
+        else:
+            # (three roundings: one sample of what rounding does says little about a single position)
+            draws = [self.error(forward(sd, cfg, ids, rnd=lambda a, k=k: bf16(a * (1 + k)) / (1 + k))).max() for k in (0, 0.13, 0.31)]
+            self.limit = 2.0 * max(draws) + 0.01
+
+    def error(self, got, at=slice(None)):
+        return np.sqrt(((got - self.logits[at]) ** 2).mean(-1)) / self.scale
+
+    def check(self, got, at=slice(None)):
+        got = got.float().cpu().numpy() if hasattr(got, "cpu") else got
+        err = self.error(got, at)
+        assert err.max() < self.limit, f"place {int(err.argmax())}: {err.max():.2e}, limit {self.limit:.2e}"
+
+
+def feed(dec, slot, ids, cuts):
+    """The tokens in portions of the given sizes (the rest one by one); logits of all positions."""
+    out, p, cuts = [], 0, list(cuts)
+    while p < len(ids):
+        c = min(cuts.pop(0) if cuts else 1, len(ids) - p)
+        out.append(dec.advance([(slot, ids[p:p + c], list(range(c)))]).cpu().numpy())
+        p += c
+    return np.concatenate(out)
+
+
+def greedy(forward, cfg, sd, ids, steps, pad, tie):
+    """The loop by the oracle: container after `steps` iterations, and per row the number of comparable columns (up to the
+    first place where two logits are closer than `tie` of the largest)."""
+    out = ids.copy()
+    B, L = ids.shape
+    cols = np.full(B, min(steps + 1, L))
+    for b in range(B):
+        for t in range(min(steps, L - 1)):
+            if out[b, t + 1] != pad:
+                continue
+            logits = forward(sd, cfg, out[b, :t + 1])[-1]
+            top = np.sort(logits)[-2:]
+            if top[1] - top[0] < tie * np.abs(logits).max():
+                cols[b] = min(cols[b], t + 1)
+            out[b, t + 1] = int(logits.argmax())
+    return out, cols

@@ -10,7 +10,7 @@ import pytest
 import torch
 
 from oracle import zekilix as Z
-from tests.hybrid_models import attention, bf16, config, dense, mlstm, random_tensors, small_config
+from tests.hybrid_models import Reference, attention, config, dense, feed, greedy, mlstm, random_tensors, small_config, token_ids
 
 pytestmark = pytest.mark.gpu
 
@@ -41,42 +41,8 @@ def _decoder(cfg, sd, dtype, max_len=400, slots=2, pass_rows=None, batch=1, **kw
     return Decoder(spec, loader.hybrid_weights(sd, spec), slots=slots)
 
 
-def _ids(seed, n, cfg):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
-
-
-class Expected:
-    """The oracle's logits of one sequence, and per number format how far from them a result may be: the rms of the
-    difference over the rms of all logits is compared with what rounding alone does to this very sequence (fp32 accumulates
-    in another order: a floor)."""
-
-    def __init__(self, sd, cfg, ids, dtype):
-        self.logits = Z.forward(sd, cfg, ids)
-        self.scale = np.sqrt((self.logits ** 2).mean())
-        if dtype == "float32":
-            self.limit = 1e-4
-        else:
-            # (three roundings: one sample of what rounding does says little about a single position)
-            draws = [self.error(Z.forward(sd, cfg, ids, rnd=lambda a, k=k: bf16(a * (1 + k)) / (1 + k))).max() for k in (0, 0.13, 0.31)]
-            self.limit = 2.0 * max(draws) + 0.01
-
-    def error(self, got, at=slice(None)):
-        return np.sqrt(((got - self.logits[at]) ** 2).mean(-1)) / self.scale
-
-    def check(self, got, at=slice(None)):
-        got = got.float().cpu().numpy() if torch.is_tensor(got) else got
-        err = self.error(got, at)
-        assert err.max() < self.limit, f"place {int(err.argmax())}: {err.max():.2e}, limit {self.limit:.2e}"
-
-
-def _feed(dec, slot, ids, cuts):
-    """The tokens in portions of the given sizes (the rest one by one); logits of all positions."""
-    out, p, cuts = [], 0, list(cuts)
-    while p < len(ids):
-        c = min(cuts.pop(0) if cuts else 1, len(ids) - p)
-        out.append(dec.advance([(slot, ids[p:p + c], list(range(c)))]).cpu().numpy())
-        p += c
-    return np.concatenate(out)
+def Expected(sd, cfg, ids, dtype):
+    return Reference(Z.forward, sd, cfg, ids, dtype)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -85,13 +51,13 @@ def test_prompts_portions_and_decoding(name, dtype):
     cfg = CONFIGS[name]
     sd = random_tensors(cfg, 5)
     T = 150
-    ids = _ids(1, T, cfg)
+    ids = token_ids(1, T, cfg)
     want = Expected(sd, cfg, ids, dtype)
     dec = _decoder(cfg, sd, dtype)
     for cuts in ((T,), (2, 2, 3, 64, 65), (1, 70, 2, 63), (100,), (1,)):
         print(f"{name} {dtype} cuts {cuts}", flush=True)
         s = dec.open()                       # the slot of the sequence before
-        want.check(_feed(dec, s, ids, cuts))
+        want.check(feed(dec, s, ids, cuts))
         dec.close(s)
 
 
@@ -101,10 +67,10 @@ def test_a_short_sequence_from_its_first_token(dtype):
     sd = random_tensors(cfg, 6)
     dec = _decoder(cfg, sd, dtype)
     for n in (1, 2, 3):
-        ids = _ids(n, n, cfg)
+        ids = token_ids(n, n, cfg)
         for cuts in ((n,), (1,)):
             s = dec.open()
-            Expected(sd, cfg, ids, dtype).check(_feed(dec, s, ids, cuts))
+            Expected(sd, cfg, ids, dtype).check(feed(dec, s, ids, cuts))
             dec.close(s)
 
 
@@ -116,7 +82,7 @@ def test_unequal_batches_against_each_alone_and_slots_used_again(dtype):
     sd = random_tensors(cfg, 7)
     dec = _decoder(cfg, sd, dtype, slots=1)
     for round_, lens in enumerate(((1, 90, 33, 140), (130, 2, 64), (65, 17, 1, 3, 80, 129))):
-        seqs = [_ids(10 * round_ + i, n + 12, cfg) for i, n in enumerate(lens)]
+        seqs = [token_ids(10 * round_ + i, n + 12, cfg) for i, n in enumerate(lens)]
         want = [Expected(sd, cfg, q, dtype) for q in seqs]
         slots = [dec.open() for _ in seqs]
         got = dec.advance([(s, q[:n], list(range(n))) for s, q, n in zip(slots, seqs, lens)]).cpu().numpy()
@@ -143,7 +109,7 @@ def test_mixed_batches_and_passes_smaller_than_a_prompt(dtype):
     cfg = small_config()
     sd = random_tensors(cfg, 8)
     dec = _decoder(cfg, sd, dtype, slots=3, pass_rows=48)
-    seqs = [_ids(30 + i, 170, cfg) for i in range(3)]
+    seqs = [token_ids(30 + i, 170, cfg) for i in range(3)]
     want = [Expected(sd, cfg, q, dtype) for q in seqs]
     slots = [dec.open() for _ in seqs]
     at = [0, 0, 0]
@@ -164,9 +130,9 @@ def test_long_decoding(dtype):
     cfg = small_config()
     sd = random_tensors(cfg, 9, forget_bias=5.0)
     dec = _decoder(cfg, sd, dtype, max_len=700, pass_rows=16)
-    ids = _ids(2, 600, cfg)
+    ids = token_ids(2, 600, cfg)
     s = dec.open()
-    Expected(sd, cfg, ids, dtype).check(_feed(dec, s, ids, (16,)))
+    Expected(sd, cfg, ids, dtype).check(feed(dec, s, ids, (16,)))
 
 
 def test_requests_that_do_not_fit_are_refused():
@@ -183,24 +149,6 @@ def test_requests_that_do_not_fit_are_refused():
 
 
 # ------------------------------------------------------------------------------------------- generation
-def _greedy(cfg, sd, ids, steps, pad, tie):
-    """The loop by the oracle: container after `steps` iterations, and per row the number of comparable columns (up to the
-    first place where two logits are closer than `tie` of the largest)."""
-    out = ids.copy()
-    B, L = ids.shape
-    cols = np.full(B, min(steps + 1, L))
-    for b in range(B):
-        for t in range(min(steps, L - 1)):
-            if out[b, t + 1] != pad:
-                continue
-            logits = Z.forward(sd, cfg, out[b, :t + 1])[-1]
-            top = np.sort(logits)[-2:]
-            if top[1] - top[0] < tie * np.abs(logits).max():
-                cols[b] = min(cols[b], t + 1)
-            out[b, t + 1] = int(logits.argmax())
-    return out, cols
-
-
 def _session(cfg, sd, precision, B, L, steps, allow_fused=True, **kw):
     from poptransformer_amd.models.zekilix import ZekilixDecModel
     from poptransformer_amd.utils import prepare_model_session
@@ -222,7 +170,7 @@ def test_generation_through_the_session(name, precision, allow_fused):
         ids[b, :n] = rng.integers(2, cfg["vocab"], n)
     session, model = _session(cfg, sd, precision, B, L, steps, allow_fused, **({"strict": True} if allow_fused else {}))
     assert session.executor_kind == ("fused:zekilix" if allow_fused else "interpreter"), session.fallback_reason
-    want, cols = _greedy(cfg, sd, ids, steps, 0, 1e-4 if precision == "fp32" else 0.05)
+    want, cols = greedy(Z.forward, cfg, sd, ids, steps, 0, 1e-4 if precision == "fp32" else 0.05)
     for _ in range(2):                                       # the second run starts from a used cache
         session.run(model.build_input_dict(input_ids=[list(r[r != 0]) for r in ids]))
         got = session.anchor_arrays["Loop:0"]
@@ -288,7 +236,7 @@ def test_trace_runner(tmp_path, dtype):
     out.mkdir()
     (model / "config.json").write_text(json.dumps(cfg))
     save_file({k: torch.from_numpy(v).to(torch.bfloat16) for k, v in sd.items()}, str(model / "model.safetensors"))
-    a, b = _ids(1, 40, cfg), _ids(2, 7, cfg)
+    a, b = token_ids(1, 40, cfg), token_ids(2, 7, cfg)
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:30], "want": [29, 0]}, {"id": "b", "tokens": b[:5], "want": []}], "end": []},
              {"step": 1, "entries": [{"id": "b", "tokens": b[5:6], "want": [0]}, {"id": "a", "tokens": a[30:31], "want": [0]}], "end": ["b"]},
              {"step": 2, "entries": [{"id": "a", "tokens": a[31:32], "want": []}], "end": ["a"]},
