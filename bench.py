@@ -26,9 +26,9 @@ bytes; or, with the per-operator executor, the fused INT4 gate/up projection), a
 Other workloads (``--workload``), each printing one line of the same form: ``gemm`` = the single INT4
 weight-only operator X[M, 4096] by W[4096, 11008] at M = ``--batch``; ``chatglm2`` = ChatGLM2-6B-shape FP8
 decode; ``rwkv`` = RWKV-4-7B-shape INT4 recurrent decode; ``prompt`` = the prompt of the headline model taken in
-passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix`` = the
-Zekilix design (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights at the same sizes: decode at batch
-1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
+passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix`` and
+``ruperax`` = these designs (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights (and, for Ruperax, the
+Zekilix design) at the same sizes: decode at batch 1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
 serve the hardware-counter measurement of the HBM traffic (see their help).
 """
 import argparse
@@ -432,6 +432,17 @@ def zekilix_config(width, ff, layers):
             "norm": {"eps": 1e-5}, "residual_mult": 1.0, "streams": 2, "vocab": 32000, "width": width}
 
 
+def ruperax_config(width, ff, layers):
+    """Latent attention (heads of 128 + 64, values of 128, latents of 1536 and 512), every second layer over the cache of the
+    one before it."""
+    mixer = {"heads": width // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 1536, "kv_rank": 512, "scale": 192 ** -0.5,
+             "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": 64}}
+    entries = [{"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff}, "mixer": dict(mixer, **({"kv_from": i - 1} if i % 2 else {}))}
+               for i in range(layers)]
+    return {"architecture": "Ruperax", "embedding": {"scale": 1.0}, "layers": entries, "max_positions": 2304, "norm": {"eps": 1e-5, "groups": 4},
+            "vocab": 32000, "width": width}
+
+
 def hybrid_step_bytes(spec, weights, B, t):
     """Bytes one decode iteration of a hybrid decoder must move at context t: the weights of every layer run, the key rows
     of the windows, the memories (read and written), the head."""
@@ -439,22 +450,29 @@ def hybrid_step_bytes(spec, weights, B, t):
     for lay in spec.layers:
         n += sum(w.nbytes for w in weights.layers[lay.source].linears())
         m = lay.mixer
+        seen = min(t + 1, getattr(m, "window", None) or t + 1)
         if m.kind == "attention":
-            n += B * m.kv_heads * (2 * m.dim + 4 / m.kv_heads) * min(t + 1, m.window or t + 1)
+            n += B * m.kv_heads * (2 * m.dim + 4 / m.kv_heads) * seen
+        elif m.kind == "latent":
+            n += B * 2 * (m.kv_rank + m.rot_dim) * seen + 2 * m.heads * m.kv_rank * (m.dim + m.vdim)
         else:
             n += B * 2 * 4 * m.heads * m.dim * (m.vdim + 1)
     return n
 
 
-def zekilix_workload(args):
+def design_workload(args, design):
     """Decode iterations (contexts 1024 .. 1024 + steps - 1, replayed from a HIP graph, one launch per operator) and prompt
-    passes of the Zekilix design, and of the Llama-2 executor with fp16 weights at equal width, feed-forward size, layer
-    count, vocabulary and head size.  --layers shortens both models (for profiles)."""
+    passes of a design, beside the executors that come closest to it: Llama-2 with fp16 weights (and for Ruperax the Zekilix
+    design) at equal width, feed-forward size, layer count, vocabulary and head size.  --layers shortens all of them (for
+    profiles)."""
     import torch
-    from poptransformer_amd.engine import fused, hybrid, loader, synthetic
+    from poptransformer_amd.engine import fused, hybrid, loader, parallel, synthetic
     rng = np.random.Generator(np.random.PCG64(1234))
     first, steps, max_len = 1024, args.steps, 2048
     results = []
+    models = [design] + (["zekilix"] if design != "zekilix" else []) + ["llama2_fp16"]
+    if args.only:
+        models = [m for m in models if m.startswith(args.only)]
 
     def timed(fn):
         torch.cuda.synchronize()
@@ -463,30 +481,37 @@ def zekilix_workload(args):
         torch.cuda.synchronize()
         return time.perf_counter() - t0
 
+    def prepare(name, width, ff, layers):
+        """(decoder of (batch, length), bytes of a decode iteration at (batch, context), parameters of the Linears of a row)"""
+        if name == "llama2_fp16":
+            lcfg = dict(LLAMA2_7B, hidden_size=width, intermediate_size=ff, num_attention_heads=width // 128, num_hidden_layers=layers)
+            lw = synthetic.llama2_f16_synthetic_weights(lcfg)
+            return (lambda B, L: fused.FusedDecoder(loader.llama2_spec(lcfg, L, B), lw),
+                    lambda B, t: lw.nbytes() + B * layers * 4 * width * (t + 1), layers * (4 * width * width + 3 * width * ff))
+        if name == "zekilix":
+            cfg, spec_of, tensors, weights_of, decoder = (zekilix_config(width, ff, layers), loader.zekilix_spec, synthetic.HybridTensors,
+                                                          loader.hybrid_weights, hybrid.HybridDecoder)
+        else:
+            cfg, spec_of, tensors, weights_of, decoder = (ruperax_config(width, ff, layers), loader.ruperax_spec, synthetic.ParallelTensors,
+                                                          loader.parallel_weights, parallel.ParallelDecoder)
+        spec = spec_of(cfg, max_len, 1)
+        w = weights_of(tensors(cfg), spec)
+        params = sum(x.n_main * x.K for lay in spec.layers for x in w.layers[lay.source].linears())
+        params += sum(m.heads * m.kv_rank * (m.dim + m.vdim) for m in (lay.mixer for lay in spec.layers) if m.kind == "latent")
+        return lambda B, L: decoder(spec_of(cfg, L, B), w), lambda B, t: hybrid_step_bytes(spec, w, B, t), params
+
     for width, ff, layers in ((2048, 5632, 8), (4096, 11008, 8)):
         if args.width and args.width != width:
             continue
         layers = args.layers or layers
-        cfg = zekilix_config(width, ff, layers)
-        lcfg = dict(LLAMA2_7B, hidden_size=width, intermediate_size=ff, num_attention_heads=width // 128, num_hidden_layers=layers)
-        makers = {}
-        if args.only != "llama2":
-            spec = loader.zekilix_spec(cfg, max_len, 1)
-            hw = loader.hybrid_weights(synthetic.HybridTensors(cfg), spec)
-            makers["zekilix"] = (lambda B: hybrid.HybridDecoder(loader.zekilix_spec(cfg, max_len, B), hw),
-                                 lambda B, t: hybrid_step_bytes(spec, hw, B, t), sum(w.n_main * w.K for lay in spec.layers for w in
-                                                                                    hw.layers[lay.source].linears()))
-        if args.only != "zekilix":
-            lw = synthetic.llama2_f16_synthetic_weights(lcfg)
-            makers["llama2_fp16"] = (lambda B: fused.FusedDecoder(loader.llama2_spec(lcfg, max_len, B), lw),
-                                     lambda B, t: lw.nbytes() + B * layers * 4 * width * (t + 1), layers * (4 * width * width + 3 * width * ff))
         row = {"width": width, "ff": ff, "layers": layers}
-        for name, (make, step_bytes, params) in makers.items():
+        for name in models:
+            make, step_bytes, params = prepare(name, width, ff, layers)
             r = row[name] = {"linear_parameters": params}
             for B in (1, 16):
                 if args.rows_only:
                     break
-                dec = make(B)
+                dec = make(B, max_len)
                 dec.capture()
                 ids = np.zeros((B, max_len), np.int32)
                 ids[:, :first] = rng.integers(3, 32000, (B, first))
@@ -505,9 +530,7 @@ def zekilix_workload(args):
                 if args.decode_only:
                     break
                 L = rows + 2
-                spec_L = (lambda B: hybrid.HybridDecoder(loader.zekilix_spec(cfg, L, B), hw)) if name == "zekilix" else \
-                    (lambda B: fused.FusedDecoder(loader.llama2_spec(lcfg, L, B), lw))
-                dec = spec_L(1)
+                dec = make(1, L)
                 ids = np.zeros((1, L), np.int32)
                 ids[:, :rows + 1] = rng.integers(3, 32000, (1, rows + 1))
 
@@ -521,16 +544,16 @@ def zekilix_workload(args):
                 note(f"{name} width {width} prompt {rows}: {best * 1e3:.3f} ms")
                 del dec
                 torch.cuda.empty_cache()
+            del make, step_bytes
+            torch.cuda.empty_cache()
         results.append(row)
-        makers.clear()
-        hw = lw = None
-        torch.cuda.empty_cache()
-    last = results[-1].get("zekilix") or results[-1]["llama2_fp16"]
+    last = results[-1][models[0]]
     head = last.get("decode_b1") or {"tokens_per_s": last["prompt_2048"]["tokens_per_s"], "ms_per_step": last["prompt_2048"]["ms"]}
     return {"metric": "decode tokens/s", "value": head["tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": args.warmup,
             "ms_per_step": head["ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
             "dtype": "bf16 weights and activations, f32 accumulation, residual and state", "data": "synthetic",
-            "config": {"workload": "Zekilix-shaped decode at batch 1 beside Llama-2 with fp16 weights at equal size", "executor": "operators"},
+            "config": {"workload": f"{design.capitalize()}-shaped decode at batch 1 beside {' and '.join(models[1:]) or 'nothing'} at equal size",
+                       "executor": "operators"},
             "sizes": results}
 
 
@@ -544,17 +567,17 @@ def main():
     ap.add_argument("--batch", type=int, default=1)
     ap.add_argument("--executor", choices=["persistent", "operators"], default=None,
                     help="default: persistent when the batch fits it (<= 16, fp16 cache), else operators")
-    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix", "ruperax"], default="decode",
                     help="decode: the Llama2-7B-shape INT4 decode loop (the headline); gemm: the single INT4 "
                          "weight-only operator at M = --batch rows; chatglm2: ChatGLM2-6B-shape FP8 decode; "
                          "rwkv: RWKV-4-7B-shape INT4 recurrent decode; prompt: the headline model's prompt in passes "
-                         "of --rows-per-pass rows (--steps passes); zekilix: the Zekilix design beside Llama-2 with fp16 weights at "
-                         "equal sizes, decode and prompts")
-    ap.add_argument("--width", type=int, default=0, help="zekilix workload: only this width")
-    ap.add_argument("--layers", type=int, default=0, help="zekilix workload: layers of both models (even)")
-    ap.add_argument("--only", choices=["zekilix", "llama2"], default=None, help="zekilix workload: one of the two models")
-    ap.add_argument("--decode-only", action="store_true", help="zekilix workload: no prompts")
-    ap.add_argument("--rows-only", action="store_true", help="zekilix workload: prompts only")
+                         "of --rows-per-pass rows (--steps passes); zekilix, ruperax: that design beside Llama-2 with fp16 weights "
+                         "(ruperax: and Zekilix) at equal sizes, decode and prompts")
+    ap.add_argument("--width", type=int, default=0, help="zekilix and ruperax workloads: only this width")
+    ap.add_argument("--layers", type=int, default=0, help="zekilix and ruperax workloads: layers of the models (even)")
+    ap.add_argument("--only", choices=["zekilix", "ruperax", "llama2"], default=None, help="zekilix and ruperax workloads: one of the models")
+    ap.add_argument("--decode-only", action="store_true", help="zekilix and ruperax workloads: no prompts")
+    ap.add_argument("--rows-only", action="store_true", help="zekilix and ruperax workloads: prompts only")
     ap.add_argument("--rows-per-pass", type=int, default=64,
                     help="prompt workload: rows (batch x positions) per pass, up to 2048")
     ap.add_argument("--fp8-cache", action="store_true",
@@ -603,8 +626,8 @@ def main():
     if args.workload == "prompt":
         print(json.dumps(prompt_workload(args)))
         return
-    if args.workload == "zekilix":
-        print(json.dumps(zekilix_workload(args)))
+    if args.workload in ("zekilix", "ruperax"):
+        print(json.dumps(design_workload(args, args.workload)))
         return
     B, cfg = args.batch, LLAMA2_7B
     executor = args.executor or ("persistent" if B <= 16 else "operators")

@@ -37,28 +37,78 @@ __device__ __forceinline__ void rotate8(const float* cs, float (&v)[8]) {
 // ------------------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void latent_append_kernel(LA a) {
+  constexpr int U = 2;                                    // pieces of eight features a thread holds (more: read again)
   __shared__ float red[2][4];
-  const int r = blockIdx.x, Qp = (a.q_rank + 7) & ~7;
+  const int r = blockIdx.x, Qp = (a.q_rank + 7) & ~7, own = a.kv_norm != nullptr;
   const T* p = reinterpret_cast<const T*>(a.proj) + (size_t)r * a.ld;
   const T* c = p + Qp;
-  float sq = 0.f, sc = 0.f;
-  for (int i = threadIdx.x; i < a.q_rank; i += 256) { const float v = (float)p[i]; sq = __builtin_fmaf(v, v, sq); }
-  if (a.kv_norm)
-    for (int i = threadIdx.x; i < a.kv_rank; i += 256) { const float v = (float)c[i]; sc = __builtin_fmaf(v, v, sc); }
-  const float iq = 1.0f / sqrtf(workgroup_sum<4>(sq, red[0]) / (float)a.q_rank + a.eps);
-  T* cq = reinterpret_cast<T*>(a.cq) + (size_t)r * Qp;
-  for (int i = threadIdx.x; i < Qp; i += 256) cq[i] = i < a.q_rank ? (T)((float)p[i] * iq * a.q_norm[i]) : (T)0.0f;
-  if (!a.kv_norm) return;
-  const float ic = 1.0f / sqrtf(workgroup_sum<4>(sc, red[1]) / (float)a.kv_rank + a.eps);
   const int pos = position_of(a, r);
-  T* dst = reinterpret_cast<T*>(a.ring) + ((size_t)a.slot[r] * a.ring_len + pos % a.ring_len) * (a.R + a.P);
-  for (int i = threadIdx.x; i < a.R; i += 256) dst[i] = i < a.kv_rank ? (T)((float)c[i] * ic * a.kv_norm[i]) : (T)0.0f;
   const float* cs = a.cos_sin + (size_t)pos * a.P;
-  for (int i = threadIdx.x; i < a.P / 2; i += 256) {
-    const float x = (float)c[a.R + 2 * i], y = (float)c[a.R + 2 * i + 1];
-    dst[a.R + 2 * i] = (T)(x * cs[2 * i] - y * cs[2 * i + 1]);
-    dst[a.R + 2 * i + 1] = (T)(y * cs[2 * i] + x * cs[2 * i + 1]);
+  const int nq = Qp / 8, nc = a.R / 8, np = own ? a.P / 8 : 0, rot_at = 255 - (int)threadIdx.x;     // (the last threads turn the rotated part)
+  // everything is requested before the first sum: latents, norms' weights, angles (padding columns of proj are zero)
+  float v[U][8], w[U][8], l[8], lw[8], t[8];
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int i = threadIdx.x + u * 256 < nq ? threadIdx.x + u * 256 : 0;
+    load8(p + i * 8, true, 8, v[u]);
+    load8(a.q_norm + i * 8, i * 8 + 8 <= a.q_rank, a.q_rank - i * 8, w[u]);
   }
+  const int lc = threadIdx.x < nc ? threadIdx.x : 0, rc = rot_at < np ? rot_at : 0;
+  if (own) {
+    load8(c + lc * 8, true, 8, l);
+    load8(a.kv_norm + lc * 8, lc * 8 + 8 <= a.kv_rank, a.kv_rank - lc * 8, lw);
+    load8(c + a.R + rc * 8, true, 8, t);
+    rotate8(cs + rc * 8, t);
+  }
+  float sq = 0.f, sc = 0.f;
+#pragma unroll
+  for (int u = 0; u < U; ++u)
+    if (threadIdx.x + u * 256 < nq)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) sq = __builtin_fmaf(v[u][e], v[u][e], sq);
+  for (int i = threadIdx.x + U * 256; i < nq; i += 256) {
+    float y[8];
+    load8(p + i * 8, true, 8, y);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sq = __builtin_fmaf(y[e], y[e], sq);
+  }
+  if (own && threadIdx.x < nc)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sc = __builtin_fmaf(l[e], l[e], sc);
+  sq = wave_total_dpp(sq);
+  sc = wave_total_dpp(sc);
+  if ((threadIdx.x & 63) == 0) {
+    red[0][threadIdx.x >> 6] = sq;
+    red[1][threadIdx.x >> 6] = sc;
+  }
+  __syncthreads();
+  const float iq = 1.0f / sqrtf((red[0][0] + red[0][1] + red[0][2] + red[0][3]) / (float)a.q_rank + a.eps);
+  T* cq = reinterpret_cast<T*>(a.cq) + (size_t)r * Qp;
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int i = threadIdx.x + u * 256;
+    if (i >= nq) break;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[u][e] = v[u][e] * iq * w[u][e];
+    store8(cq + i * 8, v[u]);
+  }
+  for (int i = threadIdx.x + U * 256; i < nq; i += 256) {
+    float y[8], yw[8];
+    load8(p + i * 8, true, 8, y);
+    load8(a.q_norm + i * 8, i * 8 + 8 <= a.q_rank, a.q_rank - i * 8, yw);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y[e] = y[e] * iq * yw[e];
+    store8(cq + i * 8, y);
+  }
+  if (!own) return;
+  const float ic = 1.0f / sqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)a.kv_rank + a.eps);
+  T* dst = reinterpret_cast<T*>(a.ring) + ((size_t)a.slot[r] * a.ring_len + pos % a.ring_len) * (a.R + a.P);
+  if (threadIdx.x < nc) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) l[e] = l[e] * ic * lw[e];
+    store8(dst + lc * 8, l);
+  }
+  if (rot_at < np) store8(dst + a.R + rc * 8, t);
 }
 
 // ------------------------------------------------------------------------------------------
@@ -332,44 +382,76 @@ __device__ __forceinline__ float part_weight(const LA& a, int r, int head, int l
   return w / wave_sum(w * l);
 }
 
-// 16 rows and NB * 16 value channels of one head per workgroup; the waves share the latent features
+// 16 rows and NB * 16 value channels of one head per workgroup.  The parts meet first: 16 lanes take 128 latent features of a
+// row, and the weighted sums go to LDS, where the waves share the latent features of the product.
 constexpr int LV_NB = 2;
 
 __global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks) {
+  constexpr int AHEAD = 4;                                // steps of the product whose weights are requested at the start
+  extern __shared__ __align__(16) bf16 xs[];              // [16][R + 8]
   __shared__ float weight[16][64];
   __shared__ f32x4 red[4][LV_NB][64];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15, XS = a.R + 8;
   const int head = blockIdx.x / blocks, n0 = (blockIdx.x % blocks) * LV_NB * 16, r0 = blockIdx.y * 16;
   const int count = a.rows - r0 < 16 ? a.rows - r0 : 16, row = r0 + (lc < count ? lc : count - 1);
-  for (int n = wave; n < count; n += 4) weight[n][lane] = part_weight(a, r0 + n, head, lane);
-  const float* po = a.part_o + ((size_t)row * a.H + head) * a.splits * a.R + lg * 8;
-  const bf16* w = reinterpret_cast<const bf16*>(a.uv) + (size_t)head * a.E * a.R + lg * 8;
-  const float* wt = weight[lc < count ? lc : count - 1];
-  f32x4 acc[LV_NB];
+  const bf16* w[LV_NB];
+  bf16x8 wv[AHEAD][LV_NB];
 #pragma unroll
-  for (int n = 0; n < LV_NB; ++n) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
-  __syncthreads();
-  for (int k = wave * 32; k < a.R; k += 128) {
-    bf16x8 wv[LV_NB];
+  for (int n = 0; n < LV_NB; ++n) {
+    const int ch = n0 + n * 16 + lc;
+    w[n] = reinterpret_cast<const bf16*>(a.uv) + ((size_t)head * a.E + (ch < a.E ? ch : a.E - 1)) * a.R + lg * 8;
 #pragma unroll
-    for (int n = 0; n < LV_NB; ++n) {
-      const int ch = n0 + n * 16 + lc;
-      wv[n] = *reinterpret_cast<const bf16x8*>(w + (size_t)(ch < a.E ? ch : a.E - 1) * a.R + k);
+    for (int i = 0; i < AHEAD; ++i) {
+      const int k = wave * 32 + i * 128;
+      wv[i][n] = *reinterpret_cast<const bf16x8*>(w[n] + (k < a.R ? k : 0));
     }
+  }
+  for (int n = wave; n < count; n += 4) weight[n][lane] = part_weight(a, r0 + n, head, lane);
+  __syncthreads();
+  const int chunks = (a.R + 127) / 128, units = count * chunks;
+  for (int u = wave * 4 + lg; u < units; u += 16) {
+    const int n = u / chunks, c = (u % chunks) * 128 + lc * 8;
+    if (c >= a.R) continue;
+    const float* po = a.part_o + ((size_t)(r0 + n) * a.H + head) * a.splits * a.R + c;
     float x[8] = {};
-#pragma unroll 4
-    for (int s = 0; s < a.splits; ++s) {
+    int s = 0;
+    for (; s + 8 <= a.splits; s += 8) {
+      float v[8][8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) load8(po + (size_t)(s + i) * a.R, true, 8, v[i]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float f = weight[n][s + i];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = __builtin_fmaf(f, v[i][e], x[e]);
+      }
+    }
+    for (; s < a.splits; ++s) {
       float v[8];
-      load8(po + (size_t)s * a.R + k, true, 8, v);
-      const float f = wt[s];
+      load8(po + (size_t)s * a.R, true, 8, v);
+      const float f = weight[n][s];
 #pragma unroll
       for (int e = 0; e < 8; ++e) x[e] = __builtin_fmaf(f, v[e], x[e]);
     }
-    bf16x8 xb;
+    store8(xs + n * XS + c, x);
+  }
+  __syncthreads();
+  f32x4 acc[LV_NB];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) xb[e] = (bf16)x[e];
+  for (int n = 0; n < LV_NB; ++n) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const bf16* xr = xs + (lc < count ? lc : count - 1) * XS + lg * 8;
 #pragma unroll
-    for (int n = 0; n < LV_NB; ++n) acc[n] = mma(wv[n], xb, acc[n]);
+  for (int i = 0; i < AHEAD; ++i) {
+    const int k = wave * 32 + i * 128;
+    if (k >= a.R) break;
+    const bf16x8 xb = *reinterpret_cast<const bf16x8*>(xr + k);
+#pragma unroll
+    for (int n = 0; n < LV_NB; ++n) acc[n] = mma(wv[i][n], xb, acc[n]);
+  }
+  for (int k = wave * 32 + AHEAD * 128; k < a.R; k += 128) {
+    const bf16x8 xb = *reinterpret_cast<const bf16x8*>(xr + k);
+#pragma unroll
+    for (int n = 0; n < LV_NB; ++n) acc[n] = mma(*reinterpret_cast<const bf16x8*>(w[n] + k), xb, acc[n]);
   }
 #pragma unroll
   for (int n = 0; n < LV_NB; ++n) red[wave][n][lane] = acc[n];
@@ -616,7 +698,10 @@ extern "C" int pta_latent_append(const LA* args, pta_stream_t stream) {
   const int Qp = (a.q_rank + 7) & ~7;
   PTA_REQUIRE(a.proj && a.q_norm && a.cq && a.q_rank > 0, "pta_latent_append: null pointer, or query latent of %d", a.q_rank);
   PTA_REQUIRE(a.ld >= Qp + (a.kv_norm ? a.R + a.P : 0), "pta_latent_append: rows of %d do not hold the latents", a.ld);
-  PTA_REQUIRE(!a.kv_norm || (a.kv_rank > 0 && a.kv_rank <= a.R), "pta_latent_append: latent of %d in %d", a.kv_rank, a.R);
+  PTA_REQUIRE(!a.kv_norm || (a.kv_rank > 0 && a.kv_rank <= a.R && a.P <= 256 * 8), "pta_latent_append: latent of %d in %d, rotated part of %d",
+              a.kv_rank, a.R, a.P);
+  PTA_REQUIRE(a.ld % 8 == 0 && pta_aligned(a.proj, 16) && pta_aligned(a.cq, 16) && pta_aligned(a.q_norm, 16) &&
+              (!a.kv_norm || pta_aligned(a.kv_norm, 16)), "pta_latent_append: unaligned operand");
   if (a.dtype == PTA_BF16) hipLaunchKernelGGL((latent_append_kernel<bf16>), dim3(a.rows), dim3(256), 0, s, a);
   else hipLaunchKernelGGL((latent_append_kernel<float>), dim3(a.rows), dim3(256), 0, s, a);
   PTA_CHECK_LAUNCH("pta_latent_append");
@@ -678,7 +763,10 @@ extern "C" int pta_latent_values(const LA* args, pta_stream_t stream) {
   PTA_REQUIRE(pta_aligned(a.part_o, 16) && pta_aligned(a.uv, 16) && pta_aligned(a.out, 16), "pta_latent_values: unaligned operand");
   if (a.dtype == PTA_BF16) {
     const int blocks = (a.E + LV_NB * 16 - 1) / (LV_NB * 16);
-    hipLaunchKernelGGL(latent_values_kernel, dim3(a.H * blocks, (a.rows + 15) / 16), dim3(256), 0, s, a, blocks);
+    const size_t smem = (size_t)16 * (a.R + 8) * sizeof(bf16);      // (up to 64 KiB more than its fixed LDS)
+    PTA_REQUIRE(smem <= 48 * 1024 || hipFuncSetAttribute((const void*)latent_values_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                         (int)smem) == hipSuccess, "pta_latent_values: %zu bytes of LDS refused", smem);
+    hipLaunchKernelGGL(latent_values_kernel, dim3(a.H * blocks, (a.rows + 15) / 16), dim3(256), smem, s, a, blocks);
   } else {
     hipLaunchKernelGGL((latent_values_vector_kernel<float>), dim3(a.rows, a.H), dim3(256), a.R * sizeof(float), s, a);
   }

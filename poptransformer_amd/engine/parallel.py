@@ -49,6 +49,9 @@ class ParallelLayerWeights:
         """Every weight once, as a decode iteration reads them."""
         return [w for w in (self.gate1, self.proj, self.uq, self.out, self.gate2, self.gate, self.up, self.down) if w is not None]
 
+    def feed_forward_bytes(self):
+        return sum(w.nbytes for w in (self.gate2, self.gate, self.up, self.down))
+
 
 @dataclass
 class ParallelWeights:
@@ -97,10 +100,15 @@ class ParallelBuffers:
 
 class ParallelDecoder(HybridDecoder):
     absorbed_rows = 16               # sequences with up to this many rows in a pass work on the cached rows themselves
+    # passes of up to branch_rows single rows run a feed-forward of at least branch_bytes on a stream beside the mixer: what two
+    # streams cost to part and meet (measured: feed-forwards of 80 MB lose 4 us per layer by it, of 300 MB gain 11)
+    branch_rows = 16
+    branch_bytes = 128 << 20
 
     def __init__(self, spec, weights, device="cuda", slots=None):
         super().__init__(spec, weights, device, slots)
         self._angles = {}
+        self._side = torch.cuda.Stream()
         self._key_lists = None
 
     def _rows_buffers(self, rows):
@@ -143,6 +151,7 @@ class ParallelDecoder(HybridDecoder):
         return lists[window]
 
     def _mixer(self, i, b, rows):
+        """The heads' gated results, before the output projection."""
         m, lw, n = self.spec.layers[i].mixer, self.w.layers[i], rows.n
         heads, D, P, E, R = m.sizes[:5]
         proj, cq, q = b.proj[lw.proj.n_main], b.cq[lw.uq.K], b.q[lw.uq.n_main]
@@ -163,7 +172,21 @@ class ParallelDecoder(HybridDecoder):
             flat = self._scratch(2 * sum(sizes))[:2 * sum(sizes)].view(self.dtype)
             latent, rot, kv = torch.split(flat, sizes)
             att.over_heads(q, keys, latent.view(count, R), rot.view(count, P), lw.kv, kv.view(count, -1), tiles, gates, ctx)
-        HK.linear(ctx, lw.out, b.x, n, ld=self.spec.width, mul=b.gate1, accumulate=True, workspace=b.workspace)
+        return ctx
+
+    def _projections(self, i, b, n, mixer=True, ff=True):
+        """The sublayers' residual gates, and the mixer's down-projections."""
+        lw, ld, calls = self.w.layers[i], self.spec.width, []
+        if mixer:
+            calls += [(b.h1, lw.gate1, b.gate1, dict(ld=ld, bias=lw.gate1_bias, sigmoid=True, workspace=b.workspace)),
+                      (b.hm, lw.proj, b.proj[lw.proj.n_main], dict(tail=b.head_gates[self.spec.layers[i].mixer.heads], workspace=b.workspace))]
+        if ff:
+            calls.append((b.h2, lw.gate2, b.gate2, dict(ld=ld, bias=lw.gate2_bias, sigmoid=True, workspace=b.workspace)))
+        HK.linear_group(n, *calls)
+
+    def _output(self, i, b, n, ctx):
+        """x += gate1 * (W_o ctx)"""
+        HK.linear(ctx, self.w.layers[i].out, b.x, n, ld=self.spec.width, mul=b.gate1, accumulate=True, workspace=b.workspace)
 
     def _feed_forward(self, i, b, rows):
         lw, n = self.w.layers[i], rows.n
@@ -182,14 +205,22 @@ class ParallelDecoder(HybridDecoder):
                          pos_out=pos_out) if i == 0 else {}
             HK.shift_norm(b.x, n, spec.norm_groups, spec.eps, lw.norm1, b.h1, lw.norm2, b.h2 if ff else None, lw.shift, b.hm,
                           store.shifted[i], rows.slot, last, rows.pos, store.max_len, **first)
-            calls = [(b.h1, lw.gate1, b.gate1, dict(ld=spec.width, bias=lw.gate1_bias, sigmoid=True, workspace=b.workspace)),
-                     (b.hm, lw.proj, b.proj[lw.proj.n_main], dict(tail=b.head_gates[layer.mixer.heads], workspace=b.workspace))]
-            if ff:
-                calls.append((b.h2, lw.gate2, b.gate2, dict(ld=spec.width, bias=lw.gate2_bias, sigmoid=True, workspace=b.workspace)))
-            HK.linear_group(n, *calls)
-            self._mixer(i, b, rows)
-            if ff:
-                self._feed_forward(i, b, rows)
+            if ff and rows.single and n <= self.branch_rows and lw.feed_forward_bytes() >= self.branch_bytes:
+                # the feed-forward is bound by its weights, the mixer by a chain of short launches; they meet in the residual
+                main = torch.cuda.current_stream()
+                self._side.wait_stream(main)
+                with torch.cuda.stream(self._side):
+                    self._projections(i, b, n, mixer=False)
+                    self._feed_forward(i, b, rows)
+                self._projections(i, b, n, ff=False)
+                ctx = self._mixer(i, b, rows)
+                main.wait_stream(self._side)
+                self._output(i, b, n, ctx)
+            else:
+                self._projections(i, b, n, ff=ff)
+                self._output(i, b, n, self._mixer(i, b, rows))
+                if ff:
+                    self._feed_forward(i, b, rows)
             if self.probe is not None:
                 self.probe(i, b.x[:n].clone())
         return b, None

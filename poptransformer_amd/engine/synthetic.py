@@ -222,3 +222,23 @@ class HybridTensors(dict):
             return torch.full(shape, 3.0 if name.endswith("f.b") else 1.0 / shape[0] if ".hc" in name and name.endswith(".in") else 1.0,
                               device=self.dev)
         return torch.randn(shape, generator=self.gen, device=self.dev, dtype=torch.float32).mul_(0.02).to(torch.bfloat16)
+
+
+class ParallelTensors(HybridTensors):
+    """As HybridTensors, for a configuration with latent attention and parallel sublayers."""
+
+    def __init__(self, cfg, seed=0, device="cuda"):
+        super().__init__(dict(cfg, layers=[], streams=None), seed, device)
+        d = cfg["width"]
+        self.shapes["pos"] = (cfg["max_positions"], d)
+        for i, lay in enumerate(cfg["layers"]):
+            p, m, ff = f"l{i}.", lay["mixer"], lay["mlp"]["ff"]
+            H = m["heads"]
+            mix = {"dq": (m["q_rank"], d), "dq.norm": (m["q_rank"],), "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]),
+                   "uk": (H * m["dim"], m["kv_rank"]), "uv": (H * m["vdim"], m["kv_rank"]), "g": (H, d), "o": (d, H * m["vdim"])}
+            if m.get("kv_from") is None:
+                mix.update({"dkv": (m["kv_rank"] + m["rot_dim"], d), "dkv.norm": (m["kv_rank"],)})
+            mlp = {"gate": (ff, d), "up": (ff, d), "down": (d, ff), "gate.b": (ff,), "up.b": (ff,), "down.b": (d,)}
+            rest = {"shift": (d,), "rg1": (d, d), "rg2": (d, d), "rg1.b": (d,), "rg2.b": (d,), "norm1": (d,), "norm2": (d,)}
+            for group, names in (("mix.", mix), ("mlp.", mlp), ("", rest)):
+                self.shapes.update({p + group + n: shape for n, shape in names.items()})

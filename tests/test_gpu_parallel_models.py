@@ -18,7 +18,7 @@ ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 DTYPES = ["float32", "bfloat16"]
 
 
-def _decoder(cfg, sd, dtype, max_len=400, slots=2, pass_rows=None, absorbed_rows=None, batch=1, **kw):
+def _decoder(cfg, sd, dtype, max_len=400, slots=2, pass_rows=None, absorbed_rows=None, batch=1, branch_bytes=None, **kw):
     from poptransformer_amd.engine import loader, parallel
     spec = loader.ruperax_spec(cfg, max_len, batch, dtype=dtype, **kw)
 
@@ -28,6 +28,8 @@ def _decoder(cfg, sd, dtype, max_len=400, slots=2, pass_rows=None, absorbed_rows
         Decoder.pass_rows = pass_rows
     if absorbed_rows is not None:
         Decoder.absorbed_rows = absorbed_rows
+    if branch_bytes is not None:
+        Decoder.branch_bytes = branch_bytes
     return Decoder(spec, loader.parallel_weights(sd, spec), slots=slots)
 
 
@@ -135,7 +137,7 @@ def test_long_decoding(dtype):
     """Several windows and ring lengths of decoded tokens (the rings of a decoder whose passes are short wrap often)."""
     cfg = small_parallel()
     sd = random_parallel(cfg, 9)
-    dec = _decoder(cfg, sd, dtype, max_len=700, pass_rows=16)
+    dec = _decoder(cfg, sd, dtype, max_len=700, pass_rows=16, branch_bytes=0)
     ids = token_ids(2, 500, cfg)
     _reference(sd, cfg, ids, dtype).check(feed(dec, dec.open(), ids, (16,)))
 
@@ -225,8 +227,9 @@ def test_generation_ends_early_and_draws_from_the_top_k():
     assert int(np.asarray(session.anchor_arrays["Loop:1"]).reshape(-1)[0]) < 39
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-def test_prompt_passes_leave_what_the_loop_leaves(dtype):
+@pytest.mark.parametrize("dtype,branch_bytes", [("float32", 0), ("bfloat16", 0), ("bfloat16", 1 << 60)])
+def test_prompt_passes_leave_what_the_loop_leaves(dtype, branch_bytes):
+    """The loop with the feed-forwards on a stream of their own, and without."""
     cfg = small_parallel()
     sd = random_parallel(cfg, 13)
     B, L, n = 3, 120, 90
@@ -237,7 +240,7 @@ def test_prompt_passes_leave_what_the_loop_leaves(dtype):
     def check():
         for b in range(B):
             want[b].check(dec.logits[b:b + 1], [n - 1])
-    dec = _decoder(cfg, sd, dtype, max_len=L, batch=B)
+    dec = _decoder(cfg, sd, dtype, max_len=L, batch=B, branch_bytes=branch_bytes)
     dec.capture()
     for passes in (None, 7, 64):
         dec.reset(ids)
