@@ -66,7 +66,8 @@ typedef struct pta_wide_linear_args {
 
 size_t pta_wide_linear_workspace_bytes(int M, int N);
 int pta_wide_linear(const pta_wide_linear_args* host_args, pta_stream_t stream);
-/* up to four single weights over inputs of the same shape, each with its own input and result: one launch for up to 16 rows */
+/* up to four single weights over inputs of the same shape, each with its own input and result: one launch where
+ * there are few rows, or many rows and whole tiles of channels */
 int pta_wide_linear_group(const pta_wide_linear_args* host_list, int count, pta_stream_t stream);
 
 /* ---- Residual streams (hyper-connections) and layer norm ---------------------------------------------------------

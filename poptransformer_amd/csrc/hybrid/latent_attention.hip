@@ -382,22 +382,21 @@ __device__ __forceinline__ float part_weight(const LA& a, int r, int head, int l
   return w / wave_sum(w * l);
 }
 
-// 16 rows and NB * 16 value channels of one head per workgroup.  The parts meet first: 16 lanes take 128 latent features of a
-// row, and the weighted sums go to LDS, where the waves share the latent features of the product.
-constexpr int LV_NB = 2;
-
-__global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks) {
+// Up to 16 rows (`each`) and NB * 16 value channels of one head per workgroup.  The parts meet first: 16 lanes take 128 latent
+// features of a row, and the weighted sums go to LDS, where the waves share the latent features of the product.
+template <int NB>
+__global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks, int each) {
   constexpr int AHEAD = 4;                                // steps of the product whose weights are requested at the start
   extern __shared__ __align__(16) bf16 xs[];              // [16][R + 8]
   __shared__ float weight[16][64];
-  __shared__ f32x4 red[4][LV_NB][64];
+  __shared__ f32x4 red[4][NB][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15, XS = a.R + 8;
-  const int head = blockIdx.x / blocks, n0 = (blockIdx.x % blocks) * LV_NB * 16, r0 = blockIdx.y * 16;
-  const int count = a.rows - r0 < 16 ? a.rows - r0 : 16, row = r0 + (lc < count ? lc : count - 1);
-  const bf16* w[LV_NB];
-  bf16x8 wv[AHEAD][LV_NB];
+  const int head = blockIdx.x / blocks, n0 = (blockIdx.x % blocks) * NB * 16, r0 = blockIdx.y * each;
+  const int count = a.rows - r0 < each ? a.rows - r0 : each, row = r0 + (lc < count ? lc : count - 1);
+  const bf16* w[NB];
+  bf16x8 wv[AHEAD][NB];
 #pragma unroll
-  for (int n = 0; n < LV_NB; ++n) {
+  for (int n = 0; n < NB; ++n) {
     const int ch = n0 + n * 16 + lc;
     w[n] = reinterpret_cast<const bf16*>(a.uv) + ((size_t)head * a.E + (ch < a.E ? ch : a.E - 1)) * a.R + lg * 8;
 #pragma unroll
@@ -436,9 +435,9 @@ __global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks) {
     store8(xs + n * XS + c, x);
   }
   __syncthreads();
-  f32x4 acc[LV_NB];
+  f32x4 acc[NB];
 #pragma unroll
-  for (int n = 0; n < LV_NB; ++n) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int n = 0; n < NB; ++n) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   const bf16* xr = xs + (lc < count ? lc : count - 1) * XS + lg * 8;
 #pragma unroll
   for (int i = 0; i < AHEAD; ++i) {
@@ -446,17 +445,17 @@ __global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks) {
     if (k >= a.R) break;
     const bf16x8 xb = *reinterpret_cast<const bf16x8*>(xr + k);
 #pragma unroll
-    for (int n = 0; n < LV_NB; ++n) acc[n] = mma(wv[i][n], xb, acc[n]);
+    for (int n = 0; n < NB; ++n) acc[n] = mma(wv[i][n], xb, acc[n]);
   }
   for (int k = wave * 32 + AHEAD * 128; k < a.R; k += 128) {
     const bf16x8 xb = *reinterpret_cast<const bf16x8*>(xr + k);
 #pragma unroll
-    for (int n = 0; n < LV_NB; ++n) acc[n] = mma(*reinterpret_cast<const bf16x8*>(w[n] + k), xb, acc[n]);
+    for (int n = 0; n < NB; ++n) acc[n] = mma(*reinterpret_cast<const bf16x8*>(w[n] + k), xb, acc[n]);
   }
 #pragma unroll
-  for (int n = 0; n < LV_NB; ++n) red[wave][n][lane] = acc[n];
+  for (int n = 0; n < NB; ++n) red[wave][n][lane] = acc[n];
   __syncthreads();
-  if (wave >= LV_NB || lc >= count) return;
+  if (wave >= NB || lc >= count) return;
   const int ch = n0 + wave * 16 + lg * 4;
   if (ch >= a.E) return;
   f32x4 y = red[0][wave][lane];
@@ -756,17 +755,25 @@ extern "C" int pta_latent_rows(const LA* args, pta_stream_t stream) {
   return PTA_OK;
 }
 
+template <int NB>
+static int launch_latent_values(const LA& a, int each, hipStream_t s) {
+  const int blocks = (a.E + NB * 16 - 1) / (NB * 16);
+  const size_t smem = (size_t)16 * (a.R + 8) * sizeof(bf16);        // (beside up to 20 KiB of fixed LDS)
+  PTA_REQUIRE(smem <= 40 * 1024 || hipFuncSetAttribute((const void*)latent_values_kernel<NB>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                       (int)smem) == hipSuccess, "pta_latent_values: %zu bytes of LDS refused", smem);
+  hipLaunchKernelGGL((latent_values_kernel<NB>), dim3(a.H * blocks, (a.rows + each - 1) / each), dim3(256), smem, s, a, blocks, each);
+  return PTA_OK;
+}
+
 extern "C" int pta_latent_values(const LA* args, pta_stream_t stream) {
   LATENT_ENTRY("pta_latent_values")
   PTA_REQUIRE(a.part_o && a.part_ml && a.uv && a.gate && a.out && a.splits >= 1 && a.splits <= 64,
               "pta_latent_values: null pointer, or splits %d (1 .. 64)", a.splits);
   PTA_REQUIRE(pta_aligned(a.part_o, 16) && pta_aligned(a.uv, 16) && pta_aligned(a.out, 16), "pta_latent_values: unaligned operand");
   if (a.dtype == PTA_BF16) {
-    const int blocks = (a.E + LV_NB * 16 - 1) / (LV_NB * 16);
-    const size_t smem = (size_t)16 * (a.R + 8) * sizeof(bf16);      // (up to 64 KiB more than its fixed LDS)
-    PTA_REQUIRE(smem <= 48 * 1024 || hipFuncSetAttribute((const void*)latent_values_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
-                                                         (int)smem) == hipSuccess, "pta_latent_values: %zu bytes of LDS refused", smem);
-    hipLaunchKernelGGL(latent_values_kernel, dim3(a.H * blocks, (a.rows + 15) / 16), dim3(256), smem, s, a, blocks);
+    // few rows: many workgroups with few channels; a batch: fewer rows each, so that its parts are not read by too many
+    const int rc = a.rows <= 4 ? launch_latent_values<2>(a, 16, s) : launch_latent_values<4>(a, a.rows <= 64 ? 4 : 16, s);
+    if (rc) return rc;
   } else {
     hipLaunchKernelGGL((latent_values_vector_kernel<float>), dim3(a.rows, a.H), dim3(256), a.R * sizeof(float), s, a);
   }

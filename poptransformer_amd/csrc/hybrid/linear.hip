@@ -222,7 +222,10 @@ extern "C" int pta_wide_linear_group(const pta_wide_linear_args* list, int count
                 "%s: single matrices with the same rows and features", name);
   }
   hipStream_t s = (hipStream_t)stream;
-  if (list[0].dtype == PTA_FP32 || list[0].M > 16) {         // many rows: each fills the machine by itself
+  // one launch: up to 16 rows, and whole tiles of more than 64 (whose workgroups would not fill the machine evenly one by one)
+  bool together = list[0].dtype == PTA_BF16 && (list[0].M <= 16 || (list[0].M > 64 && list[0].K >= 512));
+  for (int i = 0; i < count && list[0].M > 64; ++i) together = together && list[i].N % 128 == 0;
+  if (!together) {
     for (int i = 0; i < count; ++i) {
       const int rc = wide_linear(list[i], s, name);
       if (rc) return rc;

@@ -5,7 +5,13 @@
 
 typedef pta_shift_norm_args SN;
 
-constexpr int SN_ROWS = 4;               // rows a workgroup walks through where there are many (and the row before them)
+constexpr int SN_ROWS = 4;               // rows a workgroup walks through at most (and the row before them)
+
+// many rows: fewer of them made twice; not so few workgroups that their walks show
+static int rows_of_a_workgroup(const pta_shift_norm_args& a) {
+  const int n = a.rows / 1024;
+  return !a.shift || n < 1 ? 1 : (n > SN_ROWS ? SN_ROWS : n);
+}
 
 // A workgroup takes `rows_each` rows one after the other.  A thread owns the same columns of all of them, so the row before
 // (normed, fp32) waits for it in LDS; the row before the first comes from the sequence's state, or is made once more.
@@ -284,7 +290,7 @@ static void launch_wide(const SN& a, int rows_each, hipStream_t s) {
 template <typename T>
 static int launch_shift_norm(const SN& a, hipStream_t s) {
   const bool few = a.rows <= 64 && a.width >= 2048;        // a row of 1024 threads shortens the chain of a row
-  const int rows_each = a.rows <= 256 || !a.shift ? 1 : SN_ROWS;
+  const int rows_each = rows_of_a_workgroup(a);
   if ((a.width / a.groups) % 256 == 0 && a.h_ld == a.width) {
     if (few || a.width > 4096) {
       if (a.width <= 4096) launch_wide<T, 1024, 1>(a, rows_each, s);

@@ -47,6 +47,7 @@ class DecodeLoop:
         """Record one loop iteration into a HIP graph (after an eager iteration has warmed up
         every code path).  The iteration depends on device state only, so it can be replayed."""
         self.reset(np.zeros((self.spec.batch, self.spec.max_len), np.int32))
+        torch.cuda.synchronize()         # the stream of the recording does not wait for what prepared the buffers
         with torch.cuda.stream(self._stream):
             self.step_fn()
             torch.cuda.synchronize()

@@ -55,7 +55,7 @@ def test_linear_bias_gate_and_accumulation(dtype, rows):
 def test_linears_with_inputs_of_their_own(dtype, rows):
     HK, T = _hk()
     rng = np.random.default_rng(rows)
-    for k, sizes in ((48, (30, 16, 100)), (1032, (1032, 700, 1032))):
+    for k, sizes in ((48, (30, 16, 100)), (1032, (1032, 700, 1032)), (1032, (1032, 1100, 1150))):
         print(f"group {dtype} rows {rows} k {k}", flush=True)
         calls, want, tail = [], [], torch.empty((rows, 5), device="cuda")
         for i, n in enumerate(sizes):
