@@ -470,6 +470,8 @@ def design_workload(args, design):
     rng = np.random.Generator(np.random.PCG64(1234))
     first, steps, max_len = 1024, args.steps, 2048
     results = []
+    if args.one_stream:
+        parallel.ParallelDecoder.branch_rows = 0
     models = [design] + (["zekilix"] if design != "zekilix" else []) + ["llama2_fp16"]
     if args.only:
         models = [m for m in models if m.startswith(args.only)]
@@ -578,6 +580,7 @@ def main():
     ap.add_argument("--only", choices=["zekilix", "ruperax", "llama2"], default=None, help="zekilix and ruperax workloads: one of the models")
     ap.add_argument("--decode-only", action="store_true", help="zekilix and ruperax workloads: no prompts")
     ap.add_argument("--rows-only", action="store_true", help="zekilix and ruperax workloads: prompts only")
+    ap.add_argument("--one-stream", action="store_true", help="ruperax workload: no feed-forward on a stream beside the mixer (for profiles)")
     ap.add_argument("--rows-per-pass", type=int, default=64,
                     help="prompt workload: rows (batch x positions) per pass, up to 2048")
     ap.add_argument("--fp8-cache", action="store_true",

@@ -277,8 +277,9 @@ def latent_layers(layers):
 
 def ruperax_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
     from .hybrid import HybridSpec
+    scale = (cfg.get("embedding") or {}).get("scale")
     return HybridSpec("ruperax", latent_layers(cfg["layers"]), cfg["width"], cfg["vocab"], 1, cfg["norm"]["eps"], 1.0,
-                      cfg["embedding"]["scale"], 0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype,
+                      1.0 if scale is None else scale, 0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype,
                       norm_groups=cfg["norm"].get("groups") or 1, positions=cfg["max_positions"])
 
 

@@ -88,7 +88,7 @@ def test_swiglu_with_biases(dtype, rows):
 
 # ---------------------------------------------------------------------------------------------- norm and shift
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("width,groups", [(36, 3), (75, 5), (75, 1), (130, 26), (1028, 2), (4096, 4)])
+@pytest.mark.parametrize("width,groups", [(36, 3), (75, 5), (75, 1), (130, 26), (1028, 2), (1024, 4), (2048, 1), (4096, 4), (5120, 2), (8448, 3)])
 def test_grouped_norm_and_token_shift(dtype, width, groups):
     """Sequences of unequal length in one pass; one of them goes on where an earlier pass left it, one is in a used slot."""
     HK, T = _hk()
@@ -96,11 +96,12 @@ def test_grouped_norm_and_token_shift(dtype, width, groups):
     tol = 5e-6 if dtype == "float32" else 6e-3
     w1, w2, mix = (rng.standard_normal(width) for _ in range(3))
     state = torch.full((8, width), 9.0, device="cuda")
-    seqs = {5: rng.standard_normal((400, width)), 0: rng.standard_normal((400, width)), 3: rng.standard_normal((400, width))}
+    many = 2100 if width <= 2048 else 300                        # (a workgroup walks through several rows)
+    seqs = {s: rng.standard_normal((many + 320, width)) for s in (5, 0, 3)}
     want = {s: R.group_rms_norm(x, w1, groups, 1e-5) for s, x in seqs.items()}
     shifted = {s: R.token_shift(h, mix) for s, h in want.items()}
     at = dict.fromkeys(seqs, 0)
-    for counts in ({5: 1, 0: 1, 3: 1}, {5: 7, 3: 300}, {0: 2, 5: 3}, {5: 1, 3: 1}, {3: 2}, {0: 9, 5: 4, 3: 5}):
+    for counts in ({5: 1, 0: 1, 3: 1}, {5: 7, 3: many}, {0: 2, 5: 3}, {5: 1, 3: 1}, {3: 2}, {0: 9, 5: 4, 3: 5}, {0: 300, 5: 299}):
         print(f"shift {dtype} width {width} counts {counts}", flush=True)
         rows = sum(counts.values())
         x = np.concatenate([seqs[s][at[s]:at[s] + c] for s, c in counts.items()])
@@ -114,7 +115,7 @@ def test_grouped_norm_and_token_shift(dtype, width, groups):
         h1, h2, hm = (torch.full((rows, ld), 7.0, dtype=T[dtype], device="cuda") for _ in range(3))
         single = all(c == 1 for c in counts.values())
         HK.shift_norm(_dev(x), rows, groups, 1e-5, _dev(w1), h1, _dev(w2), h2, _dev(mix), hm, state, _dev(slot, torch.int32),
-                      None if single else _dev(last, torch.int32), _dev(pos, torch.int32), 1000)
+                      None if single else _dev(last, torch.int32), _dev(pos, torch.int32), 4000)
         sel = [(s, slice(at[s], at[s] + c)) for s, c in counts.items()]
         assert _rel(_np(h1)[:, :width], np.concatenate([want[s][k] for s, k in sel])) < tol
         assert _rel(_np(h2)[:, :width], np.concatenate([R.group_rms_norm(seqs[s][k], w2, groups, 1e-5) for s, k in sel])) < tol
