@@ -107,7 +107,7 @@ class Reference:
         self.logits = forward(sd, cfg, ids)
         self.scale = np.sqrt((self.logits ** 2).mean())
         if dtype == "float32":
-            self.limit = 1e-4
+            self.limit = 2e-5
         else:
             # (three roundings: one sample of what rounding does says little about a single position)
             draws = [self.error(forward(sd, cfg, ids, rnd=lambda a, k=k: bf16(a * (1 + k)) / (1 + k))).max() for k in (0, 0.13, 0.31)]
