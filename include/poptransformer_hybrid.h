@@ -252,6 +252,144 @@ int pta_latent_gather(const pta_latent_args* host_args, pta_stream_t stream);
 int pta_latent_tiles_fit(int dtype, int D, int P, int E);
 int pta_latent_tiles(const pta_latent_args* host_args, pta_stream_t stream);
 
+/* ---- Attention over cached keys and values, by heads ---------------------------------------------------------------
+ * H query heads on G key/value heads.  Query and key: RMS norm per head (plain weights), rotation of the first `rot`
+ * features (pairs 2 i and 2 i + 1 turned by cos_sin[position][i]; any other pairing after a permutation of the weights'
+ * rows).  The values are a projection of their own, or the keys as projected (v points at k).
+ *   score(i, j) = scale * (q_i . k_j)   for j <= i with (i - j < window or j < keep) and floor(i / chunk) = floor(j / chunk)
+ * and a softmax, whose denominator also holds exp(sink) of the head where there are sinks.  With maps = 2 every head has two
+ * queries and keys [map 1 | map 2] over the same values, and its result is  o = a1 - lambda * a2,  o / sqrt(mean(o^2) + eps) *
+ * (1 - diff).  Then the gates: sigmoid per head, or per feature.
+ * Sizes as stored: D and E (query / key and value features) are multiples of 8, zero past `dim` and `vdim`.
+ * Cache of a layer: keys (normed, rotated) [slots][G][maps][ring_len][D], values [slots][G][ring_len][E].  The first `keep`
+ * positions have rows of their own; position p past them is row keep + (p - keep) % (ring_len - keep), and ring_len - keep >=
+ * min(window, chunk) - 1 + (most rows a sequence has in one pass). */
+typedef struct pta_head_attention_args {
+  int dtype;
+  int rows, H, G, maps, D, E;
+  int dim, vdim;          /* true sizes                                                                            */
+  const void* q;          /* [rows, ld], first query channel: [H][maps][D]                                         */
+  const void* k;          /* [G][maps][D]                                                                          */
+  const void* v;          /* [G][E]                                                                                */
+  int ld;                 /* a multiple of 8                                                                       */
+  const float* q_norm;    /* [D] or NULL: no norm                                                                  */
+  const float* k_norm;    /* [D] or NULL                                                                           */
+  float eps, scale;
+  const float* cos_sin;   /* [positions][rot / 2][2]                                                               */
+  int positions, rot;     /* rot: a multiple of 8, at most D; 0: no rotation                                       */
+  int window;             /* > 0; past any position: all                                                           */
+  int keep;               /* first positions that stay visible, 0: none                                            */
+  int chunk;              /* 0: none (with keep = 0 only)                                                          */
+  void* keys;
+  void* values;
+  int ring_len;
+  const int32_t* slot;    /* [rows]                                                                                */
+  const int32_t* pos;     /* [rows]                                                                                */
+  const float* sink;      /* [H] or NULL                                                                           */
+  float lambda, diff;     /* maps = 2                                                                              */
+  const float* head_gate; /* [rows, H] before the sigmoid, or NULL                                                 */
+  const void* gate;       /* [rows, ld], first channel of [H][E] before the sigmoid, or NULL                       */
+  const int32_t* tile_row;   /* [tiles] first row of a tile: rows of one sequence, at most PTA_HEAD_TILE            */
+  const int32_t* tile_count; /* [tiles]                                                                            */
+  int tiles;
+  int splits;             /* decode: parts the visible keys are cut into, 1 .. 64                                  */
+  void* workspace;        /* decode with splits > 1: pta_head_attention_workspace_bytes                            */
+  size_t workspace_bytes;
+  void* out;              /* [rows, H * E]                                                                         */
+} pta_head_attention_args;
+
+enum { PTA_HEAD_TILE = 128 };
+
+size_t pta_head_attention_workspace_bytes(int rows, int H, int maps, int E, int splits);
+/* every row's keys and values into the cache */
+int pta_head_append(const pta_head_attention_args* host_args, pta_stream_t stream);
+/* rows whose keys are in the cache already (pta_head_append): bf16 on the matrix unit over tiles of rows where D and E <= 256,
+ * else row by row */
+int pta_head_attention(const pta_head_attention_args* host_args, pta_stream_t stream);
+/* one row per sequence: norm, rotation, append and attention in one launch (two with splits > 1) */
+int pta_head_decode(const pta_head_attention_args* host_args, pta_stream_t stream);
+
+/* ---- Residual that takes normed results, and routing ---------------------------------------------------------------
+ * x fp32 [rows][width]:  x <- x + rms_norm(y) * weight  for a finished sublayer's result y, which is
+ *   y[r] * (y_weight ? y_weight[r * weights_ld] : 1)  +  sum_p part_weight[r * weights_ld + p] * parts[r][p],
+ * or with `table` x = table[id] * embed_scale; then h = x (what the next sublayer reads), or with final_weight the model's norm
+ * of x.  With `router` the row is routed as well, by what h holds of it (pta_route_args). */
+typedef struct pta_routing {
+  int experts, top;       /* 1 <= top <= experts <= PTA_MAX_EXPERTS                                                */
+  int shared;             /* 1: logit `experts` is a shared expert's: choice `top` of every row, weight = its sigmoid */
+  float scale;
+  int32_t* chosen;        /* [rows, top + shared]: largest softmax scores first (a shared expert is number `experts`) */
+  float* weights;         /* [rows, top + shared]: score * scale                                                   */
+} pta_routing;
+
+enum { PTA_MAX_EXPERTS = 1024 };
+
+typedef struct pta_result_norm_args {
+  int dtype;              /* type of h, of the embedding table, of the router                                      */
+  int rows, width;
+  float* x;
+  const void* table;      /* [vocab, width] or NULL                                                                */
+  int vocab;
+  float embed_scale;
+  const int32_t* ids;     /* id of row r: ids[r * ids_stride + (ids_index ? *ids_index : 0)]                       */
+  int ids_stride;
+  const int32_t* ids_index;
+  int32_t* pos_out;       /* with ids_index: pos_out[r] = *ids_index (may be NULL)                                 */
+  const float* y;         /* [rows, width] or NULL                                                                 */
+  const float* y_weight;
+  const void* parts;      /* [rows, parts_ld, width] or NULL, the first n_parts of a row                           */
+  int n_parts, parts_ld;
+  int part_f32;           /* fp32 parts, else of the type of h                                                     */
+  const float* part_weight;
+  int weights_ld;
+  const float* weight;    /* [width]                                                                               */
+  float eps;
+  const float* final_weight; /* [width] or NULL                                                                    */
+  void* h;                /* [rows, h_ld], columns past width zero                                                 */
+  int h_ld;
+  const void* router;     /* [experts + shared, h_ld] of the type of h, or NULL                                    */
+  pta_routing routing;
+} pta_result_norm_args;
+
+int pta_result_norm(const pta_result_norm_args* host_args, pta_stream_t stream);
+/* the same routing of rows whose logits fp32 [rows, experts + shared] are there already */
+int pta_route(const float* logits, int rows, const pta_routing* host_routing, pta_stream_t stream);
+
+/* ---- Mixture of experts -------------------------------------------------------------------------------------------
+ * Assignment a = r * choices + c is choice c of row r, done by expert chosen[a].  Two products per expert, with the epilogues
+ * of pta_wide_linear's pairs between them:
+ *   pta_experts with W2:    Y[a] = pair(W x_r, W2 x_r)       (X [rows, ld_x])
+ *   pta_experts without:    Y[a] = W x_a                     (X [rows * choices, ld_x])
+ * Weights of an expert are tiled as pta_bf16_tile leaves them (fp32: row-major), expert after expert, N a multiple of 16 (bf16).
+ * Two ways: directly, every expert finding its rows itself (bf16, up to 16 rows), where the last choice may be a shared expert of
+ * sizes of its own; or grouped by pta_group_experts, without it. */
+typedef struct pta_expert_weights {
+  const void* W;
+  const void* W2;
+  int K, N, n_main;       /* channels n_main .. N - 1 are padding and go nowhere; K a multiple of 8                */
+  int pair;
+  float limit, slope;
+} pta_expert_weights;
+
+typedef struct pta_experts_args {
+  int dtype;
+  int rows, experts, top, choices;   /* choices = top, or top + 1 with a shared expert                             */
+  const int32_t* chosen;  /* [rows, choices]                                                                       */
+  const void* X;
+  int ld_x;
+  pta_expert_weights routed, shared; /* shared.W NULL: no shared expert in this launch                             */
+  void* Y;                /* [rows * choices, ld_y]                                                                */
+  int ld_y, out_f32;
+  /* grouped: pta_group_experts; NULL: directly */
+  const int32_t* lists;
+  int tile_rows;          /* rows of a tile of the lists, 128 or 256                                               */
+} pta_experts_args;
+
+/* int32 elements of the lists: order of the assignments (choice < top) by expert, then tiles of rows of one expert */
+size_t pta_expert_lists_size(int rows, int top, int experts, int tile_rows);
+int pta_group_experts(const int32_t* chosen, int rows, int top, int choices, int experts, int tile_rows, int32_t* lists, pta_stream_t stream);
+int pta_experts(const pta_experts_args* host_args, pta_stream_t stream);
+
 /* ---- Matrix memory (mLSTM) ---------------------------------------------------------------------------------------
  * Per head, with log gates i = cap tanh(z_i / cap), f = log sigmoid(cap tanh(z_f / cap)) from the fp32 pre-activations:
  *   m' = max(f + m, i);  S = exp(f + m - m') S + exp(i - m') k v^T;  n likewise with k alone;

@@ -14,6 +14,8 @@ PAIR_NONE, PAIR_SWIGLU, PAIR_CLAMPED = 0, 1, 2
 WINDOW_TILE = 128
 MLSTM_SLICE = 32
 LATENT_TILE = 128
+HEAD_TILE = 128
+MAX_EXPERTS = 1024
 
 
 def _struct(name, fields):
@@ -50,6 +52,22 @@ MlstmArgs = _struct("MlstmArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("E", _I), ("q", _P), ("k", _P), ("v", _P), ("ld", _I), ("gates", _P),
     ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("longest", _I), ("chunked", _I),
     ("o", _P), ("workspace", _P), ("workspace_bytes", c_size_t)])
+HeadArgs = _struct("HeadArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("G", _I), ("maps", _I), ("D", _I), ("E", _I), ("dim", _I), ("vdim", _I), ("q", _P), ("k", _P),
+    ("v", _P), ("ld", _I), ("q_norm", _P), ("k_norm", _P), ("eps", _F), ("scale", _F), ("cos_sin", _P), ("positions", _I), ("rot", _I),
+    ("window", _I), ("keep", _I), ("chunk", _I), ("keys", _P), ("values", _P), ("ring_len", _I), ("slot", _P), ("pos", _P), ("sink", _P),
+    ("lambda_", _F), ("diff", _F), ("head_gate", _P), ("gate", _P), ("tile_row", _P), ("tile_count", _P), ("tiles", _I), ("splits", _I),
+    ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P)])
+Routing = _struct("Routing", [("experts", _I), ("top", _I), ("shared", _I), ("scale", _F), ("chosen", _P), ("weights", _P)])
+ResultNormArgs = _struct("ResultNormArgs", [
+    ("dtype", _I), ("rows", _I), ("width", _I), ("x", _P), ("table", _P), ("vocab", _I), ("embed_scale", _F), ("ids", _P),
+    ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("y", _P), ("y_weight", _P), ("parts", _P), ("n_parts", _I), ("parts_ld", _I), ("part_f32", _I),
+    ("part_weight", _P), ("weights_ld", _I), ("weight", _P), ("eps", _F), ("final_weight", _P), ("h", _P), ("h_ld", _I), ("router", _P),
+    ("routing", Routing)])
+ExpertWeights = _struct("ExpertWeights", [("W", _P), ("W2", _P), ("K", _I), ("N", _I), ("n_main", _I), ("pair", _I), ("limit", _F), ("slope", _F)])
+ExpertsArgs = _struct("ExpertsArgs", [
+    ("dtype", _I), ("rows", _I), ("experts", _I), ("top", _I), ("choices", _I), ("chosen", _P), ("X", _P), ("ld_x", _I),
+    ("routed", ExpertWeights), ("shared", ExpertWeights), ("Y", _P), ("ld_y", _I), ("out_f32", _I), ("lists", _P), ("tile_rows", _I)])
 
 SIGNATURES = {
     "pta_hybrid_last_error": (c_char_p, []),
@@ -66,6 +84,13 @@ SIGNATURES = {
     "pta_window_append": (_I, [POINTER(WindowArgs), _P]),
     "pta_window_attention": (_I, [POINTER(WindowArgs), _P]),
     "pta_window_decode": (_I, [POINTER(WindowArgs), _P]),
+    "pta_head_attention_workspace_bytes": (c_size_t, [_I, _I, _I, _I, _I]),
+    **{f"pta_head_{n}": (_I, [POINTER(HeadArgs), _P]) for n in ("append", "attention", "decode")},
+    "pta_result_norm": (_I, [POINTER(ResultNormArgs), _P]),
+    "pta_route": (_I, [_P, _I, POINTER(Routing), _P]),
+    "pta_expert_lists_size": (c_size_t, [_I, _I, _I, _I]),
+    "pta_group_experts": (_I, [_P, _I, _I, _I, _I, _I, _P, _P]),
+    "pta_experts": (_I, [POINTER(ExpertsArgs), _P]),
     "pta_mlstm_state_floats": (c_size_t, [_I, _I, _I]),
     "pta_mlstm_workspace_bytes": (c_size_t, [POINTER(MlstmArgs)]),
     "pta_mlstm": (_I, [POINTER(MlstmArgs), _P]),

@@ -1326,9 +1326,21 @@ constexpr int ROWS_CB = 8;                  // streams per workgroup: one per wa
 constexpr int ROWS_XSTRIDE = 128 + 8;
 constexpr int ROWS_AVEC = ROWS_CB * 4 * 64; // A operands (16 bytes each) of one feature tile: [stream][step][lane]
 
+// Which rows a workgroup takes: all of X and Y in order; or those of a tile from a list, each tile with weights of its own
+// (the same matrices, `weight_bytes` further per expert): entry a of `order` is read from row a / x_div of X and goes to row a of Y.
+struct AllRows { static constexpr bool kListed = false; };
+struct ListedRows {
+  static constexpr bool kListed = true;
+  const int32_t* n_tiles;
+  const int32_t* tiles;        // [..][4]: expert, first entry, entries
+  const int32_t* order;
+  size_t weight_bytes;
+  int x_div;
+};
+
 // (two waves per SIMD: the whole register file of 256 per lane is this kernel's to use)
-template <class Fmt, int RG, bool PAIR>
-__global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu(2, 2))) void gemm_rows_kernel(GemmArgs a, int groups, int row_blocks) {
+template <class Fmt, int RG, bool PAIR, class Rows = AllRows>
+__global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu(2, 2))) void gemm_rows_kernel(GemmArgs a, int groups, int row_blocks, Rows rows) {
   constexpr int KV = Fmt::kVec;
   constexpr int XROWS = RG * 16;
   static_assert(ROWS_CB == ROWS_WAVES, "wave w decodes stream w");
@@ -1336,14 +1348,28 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
   f16x8* abuf = reinterpret_cast<f16x8*>(smem);                                          // [2][ROWS_AVEC]
   f16* xbuf = reinterpret_cast<f16*>(smem + (size_t)2 * ROWS_AVEC * 16);                 // [waves][XROWS][ROWS_XSTRIDE]
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int K = a.K, M = a.M;
+  const int K = a.K;
   // Workgroups are dealt to the eight XCDs (each with an L2 of its own) in turn: workgroup id of the launch takes
   // tile (id % 8) * per + id / 8 of the list (row block, channel group), row block slowest - so an XCD works through
   // a contiguous stretch of the list, i.e. on one row block at a time, whose activations stay in its L2.
-  const int per = (int)gridDim.x / 8;
+  int per = (int)gridDim.x / 8;
+  if constexpr (Rows::kListed) {            // (the launch has room for the most tiles there can be)
+    row_blocks = *rows.n_tiles;
+    per = (groups * row_blocks + 7) / 8;
+    if ((int)blockIdx.x / 8 >= per) return;
+  }
   const int tile = ((int)blockIdx.x % 8) * per + (int)blockIdx.x / 8;
   if (tile >= groups * row_blocks) return;
   const int group = tile % groups, row_block = tile / groups;
+  int M = a.M;
+  const int32_t* order = nullptr;
+  size_t weight_at = 0;
+  if constexpr (Rows::kListed) {
+    const int32_t* t = rows.tiles + row_block * 4;
+    weight_at = (size_t)t[0] * rows.weight_bytes;
+    order = rows.order + t[1];
+    M = t[2];
+  }
   const int nsl = a.ksplit > 1 ? a.ksplit : 1;
   const int per_slice = (a.KT + nsl - 1) / nsl;
   const int kt_first = (int)blockIdx.y * per_slice;
@@ -1361,10 +1387,25 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
   auto stream_mat = [&](int st) -> const GemmMat& { return a.mat[PAIR ? (st < ROWS_CB / 2 ? 0 : 1) : mi]; };
   auto stream_blk = [&](int st) { return PAIR ? first_blk + st % (ROWS_CB / 2) : first_blk - a.mat[mi].nb_begin + st; };
   const GemmMat& own = stream_mat(wave);
-  const typename Fmt::Scale own_sc = Fmt::load_scale(own.scale, a.x_scale, stream_blk(wave) * 16 + (lane & 15), own.N);
-  const u32x4* own_w = reinterpret_cast<const u32x4*>(own.tiled) + (size_t)stream_blk(wave) * a.KT * (KV * 64) + lane;
+  int own_blk = stream_blk(wave);
+  if constexpr (Rows::kListed) own_blk = own_blk < own.N / 16 ? own_blk : own.N / 16 - 1;      // (channels past N go nowhere)
+  const typename Fmt::Scale own_sc = Fmt::load_scale(own.scale, a.x_scale, own_blk * 16 + (lane & 15), own.N);
+  const u32x4* own_w = reinterpret_cast<const u32x4*>(reinterpret_cast<const unsigned char*>(own.tiled) + weight_at) +
+                       (size_t)own_blk * a.KT * (KV * 64) + lane;
   const f16* X = a.mat[mi].X ? a.mat[mi].X : a.X;
-  const int row0 = (row_block * ROWS_WAVES + wave) * XROWS;      // first row of this wave
+  const int row0 = ((Rows::kListed ? 0 : row_block) * ROWS_WAVES + wave) * XROWS;      // first row of this wave
+  int listed[RG * 4];                                            // (the rows of X this lane fetches)
+  if constexpr (Rows::kListed) {
+#pragma unroll
+    for (int j = 0; j < RG * 4; ++j) {
+      const int row = row0 + j * 4 + (lane >> 4);
+      listed[j] = row < M ? order[row] / rows.x_div : -1;
+    }
+  }
+  auto result_row = [&](int m) {
+    if constexpr (Rows::kListed) return order[m];
+    else return m;
+  };
   f16* xw = xbuf + (size_t)wave * XROWS * ROWS_XSTRIDE;
 
   auto fetch_w = [&](int kt, u32x4 (&wv)[KV]) {
@@ -1379,8 +1420,9 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
   auto fetch_x = [&](int kt, u32x4 (&xr)[RG * 4]) {
 #pragma unroll
     for (int j = 0; j < RG * 4; ++j) {
-      const int row = row0 + j * 4 + (lane >> 4), k = kt * 128 + (lane & 15) * 8;
-      xr[j] = (row < M && k < K) ? *reinterpret_cast<const u32x4*>(X + (size_t)row * K + k) : u32x4{0, 0, 0, 0};
+      const int row = Rows::kListed ? listed[j] : row0 + j * 4 + (lane >> 4), k = kt * 128 + (lane & 15) * 8;
+      const bool there = Rows::kListed ? row >= 0 : row < M;
+      xr[j] = (there && k < K) ? *reinterpret_cast<const u32x4*>(X + (size_t)row * K + k) : u32x4{0, 0, 0, 0};
     }
   };
   // through the wave's own strip of LDS into fragment order (a wave's LDS accesses complete in order)
@@ -1459,7 +1501,7 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const int m = row0 + rg * 16 + (lane & 15);
       const f32x4 g4 = sums[(rg * ROWS_CB + st) * 64 + lane], u4 = sums[(rg * ROWS_CB + st + ROWS_CB / 2) * 64 + lane];
       if constexpr (Fmt::kWide) {
-        if (m < M) wide_put_pair4(mat, m, (first_blk + st) * 16 + (lane >> 4) * 4, g4, u4);
+        if (m < M) wide_put_pair4(mat, result_row(m), (first_blk + st) * 16 + (lane >> 4) * 4, g4, u4);
         continue;
       }
 #pragma unroll
@@ -1480,7 +1522,7 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
       const f32x4 v4 = sums[i * 64 + lane];
       if constexpr (Fmt::kWide) {
         if (nsl == 1) {
-          if (m < M) wide_put4(mat, m, stream_blk(st) * 16 + (lane >> 4) * 4, v4);
+          if (m < M) wide_put4(mat, result_row(m), stream_blk(st) * 16 + (lane >> 4) * 4, v4);
           continue;
         }
       }
@@ -1495,22 +1537,43 @@ __global__ __launch_bounds__(ROWS_WAVES * 64) __attribute__((amdgpu_waves_per_eu
   }
 }
 
-template <class Fmt, int RG, bool PAIR>
-static int launch_gemm_rows(const GemmArgs& a, int total_nb, hipStream_t s, const char* name) {
+template <class Fmt, int RG, bool PAIR, class Rows>
+static int reserve_gemm_rows(size_t* smem, const char* name) {
   static bool ready = false;
-  const size_t smem = (size_t)2 * ROWS_AVEC * 16 + (size_t)ROWS_WAVES * RG * 16 * ROWS_XSTRIDE * 2;
+  *smem = (size_t)2 * ROWS_AVEC * 16 + (size_t)ROWS_WAVES * RG * 16 * ROWS_XSTRIDE * 2;
   static_assert((size_t)2 * ROWS_AVEC * 16 + (size_t)ROWS_WAVES * RG * 16 * ROWS_XSTRIDE * 2 <= 160 * 1024, "LDS");
   if (!ready) {
-    PTA_REQUIRE(hipFuncSetAttribute((const void*)gemm_rows_kernel<Fmt, RG, PAIR>, hipFuncAttributeMaxDynamicSharedMemorySize,
-                                    (int)smem) == hipSuccess,
-                "%s: cannot reserve %zu bytes of LDS", name, smem);
+    PTA_REQUIRE(hipFuncSetAttribute((const void*)gemm_rows_kernel<Fmt, RG, PAIR, Rows>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                    (int)*smem) == hipSuccess,
+                "%s: cannot reserve %zu bytes of LDS", name, *smem);
     ready = true;
   }
+  return PTA_OK;
+}
+
+// Tiles of listed rows (at most RG * 128 each, up to max_tiles of them) of a matrix, or of a gate / up pair; wide formats.
+template <class Fmt, int RG, bool PAIR>
+static int launch_gemm_listed(const GemmArgs& a, int total_nb, int max_tiles, const ListedRows& rows, hipStream_t s, const char* name) {
+  size_t smem;
+  const int rc = reserve_gemm_rows<Fmt, RG, PAIR, ListedRows>(&smem, name);
+  if (rc) return rc;
+  constexpr int per_wg = PAIR ? ROWS_CB / 2 : ROWS_CB;
+  const int groups = (total_nb + per_wg - 1) / per_wg;
+  hipLaunchKernelGGL((gemm_rows_kernel<Fmt, RG, PAIR, ListedRows>), dim3((groups * max_tiles + 7) / 8 * 8), dim3(ROWS_WAVES * 64), smem, s, a,
+                     groups, max_tiles, rows);
+  return PTA_OK;
+}
+
+template <class Fmt, int RG, bool PAIR>
+static int launch_gemm_rows(const GemmArgs& a, int total_nb, hipStream_t s, const char* name) {
+  size_t smem;
+  const int rc = reserve_gemm_rows<Fmt, RG, PAIR, AllRows>(&smem, name);
+  if (rc) return rc;
   const int groups = total_nb / (PAIR ? ROWS_CB / 2 : ROWS_CB);
   const int row_blocks = (a.M + ROWS_WAVES * RG * 16 - 1) / (ROWS_WAVES * RG * 16);
   const int nsl = a.ksplit > 1 ? a.ksplit : 1;
   const int per = (groups * row_blocks + 7) / 8;
-  hipLaunchKernelGGL((gemm_rows_kernel<Fmt, RG, PAIR>), dim3(per * 8, nsl), dim3(ROWS_WAVES * 64), smem, s, a, groups, row_blocks);
+  hipLaunchKernelGGL((gemm_rows_kernel<Fmt, RG, PAIR>), dim3(per * 8, nsl), dim3(ROWS_WAVES * 64), smem, s, a, groups, row_blocks, AllRows{});
   if (nsl > 1) {
     const size_t total = (size_t)a.M * a.mat[0].N;
     hipLaunchKernelGGL((splitk_finish_kernel<Fmt>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0, s, a);

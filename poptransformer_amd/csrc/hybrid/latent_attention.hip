@@ -2,34 +2,13 @@
 //
 // Absorbed form: W_uk^T q meets the cached rows, so all heads of a row share every key that is read; the 16 columns of a
 // matrix instruction are 16 heads.  Over heads: prompts, with keys and values of every head in buffers of their own.
-#include "hybrid.h"
-#include <type_traits>
+#include "attention.h"
 
 typedef pta_latent_args LA;
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ f32x4 mma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-
-// Transposed read of a row-major LDS tile: of the 16 lanes of a group, lane i gives the address of four elements of row i / 4
-// (columns 4 (i % 4) ..) and gets column i of the four rows.
-__device__ __forceinline__ bf16x4 read_transposed(const bf16* p) {
-  return bitcast<bf16x4>(__builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)p));
-}
-__device__ __forceinline__ bf16x8 join(bf16x4 lo, bf16x4 hi) { return __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7); }
 
 __device__ __forceinline__ int position_of(const LA& a, int r) {
   const int p = a.pos[r];
   return p < 0 ? 0 : (p >= a.positions ? a.positions - 1 : p);
-}
-
-// eight features from f on (f a multiple of eight) of a rotated part, turned by the row's angles
-__device__ __forceinline__ void rotate8(const float* cs, float (&v)[8]) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const float c = cs[2 * i], s = cs[2 * i + 1], x = v[2 * i], y = v[2 * i + 1];
-    v[2 * i] = x * c - y * s;
-    v[2 * i + 1] = y * c + x * s;
-  }
 }
 
 // ------------------------------------------------------------------------------------------

@@ -1,0 +1,263 @@
+// A residual that takes normed results: x <- x + rms_norm(y) * weight, with what follows in the same launch: the rounded row that
+// the next sublayer reads, or the model's norm of it, and the routing of the row to its experts.
+#include "hybrid.h"
+#include <type_traits>
+
+typedef pta_result_norm_args RN;
+
+// Routing of one row by THREADS threads: z holds the logits (in LDS, visible to all; overwritten).  Expert e's place among the
+// chosen is the number of larger scores (of equal ones the first comes first), so no choice waits for another.
+template <int THREADS>
+__device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r) {
+  const int E = g.experts, choices = g.top + g.shared;
+  int32_t* chosen = g.chosen + (size_t)r * choices;
+  float* weights = g.weights + (size_t)r * choices;
+  constexpr int PER = (PTA_MAX_EXPERTS + THREADS - 1) / THREADS;
+  int rank[PER];
+  float p[PER];
+#pragma unroll
+  for (int k = 0; k < PER; ++k) {
+    const int e = threadIdx.x + k * THREADS;
+    rank[k] = E;
+    p[k] = 0.f;
+    if (e >= E) continue;
+    const float mine = z[e];
+    float top = mine;
+    int above = 0;
+    for (int j = 0; j < E; ++j) {
+      const float v = z[j];
+      top = fmaxf(top, v);
+      above += v > mine || (v == mine && j < e);
+    }
+    rank[k] = above;
+    p[k] = expf(mine - top);
+  }
+  const float shared = g.shared && threadIdx.x == 0 ? sigmoid_f32(z[E]) : 0.f;
+  __syncthreads();
+#pragma unroll
+  for (int k = 0; k < PER; ++k)
+    if (threadIdx.x + k * THREADS < E) z[threadIdx.x + k * THREADS] = p[k];
+  __syncthreads();
+  bool any = false;
+#pragma unroll
+  for (int k = 0; k < PER; ++k) any = any || rank[k] < g.top;
+  if (any) {
+    float sum = 0.f;
+    for (int j = 0; j < E; ++j) sum += z[j];
+#pragma unroll
+    for (int k = 0; k < PER; ++k)
+      if (rank[k] < g.top) {
+        chosen[rank[k]] = threadIdx.x + k * THREADS;
+        weights[rank[k]] = p[k] / sum * g.scale;
+      }
+  }
+  if (g.shared && threadIdx.x == 0) {
+    chosen[g.top] = E;
+    weights[g.top] = shared;
+  }
+}
+
+__global__ __launch_bounds__(64) void route_kernel(const float* logits, pta_routing g) {
+  __shared__ float z[PTA_MAX_EXPERTS + 1];
+  const int n = g.experts + g.shared;
+  for (int c = threadIdx.x; c < n; c += 64) z[c] = logits[(size_t)blockIdx.x * n + c];
+  __syncthreads();
+  route_row<64>(g, z, blockIdx.x);
+}
+
+__device__ __forceinline__ float rounded(float v, bf16) { return (float)(bf16)v; }
+__device__ __forceinline__ float rounded(float v, float) { return v; }
+
+// One workgroup per row; a thread owns the columns c, c + 4 * THREADS, ... (four at a time) from the result to h.
+template <typename T, int THREADS>
+__global__ __launch_bounds__(THREADS) void result_norm_kernel(RN a) {
+  constexpr int WAVES = THREADS / 64;
+  extern __shared__ __align__(16) float u_row[];             // the result, then what h holds
+  __shared__ float red[2][WAVES];
+  __shared__ float z[PTA_MAX_EXPERTS + 1];
+  __shared__ float pw[64];
+  const int r = blockIdx.x, d = a.width;
+  float* x = a.x + (size_t)r * d;
+  T* h = reinterpret_cast<T*>(a.h) + (size_t)r * a.h_ld;
+  const bool vec = (d & 3) == 0;
+  const int step = vec ? THREADS * 4 : THREADS, span = vec ? 4 : 1;
+  const T* row = nullptr;
+  if (a.table) {
+    int col = a.ids_index ? *a.ids_index : 0;
+    col = col < 0 ? 0 : (col >= a.ids_stride ? a.ids_stride - 1 : col);
+    int id = a.ids[(size_t)r * a.ids_stride + col];
+    id = id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id);
+    row = reinterpret_cast<const T*>(a.table) + (size_t)id * d;
+    if (a.pos_out && threadIdx.x == 0) a.pos_out[r] = a.ids_index ? *a.ids_index : 0;
+  }
+  float inv = 0.f;
+  if (!row) {
+    const float* y = a.y ? a.y + (size_t)r * d : nullptr;
+    const float yw = a.y && a.y_weight ? a.y_weight[(size_t)r * a.weights_ld] : 1.0f;
+    if (a.parts) {
+      if ((int)threadIdx.x < a.n_parts) pw[threadIdx.x] = a.part_weight[(size_t)r * a.weights_ld + threadIdx.x];
+      __syncthreads();
+    }
+    float sq = 0.f;
+    auto column = [&](auto width_tag, int c) {
+      constexpr int V = decltype(width_tag)::value;
+      float u[V] = {};
+      if (y) {
+        if constexpr (V == 4) {
+          const f32x4 t = *reinterpret_cast<const f32x4*>(y + c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) u[e] = t[e] * yw;
+        } else {
+          u[0] = y[c] * yw;
+        }
+      }
+      if (a.parts) {
+        const size_t at = (size_t)r * a.parts_ld * d + c;
+#pragma unroll 4
+        for (int p = 0; p < a.n_parts; ++p) {
+          float t[V];
+          if (a.part_f32) {
+            const float* s = reinterpret_cast<const float*>(a.parts) + at + (size_t)p * d;
+            if constexpr (V == 4) {
+              const f32x4 q = *reinterpret_cast<const f32x4*>(s);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) t[e] = q[e];
+            } else t[0] = s[0];
+          } else {
+            const T* s = reinterpret_cast<const T*>(a.parts) + at + (size_t)p * d;
+            if constexpr (V == 4 && sizeof(T) == 2) {
+              const bf16x4 q = *reinterpret_cast<const bf16x4*>(s);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) t[e] = (float)q[e];
+            } else {
+#pragma unroll
+              for (int e = 0; e < V; ++e) t[e] = (float)s[e];
+            }
+          }
+#pragma unroll
+          for (int e = 0; e < V; ++e) u[e] = __builtin_fmaf(pw[p], t[e], u[e]);
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        u_row[c + e] = u[e];
+        sq = __builtin_fmaf(u[e], u[e], sq);
+      }
+    };
+    if (vec) for (int c = threadIdx.x * 4; c < d; c += step) column(std::integral_constant<int, 4>{}, c);
+    else for (int c = threadIdx.x; c < d; c += step) column(std::integral_constant<int, 1>{}, c);
+    inv = 1.0f / sqrtf(workgroup_sum<WAVES>(sq, red[0]) / (float)d + a.eps);
+  }
+  float sq = 0.f;
+  auto update = [&](auto width_tag, int c) {
+    constexpr int V = decltype(width_tag)::value;
+    float v[V];
+    if (row) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = (float)row[c + e] * a.embed_scale;
+    } else if constexpr (V == 4) {
+      const f32x4 t = *reinterpret_cast<const f32x4*>(x + c), w = *reinterpret_cast<const f32x4*>(a.weight + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = t[e] + u_row[c + e] * inv * w[e];
+    } else {
+      v[0] = x[c] + u_row[c] * inv * a.weight[c];
+    }
+    if constexpr (V == 4) *reinterpret_cast<f32x4*>(x + c) = f32x4{v[0], v[1], v[2], v[3]};
+    else x[c] = v[0];
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      u_row[c + e] = a.final_weight ? v[e] : rounded(v[e], T{});
+      sq = __builtin_fmaf(v[e], v[e], sq);
+    }
+    if (!a.final_weight) {
+      if constexpr (V == 4 && sizeof(T) == 2) {
+        if ((a.h_ld & 3) == 0) {
+          bf16x4 o;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[e] = (bf16)v[e];
+          *reinterpret_cast<bf16x4*>(h + c) = o;
+          return;
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) h[c + e] = (T)v[e];
+    }
+  };
+  if (vec) for (int c = threadIdx.x * 4; c < d; c += step) update(std::integral_constant<int, 4>{}, c);
+  else for (int c = threadIdx.x; c < d; c += step) update(std::integral_constant<int, 1>{}, c);
+  if (a.final_weight) {
+    const float f = 1.0f / sqrtf(workgroup_sum<WAVES>(sq, red[1]) / (float)d + a.eps);
+    for (int c = threadIdx.x * span; c < d; c += step)
+      for (int e = 0; e < span; ++e) h[c + e] = (T)(u_row[c + e] * f * a.final_weight[c + e]);
+  }
+  for (int c = d + threadIdx.x; c < a.h_ld; c += THREADS) h[c] = (T)0.0f;
+  if (!a.router) return;
+  // one wave per expert at a time
+  for (int c = d + threadIdx.x; c < a.h_ld; c += THREADS) u_row[c] = 0.f;
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = a.routing.experts + a.routing.shared;
+  for (int e = wave; e < n; e += WAVES) {
+    const T* w = reinterpret_cast<const T*>(a.router) + (size_t)e * a.h_ld;
+    float s = 0.f;
+#pragma unroll 4
+    for (int c = lane * 8; c < a.h_ld; c += 512) {
+      float t[8];
+      load8(w + c, true, 8, t);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) s = __builtin_fmaf(t[k], u_row[c + k], s);
+    }
+    s = wave_total_dpp(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  route_row<THREADS>(a.routing, z, r);
+}
+
+static int check_routing(const pta_routing& g, const char* name) {
+  PTA_REQUIRE(g.experts >= 1 && g.experts <= PTA_MAX_EXPERTS && g.top >= 1 && g.top <= g.experts && (g.shared == 0 || g.shared == 1),
+              "%s: top %d of %d experts (at most %d)", name, g.top, g.experts, PTA_MAX_EXPERTS);
+  PTA_REQUIRE(g.chosen && g.weights, "%s: the routing has nowhere to go", name);
+  return PTA_OK;
+}
+
+extern "C" int pta_route(const float* logits, int rows, const pta_routing* routing, pta_stream_t stream) {
+  PTA_REQUIRE(logits && routing && rows > 0, "pta_route: null pointer, or %d rows", rows);
+  const int rc = check_routing(*routing, "pta_route");
+  if (rc) return rc;
+  hipLaunchKernelGGL(route_kernel, dim3(rows), dim3(64), 0, (hipStream_t)stream, logits, *routing);
+  PTA_CHECK_LAUNCH("pta_route");
+  return PTA_OK;
+}
+
+extern "C" int pta_result_norm(const RN* args, pta_stream_t stream) {
+  const char* name = "pta_result_norm";
+  PTA_REQUIRE(args, "%s: null arguments", name);
+  const RN& a = *args;
+  PTA_REQUIRE(a.dtype == PTA_BF16 || a.dtype == PTA_FP32, "%s: unknown type %d", name, a.dtype);
+  PTA_REQUIRE(a.rows > 0 && a.width > 0 && a.width <= 14000, "%s: rows %d, width %d (1 .. 14000)", name, a.rows, a.width);
+  PTA_REQUIRE(a.x && a.h && a.h_ld >= a.width && a.h_ld <= a.width + 7 && pta_aligned(a.x, 16) && pta_aligned(a.h, 16),
+              "%s: x or h null or unaligned, h rows of %d", name, a.h_ld);
+  PTA_REQUIRE(a.table ? (a.ids && a.vocab > 0 && a.ids_stride > 0 && !a.y && !a.parts) : ((a.y || a.parts) && a.weight),
+              "%s: either an embedding with ids, or a result with its norm's weight", name);
+  PTA_REQUIRE(pta_aligned(a.y, 16) && pta_aligned(a.parts, 16) && pta_aligned(a.weight, 16), "%s: unaligned result or weight", name);
+  PTA_REQUIRE(!a.parts || (a.n_parts >= 1 && a.n_parts <= 64 && a.parts_ld >= a.n_parts && a.part_weight && a.weights_ld >= a.n_parts), "%s: %d parts (1 .. 64)", name, a.n_parts);
+  PTA_REQUIRE(!a.y_weight || a.weights_ld >= 1, "%s: the weights' stride", name);
+  if (a.router) {
+    const int rc = check_routing(a.routing, name);
+    if (rc) return rc;
+    PTA_REQUIRE(!a.final_weight && a.h_ld % 8 == 0 && pta_aligned(a.router, 16), "%s: a router reads h, in whole pieces of eight", name);
+  }
+  hipStream_t s = (hipStream_t)stream;
+  const size_t smem = (size_t)a.h_ld * sizeof(float);
+  // few rows: a whole row of 1024 threads shortens the chain of a row; many rows: the machine is full either way
+  const bool few = a.rows <= 64 && a.width >= 2048;
+  auto launch = [&](auto threads) {
+    constexpr int N = decltype(threads)::value;
+    if (a.dtype == PTA_BF16) hipLaunchKernelGGL((result_norm_kernel<bf16, N>), dim3(a.rows), dim3(N), smem, s, a);
+    else hipLaunchKernelGGL((result_norm_kernel<float, N>), dim3(a.rows), dim3(N), smem, s, a);
+  };
+  if (few) launch(std::integral_constant<int, 1024>{});
+  else launch(std::integral_constant<int, 256>{});
+  PTA_CHECK_LAUNCH(name);
+  return PTA_OK;
+}

@@ -4,31 +4,11 @@
 // The cache keeps one raw key row per token and key head, which is read once for both products, and the inverse root
 // mean square of the token's keys; the key norm's weight, the query norm and the score scale are folded into the query:
 //   score(i, j) = rinv_j * (q'_i . k_j) - slope * (i - j),   q' = q * rinv_q * w_q * w_k * scale.
-#include "hybrid.h"
-#include <type_traits>
+#include "attention.h"
 
 typedef pta_window_attention_args WA;
 
 static __host__ __device__ inline int padded8(int d) { return (d + 7) & ~7; }
-
-template <typename T> __device__ __forceinline__ float exp_of(float x);
-template <> __device__ __forceinline__ float exp_of<float>(float x) { return expf(x); }
-template <> __device__ __forceinline__ float exp_of<bf16>(float x) { return __expf(x); }
-
-// Sum over each group of L consecutive lanes, in every lane of the group (all lanes active).
-template <int L>
-__device__ __forceinline__ float group_sum(float v) {
-  auto dpp = [](float x, auto ctrl) {
-    return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), decltype(ctrl)::value, 0xF, 0xF, true));
-  };
-  if (L >= 2) v += dpp(v, std::integral_constant<int, 0xB1>{});       // quad_perm [1, 0, 3, 2]
-  if (L >= 4) v += dpp(v, std::integral_constant<int, 0x4E>{});       // quad_perm [2, 3, 0, 1]
-  if (L >= 8) v += dpp(v, std::integral_constant<int, 0x141>{});      // row_half_mirror
-  if (L >= 16) v += dpp(v, std::integral_constant<int, 0x140>{});     // row_mirror
-  if (L >= 32) v += __shfl_xor(v, 16, 64);
-  if (L >= 64) v += __shfl_xor(v, 32, 64);
-  return v;
-}
 
 // this thread's share of the sum of squares of n consecutive elements (256 threads)
 template <typename T>
@@ -72,34 +52,6 @@ __global__ __launch_bounds__(256) void window_append_kernel(WA a, bool vec) {
 // FUSED: the row's own key comes from the projection and is put into the ring by this launch.
 // ------------------------------------------------------------------------------------------
 constexpr int WR_KEYS = 4;               // keys a lane group takes per step
-
-// eight elements on their way from memory
-template <typename T> struct Raw8;
-template <> struct Raw8<bf16> {
-  u32x4 w;
-  __device__ __forceinline__ void load(const bf16* p, bool vec, int valid) {
-    if (vec) {
-      w = *reinterpret_cast<const u32x4*>(p);
-    } else {
-      bf16x8 z;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) z[e] = e < valid ? p[e] : (bf16)0.0f;
-      w = bitcast<u32x4>(z);
-    }
-  }
-  __device__ __forceinline__ void unpack(float (&v)[8]) const {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) { v[2 * e] = bitcast<float>(w[e] << 16); v[2 * e + 1] = bitcast<float>(w[e] & 0xffff0000u); }
-  }
-};
-template <> struct Raw8<float> {
-  float w[8];
-  __device__ __forceinline__ void load(const float* p, bool vec, int valid) { load8(p, vec, valid, w); }
-  __device__ __forceinline__ void unpack(float (&v)[8]) const {
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = w[e];
-  }
-};
 
 template <typename T, int RG, int LPK>
 __global__ __launch_bounds__(256) void window_rows_kernel(WA a, bool vec, int fused, int groups, float* part_o, float* part_ml) {

@@ -1,5 +1,6 @@
 """Executor of decoders that mix windowed attention with recurrent (matrix memory) layers over fp32 residual streams; the
-mixers, feed-forwards and the row handling that `parallel` uses for layers whose sublayers stand side by side.
+mixers, feed-forwards and the row handling that `parallel` uses for layers whose sublayers stand side by side, and
+`result_norm` for layers whose residual takes the norms of their sublayers' results.
 
 The model is a list of layers, each described by its mixer, its feed-forward (or none) and the layer whose tensors it
 uses.  One forward function serves everything: it takes the ROWS of a pass (row = one token of the sequence in a slot, at
@@ -11,6 +12,7 @@ Per layer with a feed-forward the launches of a decode iteration are: projection
 window merged by a second launch; or recurrence and head norm), output projection, stream update + norm, gate / up pair,
 down projection, stream update + norm.
 """
+import math
 from dataclasses import dataclass
 from typing import List, Optional
 
@@ -115,6 +117,96 @@ class LatentMixer:
 
 
 @dataclass
+class Rotation:
+    """Rotary positions on the first `dims` features of a head, in pairs (i, i + dims / 2) or (`neighbours`) (2 i, 2 i + 1).  The
+    frequencies base^(-2 i / dims) are divided by `factor`; with yarn = (original, fast, slow) only those that make fewer than
+    `slow` turns in `original` positions, those of more than `fast` turns not at all, with a ramp in between."""
+    base: float
+    dims: int
+    neighbours: bool = False
+    factor: float = 1.0
+    yarn: Optional[tuple] = None
+
+    def frequencies(self):
+        """(frequencies, factor of cos and sin)"""
+        i = np.arange(self.dims // 2)
+        f = float(self.base) ** (-2.0 * i / self.dims)
+        if self.yarn is None:
+            return f / self.factor, 1.0
+        original, fast, slow = self.yarn
+
+        def feature(turns):
+            return self.dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(self.base))
+        low, high = max(math.floor(feature(fast)), 0), min(math.ceil(feature(slow)), self.dims - 1)
+        slowed = np.clip((i - low) / max(high - low, 0.001), 0.0, 1.0)
+        return f * (slowed / self.factor + (1.0 - slowed)), 0.1 * math.log(self.factor) + 1.0
+
+    def pairs(self, size):
+        """Order of `size` features in which the two of a pair follow each other."""
+        turned = np.arange(self.dims)
+        if not self.neighbours:
+            turned = turned.reshape(2, -1).T.reshape(-1)
+        return np.concatenate([turned, np.arange(self.dims, size)])
+
+    def angles(self, positions):
+        """fp32 [positions, pairs, (cos, sin)] of those pairs; whole pieces of eight features, the ones past `dims` stay as they are."""
+        f, amplitude = self.frequencies()
+        a = np.arange(positions)[:, None] * f
+        out = np.zeros((positions, HK.pad8(self.dims) // 2, 2), np.float32)
+        out[..., 0] = 1.0
+        out[:, :len(f), 0], out[:, :len(f), 1] = np.cos(a) * amplitude, np.sin(a) * amplitude
+        return out
+
+
+@dataclass
+class HeadMixer:
+    """Attention over cached keys and values of kv_heads heads: norms of queries and keys per head, rotation, and what is set of
+    the rest.  Visible are the newest `window` positions (None: all) with the first `keep`, or those of the same `chunk`."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot: Optional[Rotation] = None
+    window: Optional[int] = None
+    keep: int = 0
+    chunk: Optional[int] = None
+    keys_are_values: bool = False    # the values are the keys as projected
+    biases: str = ""                 # which of "qkv" have biases
+    sink: bool = False               # a learned score per head in the softmax's denominator
+    gate: Optional[str] = None       # sigmoid gate of the result, one number per "head" or per "feature"
+    diff: Optional[float] = None     # two maps per head, the second subtracted; part of their weight, and 1 - diff of the result
+    kind = "heads"
+
+    @property
+    def maps(self):
+        return 1 if self.diff is None else 2
+
+    @property
+    def stored_dim(self):
+        return HK.pad8(self.dim)
+
+    @property
+    def stored_vdim(self):
+        return HK.pad8(self.vdim)
+
+    @property
+    def span(self):
+        """Most positions, besides the kept ones, that one sees."""
+        return min(self.window or 1 << 30, self.chunk or 1 << 30)
+
+    @property
+    def out_channels(self):
+        return self.heads * self.stored_vdim
+
+
+@dataclass
+class SwiGLU:
+    """silu(g) u between the gate / up pair and the down projection."""
+    ff: int
+
+
+@dataclass
 class BiasedSwiGLU:
     """silu(g) u between the gate / up pair and the down projection, all three with biases."""
     ff: int
@@ -126,6 +218,17 @@ class ClampedGLU:
     ff: int
     limit: float
     slope: float = 1.702
+
+
+@dataclass
+class Experts:
+    """Mixture of experts: of `count` feed-forwards every token has the `top` with the largest router softmax scores, weighted by
+    score * scale; `shared` runs for every token, weighted by a sigmoid of its own."""
+    count: int
+    top: int
+    scale: float
+    expert: ClampedGLU
+    shared: Optional[ClampedGLU] = None
 
 
 @dataclass

@@ -333,3 +333,126 @@ def parallel_weights(tensors, spec, device="cuda"):
         layers.append(ParallelLayerWeights(**lw))
     return ParallelWeights(get("embed", (spec.vocab, d)).to(dtype).contiguous(), get("pos", (spec.positions, d)).to(dtype).contiguous(),
                            layers, vec("final.norm", d), HK.WideWeight(get("head", (spec.vocab, d)), dtype))
+
+
+# ----------------------------------------------------------------------------------- residual that takes normed results
+def _rotation(rot, neighbours, yarn, where):
+    from .hybrid import Rotation
+    if rot is None:
+        return None
+    if rot["dims"] % 2 or rot["dims"] < 2:
+        raise ValueError(f"{where}: {rot['dims']} rotated features")
+    s = rot.get("scaling")
+    if s is None:
+        return Rotation(float(rot["base"]), rot["dims"], neighbours)
+    return Rotation(float(rot["base"]), rot["dims"], neighbours, float(s["factor"]),
+                    (float(s["original"]), float(s["fast"]), float(s["slow"])) if yarn else None)
+
+
+def head_layers(layers):
+    """The `layers` list of a configuration with attention by heads and feed-forwards that may be mixtures of experts ->
+    [HybridLayer].  Types: `attention` (sliding window with kept first positions, sinks, values that are the keys), `attention_2`
+    (differential, within chunks, no rotation), `attention_3` (within chunks)."""
+    from .hybrid import ClampedGLU, Experts, HeadMixer, HybridLayer, SwiGLU
+    out = []
+    for i, c in enumerate(layers):
+        m, kind = c["mixer"], c["type"]
+        mask, where = m.get("mask") or {}, f"layer {i}"
+        mixer = HeadMixer(m["heads"], m["kv_heads"], m["dim"], m["vdim"], float(m["scale"]))
+        if kind == "attention":
+            mixer.window, mixer.keep = mask.get("size"), mask.get("keep_first") or 0
+            mixer.rot = _rotation(m.get("rot"), False, False, where)
+            mixer.keys_are_values, mixer.biases, mixer.sink, mixer.gate = True, "qk", True, "head"
+            if mixer.vdim != mixer.dim:
+                raise ValueError(f"{where}: the values are the keys, so vdim ({mixer.vdim}) must equal dim ({mixer.dim})")
+        elif kind == "attention_2":
+            mixer.chunk, mixer.diff = mask.get("size"), float(m["diff"])
+        elif kind == "attention_3":
+            mixer.chunk, mixer.biases, mixer.gate = mask.get("size"), "qkv", "feature"
+            mixer.rot = _rotation(m.get("rot"), True, True, where)
+        else:
+            raise NotImplementedError(f"{where}: mixer {kind}")
+        if mixer.heads % mixer.kv_heads or (mixer.rot is not None and mixer.rot.dims > mixer.dim):
+            raise ValueError(f"{where}: {mixer.heads} heads on {mixer.kv_heads}, rotation {m.get('rot')} of {mixer.dim} features")
+        f, mlp = c.get("mlp"), None
+        if f is not None and f.get("kind", "dense") == "dense":
+            mlp = SwiGLU(f["ff"])
+        elif f is not None and f["kind"] == "moe":
+            r, s = f["router"], f.get("shared")
+            mlp = Experts(r["experts"], r["top"], float(r["scale"]), ClampedGLU(f["expert"]["ff"], float(f["expert"]["limit"])),
+                          ClampedGLU(s["ff"], float(s["limit"])) if s is not None else None)
+        elif f is not None:
+            raise NotImplementedError(f"{where}: feed-forward {f['kind']}")
+        out.append(HybridLayer(mixer, mlp, i))
+    return out
+
+
+def golapel_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
+    from .hybrid import HybridSpec
+    return HybridSpec("golapel", head_layers(cfg["layers"]), cfg["width"], cfg["vocab"], 1, cfg["norm"]["eps"], 1.0, cfg["embedding"]["scale"],
+                      0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype)
+
+
+def result_norm_weights(tensors, spec, device="cuda"):
+    """As hybrid_weights, for layers with attention by heads.  Head sizes are rounded up to whole pieces of eight features with
+    zeros; the two features of a rotated pair come to stand side by side in queries and keys (and so in values that are keys)."""
+    from .. import hybrid_kernels as HK
+    from .hybrid import Experts
+    from .result_norm import FeedForwardWeights, ResultNormLayerWeights, ResultNormWeights
+    dtype = HK.DTYPES[spec.dtype]
+    get, vec = _lookup(tensors, device)
+    d = spec.width
+
+    def feed_forward(make, names, ff):
+        """make(tensors of the experts, further keywords) -> weight; names: prefixes of the experts' tensors"""
+        n = HK.pad8(ff)
+        gate, up = (make([get(p + part, (ff, d)) for p in names], dtype, main_to=n) for part in ("gate", "up"))
+        return FeedForwardWeights(gate, up, make([get(p + "down", (d, ff)) for p in names], dtype))
+
+    layers = []
+    for i, lay in enumerate(spec.layers):
+        p, m, mlp = f"l{i}.", lay.mixer, lay.mlp
+        mix = p + "mix."
+        H, G, M, D, E = m.heads, m.kv_heads, m.maps, m.stored_dim, m.stored_vdim
+        pairs = torch.from_numpy(m.rot.pairs(m.dim) if m.rot is not None else np.arange(m.dim)).to(device)
+        order = pairs if m.keys_are_values else torch.arange(m.vdim, device=device)
+
+        def rows(t, heads, size, which, stored):
+            """[heads * size, ...] in the order `which` of every head's features, each head padded to `stored`"""
+            t = t.view(heads, size, -1)[:, which]
+            return _padded(t, heads, stored, t.shape[2]).reshape(heads * stored, -1)
+        parts = [("q", H * M, m.dim, pairs, D), ("k", G * M, m.dim, pairs, D)]
+        if not m.keys_are_values:
+            parts.append(("v", G, m.vdim, order, E))
+        if m.gate == "feature":
+            parts.append(("g", H, m.vdim, order, E))
+        weights = [rows(get(mix + n, (heads * size, d)), heads, size, which, stored) for n, heads, size, which, stored in parts]
+        if m.gate == "head":
+            weights.append(get(mix + "g", (H, d)))
+        bias = None
+        if m.biases:
+            bias = torch.cat([rows(vec(mix + n + ".b", heads * size) if n in m.biases else torch.zeros(heads * size, device=device),
+                                   heads, size, which, stored).reshape(-1) for n, heads, size, which, stored in parts]).contiguous()
+        o = get(mix + "o", (d, H * m.vdim)).view(d, H, m.vdim)[:, :, order]
+        lw = dict(norm1=vec(p + "norm1", d), proj=HK.WideWeight(torch.cat(weights), dtype, tail=H if m.gate == "head" else 0), proj_bias=bias,
+                  out=HK.WideWeight(_padded(o, d, H, E).reshape(d, -1), dtype), q_norm=_padded(vec(mix + "q.norm", m.dim)[pairs], D),
+                  k_norm=_padded(vec(mix + "k.norm", m.dim)[pairs], D), sink=vec(mix + "sink", H) if m.sink else None)
+        if m.diff is not None:
+            a1, b1, a2, b2 = (vec(mix + n, m.dim).double() for n in ("lq1", "lk1", "lq2", "lk2"))
+            lw.update(lam=float(torch.exp((a1 * b1).sum()) - torch.exp((a2 * b2).sum())) + m.diff)
+        if mlp is not None:
+            lw.update(norm2=vec(p + "norm2", d))
+        mp = p + "mlp."
+        if isinstance(mlp, Experts):
+            lw.update(ff=feed_forward(HK.ExpertWeight, [f"{mp}e{e}." for e in range(mlp.count)], mlp.expert.ff), top=mlp.top)
+            router = [get(mp + "router", (mlp.count, d))]
+            if mlp.shared is not None:
+                lw.update(shared=feed_forward(HK.ExpertWeight, [mp + "shared."], mlp.shared.ff))
+                router.append(get(mp + "shared.sg", (1, d)))
+            router = torch.cat(router)
+            lw.update(router=_padded(router, router.shape[0], HK.pad8(d)).to(dtype).contiguous(), router_linear=HK.WideWeight(router, dtype))
+        elif mlp is not None:
+            lw.update(ff=feed_forward(lambda w, *a, **kw: HK.WideWeight(w[0], *a, **kw), [mp], mlp.ff))
+        layers.append(ResultNormLayerWeights(**lw))
+    embed = get("embed", (spec.vocab, d)).to(dtype).contiguous()
+    return ResultNormWeights(embed, layers, vec("final.norm", d), HK.WideWeight(embed, dtype))

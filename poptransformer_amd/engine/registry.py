@@ -19,6 +19,13 @@ def _ruperax(cfg, path, max_len, batch, dtype, slots):
     return ParallelDecoder(spec, loader.parallel_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
 
 
+def _golapel(cfg, path, max_len, batch, dtype, slots):
+    from ..utils import checkpoint
+    from .result_norm import ResultNormDecoder
+    spec = loader.golapel_spec(cfg, max_len, batch, dtype=dtype)
+    return ResultNormDecoder(spec, loader.result_norm_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
+
+
 def _fused(spec_of, weights_of):
     def make(cfg, path, max_len, batch, dtype, slots):
         from ..utils import checkpoint
@@ -44,6 +51,7 @@ def _only_fp16(dtype):
 ARCHITECTURES = {
     "Zekilix": (("hybrid",), _zekilix),
     "Ruperax": (("hybrid",), _ruperax),
+    "Golapel": (("hybrid",), _golapel),
     "GPT2LMHeadModel": (("hip", "hybrid"), _fused(loader.gpt2_spec, loader.gpt2_weights)),
     "LlamaForCausalLM": (("hip", "hybrid"), _fused(loader.llama2_spec, loader.llama2_weights)),
     "ChatGLMModel": (("hip", "hybrid"), _fused(loader.chatglm2_spec, loader.chatglm2_weights)),

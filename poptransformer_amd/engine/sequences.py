@@ -3,6 +3,8 @@
 A sequence holds one SLOT while it lives.  Per layer run (a layer whose weights are another layer's has a cache of its
 own) a slot is
   * for windowed attention: a ring of key rows, position p in row p % ring_len, and one fp32 factor per position;
+  * for attention by heads: rings of keys (normed, rotated) and values, the first `keep` positions in rows of their own before
+    the ring of the others;
   * for latent attention: a ring of latents with their rotated key part - a layer that reads another one's cache has none;
   * for matrix memory: the fp32 state, zero before the first token;
 and with a token shift per layer the normed fp32 row of the newest token.
@@ -34,6 +36,10 @@ class SequenceStore:
         return None if None in windows else max(windows)
 
     def ring_len(self, i):
+        m = self.spec.layers[i].mixer
+        if m.kind == "heads":
+            n = max(min(self.max_len, m.keep + m.span - 1 + self.portion), m.keep + 1)
+            return (n + 63) // 64 * 64
         window = self.cache_window(i)
         n = self.max_len if window is None else min(self.max_len, window - 1 + self.portion)
         return (n + 63) // 64 * 64
@@ -51,6 +57,9 @@ class SequenceStore:
             if m.kind == "attention":
                 n = self.ring_len(i)
                 new = (zeros(slots, m.kv_heads, n, HK.pad8(m.dim)), zeros(slots, n, dtype=torch.float32))
+            elif m.kind == "heads":
+                n = self.ring_len(i)
+                new = (zeros(slots, m.kv_heads, m.maps, n, m.stored_dim), zeros(slots, m.kv_heads, n, m.stored_vdim))
             elif m.kind == "latent":
                 new = (zeros(slots, self.ring_len(i), m.cache_row),) if m.source is None else ()
             else:

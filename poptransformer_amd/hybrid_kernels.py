@@ -286,6 +286,192 @@ def latent_tiles_fit(dtype, D, P, E):
     return bool(H.load().pta_latent_tiles_fit(_CODE[dtype], D, P, E))
 
 
+class HeadAttention:
+    """The calls of attention over cached keys and values of one layer.  `mixer` gives the sizes, the visible positions and what the
+    result goes through (engine/hybrid.py HeadMixer); proj rows hold q | k | v (none where the values are the keys) | gate per
+    feature (where there is one)."""
+
+    def __init__(self, mixer, eps, q_norm, k_norm, cos_sin, sink, lam, keys, values, proj, rows, slot, pos, head_gate, out):
+        m = mixer
+        heads, G, M, D, E = m.heads, m.kv_heads, m.maps, m.stored_dim, m.stored_vdim
+        es, ld = proj.element_size(), proj.shape[-1]
+        for t, n in ((keys, (G, M, D)), (values, (G, E))):
+            _need(t, proj.dtype, "cache")
+            if (*t.shape[1:-2], t.shape[-1]) != n or t.shape[-2] != keys.shape[-2]:
+                raise ValueError(f"the cache must be [slots, {n[:-1]}, length, {n[-1]}], got {tuple(t.shape)}")
+        if keys.shape[-2] < m.keep + min(m.span, keys.shape[-2] - m.keep):
+            raise ValueError("the cache is shorter than the positions that are visible")
+        _need(proj, proj.dtype, "projection", rows * ld)
+        _need(slot, I32, "slot", rows)
+        _need(pos, I32, "pos", rows)
+        _need(out, proj.dtype, "out", rows * heads * E)
+        for t, n in ((q_norm, D), (k_norm, D), (sink, heads), (head_gate, rows * heads)):
+            if t is not None:
+                _need(t, F32, "norms, sinks and gates", n)
+        at_k = heads * M * D
+        at_v = at_k if m.keys_are_values else at_k + G * M * D
+        at_gate = at_k + G * M * D + (0 if m.keys_are_values else G * E)
+        if ld < at_gate + (heads * E if m.gate == "feature" else 0):
+            raise ValueError("the projection rows do not hold queries, keys, values and gate")
+        base = proj.data_ptr()
+        a = self.a = H.HeadArgs(_CODE[proj.dtype], rows, heads, G, M, D, E, m.dim, m.vdim, base, base + at_k * es, base + at_v * es, ld)
+        a.q_norm, a.k_norm, a.eps, a.scale = _p(q_norm), _p(k_norm), eps, m.scale
+        if cos_sin is not None:
+            _need(cos_sin, F32, "cos_sin")
+            a.cos_sin, a.positions, a.rot = _p(cos_sin), cos_sin.shape[0], cos_sin.shape[1] * 2
+        a.window, a.keep, a.chunk = m.window or (1 << 30), m.keep, m.chunk or 0
+        a.keys, a.values, a.ring_len, a.slot, a.pos, a.sink = _p(keys), _p(values), keys.shape[-2], _p(slot), _p(pos), _p(sink)
+        a.lambda_, a.diff, a.out, a.splits = lam, m.diff or 0.0, _p(out), 1
+        a.head_gate = _p(head_gate)
+        a.gate = base + at_gate * es if m.gate == "feature" else None
+
+    def decode(self, splits, workspace):
+        """One row per sequence: norms, rotation, append and attention."""
+        a = self.a
+        a.splits, a.workspace, a.workspace_bytes = splits, _p(workspace), workspace.numel() if workspace is not None else 0
+        H.check(H.load().pta_head_decode(ctypes.byref(a), _stream()))
+
+    def prompt(self, tiles):
+        """Rows of a pass with several rows per sequence; tiles = (first rows, row counts, how many)."""
+        a, lib = self.a, H.load()
+        tr, tc, n = tiles
+        _need(tr, I32, "tiles", n)
+        _need(tc, I32, "tiles", n)
+        a.tile_row, a.tile_count, a.tiles = _p(tr), _p(tc), n
+        H.check(lib.pta_head_append(ctypes.byref(a), _stream()))
+        H.check(lib.pta_head_attention(ctypes.byref(a), _stream()))
+
+
+def head_workspace(rows, mixer, splits, device):
+    n = H.load().pta_head_attention_workspace_bytes(rows, mixer.heads, mixer.maps, mixer.stored_vdim, splits)
+    return torch.empty(max(n, 16), dtype=torch.uint8, device=device)
+
+
+class Routing:
+    """Where the routing of up to `rows` rows goes: choice c of row r in chosen[r, c], its weight beside it."""
+
+    def __init__(self, rows, experts, top, shared, scale, device):
+        self.experts, self.top, self.shared, self.scale, self.choices = experts, top, bool(shared), scale, top + bool(shared)
+        self.chosen = torch.zeros((rows, self.choices), dtype=I32, device=device)
+        self.weights = torch.zeros((rows, self.choices), dtype=F32, device=device)
+
+    def args(self, rows):
+        _need(self.chosen, I32, "routing", rows * self.choices)
+        return H.Routing(self.experts, self.top, int(self.shared), self.scale, _p(self.chosen), _p(self.weights))
+
+    def __call__(self, logits, rows):
+        """Routes rows by their logits fp32 [rows, experts + shared]."""
+        _need(logits, F32, "router logits", rows * (self.experts + self.shared))
+        a = self.args(rows)
+        H.check(H.load().pta_route(_p(logits), rows, ctypes.byref(a), _stream()))
+
+
+def result_norm(x, rows, eps, h, weight=None, table=None, embed_scale=1.0, ids=None, ids_index=None, pos_out=None, y=None, y_weight=None,
+                parts=None, n_parts=0, parts_ld=None, part_weight=None, final_weight=None, router=None, routing=None):
+    """x += norm(result), h = x (pta_result_norm).  The result is y (times y_weight [rows, n][:, c], given as (weights, c)) plus the
+    weighted parts [rows, parts_ld, width] (the first n_parts of a row, default: all); with `router` the rows are routed into `routing`."""
+    width = x.shape[-1]
+    _need(x, F32, "x", rows * width)
+    _need(h, h.dtype, "h", rows * h.shape[-1])
+    if table is not None:
+        _need(table, h.dtype, "table")
+        _need(ids, I32, "ids")
+    else:
+        _need(weight, F32, "weight", width)
+    if final_weight is not None:
+        _need(final_weight, F32, "final_weight", width)
+    if y is not None:
+        _need(y, F32, "y", rows * width)
+    stride = ids.shape[-1] if ids is not None and ids.dim() == 2 else 1
+    a = H.ResultNormArgs(_CODE[h.dtype], rows, width, _p(x), _p(table), table.shape[0] if table is not None else 0, embed_scale, _p(ids), stride,
+                         _p(ids_index), _p(pos_out), _p(y))
+    if y_weight is not None:
+        w, c = y_weight
+        _need(w, F32, "y_weight", rows * w.shape[-1])
+        a.y_weight, a.weights_ld = w.data_ptr() + 4 * c, w.shape[-1]
+    if parts is not None:
+        if parts.dtype not in (F32, h.dtype):
+            raise ValueError(f"parts must be float32 or {h.dtype}")
+        parts_ld = parts_ld or n_parts
+        _need(parts, parts.dtype, "parts", rows * parts_ld * width)
+        _need(part_weight, F32, "part_weight", rows * part_weight.shape[-1])
+        if a.weights_ld not in (0, part_weight.shape[-1]):
+            raise ValueError("the weights of y and of the parts belong to one buffer")
+        a.parts, a.n_parts, a.parts_ld, a.part_f32 = _p(parts), n_parts, parts_ld, int(parts.dtype == F32)
+        a.part_weight, a.weights_ld = _p(part_weight), part_weight.shape[-1]
+    a.weight, a.eps, a.final_weight, a.h, a.h_ld = _p(weight), eps, _p(final_weight), _p(h), h.shape[-1]
+    if router is not None:
+        _need(router, h.dtype, "router", (routing.experts + routing.shared) * h.shape[-1])
+        a.router, a.routing = _p(router), routing.args(rows)
+    H.check(H.load().pta_result_norm(ctypes.byref(a), _stream()))
+
+
+class ExpertWeight:
+    """Linear weights of one shape, one per expert, one after the other: bf16 tiled (channels rounded up to 16, many to 128), fp32
+    as they are.  main_to: further zero channels, as WideWeight's.  That of a single expert also serves `linear`."""
+    tail, tail_bias = 0, None
+
+    def __init__(self, weights, dtype, main_to=None):
+        """weights: an iterable of [N, K] tensors"""
+        parts = []
+        for w in weights:
+            n, k = w.shape
+            self.n_main, self.K, self.dtype = n if main_to is None else main_to, pad8(k), dtype
+            tile = 128 if self.n_main >= 1024 else 16
+            self.N = (self.n_main + tile - 1) // tile * tile
+            full = torch.zeros((self.N, self.K), dtype=dtype, device=w.device)
+            full[:n, :k] = w.to(dtype)
+            if dtype == torch.bfloat16:
+                lib = H.load()
+                data = torch.empty(lib.pta_bf16_tiled_bytes(self.N, self.K), dtype=torch.uint8, device=w.device)
+                H.check(lib.pta_bf16_tile(full.data_ptr(), data.data_ptr(), self.N, self.K, _stream()))
+                torch.cuda.current_stream().synchronize()      # `full` goes back to the allocator here
+                full = data
+            parts.append(full)
+        self.count, self.data = len(parts), torch.stack(parts)
+
+    @property
+    def nbytes(self):
+        """Bytes of one expert's."""
+        return self.n_main * self.K * (2 if self.dtype == torch.bfloat16 else 4)
+
+    def args(self, up=None, pair=H.PAIR_NONE, limit=0.0, slope=0.0):
+        if up is not None and (up.N, up.K, up.count) != (self.N, self.K, self.count):
+            raise ValueError("the weights of a pair must be alike")
+        return H.ExpertWeights(_p(self.data), _p(up.data) if up is not None else None, self.K, self.N, self.n_main, pair, limit, slope)
+
+
+def expert_lists(rows, top, experts, tile_rows, device):
+    return torch.zeros(H.load().pta_expert_lists_size(rows, top, experts, tile_rows), dtype=I32, device=device)
+
+
+def group_experts(routing, rows, tile_rows, lists):
+    _need(lists, I32, "lists", H.load().pta_expert_lists_size(rows, routing.top, routing.experts, tile_rows))
+    H.check(H.load().pta_group_experts(_p(routing.chosen), rows, routing.top, routing.choices, routing.experts, tile_rows, _p(lists), _stream()))
+
+
+def experts(x, routing, rows, routed, out, shared=None, lists=None, tile_rows=0):
+    """One product of every row's experts (pta_experts).  routed, shared: dict(w=ExpertWeight, and of a pair up=, pair=, limit=, slope=);
+    x [rows, ld] for a pair, else [rows * choices, ld]; out [rows * choices, ld]."""
+    w, dtype, n = routed["w"], routed["w"].dtype, rows * routing.choices
+    pair = routed.get("up") is not None
+    _need(x, dtype, "x", (rows if pair else n) * x.shape[-1])
+    if out.dtype not in (dtype, F32):
+        raise ValueError(f"out must be {dtype} or float32")
+    _need(out, out.dtype, "out", n * out.shape[-1])
+    if w.count != routing.experts or (shared is not None and (shared["w"].dtype != dtype or not routing.shared or (shared.get("up") is not None) != pair)):
+        raise ValueError("the experts' weights do not fit the routing")
+    pack = lambda d: d["w"].args(**{k: v for k, v in d.items() if k != "w"})
+    a = H.ExpertsArgs(_CODE[dtype], rows, routing.experts, routing.top, routing.choices, _p(routing.chosen), _p(x), x.shape[-1], pack(routed))
+    if shared is not None:
+        a.shared = pack(shared)
+    a.Y, a.ld_y, a.out_f32 = _p(out), out.shape[-1], int(out.dtype == F32)
+    if lists is not None:
+        _need(lists, I32, "lists", H.load().pta_expert_lists_size(rows, routing.top, routing.experts, tile_rows))
+        a.lists, a.tile_rows = _p(lists), tile_rows
+    H.check(H.load().pta_experts(ctypes.byref(a), _stream()))
+
+
 def mlstm_state(slots, heads, dim, vdim, device):
     return torch.zeros((slots, H.load().pta_mlstm_state_floats(heads, dim, vdim)), dtype=F32, device=device)
 
