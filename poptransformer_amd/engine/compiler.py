@@ -1,7 +1,7 @@
 """From a recorded graph to something that runs: `Session.compile` ends here.
 
 Every graph can run op by op (engine/interpreter.py).  A graph that is one of the decoder loops
-this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix, Ruperax as the models build them through the operator
+this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix, Ruperax, Golapel as the models build them through the operator
 API - is additionally mapped onto the fused executor for its family: the family is read off the
 state-dict keys the layers registered as initializer names, the shapes off a one-iteration probe of
 the interpreter, and the weights off the initializers.  The fused executor is then VALIDATED: it
@@ -291,6 +291,37 @@ def _build_parallel(facts, topk=1):
     return ParallelDecoder(spec, parallel_weights(facts.init, spec))
 
 
+def _build_result_norm(facts, topk=1):
+    """As _build_hybrid, for layers with attention by heads whose results are normed: the layers recorded the numbers of their
+    mixers, rotations and mixtures of experts as one constant each."""
+    from .hybrid import ClampedGLU, Experts, HeadMixer, HybridLayer, HybridSpec, Rotation, SwiGLU
+    from .loader import result_norm_weights
+    from .result_norm import ResultNormDecoder
+    const = _const_reader(facts)
+    layers = []
+    while const(f"l{len(layers)}.mixer", False) is not None:
+        i = len(layers)
+        mix, mlp = f"l{i}.mix.", f"l{i}.mlp."
+        numbers, rot = const(f"l{i}.mixer"), const(f"l{i}.rotation", False)
+        dim = _need(facts, mix + "q.norm").shape[0]
+        vdim = facts.init[mix + "v"].shape[0] // int(numbers[1]) if facts.has(mix + "v") else dim
+        mixer = HeadMixer.of(numbers, dim, vdim, "".join(n for n in "qkv" if facts.has(mix + n + ".b")), Rotation.of(rot) if rot is not None else None)
+        experts, ff = const(f"l{i}.experts", False), None
+        if experts is not None:
+            count, top, scale, limit, *shared = (float(v) for v in experts)
+            ff = Experts(int(count), int(top), scale, ClampedGLU(_need(facts, mlp + "e0.gate").shape[0], limit),
+                         ClampedGLU(_need(facts, mlp + "shared.gate").shape[0], shared[0]) if shared else None)
+        elif facts.has(mlp + "gate"):
+            ff = SwiGLU(facts.init[mlp + "gate"].shape[0])
+        layers.append(HybridLayer(mixer, ff, i))
+    if not layers:
+        raise ValueError("no layers found among the graph's constants")
+    vocab, width = _need(facts, "embed").shape
+    spec = HybridSpec("golapel", layers, width, vocab, 1, float(const("eps")), 1.0, float(const("embedding_scale")), 0.0, facts.max_len,
+                      facts.batch, facts.pad_id, facts.eos_id, facts.early_stop, topk, _executor_dtype())
+    return ResultNormDecoder(spec, result_norm_weights(facts.init, spec))
+
+
 def _build_hybrid(facts, topk=1):
     """The hybrid executor of a graph whose layers are tensors `l<i>.*`: sizes from the tensors, constants from the named
     constants the layers recorded, the arithmetic ('bf16' or 'fp32') from the precision the graph was built with."""
@@ -334,8 +365,10 @@ def _family(facts):
         return "gpt2"
     if facts.has("rwkv.blocks.0.attention.key.weight"):
         return "rwkv"
-    if facts.has("l0.mix.q") and facts.has("l0.norm1"):
+    if facts.has("l0.mix.q") and facts.has("l0.norm1") and facts.has("head"):
         return "zekilix"
+    if facts.has("l0.mix.q.norm") and facts.has("l0.norm1"):          # the embedding is the head
+        return "golapel"
     if facts.has("l0.mix.uk") and facts.has("l0.rg1"):
         return "ruperax"
     return None
@@ -533,7 +566,7 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
         prog.interp_outputs = list(graph.outputs)
         k = _sampling_k(facts)
         use_fp8_cache = _fp8_cache_of(facts, fp8_cache)
-        if use_fp8_cache and family in ("rwkv", "zekilix", "ruperax"):
+        if use_fp8_cache and family in ("rwkv", "zekilix", "ruperax", "golapel"):
             raise ValueError(f"fp8_cache: the {family} executor has no FP8 KV cache")
         steps = min(PROBE_STEPS, facts.max_loop)
         # one-iteration probe: operand shapes of the native operators
@@ -548,6 +581,8 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
             decoder = _build_hybrid(facts, k)
         elif family == "ruperax":
             decoder = _build_parallel(facts, k)
+        elif family == "golapel":
+            decoder = _build_result_norm(facts, k)
         else:
             spec, weights = _build_transformer(facts, shapes, family, k, use_fp8_cache)
             decoder = fused.FusedDecoder(spec, weights)

@@ -141,6 +141,15 @@ class Rotation:
         slowed = np.clip((i - low) / max(high - low, 0.001), 0.0, 1.0)
         return f * (slowed / self.factor + (1.0 - slowed)), 0.1 * math.log(self.factor) + 1.0
 
+    def numbers(self):
+        """The fields as a flat list, which `Rotation.of` reads."""
+        return [self.base, self.dims, self.neighbours, self.factor, *(self.yarn or ())]
+
+    @staticmethod
+    def of(numbers):
+        base, dims, neighbours, factor, *yarn = (float(v) for v in numbers)
+        return Rotation(base, int(dims), bool(neighbours), factor, tuple(yarn) or None)
+
     def pairs(self, size):
         """Order of `size` features in which the two of a pair follow each other."""
         turned = np.arange(self.dims)
@@ -177,6 +186,28 @@ class HeadMixer:
     gate: Optional[str] = None       # sigmoid gate of the result, one number per "head" or per "feature"
     diff: Optional[float] = None     # two maps per head, the second subtracted; part of their weight, and 1 - diff of the result
     kind = "heads"
+
+    def numbers(self):
+        """Everything but the feature sizes, the biases and the rotation as a flat list, which `HeadMixer.of` reads."""
+        return [self.heads, self.kv_heads, self.scale, self.window or 0, self.keep, self.chunk or 0, self.keys_are_values, self.sink,
+                (None, "head", "feature").index(self.gate), *(() if self.diff is None else (self.diff,))]
+
+    @staticmethod
+    def of(numbers, dim, vdim, biases, rot):
+        heads, kv_heads, scale, window, keep, chunk, keys_are_values, sink, gate, *diff = (float(v) for v in numbers)
+        return HeadMixer(int(heads), int(kv_heads), dim, vdim, scale, rot, int(window) or None, int(keep), int(chunk) or None,
+                         bool(keys_are_values), biases, bool(sink), (None, "head", "feature")[int(gate)], diff[0] if diff else None)
+
+    def visible(self, positions):
+        """bool [position of the query, distance back to the key]."""
+        i, back = np.arange(positions)[:, None], np.arange(positions)[None]
+        j = i - back
+        near = j >= 0
+        if self.window is not None:
+            near &= (back < self.window) | (j < self.keep)
+        if self.chunk is not None:
+            near &= i // self.chunk == j // self.chunk
+        return near
 
     @property
     def maps(self):

@@ -299,8 +299,6 @@ class HeadAttention:
             _need(t, proj.dtype, "cache")
             if (*t.shape[1:-2], t.shape[-1]) != n or t.shape[-2] != keys.shape[-2]:
                 raise ValueError(f"the cache must be [slots, {n[:-1]}, length, {n[-1]}], got {tuple(t.shape)}")
-        if keys.shape[-2] < m.keep + min(m.span, keys.shape[-2] - m.keep):
-            raise ValueError("the cache is shorter than the positions that are visible")
         _need(proj, proj.dtype, "projection", rows * ld)
         _need(slot, I32, "slot", rows)
         _need(pos, I32, "pos", rows)

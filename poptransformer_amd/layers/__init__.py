@@ -10,6 +10,8 @@ from .mlp import MLP
 from .lm_head import LMHead
 from .streams import NamedLinear, StreamConnection, WeightNorm
 from .parallel import BiasedSwiGLU, GroupedRMSNorm, ResultGate, RotaryTable, TokenShift
+from .heads import ExpertMixture, HeadAttention, SwiGLU
 
 __all__ = ["BaseLayer", "Linear", "LayerNorm", "RMSLayerNorm", "Embedding", "MLP", "LMHead", "NamedLinear", "StreamConnection",
-           "WeightNorm", "BiasedSwiGLU", "GroupedRMSNorm", "ResultGate", "RotaryTable", "TokenShift"]
+           "WeightNorm", "BiasedSwiGLU", "GroupedRMSNorm", "ResultGate", "RotaryTable", "TokenShift", "HeadAttention",
+           "SwiGLU", "ExpertMixture"]

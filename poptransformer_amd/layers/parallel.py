@@ -75,21 +75,39 @@ class BiasedSwiGLU(BaseLayer):
 
 
 class RotaryTable(BaseLayer):
-    """cos and sin of every position, [positions, dims / 2] each, for features i and i + dims / 2 turned together."""
+    """cos and sin of every position, [positions, dims / 2] each, for features i and i + dims / 2 turned together, or
+    (`neighbours`) features 2 i and 2 i + 1.  Frequencies other than base^(-2 i / dims), and a factor of both, may be given."""
 
-    def __init__(self, name, positions, base, dims):
+    def __init__(self, name, positions, base, dims, neighbours=False, frequencies=None, amplitude=1.0):
         super().__init__(None, name)
-        self.dims = dims
-        angle = np.arange(positions)[:, None] * float(base) ** (-2.0 * np.arange(dims // 2) / dims)
-        self.ids = [self.add_initialized_input_tensor(f(angle).astype(np.float32), f"{name}.{n}") for f, n in ((np.cos, "cos"), (np.sin, "sin"))]
+        self.dims, self.neighbours = dims, neighbours
+        f = float(base) ** (-2.0 * np.arange(dims // 2) / dims) if frequencies is None else frequencies
+        angle = np.arange(positions)[:, None] * f
+        self.ids = [self.add_initialized_input_tensor((f(angle) * amplitude).astype(np.float32), f"{name}.{n}")
+                    for f, n in ((np.cos, "cos"), (np.sin, "sin"))]
 
     def __call__(self, graph, x, step, size):
         """x [B, n, size], its first `dims` features turned by the angles of position `step`."""
         half, rest = self.dims // 2, size - self.dims
         cos, sin = (ops.reshape(graph, ops.dynamic_slice(graph, t, step, axes=[0], sizes=[1]), [1, 1, half]) for t in self.ids)
+        if self.neighbours:
+            return self._neighbours(graph, x, cos, sin, size)
         parts = [half, half] + ([rest] if rest else [])
         u, v, *tail = ops.split(graph, x, len(parts), axis=2, splits=parts, name="split_rotated")
         a = ops.sub(graph, ops.mul(graph, u, cos), ops.mul(graph, v, sin))
         b = ops.add(graph, ops.mul(graph, v, cos), ops.mul(graph, u, sin))
         y = ops.concat(graph, a, b, 2)
         return ops.concat(graph, y, tail[0], 2) if tail else y
+
+    def _neighbours(self, graph, x, cos, sin, size):
+        half, rest = self.dims // 2, size - self.dims
+        B, n = self.batch_size, -1
+        turned = x
+        if rest:
+            turned, tail = ops.split(graph, x, 2, axis=2, splits=[self.dims, rest], name="split_rotated")
+        u, v = ops.split(graph, ops.reshape(graph, turned, [B, n, half, 2]), 2, axis=3, splits=[1, 1], name="split_neighbours")
+        u, v = (ops.squeeze(graph, t, [3]) for t in (u, v))
+        a = ops.sub(graph, ops.mul(graph, u, cos), ops.mul(graph, v, sin))
+        b = ops.add(graph, ops.mul(graph, v, cos), ops.mul(graph, u, sin))
+        y = ops.reshape(graph, ops.concat(graph, ops.unsqueeze(graph, a, [3]), ops.unsqueeze(graph, b, [3]), 3), [B, n, self.dims])
+        return ops.concat(graph, y, tail, 2) if rest else y
