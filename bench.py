@@ -26,9 +26,9 @@ bytes; or, with the per-operator executor, the fused INT4 gate/up projection), a
 Other workloads (``--workload``), each printing one line of the same form: ``gemm`` = the single INT4
 weight-only operator X[M, 4096] by W[4096, 11008] at M = ``--batch``; ``chatglm2`` = ChatGLM2-6B-shape FP8
 decode; ``rwkv`` = RWKV-4-7B-shape INT4 recurrent decode; ``prompt`` = the prompt of the headline model taken in
-passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix`` and
-``ruperax`` = these designs (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights (and, for Ruperax, the
-Zekilix design) at the same sizes: decode at batch 1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
+passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix``,
+``ruperax`` and ``golapel`` = these designs (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights (and, for
+Ruperax and Golapel, the Zekilix design) at the same sizes: decode at batch 1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
 serve the hardware-counter measurement of the HBM traffic (see their help).
 """
 import argparse
@@ -443,13 +443,33 @@ def ruperax_config(width, ff, layers):
             "vocab": 32000, "width": width}
 
 
+def golapel_config(width, ff, layers):
+    """A window with a dense feed-forward before every layer within chunks (plain and differential in turn) that has a mixture of
+    experts: 6 of 32 with a shared one of twice their size, together as large as the dense feed-forward."""
+    scale, kv = 128 ** -0.5, width // 512
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // 8, "limit": 7.0}, "router": {"experts": 32, "top": 6, "scale": 1.5},
+           "shared": {"ff": ff // 4, "limit": 7.0}}
+    window = {"type": "attention", "mlp": dense, "mixer": {"heads": width // 128, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": scale,
+              "mask": {"size": 1024, "keep_first": 4}, "rot": {"base": 1e6, "dims": 128, "scaling": {"factor": 2.0}}}}
+    chunk = {"type": "attention_3", "mlp": moe, "mixer": {"heads": width // 128, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": scale,
+             "mask": {"size": 2048}, "rot": {"base": 5e5, "dims": 128, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}}
+    maps = {"type": "attention_2", "mlp": moe, "mixer": {"heads": width // 128, "kv_heads": kv, "dim": 64, "vdim": 128, "scale": 64 ** -0.5,
+            "diff": 0.5, "mask": {"size": 2048}}}
+    return {"architecture": "Golapel", "embedding": {"scale": 16.0}, "layers": ([window, chunk, window, maps] * layers)[:layers],
+            "norm": {"eps": 1e-5}, "vocab": 32000, "width": width}
+
+
 def hybrid_step_bytes(spec, weights, B, t):
-    """Bytes one decode iteration of a hybrid decoder must move at context t: the weights of every layer run, the key rows
-    of the windows, the memories (read and written), the head."""
-    n = weights.head.nbytes
+    """Bytes one decode iteration of a hybrid decoder must move at context t: the weights of every layer run (of a mixture the
+    experts that the rows choose on average), the key rows that are seen, the memories (read and written), the head."""
+    n = weights.head.nbytes if spec.family != "golapel" else weights.nbytes(B)
     for lay in spec.layers:
-        n += sum(w.nbytes for w in weights.layers[lay.source].linears())
         m = lay.mixer
+        if m.kind == "heads":
+            n += B * m.kv_heads * 2 * (m.maps * m.dim + m.vdim) * (min(t + 1, m.keep + m.window) if m.window else t % m.chunk + 1)
+            continue
+        n += sum(w.nbytes for w in weights.layers[lay.source].linears())
         seen = min(t + 1, getattr(m, "window", None) or t + 1)
         if m.kind == "attention":
             n += B * m.kv_heads * (2 * m.dim + 4 / m.kv_heads) * seen
@@ -462,11 +482,11 @@ def hybrid_step_bytes(spec, weights, B, t):
 
 def design_workload(args, design):
     """Decode iterations (contexts 1024 .. 1024 + steps - 1, replayed from a HIP graph, one launch per operator) and prompt
-    passes of a design, beside the executors that come closest to it: Llama-2 with fp16 weights (and for Ruperax the Zekilix
-    design) at equal width, feed-forward size, layer count, vocabulary and head size.  --layers shortens all of them (for
+    passes of a design, beside the executors that come closest to it: Llama-2 with fp16 weights (and for the later designs
+    Zekilix) at equal width, feed-forward size, layer count, vocabulary and head size.  --layers shortens all of them (for
     profiles)."""
     import torch
-    from poptransformer_amd.engine import fused, hybrid, loader, parallel, synthetic
+    from poptransformer_amd.engine import fused, hybrid, loader, parallel, result_norm, synthetic
     rng = np.random.Generator(np.random.PCG64(1234))
     first, steps, max_len = 1024, args.steps, 2048
     results = []
@@ -493,11 +513,17 @@ def design_workload(args, design):
         if name == "zekilix":
             cfg, spec_of, tensors, weights_of, decoder = (zekilix_config(width, ff, layers), loader.zekilix_spec, synthetic.HybridTensors,
                                                           loader.hybrid_weights, hybrid.HybridDecoder)
+        elif name == "golapel":
+            cfg, spec_of, tensors, weights_of, decoder = (golapel_config(width, ff, layers), loader.golapel_spec, synthetic.HeadTensors,
+                                                          loader.result_norm_weights, result_norm.ResultNormDecoder)
         else:
             cfg, spec_of, tensors, weights_of, decoder = (ruperax_config(width, ff, layers), loader.ruperax_spec, synthetic.ParallelTensors,
                                                           loader.parallel_weights, parallel.ParallelDecoder)
         spec = spec_of(cfg, max_len, 1)
         w = weights_of(tensors(cfg), spec)
+        if name == "golapel":
+            params = sum(lw.active_parameters() for lw in w.layers)
+            return lambda B, L: decoder(spec_of(cfg, L, B), w), lambda B, t: hybrid_step_bytes(spec, w, B, t), params
         params = sum(x.n_main * x.K for lay in spec.layers for x in w.layers[lay.source].linears())
         params += sum(m.heads * m.kv_rank * (m.dim + m.vdim) for m in (lay.mixer for lay in spec.layers) if m.kind == "latent")
         return lambda B, L: decoder(spec_of(cfg, L, B), w), lambda B, t: hybrid_step_bytes(spec, w, B, t), params
@@ -569,17 +595,17 @@ def main():
     ap.add_argument("--batch", type=int, default=1)
     ap.add_argument("--executor", choices=["persistent", "operators"], default=None,
                     help="default: persistent when the batch fits it (<= 16, fp16 cache), else operators")
-    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix", "ruperax"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix", "ruperax", "golapel"], default="decode",
                     help="decode: the Llama2-7B-shape INT4 decode loop (the headline); gemm: the single INT4 "
                          "weight-only operator at M = --batch rows; chatglm2: ChatGLM2-6B-shape FP8 decode; "
                          "rwkv: RWKV-4-7B-shape INT4 recurrent decode; prompt: the headline model's prompt in passes "
-                         "of --rows-per-pass rows (--steps passes); zekilix, ruperax: that design beside Llama-2 with fp16 weights "
-                         "(ruperax: and Zekilix) at equal sizes, decode and prompts")
-    ap.add_argument("--width", type=int, default=0, help="zekilix and ruperax workloads: only this width")
-    ap.add_argument("--layers", type=int, default=0, help="zekilix and ruperax workloads: layers of the models (even)")
-    ap.add_argument("--only", choices=["zekilix", "ruperax", "llama2"], default=None, help="zekilix and ruperax workloads: one of the models")
-    ap.add_argument("--decode-only", action="store_true", help="zekilix and ruperax workloads: no prompts")
-    ap.add_argument("--rows-only", action="store_true", help="zekilix and ruperax workloads: prompts only")
+                         "of --rows-per-pass rows (--steps passes); zekilix, ruperax, golapel: that design beside Llama-2 with fp16 "
+                         "weights (the latter two: and Zekilix) at equal sizes, decode and prompts")
+    ap.add_argument("--width", type=int, default=0, help="workloads of a design: only this width")
+    ap.add_argument("--layers", type=int, default=0, help="workloads of a design: layers of the models (even)")
+    ap.add_argument("--only", choices=["zekilix", "ruperax", "golapel", "llama2"], default=None, help="workloads of a design: one of the models")
+    ap.add_argument("--decode-only", action="store_true", help="workloads of a design: no prompts")
+    ap.add_argument("--rows-only", action="store_true", help="workloads of a design: prompts only")
     ap.add_argument("--one-stream", action="store_true", help="ruperax workload: no feed-forward on a stream beside the mixer (for profiles)")
     ap.add_argument("--rows-per-pass", type=int, default=64,
                     help="prompt workload: rows (batch x positions) per pass, up to 2048")
@@ -629,7 +655,7 @@ def main():
     if args.workload == "prompt":
         print(json.dumps(prompt_workload(args)))
         return
-    if args.workload in ("zekilix", "ruperax"):
+    if args.workload in ("zekilix", "ruperax", "golapel"):
         print(json.dumps(design_workload(args, args.workload)))
         return
     B, cfg = args.batch, LLAMA2_7B

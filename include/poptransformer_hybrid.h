@@ -352,7 +352,10 @@ typedef struct pta_result_norm_args {
 } pta_result_norm_args;
 
 int pta_result_norm(const pta_result_norm_args* host_args, pta_stream_t stream);
-/* the same routing of rows whose logits fp32 [rows, experts + shared] are there already */
+/* the same routing of many bf16 rows by their products with the router [experts + shared, ld] as pta_bf16_tile leaves it, ld a multiple
+ * of 8 */
+int pta_route_rows(const uint16_t* h, int ld, int rows, const void* router, const pta_routing* host_routing, pta_stream_t stream);
+/* and of rows whose logits fp32 [rows, experts + shared] are there already */
 int pta_route(const float* logits, int rows, const pta_routing* host_routing, pta_stream_t stream);
 
 /* ---- Mixture of experts -------------------------------------------------------------------------------------------

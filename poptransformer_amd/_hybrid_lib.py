@@ -88,6 +88,7 @@ SIGNATURES = {
     **{f"pta_head_{n}": (_I, [POINTER(HeadArgs), _P]) for n in ("append", "attention", "decode")},
     "pta_result_norm": (_I, [POINTER(ResultNormArgs), _P]),
     "pta_route": (_I, [_P, _I, POINTER(Routing), _P]),
+    "pta_route_rows": (_I, [_P, _I, _I, _P, POINTER(Routing), _P]),
     "pta_expert_lists_size": (c_size_t, [_I, _I, _I, _I]),
     "pta_group_experts": (_I, [_P, _I, _I, _I, _I, _I, _P, _P]),
     "pta_experts": (_I, [POINTER(ExpertsArgs), _P]),

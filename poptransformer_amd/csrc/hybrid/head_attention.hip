@@ -297,43 +297,49 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
   }
 }
 
-// the parts of a row's keys (at most 64) meet: one wave per (row, head)
+// the parts of a row's keys (at most 64) meet: one workgroup per (row, head), a thread per map and feature
 template <typename T, int MAPS>
-__global__ __launch_bounds__(64) void head_merge_kernel(HA a, const float* part_o, const float* part_ml) {
-  __shared__ float weight[MAPS][64];
-  __shared__ float res[MAPS][512];
-  const int r = blockIdx.x / a.H, head = blockIdx.x % a.H, E = a.E, lane = threadIdx.x, n = a.splits;
+__global__ __launch_bounds__(256) void head_merge_kernel(HA a, const float* part_o, const float* part_ml) {
+  __shared__ float weight[MAPS][64], inv_s[MAPS];
+  __shared__ float res[MAPS * 512];
+  const int r = blockIdx.x / a.H, head = blockIdx.x % a.H, E = a.E, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = a.splits;
   const size_t at = ((size_t)r * a.H + head) * MAPS * n;
-  // the first eight parts of this lane's first feature are requested before the weights are known
-  float v[MAPS][8], inv[MAPS];
+  // the first eight parts of this thread's first feature are requested before the weights are known
+  auto fetch = [&](int i, int s, float (&v)[8]) {
+    const int t = i / E, d = i % E;
 #pragma unroll
-  for (int t = 0; t < MAPS; ++t)
-#pragma unroll
-    for (int u = 0; u < 8; ++u) v[t][u] = u < n && lane < E ? part_o[(at + t * n + u) * E + lane] : 0.f;
-#pragma unroll
-  for (int t = 0; t < MAPS; ++t) {
+    for (int u = 0; u < 8; ++u) v[u] = i < MAPS * E && s + u < n ? part_o[(at + t * n + s + u) * E + d] : 0.f;
+  };
+  float v[8];
+  fetch(threadIdx.x, 0, v);
+  if (wave < MAPS) {
     float m = -1e30f, l = 0.f;
-    if (lane < n) { m = part_ml[(at + t * n + lane) * 2]; l = part_ml[(at + t * n + lane) * 2 + 1]; }
+    if (lane < n) { m = part_ml[(at + wave * n + lane) * 2]; l = part_ml[(at + wave * n + lane) * 2 + 1]; }
     const float top = wave_max(m), w = lane < n ? exp_of<T>(m - top) : 0.f;
-    weight[t][lane] = w;
-    inv[t] = 1.0f / wave_sum(w * l);
+    weight[wave][lane] = w;
+    const float total = wave_sum(w * l);
+    if (lane == 0) inv_s[wave] = 1.0f / total;
   }
   __syncthreads();
+  for (int i = threadIdx.x; i < MAPS * E; i += 256) {
+    float sum = 0.f;
+    for (int s = 0; s < n; s += 8) {
+      float next[8];
+      if (s + 8 < n) fetch(i, s + 8, next);
+      else fetch(i + 256, 0, next);
 #pragma unroll
-  for (int t = 0; t < MAPS; ++t)
-    for (int d = lane; d < E; d += 64) {
-      float sum = 0.f;
-      for (int s = 0; s < n; s += 8) {
-        if (s > 0 || d != lane) {
+      for (int u = 0; u < 8; ++u) sum = __builtin_fmaf(s + u < n ? weight[i / E][s + u] : 0.f, v[u], sum);
 #pragma unroll
-          for (int u = 0; u < 8; ++u) v[t][u] = s + u < n ? part_o[(at + t * n + s + u) * E + d] : 0.f;
-        }
-#pragma unroll
-        for (int u = 0; u < 8; ++u) sum = __builtin_fmaf(s + u < n ? weight[t][s + u] : 0.f, v[t][u], sum);
-      }
-      res[t][d] = sum;
+      for (int u = 0; u < 8; ++u) v[u] = next[u];
     }
-  finish_head<T, MAPS>(a, r, head, lane, inv, [&](int t, int d) { return res[t][d]; });     // (a lane reads what it wrote)
+    res[i] = sum;
+  }
+  __syncthreads();
+  if (wave > 0) return;
+  float inv[MAPS];
+#pragma unroll
+  for (int t = 0; t < MAPS; ++t) inv[t] = inv_s[t];
+  finish_head<T, MAPS>(a, r, head, lane, inv, [&](int t, int d) { return res[t * E + d]; });
 }
 
 // ------------------------------------------------------------------------------------------
@@ -699,10 +705,10 @@ extern "C" int pta_head_decode(const HA* args, pta_stream_t stream) {
   if (a.dtype == PTA_BF16) launch_rows<bf16>(a, 1, po, pml, s);
   else launch_rows<float>(a, 1, po, pml, s);
   if (a.splits > 1) {
-    if (a.dtype == PTA_BF16 && a.maps == 2) hipLaunchKernelGGL((head_merge_kernel<bf16, 2>), heads, dim3(64), 0, s, a, po, pml);
-    else if (a.dtype == PTA_BF16) hipLaunchKernelGGL((head_merge_kernel<bf16, 1>), heads, dim3(64), 0, s, a, po, pml);
-    else if (a.maps == 2) hipLaunchKernelGGL((head_merge_kernel<float, 2>), heads, dim3(64), 0, s, a, po, pml);
-    else hipLaunchKernelGGL((head_merge_kernel<float, 1>), heads, dim3(64), 0, s, a, po, pml);
+    if (a.dtype == PTA_BF16 && a.maps == 2) hipLaunchKernelGGL((head_merge_kernel<bf16, 2>), heads, dim3(256), 0, s, a, po, pml);
+    else if (a.dtype == PTA_BF16) hipLaunchKernelGGL((head_merge_kernel<bf16, 1>), heads, dim3(256), 0, s, a, po, pml);
+    else if (a.maps == 2) hipLaunchKernelGGL((head_merge_kernel<float, 2>), heads, dim3(256), 0, s, a, po, pml);
+    else hipLaunchKernelGGL((head_merge_kernel<float, 1>), heads, dim3(256), 0, s, a, po, pml);
   }
   PTA_CHECK_LAUNCH("pta_head_decode");
   return PTA_OK;

@@ -1,14 +1,14 @@
 // A residual that takes normed results: x <- x + rms_norm(y) * weight, with what follows in the same launch: the rounded row that
 // the next sublayer reads, or the model's norm of it, and the routing of the row to its experts.
-#include "hybrid.h"
-#include <type_traits>
+#include "attention.h"
 
 typedef pta_result_norm_args RN;
 
-// Routing of one row by THREADS threads: z holds the logits (in LDS, visible to all; overwritten).  Expert e's place among the
-// chosen is the number of larger scores (of equal ones the first comes first), so no choice waits for another.
+// Routing of row r by THREADS threads, of which this is `tid`: z holds the logits (in LDS, visible to all; overwritten).  Expert e's
+// place among the chosen is the number of larger scores (of equal ones the first comes first), so no choice waits for another.
+// The whole workgroup calls it, each group of THREADS for a row of its own; with `store` unset nothing is kept.
 template <int THREADS>
-__device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r) {
+__device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r, int tid, bool store) {
   const int E = g.experts, choices = g.top + g.shared;
   int32_t* chosen = g.chosen + (size_t)r * choices;
   float* weights = g.weights + (size_t)r * choices;
@@ -17,13 +17,14 @@ __device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r)
   float p[PER];
 #pragma unroll
   for (int k = 0; k < PER; ++k) {
-    const int e = threadIdx.x + k * THREADS;
+    const int e = tid + k * THREADS;
     rank[k] = E;
     p[k] = 0.f;
     if (e >= E) continue;
     const float mine = z[e];
     float top = mine;
     int above = 0;
+#pragma unroll 8
     for (int j = 0; j < E; ++j) {
       const float v = z[j];
       top = fmaxf(top, v);
@@ -32,29 +33,76 @@ __device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r)
     rank[k] = above;
     p[k] = expf(mine - top);
   }
-  const float shared = g.shared && threadIdx.x == 0 ? sigmoid_f32(z[E]) : 0.f;
+  const float shared = g.shared && tid == 0 ? sigmoid_f32(z[E]) : 0.f;
   __syncthreads();
 #pragma unroll
   for (int k = 0; k < PER; ++k)
-    if (threadIdx.x + k * THREADS < E) z[threadIdx.x + k * THREADS] = p[k];
+    if (tid + k * THREADS < E) z[tid + k * THREADS] = p[k];
   __syncthreads();
   bool any = false;
 #pragma unroll
   for (int k = 0; k < PER; ++k) any = any || rank[k] < g.top;
-  if (any) {
+  if (any && store) {
     float sum = 0.f;
+#pragma unroll 8
     for (int j = 0; j < E; ++j) sum += z[j];
 #pragma unroll
     for (int k = 0; k < PER; ++k)
       if (rank[k] < g.top) {
-        chosen[rank[k]] = threadIdx.x + k * THREADS;
+        chosen[rank[k]] = tid + k * THREADS;
         weights[rank[k]] = p[k] / sum * g.scale;
       }
   }
-  if (g.shared && threadIdx.x == 0) {
+  if (g.shared && store && tid == 0) {
     chosen[g.top] = E;
     weights[g.top] = shared;
   }
+}
+
+// Many rows (bf16): sixteen of them per workgroup, whose waves share the features; BLOCKS * 16 logits of each at a time.
+constexpr int RR_WAVES = 8;
+
+template <int BLOCKS>
+__global__ __launch_bounds__(RR_WAVES * 64) void route_rows_kernel(const bf16* h, int ld, int rows, const bf16x8* router, pta_routing g, int z_ld) {
+  extern __shared__ __align__(16) float z_rows[];            // [16][z_ld]
+  __shared__ f32x4 red[RR_WAVES][BLOCKS][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15;
+  const int row0 = blockIdx.x * 16, n = g.experts + g.shared, pieces = (ld + 127) / 128 * 4, last = (n + 15) / 16 - 1;
+  const bf16* x = h + (size_t)(row0 + lc < rows ? row0 + lc : rows - 1) * ld;
+  for (int e0 = 0; e0 < n; e0 += BLOCKS * 16) {
+    const bf16x8* w[BLOCKS];
+    f32x4 acc[BLOCKS];
+#pragma unroll
+    for (int b = 0; b < BLOCKS; ++b) {
+      w[b] = router + (size_t)(e0 / 16 + b < last ? e0 / 16 + b : last) * pieces * 64 + lane;
+      acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll 4
+    for (int c = wave; c < pieces; c += RR_WAVES) {
+      const int k = c * 32 + lg * 8;
+      bf16x8 xv = *reinterpret_cast<const bf16x8*>(x + (k < ld ? k : 0));
+#pragma unroll
+      for (int i = 0; i < 8; ++i) xv[i] = k < ld ? xv[i] : (bf16)0.0f;
+#pragma unroll
+      for (int b = 0; b < BLOCKS; ++b) acc[b] = mma(w[b][(size_t)c * 64], xv, acc[b]);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int b = 0; b < BLOCKS; ++b) red[wave][b][lane] = acc[b];
+    __syncthreads();
+    for (int i = threadIdx.x; i < BLOCKS * 64; i += RR_WAVES * 64) {
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int v = 0; v < RR_WAVES; ++v) s += red[v][i / 64][i % 64];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int e = e0 + i / 64 * 16 + i % 64 / 16 * 4 + r;
+        if (e < n) z_rows[(i & 15) * z_ld + e] = s[r];
+      }
+    }
+  }
+  __syncthreads();
+  for (int m = wave; m < 16; m += RR_WAVES) route_row<64>(g, z_rows + m * z_ld, row0 + m, lane, row0 + m < rows);
 }
 
 __global__ __launch_bounds__(64) void route_kernel(const float* logits, pta_routing g) {
@@ -62,7 +110,7 @@ __global__ __launch_bounds__(64) void route_kernel(const float* logits, pta_rout
   const int n = g.experts + g.shared;
   for (int c = threadIdx.x; c < n; c += 64) z[c] = logits[(size_t)blockIdx.x * n + c];
   __syncthreads();
-  route_row<64>(g, z, blockIdx.x);
+  route_row<64>(g, z, blockIdx.x, threadIdx.x, true);
 }
 
 __device__ __forceinline__ float rounded(float v, bf16) { return (float)(bf16)v; }
@@ -210,7 +258,7 @@ __global__ __launch_bounds__(THREADS) void result_norm_kernel(RN a) {
     if (lane == 0) z[e] = s;
   }
   __syncthreads();
-  route_row<THREADS>(a.routing, z, r);
+  route_row<THREADS>(a.routing, z, r, threadIdx.x, true);
 }
 
 static int check_routing(const pta_routing& g, const char* name) {
@@ -226,6 +274,32 @@ extern "C" int pta_route(const float* logits, int rows, const pta_routing* routi
   if (rc) return rc;
   hipLaunchKernelGGL(route_kernel, dim3(rows), dim3(64), 0, (hipStream_t)stream, logits, *routing);
   PTA_CHECK_LAUNCH("pta_route");
+  return PTA_OK;
+}
+
+extern "C" int pta_route_rows(const uint16_t* h, int ld, int rows, const void* router, const pta_routing* routing, pta_stream_t stream) {
+  const char* name = "pta_route_rows";
+  PTA_REQUIRE(h && router && routing && rows > 0, "%s: null pointer, or %d rows", name, rows);
+  PTA_REQUIRE(ld > 0 && ld % 8 == 0 && pta_aligned(h, 16) && pta_aligned(router, 16), "%s: rows of %d, or unaligned operands", name, ld);
+  const int rc = check_routing(*routing, name);
+  if (rc) return rc;
+  const int z_ld = routing->experts + routing->shared + 1;
+  const size_t smem = (size_t)16 * z_ld * sizeof(float);
+  auto launch = [&](auto blocks) {
+    constexpr int B = decltype(blocks)::value;
+    PTA_REQUIRE(smem <= 24 * 1024 || hipFuncSetAttribute((const void*)route_rows_kernel<B>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) ==
+                                         hipSuccess, "%s: %zu bytes of LDS refused", name, smem);
+    hipLaunchKernelGGL((route_rows_kernel<B>), dim3((rows + 15) / 16), dim3(RR_WAVES * 64), smem, (hipStream_t)stream,
+                       reinterpret_cast<const bf16*>(h), ld, rows, reinterpret_cast<const bf16x8*>(router), *routing, z_ld);
+    return PTA_OK;
+  };
+  const int blocks = (z_ld + 14) / 16;
+  const int launched = blocks == 1   ? launch(std::integral_constant<int, 1>{})
+                       : blocks == 2 ? launch(std::integral_constant<int, 2>{})
+                       : blocks == 3 ? launch(std::integral_constant<int, 3>{})
+                                     : launch(std::integral_constant<int, 4>{});
+  if (launched) return launched;
+  PTA_CHECK_LAUNCH(name);
   return PTA_OK;
 }
 

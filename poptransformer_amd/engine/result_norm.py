@@ -7,8 +7,8 @@ sampling and the decode loop are HybridDecoder's.
 
 Launches of a layer in a decode iteration: projections; attention (norms, rotation and cache entry with it, the parts of the
 visible keys merged by a second launch); output projection; result norm, which also routes the row; gate / up pair and down
-projection of the chosen experts and the shared one (or of the dense feed-forward); result norm.  Passes of many rows route by
-a product of their own and work through the experts' lists of rows.
+projection of the chosen experts and the shared one (or of the dense feed-forward); result norm.  Passes of many rows work
+through the experts' lists of rows, and route in a launch of its own.
 """
 from dataclasses import dataclass
 from typing import List, Optional
@@ -45,8 +45,14 @@ class ResultNormLayerWeights:
     ff: Optional[FeedForwardWeights] = None          # dense, or the routed experts
     shared: Optional[FeedForwardWeights] = None
     router: Optional[torch.Tensor] = None            # [experts (+ the shared one's gate), padded width]
-    router_linear: Optional[HK.WideWeight] = None    # the same, for passes of many rows
+    router_linear: Optional[HK.WideWeight] = None    # the same as a Linear
     top: int = 0
+
+    def active_parameters(self):
+        """Parameters of the products that one row goes through."""
+        parts = [(w, 1) for w in (self.proj, self.out)] + [(w, max(self.top, 1)) for w in (self.ff.linears() if self.ff else ())]
+        parts += [(w, 1) for w in (self.shared.linears() if self.shared else ())]
+        return sum(w.n_main * w.K * times for w, times in parts)
 
 
 @dataclass
@@ -103,7 +109,8 @@ class ResultNormBuffers:
                 self.act[choices, n] = buf(rows * choices, n)
             if choices not in self.parts:
                 self.parts[choices] = buf(rows * choices, spec.width, dtype=F32 if direct else dtype)
-            self.logits[lw.router.shape[0]] = buf(rows, lw.router.shape[0], dtype=F32)
+            if dtype == F32:
+                self.logits[lw.router.shape[0]] = buf(rows, lw.router.shape[0], dtype=F32)
             if not direct:
                 for t in (128, 256):
                     self.lists[e.count, e.top, t] = HK.expert_lists(rows, e.top, e.count, t, device)
@@ -113,7 +120,9 @@ class ResultNormBuffers:
 
 class ResultNormDecoder(HybridDecoder):
     direct_rows = 16                 # passes of up to this many bf16 rows find their experts' rows without lists
-    router_bytes = 256 << 10         # routers up to this size are multiplied in the norm's launch by such passes
+    # routers up to this size are multiplied in the norm's launch by passes of up to so many rows (every row reads all of it: 2048
+    # rows of 4096 features and 33 logits take 43 us that way, 19 + 21 with a launch for the routing, 512 rows 16 against 10 + 15)
+    router_bytes, router_rows = 1 << 20, 512
 
     def __init__(self, spec, weights, device="cuda", slots=None):
         super().__init__(spec, weights, device, slots)
@@ -167,7 +176,7 @@ class ResultNormDecoder(HybridDecoder):
     def _routed_by_norm(self, i, b):
         """What the norm's launch needs to route the rows to layer i's experts, where it does."""
         lw = self.w.layers[i]
-        if lw.router is None or not self._direct(b.rows) or lw.router.numel() * lw.router.element_size() > self.router_bytes:
+        if lw.router is None or b.rows > self.router_rows or lw.router.numel() * lw.router.element_size() > self.router_bytes:
             return {}
         return dict(router=lw.router, routing=self._routing(i, b))
 
@@ -179,9 +188,12 @@ class ResultNormDecoder(HybridDecoder):
             return dict(y=b.y)
         r = self._routing(i, b)
         if not self._routed_by_norm(i, b):
-            logits = b.logits[lw.router.shape[0]]
-            HK.linear(b.h, lw.router_linear, logits, n)
-            r(logits, n)
+            if self.dtype == torch.bfloat16:
+                r.by_product(b.h, lw.router_linear, n)
+            else:
+                logits = b.logits[lw.router.shape[0]]
+                HK.linear(b.h, lw.router_linear, logits, n)
+                r(logits, n)
 
         def clamped(glu):
             return dict(pair=H.PAIR_CLAMPED, limit=glu.limit, slope=glu.slope)

@@ -242,3 +242,41 @@ class ParallelTensors(HybridTensors):
             rest = {"shift": (d,), "rg1": (d, d), "rg2": (d, d), "rg1.b": (d,), "rg2.b": (d,), "norm1": (d,), "norm2": (d,)}
             for group, names in (("mix.", mix), ("mlp.", mlp), ("", rest)):
                 self.shapes.update({p + group + n: shape for n, shape in names.items()})
+
+
+class HeadTensors(HybridTensors):
+    """As HybridTensors, for a configuration with attention by heads and mixtures of experts."""
+
+    def __init__(self, cfg, seed=0, device="cuda"):
+        super().__init__(dict(cfg, layers=[], streams=None), seed, device)
+        d = cfg["width"]
+        del self.shapes["head"]
+        for i, lay in enumerate(cfg["layers"]):
+            p, m, f = f"l{i}.", lay["mixer"], lay["mlp"]
+            H, G, D, E, kind = m["heads"], m["kv_heads"], m["dim"], m["vdim"], lay["type"]
+            maps = 2 if kind == "attention_2" else 1
+            mix = {"q": (H * maps * D, d), "k": (G * maps * D, d), "q.norm": (D,), "k.norm": (D,), "o": (d, H * E)}
+            if kind == "attention_2":
+                mix.update({n: (D,) for n in ("lq1", "lk1", "lq2", "lk2")})
+            else:
+                mix.update({"q.b": (H * D,), "k.b": (G * D,), "g": (H if kind == "attention" else H * E, d)})
+            mix.update({"sink": (H,)} if kind == "attention" else {"v": (G * E, d)})
+            if kind == "attention_3":
+                mix["v.b"] = (G * E,)
+            mlp = {}
+            parts = [("", f["ff"])] if f["kind"] == "dense" else [(f"e{e}.", f["expert"]["ff"]) for e in range(f["router"]["experts"])]
+            if f["kind"] == "moe":
+                mlp["router"] = (f["router"]["experts"], d)
+                if f.get("shared") is not None:
+                    parts.append(("shared.", f["shared"]["ff"]))
+                    mlp["shared.sg"] = (1, d)
+            for q, ff in parts:
+                mlp.update({q + "gate": (ff, d), q + "up": (ff, d), q + "down": (d, ff)})
+            for group, names in (("mix.", mix), ("mlp.", mlp), ("", {"norm1": (d,), "norm2": (d,)})):
+                self.shapes.update({p + group + n: shape for n, shape in names.items()})
+
+    def __getitem__(self, name):
+        shape = self.shapes[name]
+        if len(shape) == 1 and (name.endswith(".b") or name.split(".")[-1] in ("sink", "lq1", "lk1", "lq2", "lk2")):
+            return torch.zeros(shape, device=self.dev)
+        return super().__getitem__(name)

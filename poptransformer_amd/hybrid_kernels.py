@@ -363,6 +363,14 @@ class Routing:
         a = self.args(rows)
         H.check(H.load().pta_route(_p(logits), rows, ctypes.byref(a), _stream()))
 
+    def by_product(self, h, router, rows):
+        """Routes bf16 rows by their products with the router, a WideWeight."""
+        _need(h, torch.bfloat16, "rows", rows * h.shape[-1])
+        if (router.dtype, router.K, router.n_main) != (torch.bfloat16, h.shape[-1], self.experts + self.shared):
+            raise ValueError("the router does not fit the rows or the routing")
+        a = self.args(rows)
+        H.check(H.load().pta_route_rows(_p(h), h.shape[-1], rows, _p(router.data), ctypes.byref(a), _stream()))
+
 
 def result_norm(x, rows, eps, h, weight=None, table=None, embed_scale=1.0, ids=None, ids_index=None, pos_out=None, y=None, y_weight=None,
                 parts=None, n_parts=0, parts_ld=None, part_weight=None, final_weight=None, router=None, routing=None):

@@ -270,6 +270,24 @@ def test_routing(rows, experts, top, shared):
         assert (r.chosen[:rows, top] == experts).all() and _rel(_np(r.weights)[:rows, top], G.sigmoid(z[:, experts])) < 1e-5
 
 
+@pytest.mark.parametrize("rows,experts,top,shared,d", [(17, 8, 3, True, 84), (1, 5, 1, False, 53), (300, 64, 6, False, 1032), (40, 33, 2, True, 256),
+                                                       (16, 130, 4, True, 2100), (33, 1000, 8, True, 72)])
+def test_routing_by_product(rows, experts, top, shared, d):
+    HK, T = _hk()
+    rng = np.random.default_rng(rows)
+    h, w = (torch.zeros((n, HK.pad8(d)), dtype=torch.bfloat16, device="cuda") for n in (rows, experts + shared))
+    h[:, :d], w[:, :d] = _dev(rng.standard_normal((rows, d))), _dev(rng.standard_normal((experts + shared, d)) * 2 / np.sqrt(d))
+    r = HK.Routing(rows + 2, experts, top, shared, 0.8, "cuda")
+    r.chosen.fill_(-7)
+    r.by_product(h, HK.WideWeight(w[:, :d].float(), T["bfloat16"]), rows)
+    z = _np(h) @ _np(w).T
+    chosen, weight = G.route(z[:, :experts], top, 0.8)
+    assert np.array_equal(r.chosen.cpu().numpy()[:rows, :top], chosen) and _rel(_np(r.weights)[:rows, :top], weight) < 1e-4
+    assert (r.chosen[rows:] == -7).all()
+    if shared:
+        assert (r.chosen[:rows, top] == experts).all() and _rel(_np(r.weights)[:rows, top], G.sigmoid(z[:, experts])) < 1e-4
+
+
 # ---------------------------------------------------------------------------------------------- experts
 def _choices(rng, rows, experts, top, how):
     if how == "all the same":

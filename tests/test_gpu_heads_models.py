@@ -20,7 +20,7 @@ DTYPES = ["float32", "bfloat16"]
 
 def _decoder(cfg, sd, dtype, max_len=400, slots=2, batch=1, **kw):
     from poptransformer_amd.engine import loader, result_norm
-    own = {k: kw.pop(k) for k in ("pass_rows", "direct_rows", "router_bytes", "head_rows") if k in kw}
+    own = {k: kw.pop(k) for k in ("pass_rows", "direct_rows", "router_bytes", "router_rows", "head_rows") if k in kw}
     spec = loader.golapel_spec(cfg, max_len, batch, dtype=dtype, **kw)
     cls = type("Decoder", (result_norm.ResultNormDecoder,), own)
     return cls(spec, loader.result_norm_weights(sd, spec), slots=slots)
