@@ -77,14 +77,26 @@ __global__ __launch_bounds__(RR_WAVES * 64) void route_rows_kernel(const bf16* h
       w[b] = router + (size_t)(e0 / 16 + b < last ? e0 / 16 + b : last) * pieces * 64 + lane;
       acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-#pragma unroll 4
-    for (int c = wave; c < pieces; c += RR_WAVES) {
-      const int k = c * 32 + lg * 8;
-      bf16x8 xv = *reinterpret_cast<const bf16x8*>(x + (k < ld ? k : 0));
+    const int per = (pieces + RR_WAVES - 1) / RR_WAVES, end = (wave + 1) * per < pieces ? (wave + 1) * per : pieces;
+    constexpr int U = 4;                                     // pieces whose operands are requested together
+    for (int c0 = wave * per; c0 < end; c0 += U) {
+      bf16x8 xv[U], wv[U][BLOCKS];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) xv[i] = k < ld ? xv[i] : (bf16)0.0f;
+      for (int u = 0; u < U; ++u) {
+        const int c = c0 + u < end ? c0 + u : end - 1, k = c * 32 + lg * 8;
+        xv[u] = *reinterpret_cast<const bf16x8*>(x + (k < ld ? k : 0));
 #pragma unroll
-      for (int b = 0; b < BLOCKS; ++b) acc[b] = mma(w[b][(size_t)c * 64], xv, acc[b]);
+        for (int b = 0; b < BLOCKS; ++b) wv[u][b] = w[b][(size_t)c * 64];
+      }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const bool in = c0 + u < end && (c0 + u) * 32 + lg * 8 < ld;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) xv[u][i] = in ? xv[u][i] : (bf16)0.0f;
+#pragma unroll
+        for (int b = 0; b < BLOCKS; ++b) acc[b] = mma(wv[u][b], xv[u], acc[b]);
+      }
     }
     __syncthreads();
 #pragma unroll
