@@ -123,6 +123,7 @@ class ResultNormDecoder(HybridDecoder):
     # routers up to this size are multiplied in the norm's launch by passes of up to so many rows (every row reads all of it: 2048
     # rows of 4096 features and 33 logits take 43 us that way, 19 + 21 with a launch for the routing, 512 rows 16 against 10 + 15)
     router_bytes, router_rows = 1 << 20, 512
+    tall_rows = 128                  # rows per expert, on average, above which their lists are cut into tiles of 256 (else 128)
 
     def __init__(self, spec, weights, device="cuda", slots=None):
         super().__init__(spec, weights, device, slots)
@@ -210,7 +211,7 @@ class ResultNormDecoder(HybridDecoder):
             HK.experts(b.h, r, n, pair, act, shared_pair)
             HK.experts(act, r, n, down, parts, shared_down)
             return dict(result, n_parts=r.choices)
-        tile = 256 if n * mlp.top > 128 * mlp.count else 128
+        tile = 256 if n * mlp.top > self.tall_rows * mlp.count else 128
         lists, act = b.lists[mlp.count, mlp.top, tile], b.act[r.choices, lw.ff.gate.n_main]
         HK.group_experts(r, n, tile, lists)
         HK.experts(b.h, r, n, pair, act, lists=lists, tile_rows=tile)
