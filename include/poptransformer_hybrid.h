@@ -56,10 +56,10 @@ typedef struct pta_wide_linear_args {
   void* workspace;        /* NULL, or scratch of pta_wide_linear_workspace_bytes(M, N): lets bf16 launches with few
                              channels split K across workgroups                                                    */
   size_t workspace_bytes;
-  /* main channels, in this order: sum + bias, cap, sigmoid, * mul, += Y */
+  /* main channels, in this order: sum + bias, cap, act, * mul, += Y */
   const float* bias;      /* [n_main] or NULL (of a pair: the gate's)                                              */
   const float* bias2;     /* [n_main] or NULL: the up weight's of a pair                                           */
-  int sigmoid;            /* y = sigmoid(y)                                                                        */
+  int act;                /* PTA_ACT_* of poptransformer_hip.h, in fp32 (single weights)                           */
   const void* mul;        /* NULL, or [M, ld] of the type of X: y = y * mul                                        */
   int accumulate;         /* Y += y (fp32 Y only)                                                                  */
 } pta_wide_linear_args;
@@ -188,7 +188,7 @@ int pta_window_decode(const pta_window_attention_args* host_args, pta_stream_t s
 /* ---- Attention over latents ---------------------------------------------------------------------------------------
  * A token leaves one row in the cache: its normed latent c and one rotated key part that all heads share.  Head h has the
  * key (W_uk,h c | rotated part), the value W_uv,h c, and score(i, j) = scale * (q_i . k_j) for 0 <= i - j < window, an
- * ordinary softmax, and its result times sigmoid(gate_h).  Two ways to the same numbers:
+ * ordinary softmax, and its result times sigmoid(gate_h), or feature by feature.  Two ways to the same numbers:
  *   absorbed (decode, short portions, fp32): q'_h = W_uk,h^T q_h meets the cached rows themselves, and W_uv,h is applied
  *     to the weighted sum of latents;
  *   over heads (prompts): keys and values of all heads are made from the cached rows (a Linear over pta_latent_gather's
@@ -223,7 +223,9 @@ typedef struct pta_latent_args {
   float* part_o;          /* [rows, H, splits, R]: sums of weighted latents                                        */
   float* part_ml;         /* [rows, H, splits, 2]: their largest score and sum of weights                          */
   const void* uv;         /* [H, E, R]                                                                             */
-  const float* gate;      /* [rows, H], before the sigmoid                                                         */
+  const float* gate;      /* [rows, H], before the sigmoid, or NULL                                                */
+  const void* feature_gate; /* [rows, gate_ld], first channel of [H][E] before the sigmoid, or NULL                */
+  int gate_ld;            /* a multiple of 8                                                                       */
   void* out;              /* [rows, H * E]                                                                         */
   /* over heads */
   int keys;               /* rows of the key buffers                                                               */
@@ -252,12 +254,43 @@ int pta_latent_gather(const pta_latent_args* host_args, pta_stream_t stream);
 int pta_latent_tiles_fit(int dtype, int D, int P, int E);
 int pta_latent_tiles(const pta_latent_args* host_args, pta_stream_t stream);
 
+/* ---- Short causal convolutions -------------------------------------------------------------------------------------
+ * y_t = act(sum_j weight[j] * u_{t - taps + 1 + j} + bias) channel by channel, zeros before position 0; act: silu or nothing.
+ * ring [slots][taps][channels] of the rows' type keeps a sequence's newest rows, position p in row p % taps. */
+typedef struct pta_conv {
+  int channels, taps;     /* channels: a multiple of 8; 1 <= taps <= PTA_CONV_TILE                                 */
+  const float* weight;    /* [taps][channels]                                                                      */
+  const float* bias;      /* [channels] or NULL                                                                    */
+  int silu;
+  void* ring;             /* NULL where the struct is part of another's arguments: no convolution                  */
+} pta_conv;
+
+enum { PTA_CONV_TILE = 128 };
+
+typedef struct pta_short_conv_args {
+  int dtype;
+  pta_conv c;
+  const void* x;          /* [rows, ld_x]                                                                          */
+  int ld_x;
+  void* y;                /* [rows, ld_y]                                                                          */
+  int ld_y;
+  const int32_t* slot;    /* [rows]                                                                                */
+  const int32_t* pos;     /* [rows]                                                                                */
+  const int32_t* last;    /* [rows]: of a sequence's first row in the pass the row of its last token, else -1      */
+  const int32_t* tile_row;   /* [tiles] first row of a tile: rows of one sequence, at most PTA_CONV_TILE, all of them
+                                but its last that many                                                             */
+  const int32_t* tile_count; /* [tiles]                                                                            */
+  int tiles;
+} pta_short_conv_args;
+
+int pta_short_conv(const pta_short_conv_args* host_args, pta_stream_t stream);
+
 /* ---- Attention over cached keys and values, by heads ---------------------------------------------------------------
  * H query heads on G key/value heads.  Query and key: RMS norm per head (plain weights), rotation of the first `rot`
  * features (pairs 2 i and 2 i + 1 turned by cos_sin[position][i]; any other pairing after a permutation of the weights'
  * rows).  The values are a projection of their own, or the keys as projected (v points at k).
  *   score(i, j) = scale * (q_i . k_j)   for j <= i with (i - j < window or j < keep) and floor(i / chunk) = floor(j / chunk)
- * and a softmax, whose denominator also holds exp(sink) of the head where there are sinks.  With maps = 2 every head has two
+ * less the penalty of the distance where there is one, and a softmax, whose denominator also holds exp(sink) of the head where there are sinks.  With maps = 2 every head has two
  * queries and keys [map 1 | map 2] over the same values, and its result is  o = a1 - lambda * a2,  o / sqrt(mean(o^2) + eps) *
  * (1 - diff).  Then the gates: sigmoid per head, or per feature.
  * Sizes as stored: D and E (query / key and value features) are multiples of 8, zero past `dim` and `vdim`.
@@ -296,6 +329,9 @@ typedef struct pta_head_attention_args {
   void* workspace;        /* decode with splits > 1: pta_head_attention_workspace_bytes                            */
   size_t workspace_bytes;
   void* out;              /* [rows, H * E]                                                                         */
+  const float* far1;      /* [H] or NULL: far1 ln(1 + far2 (i - j)) is taken off the scores (with keep = 0 only)   */
+  const float* far2;      /* [H], not negative                                                                     */
+  pta_conv conv;          /* decode: q | k | v, one behind the other, go through it first (maps = 1)               */
 } pta_head_attention_args;
 
 enum { PTA_HEAD_TILE = 128 };
@@ -318,11 +354,17 @@ typedef struct pta_routing {
   int experts, top;       /* 1 <= top <= experts <= PTA_MAX_EXPERTS                                                */
   int shared;             /* 1: logit `experts` is a shared expert's: choice `top` of every row, weight = its sigmoid */
   float scale;
-  int32_t* chosen;        /* [rows, top + shared]: largest softmax scores first (a shared expert is number `experts`) */
+  int32_t* chosen;        /* [rows, top + shared]: largest scores first (a shared expert is number `experts`) */
   float* weights;         /* [rows, top + shared]: score * scale                                                   */
+  int score;              /* PTA_SCORE_*                                                                           */
+  const float* correction; /* [experts] or NULL: added to sigmoid scores for the choice, not for the weights       */
+  int groups, keep;       /* equal groups of neighbouring experts (1: none); only those of the `keep` groups whose two largest
+                             choice scores sum up highest can be chosen (sigmoid scores)                           */
+  int share;              /* 1: a weight is the score's share of the chosen scores' sum (+ 1e-20)                  */
 } pta_routing;
 
 enum { PTA_MAX_EXPERTS = 1024 };
+enum { PTA_SCORE_SOFTMAX = 0, PTA_SCORE_SIGMOID = 1 };
 
 typedef struct pta_result_norm_args {
   int dtype;              /* type of h, of the embedding table, of the router                                      */
@@ -429,6 +471,113 @@ int pta_mlstm(const pta_mlstm_args* host_args, pta_stream_t stream);
 /* out = (o of each head / its root mean square) * weight * sigmoid(gate); out [rows, out_ld], the rest of a row zero */
 int pta_head_norm_gate(int dtype, const float* o, const float* weight, const void* gate, int gate_ld, void* out, int out_ld,
                        int rows, int H, int E, float eps, pta_stream_t stream);
+
+/* ---- State-space recurrence (Mamba-2) -----------------------------------------------------------------------------
+ * Per head, with dt = softplus(z + dt_bias) from the fp32 pre-activations and b, c of the head's group (H / G heads share them):
+ *   S = exp(-exp(a_log) dt) S + dt b x^T,   y = S^T c + skip x.
+ * State of a layer, fp32: [slots][H][slices][D][PTA_SSD_SLICE], a head's columns of S (E of them) in slices.
+ * With conv.ring every sequence has one row, x | b | c stand one behind the other as projected and go through the convolution first. */
+enum { PTA_SSD_SLICE = 32 };
+
+typedef struct pta_ssd_args {
+  int dtype;
+  int rows, H, G, D, E;   /* D (state) and E (head size): multiples of 8                                           */
+  const void* x;          /* [rows, ld]: H * E channels                                                            */
+  const void* b;          /* G * D                                                                                 */
+  const void* c;          /* G * D                                                                                 */
+  int ld;
+  const float* dt;        /* fp32 [rows, H]                                                                        */
+  const float* dt_bias;   /* [H]                                                                                   */
+  const float* a_log;     /* [H]                                                                                   */
+  const float* skip;      /* [H]                                                                                   */
+  float* state;
+  const int32_t* slot;    /* [rows]                                                                                */
+  const int32_t* pos;     /* [rows], with conv                                                                     */
+  const int32_t* seq_row; /* [seqs] first row of each sequence of the pass, seq_count its rows                     */
+  const int32_t* seq_count;
+  int seqs;
+  int longest;            /* rows of the longest sequence of the pass                                              */
+  int chunked;            /* bf16: work through the rows in chunks on the matrix unit where D <= 256 (else: one by one) */
+  float* y;               /* fp32 [rows, H * E]                                                                    */
+  void* workspace;        /* chunked: pta_ssd_workspace_bytes (0 where the pass is not cut into segments)          */
+  size_t workspace_bytes;
+  pta_conv conv;
+} pta_ssd_args;
+
+size_t pta_ssd_state_floats(int H, int D, int E);     /* per slot */
+size_t pta_ssd_workspace_bytes(const pta_ssd_args* host_args);   /* reads the sizes only */
+int pta_ssd(const pta_ssd_args* host_args, pta_stream_t stream);
+
+/* out = n(y silu(z)) weight, n dividing each of `parts` equal stretches of the H * vdim columns by its own root mean square.
+ * Heads are stored in E columns (vdim rounded up to 8). */
+typedef struct pta_gated_norm_args {
+  int dtype;
+  int rows, H, E, vdim, parts;
+  const float* y;         /* [rows, H * E]                                                                         */
+  const void* z;          /* [rows, ld_z]                                                                          */
+  int ld_z;
+  const float* weight;    /* [H * E]                                                                               */
+  float eps;
+  void* out;              /* [rows, H * E]                                                                         */
+} pta_gated_norm_args;
+
+int pta_gated_norm(const pta_gated_norm_args* host_args, pta_stream_t stream);
+
+/* ---- Residuals of all depths ---------------------------------------------------------------------------------------
+ * history fp32 [depths][depth_stride]: the residual rows [rows][width] as the embedding (depth 0) and every layer left them.
+ * One launch per end of a layer, for the newest of `depth` of them:
+ *   newest += n(y) y_weight    (n: over the root mean square; where there is a y)
+ *   u = sum_j weights[j] history[j]   (weights NULL with depth = 1: the row itself)
+ *   next = u;  h = norm(u) norm_weight (layer norm where `centred`, else RMS norm), columns past width zero;
+ * and with `router` the row is routed by what h holds (pta_route_args).  With `table` (depth = 0) u is the embedding, which is
+ * also stored as history[0], and every layer's part of the token's row of side_table goes to side[layer][row]. */
+typedef struct pta_depth_norm_args {
+  int dtype;              /* type of h, of the tables, of the router                                               */
+  int rows, width;
+  float* history;
+  size_t depth_stride;    /* floats                                                                                */
+  int depth;
+  const float* weights;   /* [depth]                                                                               */
+  const float* y;         /* [rows, width] or NULL                                                                 */
+  const float* y_weight;  /* [width]                                                                               */
+  float* next;            /* [rows, width] or NULL                                                                 */
+  int centred;
+  const float* norm_weight; /* [width]                                                                             */
+  float eps;              /* of both norms                                                                         */
+  void* h;                /* [rows, h_ld]                                                                          */
+  int h_ld;
+  const void* table;      /* [vocab, width] or NULL                                                                */
+  int vocab;
+  float embed_scale;
+  const int32_t* ids;     /* id of row r: ids[r * ids_stride + (ids_index ? *ids_index : 0)]                       */
+  int ids_stride;
+  const int32_t* ids_index;
+  int32_t* pos_out;       /* with ids_index: pos_out[r] = *ids_index (may be NULL)                                 */
+  const void* side_table; /* [vocab, side_layers, side_ld]                                                         */
+  void* side;             /* [side_layers][side_stride], or NULL                                                   */
+  int side_layers, side_ld; /* side_ld: a multiple of 8                                                            */
+  size_t side_stride;
+  const void* router;     /* [experts + shared, h_ld] of the type of h, or NULL                                    */
+  pta_routing routing;
+} pta_depth_norm_args;
+
+int pta_depth_norm(const pta_depth_norm_args* host_args, pta_stream_t stream);
+
+/* x += sum_p part_weight[r * weights_ld + p] * parts[r][p] (where there are parts), h = x, columns past width zero */
+typedef struct pta_add_parts_args {
+  int dtype;
+  int rows, width;
+  float* x;               /* [rows, width]                                                                         */
+  const void* parts;      /* [rows, parts_ld, width] or NULL, the first n_parts of a row                           */
+  int n_parts, parts_ld;
+  int part_f32;           /* fp32 parts, else of the type of h                                                     */
+  const float* part_weight;
+  int weights_ld;
+  void* h;                /* [rows, h_ld]                                                                          */
+  int h_ld;
+} pta_add_parts_args;
+
+int pta_add_parts(const pta_add_parts_args* host_args, pta_stream_t stream);
 
 /* ---- Next-token selection over fp32 logits, and the loop's bookkeeping -------------------------------------------- */
 int pta_argmax_f32(const float* logits, int32_t* ids, float* values, int rows, int n, pta_stream_t stream);

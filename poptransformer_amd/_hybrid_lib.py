@@ -11,8 +11,11 @@ LIB_PATH = os.path.join(os.path.dirname(os.path.abspath(__file__)), "libpoptrans
 
 BF16, FP32 = 0, 1
 PAIR_NONE, PAIR_SWIGLU, PAIR_CLAMPED = 0, 1, 2
+ACT_NONE, ACT_GELU_TANH, ACT_RELU_SQUARE, ACT_SIGMOID = 0, 1, 2, 3
+SCORE_SOFTMAX, SCORE_SIGMOID = 0, 1
 WINDOW_TILE = 128
 MLSTM_SLICE = 32
+CONV_TILE = 128
 LATENT_TILE = 128
 HEAD_TILE = 128
 MAX_EXPERTS = 1024
@@ -26,7 +29,7 @@ _P, _I, _F = c_void_p, c_int, c_float
 WideLinearArgs = _struct("WideLinearArgs", [
     ("dtype", _I), ("X", _P), ("M", _I), ("K", _I), ("N", _I), ("W", _P), ("W2", _P), ("pair", _I), ("limit", _F), ("slope", _F),
     ("cap", _F), ("Y", _P), ("ld", _I), ("n_main", _I), ("out_f32", _I), ("tail", _P), ("tail_count", _I), ("tail_bias", _P),
-    ("workspace", _P), ("workspace_bytes", c_size_t), ("bias", _P), ("bias2", _P), ("sigmoid", _I), ("mul", _P), ("accumulate", _I)])
+    ("workspace", _P), ("workspace_bytes", c_size_t), ("bias", _P), ("bias2", _P), ("act", _I), ("mul", _P), ("accumulate", _I)])
 StreamsArgs = _struct("StreamsArgs", [
     ("dtype", _I), ("rows", _I), ("width", _I), ("S", _I), ("streams", _P), ("table", _P), ("vocab", _I), ("embed_scale", _F),
     ("ids", _P), ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("y", _P), ("out", _P), ("mix", _P), ("mult", _F),
@@ -45,25 +48,45 @@ LatentArgs = _struct("LatentArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("P", _I), ("E", _I), ("R", _I), ("q_rank", _I), ("kv_rank", _I), ("proj", _P),
     ("ld", _I), ("q_norm", _P), ("kv_norm", _P), ("eps", _F), ("cq", _P), ("cos_sin", _P), ("positions", _I), ("ring", _P),
     ("ring_len", _I), ("slot", _P), ("pos", _P), ("q", _P), ("uk_t", _P), ("q_latent", _P), ("scale", _F), ("window", _I),
-    ("splits", _I), ("part_o", _P), ("part_ml", _P), ("uv", _P), ("gate", _P), ("out", _P), ("keys", _I), ("key_slot", _P),
+    ("splits", _I), ("part_o", _P), ("part_ml", _P), ("uv", _P), ("gate", _P), ("feature_gate", _P), ("gate_ld", _I), ("out", _P), ("keys", _I), ("key_slot", _P),
     ("key_pos", _P), ("key_latent", _P), ("key_rot", _P), ("kv", _P), ("tile_row", _P), ("tile_count", _P), ("tile_key", _P),
     ("tiles", _I)])
 MlstmArgs = _struct("MlstmArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("D", _I), ("E", _I), ("q", _P), ("k", _P), ("v", _P), ("ld", _I), ("gates", _P),
     ("cap", _F), ("state", _P), ("slot", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I), ("longest", _I), ("chunked", _I),
     ("o", _P), ("workspace", _P), ("workspace_bytes", c_size_t)])
+Conv = _struct("Conv", [("channels", _I), ("taps", _I), ("weight", _P), ("bias", _P), ("silu", _I), ("ring", _P)])
+ShortConvArgs = _struct("ShortConvArgs", [
+    ("dtype", _I), ("c", Conv), ("x", _P), ("ld_x", _I), ("y", _P), ("ld_y", _I), ("slot", _P), ("pos", _P), ("last", _P), ("tile_row", _P),
+    ("tile_count", _P), ("tiles", _I)])
+SsdArgs = _struct("SsdArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("G", _I), ("D", _I), ("E", _I), ("x", _P), ("b", _P), ("c", _P), ("ld", _I), ("dt", _P),
+    ("dt_bias", _P), ("a_log", _P), ("skip", _P), ("state", _P), ("slot", _P), ("pos", _P), ("seq_row", _P), ("seq_count", _P), ("seqs", _I),
+    ("longest", _I), ("chunked", _I), ("y", _P), ("workspace", _P), ("workspace_bytes", c_size_t), ("conv", Conv)])
+GatedNormArgs = _struct("GatedNormArgs", [
+    ("dtype", _I), ("rows", _I), ("H", _I), ("E", _I), ("vdim", _I), ("parts", _I), ("y", _P), ("z", _P), ("ld_z", _I), ("weight", _P),
+    ("eps", _F), ("out", _P)])
 HeadArgs = _struct("HeadArgs", [
     ("dtype", _I), ("rows", _I), ("H", _I), ("G", _I), ("maps", _I), ("D", _I), ("E", _I), ("dim", _I), ("vdim", _I), ("q", _P), ("k", _P),
     ("v", _P), ("ld", _I), ("q_norm", _P), ("k_norm", _P), ("eps", _F), ("scale", _F), ("cos_sin", _P), ("positions", _I), ("rot", _I),
     ("window", _I), ("keep", _I), ("chunk", _I), ("keys", _P), ("values", _P), ("ring_len", _I), ("slot", _P), ("pos", _P), ("sink", _P),
     ("lambda_", _F), ("diff", _F), ("head_gate", _P), ("gate", _P), ("tile_row", _P), ("tile_count", _P), ("tiles", _I), ("splits", _I),
-    ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P)])
-Routing = _struct("Routing", [("experts", _I), ("top", _I), ("shared", _I), ("scale", _F), ("chosen", _P), ("weights", _P)])
+    ("workspace", _P), ("workspace_bytes", c_size_t), ("out", _P), ("far1", _P), ("far2", _P), ("conv", Conv)])
+Routing = _struct("Routing", [("experts", _I), ("top", _I), ("shared", _I), ("scale", _F), ("chosen", _P), ("weights", _P), ("score", _I),
+                              ("correction", _P), ("groups", _I), ("keep", _I), ("share", _I)])
 ResultNormArgs = _struct("ResultNormArgs", [
     ("dtype", _I), ("rows", _I), ("width", _I), ("x", _P), ("table", _P), ("vocab", _I), ("embed_scale", _F), ("ids", _P),
     ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("y", _P), ("y_weight", _P), ("parts", _P), ("n_parts", _I), ("parts_ld", _I), ("part_f32", _I),
     ("part_weight", _P), ("weights_ld", _I), ("weight", _P), ("eps", _F), ("final_weight", _P), ("h", _P), ("h_ld", _I), ("router", _P),
     ("routing", Routing)])
+DepthNormArgs = _struct("DepthNormArgs", [
+    ("dtype", _I), ("rows", _I), ("width", _I), ("history", _P), ("depth_stride", c_size_t), ("depth", _I), ("weights", _P), ("y", _P),
+    ("y_weight", _P), ("next", _P), ("centred", _I), ("norm_weight", _P), ("eps", _F), ("h", _P), ("h_ld", _I), ("table", _P), ("vocab", _I),
+    ("embed_scale", _F), ("ids", _P), ("ids_stride", _I), ("ids_index", _P), ("pos_out", _P), ("side_table", _P), ("side", _P),
+    ("side_layers", _I), ("side_ld", _I), ("side_stride", c_size_t), ("router", _P), ("routing", Routing)])
+AddPartsArgs = _struct("AddPartsArgs", [
+    ("dtype", _I), ("rows", _I), ("width", _I), ("x", _P), ("parts", _P), ("n_parts", _I), ("parts_ld", _I), ("part_f32", _I),
+    ("part_weight", _P), ("weights_ld", _I), ("h", _P), ("h_ld", _I)])
 ExpertWeights = _struct("ExpertWeights", [("W", _P), ("W2", _P), ("K", _I), ("N", _I), ("n_main", _I), ("pair", _I), ("limit", _F), ("slope", _F)])
 ExpertsArgs = _struct("ExpertsArgs", [
     ("dtype", _I), ("rows", _I), ("experts", _I), ("top", _I), ("choices", _I), ("chosen", _P), ("X", _P), ("ld_x", _I),
@@ -92,6 +115,13 @@ SIGNATURES = {
     "pta_expert_lists_size": (c_size_t, [_I, _I, _I, _I]),
     "pta_group_experts": (_I, [_P, _I, _I, _I, _I, _I, _P, _P]),
     "pta_experts": (_I, [POINTER(ExpertsArgs), _P]),
+    "pta_short_conv": (_I, [POINTER(ShortConvArgs), _P]),
+    "pta_ssd_state_floats": (c_size_t, [_I, _I, _I]),
+    "pta_ssd_workspace_bytes": (c_size_t, [POINTER(SsdArgs)]),
+    "pta_ssd": (_I, [POINTER(SsdArgs), _P]),
+    "pta_gated_norm": (_I, [POINTER(GatedNormArgs), _P]),
+    "pta_depth_norm": (_I, [POINTER(DepthNormArgs), _P]),
+    "pta_add_parts": (_I, [POINTER(AddPartsArgs), _P]),
     "pta_mlstm_state_floats": (c_size_t, [_I, _I, _I]),
     "pta_mlstm_workspace_bytes": (c_size_t, [POINTER(MlstmArgs)]),
     "pta_mlstm": (_I, [POINTER(MlstmArgs), _P]),

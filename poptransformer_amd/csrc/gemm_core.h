@@ -21,7 +21,7 @@ struct WideOut {
   float limit, slope;
   const float* bias;        // [n_main] or null, added to the sum (of a pair: to the gate's)
   const float* bias2;       // [n_main] or null, added to the sum of a pair's second weight
-  int sigmoid;              // y = sigmoid(y)
+  int act;                  // PTA_ACT_*
   const void* mul;          // [M, ld] or null, fp32 (mul_f32) or bf16: y = y * mul
   int mul_f32;
   int accumulate;           // Y (fp32) += y
@@ -133,7 +133,12 @@ struct GemmMat {
 __device__ __forceinline__ float wide_value(const WideOut& w, int n, float v) {
   if (w.bias) v += w.bias[n];
   if (w.cap > 0.f) v = w.cap * tanhf(v / w.cap);
-  return w.sigmoid ? 1.0f / (1.0f + expf(-v)) : v;
+  switch (w.act) {
+    case PTA_ACT_GELU_TANH: return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+    case PTA_ACT_RELU_SQUARE: return v > 0.f ? v * v : 0.f;
+    case PTA_ACT_SIGMOID: return 1.0f / (1.0f + expf(-v));
+    default: return v;
+  }
 }
 
 __device__ __forceinline__ float wide_pair_value(const WideOut& w, int n, float g, float u) {

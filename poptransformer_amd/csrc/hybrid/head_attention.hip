@@ -1,9 +1,9 @@
 // Attention over cached keys and values with norms per head, rotation, windows that keep the first positions, chunks, sinks,
-// differential pairs of maps and output gates.
+// differential pairs of maps, output gates, penalties of the distance and short convolutions ahead of it all.
 //
 // The keys a row sees are numbered: first the kept positions, then those from the window's (or chunk's) begin on.  Every kernel
 // works on a stretch of these numbers, so positions nobody sees cost nothing.
-#include "attention.h"
+#include "short_conv.h"
 
 typedef pta_head_attention_args HA;
 
@@ -37,6 +37,11 @@ struct KeyRange {
 __device__ __forceinline__ int ring_row(const HA& a, int p) {
   return p < a.keep ? p : a.keep + (int)((unsigned)(p - a.keep) % (unsigned)(a.ring_len - a.keep));
 }
+// what a distance takes off a score of head h
+template <typename T> __device__ __forceinline__ float log_of(float x);
+template <> __device__ __forceinline__ float log_of<float>(float x) { return logf(x); }
+template <> __device__ __forceinline__ float log_of<bf16>(float x) { return __logf(x); }
+
 __device__ __forceinline__ const float* angles_of(const HA& a, int pos) {
   return a.cos_sin + (size_t)(pos < a.positions ? pos : a.positions - 1) * a.rot;
 }
@@ -163,13 +168,22 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] = 0.f;
   };
-  float qv[NQ][8], wn[8];
+  float qv[NQ][8], wn[8], far1[RG], far2[RG];
   load8(a.q_norm ? a.q_norm + (dk ? d0 : 0) : nullptr, a.q_norm != nullptr, 0, wn);
 #pragma unroll
   for (int h = 0; h < RG; ++h) {
     const int head = g * R + (hg * RG + h < R ? hg * RG + h : R - 1);               // (a duplicate that is not stored)
 #pragma unroll
     for (int t = 0; t < MAPS; ++t) load8(proj_q + (head * MAPS + t) * D + (dk ? d0 : 0), true, 8, qv[h * MAPS + t]);
+    far1[h] = a.far1 ? a.far1[head] : 0.f;
+    far2[h] = a.far1 ? a.far2[head] : 0.f;
+    if constexpr (MAPS == 1) {
+      if (a.conv.ring && fused) {
+        const int c0 = head * D + (dk ? d0 : 0);
+        if (split == 0 && grp == 0 && dk && hg * RG + h < R) store8(conv_place<T>(a.conv, slot, i, c0), qv[h]);
+        conv8<T>(a.conv, slot, i, c0, qv[h]);
+      }
+    }
   }
 #pragma unroll
   for (int q = 0; q < NQ; ++q) {
@@ -187,8 +201,8 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
 #pragma unroll
     for (int e = 0; e < 8; ++e) o[q][e] = 0.f;
   }
-  // U keys of this lane group, those with `seen`
-  auto step = [&](auto count, const auto& kv, const auto& vv, const auto& seen) {
+  // U keys of this lane group, those with `seen`, `back` positions before the row
+  auto step = [&](auto count, const auto& kv, const auto& vv, const auto& seen, const auto& back) {
     constexpr int U = decltype(count)::value;
 #pragma unroll
     for (int q = 0; q < NQ; ++q) {
@@ -199,6 +213,7 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
 #pragma unroll
         for (int e = 0; e < 8; ++e) t = __builtin_fmaf(qv[q][e], kv[u][q % MAPS][e], t);
         t = group_sum<LPK>(t);
+        if (a.far1) t -= far1[q / MAPS] * log_of<T>(1.0f + far2[q / MAPS] * back[u]);
         s[u] = seen[u] ? t : -INFINITY;
         top = fmaxf(top, s[u]);
       }
@@ -219,15 +234,18 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
   for (int nb = n0; nb < n_end; nb += NG * HR_KEYS) {
     float kv[HR_KEYS][MAPS][8], vv[HR_KEYS][8];
     bool seen[HR_KEYS];
+    float back[HR_KEYS];
 #pragma unroll
     for (int u = 0; u < HR_KEYS; ++u) {
-      seen[u] = nb + u * NG + grp < n_end;
+      const int n = nb + u * NG + grp;
+      seen[u] = n < n_end;
+      back[u] = seen[u] ? (float)(i - keys.position(n)) : 0.f;
 #pragma unroll
       for (int t = 0; t < MAPS; ++t) kr[u][t].unpack(kv[u][t]);
       vr[u].unpack(vv[u]);
     }
     if (nb + NG * HR_KEYS < n_end) fetch(nb + NG * HR_KEYS);
-    step(std::integral_constant<int, HR_KEYS>{}, kv, vv, seen);
+    step(std::integral_constant<int, HR_KEYS>{}, kv, vv, seen, back);
   }
   if (own) {
     float kv[1][MAPS][8], vv[1][8];
@@ -236,9 +254,23 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     load8(reinterpret_cast<const T*>(a.v) + (size_t)r * a.ld + g * E + (dv ? d0 : 0), true, 8, vv[0]);
     const bool put = hg == 0 && grp == 0;
     const int row = ring_row(a, i);
+    if constexpr (MAPS == 1) {
+      if (a.conv.ring) {
+        const int c0 = (a.H + a.G) * D + g * E + (dv ? d0 : 0);
+        if (put && dv) store8(conv_place<T>(a.conv, slot, i, c0), vv[0]);
+        conv8<T>(a.conv, slot, i, c0, vv[0]);
+      }
+    }
 #pragma unroll
     for (int t = 0; t < MAPS; ++t) {
       load8(pk + t * D, true, 8, kv[0][t]);
+      if constexpr (MAPS == 1) {
+        if (a.conv.ring) {
+          const int c0 = (a.H + g) * D + (dk ? d0 : 0);
+          if (put && dk) store8(conv_place<T>(a.conv, slot, i, c0), kv[0][t]);
+          conv8<T>(a.conv, slot, i, c0, kv[0][t]);
+        }
+      }
       zero_past(dk, kv[0][t]);
       norm_rotate<LPK>(a, wn, a.k_norm != nullptr, d0, cs, kv[0][t]);
       if (put && dk) store8(const_cast<T*>(kring) + ((size_t)t * a.ring_len + row) * D, kv[0][t]);
@@ -247,7 +279,8 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     }
     if (put && dv) store8(const_cast<T*>(vring) + (size_t)row * E, vv[0]);
     const bool seen[1] = {grp == 0};
-    step(std::integral_constant<int, 1>{}, kv, vv, seen);
+    const float back[1] = {0.f};
+    step(std::integral_constant<int, 1>{}, kv, vv, seen, back);
   }
 #pragma unroll
   for (int q = 0; q < NQ; ++q) {
@@ -360,6 +393,8 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
   extern __shared__ __align__(16) unsigned char head_tile_lds[];
   bf16* sk = reinterpret_cast<bf16*>(head_tile_lds);                   // [MAPS][HT_KEYS][KS]
   bf16* sv = sk + MAPS * HT_KEYS * KS;                                 // [HT_KEYS][VS]
+  // of the distance from row n of the workgroup's to key k of a step, at k - n + (rows - 1): what is taken off the score
+  __shared__ float far[HT_KEYS + 4 * RW];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lg = lane >> 4, lc = lane & 15;
   const int head = blockIdx.x, tile = blockIdx.y, skip = (int)blockIdx.z * 4 * RW;
   const int D = a.D, E = a.E, g = head / (a.H / a.G);
@@ -435,6 +470,7 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
   f32x4 o[QW][DVT];
   float mx[QW], l[QW];
   const float sink = a.sink ? a.sink[head] * LOG2E : 0.f;
+  const float far1 = a.far1 ? a.far1[head] : 0.f, far2 = a.far1 ? a.far2[head] : 0.f;
 #pragma unroll
   for (int w = 0; w < QW; ++w) {
     mx[w] = a.sink ? sink : -1e30f;
@@ -451,6 +487,10 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
       for (int m = 0; m < DKT; ++m) *reinterpret_cast<u32x4*>(sk + (t * HT_KEYS + my_key) * KS + m * 32 + my_piece) = kf[t][m];
 #pragma unroll
     for (int m = 0; m < VIT; ++m) *reinterpret_cast<u32x4*>(sv + my_key * VS + m * 32 + my_piece) = vf[m];
+    if (a.far1 && (int)threadIdx.x < HT_KEYS + 4 * RW - 1) {           // (positions follow each other: keep = 0)
+      const int back = p0 + 4 * RW - 1 - keys.position(nt) - (int)threadIdx.x;
+      far[threadIdx.x] = far1 * __log2f(1.0f + far2 * (float)(back > 0 ? back : 0));
+    }
     __syncthreads();
     if (nt + HT_KEYS < total) fetch(nt + HT_KEYS);
     const int j_first = keys.position(nt), j_last = keys.position(nt + HT_KEYS - 1);
@@ -468,6 +508,16 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
         for (int u = 0; u < MAPS; ++u) kv[u] = *reinterpret_cast<const bf16x8*>(sk + (u * HT_KEYS + t * 16 + lc) * KS + c * 32 + lg * 8);
 #pragma unroll
         for (int w = 0; w < QW; ++w) s[w][t] = mma(kv[MAPS == 2 ? w : 0], qf[w][c], s[w][t]);
+      }
+    }
+    if (a.far1) {
+#pragma unroll
+      for (int w = 0; w < QW; ++w) {
+        const float* f = far + lg * 4 + 4 * RW - 1 - (MAPS == 2 ? wave * 16 + lc : (wave * QW + w) * 16 + lc);
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) s[w][t][e] -= f[t * 16 + e];
       }
     }
     if (!whole) {
@@ -581,6 +631,7 @@ static int check_head(const HA* args, const char* name) {
   PTA_REQUIRE(a.rot == 0 || (a.rot > 0 && a.rot % 8 == 0 && a.rot <= a.D && a.cos_sin && a.positions > 0), "%s: %d rotated features", name, a.rot);
   PTA_REQUIRE(a.window > 0 && a.keep >= 0 && a.chunk >= 0 && (a.chunk == 0 || a.keep == 0), "%s: window %d, keep %d, chunk %d", name, a.window,
               a.keep, a.chunk);
+  PTA_REQUIRE(!a.far1 || (a.far2 && a.keep == 0), "%s: a penalty of the distance needs both of its numbers, and no kept positions", name);
   PTA_REQUIRE(a.keys && a.values && pta_aligned(a.keys, 16) && pta_aligned(a.values, 16) && a.ring_len > a.keep && a.slot && a.pos,
               "%s: the cache (%d rows) or the rows' places are missing", name, a.ring_len);
   return PTA_OK;
@@ -696,6 +747,13 @@ extern "C" int pta_head_decode(const HA* args, pta_stream_t stream) {
   if (rc) return rc;
   const HA& a = *args;
   PTA_REQUIRE(a.splits >= 1 && a.splits <= 64, "%s: splits %d (1 .. 64)", name, a.splits);
+  if (a.conv.ring) {
+    rc = check_conv(a.conv, name);
+    if (rc) return rc;
+    const size_t es = a.dtype == PTA_BF16 ? 2 : 4;
+    PTA_REQUIRE(a.maps == 1 && !a.conv.silu && a.conv.channels == (a.H + a.G) * a.D + a.G * a.E && (const char*)a.k == (const char*)a.q + es * a.H * a.D &&
+                (const char*)a.v == (const char*)a.k + es * a.G * a.D, "%s: the convolution takes q | k | v of single maps", name);
+  }
   const size_t need = pta_head_attention_workspace_bytes(a.rows, a.H, a.maps, a.E, a.splits);
   PTA_REQUIRE(a.splits == 1 || (a.workspace && a.workspace_bytes >= need), "%s: the workspace needs %zu bytes", name, need);
   hipStream_t s = (hipStream_t)stream;

@@ -11,6 +11,8 @@ __device__ __forceinline__ int position_of(const LA& a, int r) {
   return p < 0 ? 0 : (p >= a.positions ? a.positions - 1 : p);
 }
 
+__device__ __forceinline__ float head_gate(const LA& a, int r, int head) { return a.gate ? sigmoid_f32(a.gate[(size_t)r * a.H + head]) : 1.0f; }
+
 // ------------------------------------------------------------------------------------------
 // Norms of the two latents, and the row's cache entry.
 // ------------------------------------------------------------------------------------------
@@ -444,7 +446,12 @@ __global__ __launch_bounds__(256) void latent_values_kernel(LA a, int blocks, in
 #pragma unroll
     for (int e = 0; e < 4; ++e) y[e] += t[e];
   }
-  const float g = sigmoid_f32(a.gate[(size_t)row * a.H + head]);
+  const float g = head_gate(a, row, head);
+  if (a.feature_gate) {
+    const bf16x4 fg = *reinterpret_cast<const bf16x4*>(reinterpret_cast<const bf16*>(a.feature_gate) + (size_t)row * a.gate_ld + head * a.E + ch);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) y[e] *= sigmoid_f32((float)fg[e]);
+  }
   bf16x4 yb;
 #pragma unroll
   for (int e = 0; e < 4; ++e) yb[e] = (bf16)(y[e] * g);
@@ -467,13 +474,14 @@ __global__ __launch_bounds__(256) void latent_values_vector_kernel(LA a) {
     x_row[c] = (float)(T)x;
   }
   __syncthreads();
-  const float g = sigmoid_f32(a.gate[(size_t)r * a.H + head]);
+  const float g = head_gate(a, r, head);
+  const T* fg = a.feature_gate ? reinterpret_cast<const T*>(a.feature_gate) + (size_t)r * a.gate_ld + head * a.E : nullptr;
   for (int n = wave; n < a.E; n += 4) {
     const T* w = reinterpret_cast<const T*>(a.uv) + ((size_t)head * a.E + n) * a.R;
     float s = 0.f;
     for (int c = lane; c < a.R; c += 64) s = __builtin_fmaf((float)w[c], x_row[c], s);
     s = wave_sum(s);
-    if (lane == 0) reinterpret_cast<T*>(a.out)[((size_t)r * a.H + head) * a.E + n] = (T)(s * g);
+    if (lane == 0) reinterpret_cast<T*>(a.out)[((size_t)r * a.H + head) * a.E + n] = (T)(fg ? s * g * sigmoid_f32((float)fg[n]) : s * g);
   }
 }
 
@@ -637,14 +645,21 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(LA a) {
     tot += __shfl_xor(tot, 32, 64);
     const int n = (wave * QW + w) * 16 + lc;
     if (n >= count) continue;
-    const float f = sigmoid_f32(a.gate[(size_t)(row0 + n) * a.H + head]) / tot;
+    const float f = head_gate(a, row0 + n, head) / tot;
+    const bf16* fg = a.feature_gate ? reinterpret_cast<const bf16*>(a.feature_gate) + (size_t)(row0 + n) * a.gate_ld + head * E : nullptr;
     bf16* out = reinterpret_cast<bf16*>(a.out) + ((size_t)(row0 + n) * a.H + head) * E;
 #pragma unroll
     for (int t = 0; t < DVT; ++t) {
       if (t * 16 >= E) break;
       bf16x4 y;
+      if (fg) {
+        const bf16x4 gv = *reinterpret_cast<const bf16x4*>(fg + t * 16 + lg * 4);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) y[e] = (bf16)(o[w][t][e] * f);
+        for (int e = 0; e < 4; ++e) y[e] = (bf16)(o[w][t][e] * f / (1.0f + __expf(-(float)gv[e])));
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = (bf16)(o[w][t][e] * f);
+      }
       *reinterpret_cast<bf16x4*>(out + t * 16 + lg * 4) = y;
     }
   }
@@ -657,6 +672,8 @@ static int check_latent(const LA& a, const char* name) {
   PTA_REQUIRE(a.D > 0 && a.D % 32 == 0 && a.P > 0 && a.P % 32 == 0 && a.R > 0 && a.R % 32 == 0 && a.E > 0 && a.E % 16 == 0,
               "%s: sizes D %d, P %d, R %d must be multiples of 32 and E %d of 16", name, a.D, a.P, a.R, a.E);
   PTA_REQUIRE(a.R <= 256 * LV_FEATURES && a.R + a.P <= 16000 && a.D <= 16000, "%s: latent of %d (at most %d)", name, a.R, 256 * LV_FEATURES);
+  PTA_REQUIRE(!a.feature_gate || (pta_aligned(a.feature_gate, 16) && a.gate_ld % 8 == 0 && a.gate_ld >= a.H * a.E), "%s: unaligned gate, or rows of %d",
+              name, a.gate_ld);
   PTA_REQUIRE(a.cos_sin && a.positions > 0 && a.ring && pta_aligned(a.ring, 16) && a.ring_len > 0 && a.slot && a.pos,
               "%s: positions, the cache or the rows' places are missing", name);
   return PTA_OK;
@@ -746,7 +763,7 @@ static int launch_latent_values(const LA& a, int each, hipStream_t s) {
 
 extern "C" int pta_latent_values(const LA* args, pta_stream_t stream) {
   LATENT_ENTRY("pta_latent_values")
-  PTA_REQUIRE(a.part_o && a.part_ml && a.uv && a.gate && a.out && a.splits >= 1 && a.splits <= 64,
+  PTA_REQUIRE(a.part_o && a.part_ml && a.uv && a.out && a.splits >= 1 && a.splits <= 64,
               "pta_latent_values: null pointer, or splits %d (1 .. 64)", a.splits);
   PTA_REQUIRE(pta_aligned(a.part_o, 16) && pta_aligned(a.uv, 16) && pta_aligned(a.out, 16), "pta_latent_values: unaligned operand");
   if (a.dtype == PTA_BF16) {
@@ -783,7 +800,7 @@ static void launch_latent_tiles(const LA& a, hipStream_t s) {
 extern "C" int pta_latent_tiles(const LA* args, pta_stream_t stream) {
   LATENT_ENTRY("pta_latent_tiles")
   PTA_REQUIRE(pta_latent_tiles_fit(a.dtype, a.D, a.P, a.E), "pta_latent_tiles: bf16 with D + P and E up to 256");
-  PTA_REQUIRE(a.q && a.kv && a.key_rot && a.gate && a.out && a.window > 0, "pta_latent_tiles: null pointer, or window %d", a.window);
+  PTA_REQUIRE(a.q && a.kv && a.key_rot && a.out && a.window > 0, "pta_latent_tiles: null pointer, or window %d", a.window);
   PTA_REQUIRE(a.tile_row && a.tile_count && a.tile_key && a.tiles > 0 && a.tiles <= 65535, "pta_latent_tiles: %d tiles (1 .. 65535)", a.tiles);
   PTA_REQUIRE(pta_aligned(a.q, 16) && pta_aligned(a.kv, 16) && pta_aligned(a.key_rot, 16) && pta_aligned(a.out, 16),
               "pta_latent_tiles: unaligned operand");

@@ -149,6 +149,7 @@ static int check_wide(const pta_wide_linear_args& a, const char* name) {
               "%s: n_main %d (ld %d) and tail %d do not fit %d channels", name, a.n_main, a.ld, a.tail_count, a.N);
   PTA_REQUIRE(a.tail_count == 0 || (a.tail && !pair), "%s: a tail needs its buffer, and a single weight", name);
   PTA_REQUIRE(a.pair != PTA_PAIR_CLAMPED || a.limit > 0.f, "%s: the clamped pair needs a positive limit", name);
+  PTA_REQUIRE(a.act >= PTA_ACT_NONE && a.act <= PTA_ACT_SIGMOID, "%s: unknown activation %d", name, a.act);
   PTA_REQUIRE(pair || !a.bias2, "%s: a second bias belongs to a pair", name);
   PTA_REQUIRE(!a.accumulate || a.out_f32 || a.dtype == PTA_FP32, "%s: only fp32 results accumulate", name);
   PTA_REQUIRE(!a.mul || pta_aligned(a.mul, 16), "%s: the multiplier must be 16-byte aligned", name);
@@ -175,7 +176,7 @@ static GemmMat wide_matrix(const pta_wide_linear_args& a, const void* W) {
   w.slope = a.slope;
   w.bias = a.bias;
   w.bias2 = a.bias2;
-  w.sigmoid = a.sigmoid;
+  w.act = a.act;
   w.mul = a.mul;
   w.mul_f32 = a.dtype == PTA_FP32;
   w.accumulate = a.accumulate;

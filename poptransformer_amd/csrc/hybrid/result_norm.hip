@@ -1,63 +1,9 @@
 // A residual that takes normed results: x <- x + rms_norm(y) * weight, with what follows in the same launch: the rounded row that
 // the next sublayer reads, or the model's norm of it, and the routing of the row to its experts.
 #include "attention.h"
+#include "routing.h"
 
 typedef pta_result_norm_args RN;
-
-// Routing of row r by THREADS threads, of which this is `tid`: z holds the logits (in LDS, visible to all; overwritten).  Expert e's
-// place among the chosen is the number of larger scores (of equal ones the first comes first), so no choice waits for another.
-// The whole workgroup calls it, each group of THREADS for a row of its own; with `store` unset nothing is kept.
-template <int THREADS>
-__device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r, int tid, bool store) {
-  const int E = g.experts, choices = g.top + g.shared;
-  int32_t* chosen = g.chosen + (size_t)r * choices;
-  float* weights = g.weights + (size_t)r * choices;
-  constexpr int PER = (PTA_MAX_EXPERTS + THREADS - 1) / THREADS;
-  int rank[PER];
-  float p[PER];
-#pragma unroll
-  for (int k = 0; k < PER; ++k) {
-    const int e = tid + k * THREADS;
-    rank[k] = E;
-    p[k] = 0.f;
-    if (e >= E) continue;
-    const float mine = z[e];
-    float top = mine;
-    int above = 0;
-#pragma unroll 8
-    for (int j = 0; j < E; ++j) {
-      const float v = z[j];
-      top = fmaxf(top, v);
-      above += v > mine || (v == mine && j < e);
-    }
-    rank[k] = above;
-    p[k] = expf(mine - top);
-  }
-  const float shared = g.shared && tid == 0 ? sigmoid_f32(z[E]) : 0.f;
-  __syncthreads();
-#pragma unroll
-  for (int k = 0; k < PER; ++k)
-    if (tid + k * THREADS < E) z[tid + k * THREADS] = p[k];
-  __syncthreads();
-  bool any = false;
-#pragma unroll
-  for (int k = 0; k < PER; ++k) any = any || rank[k] < g.top;
-  if (any && store) {
-    float sum = 0.f;
-#pragma unroll 8
-    for (int j = 0; j < E; ++j) sum += z[j];
-#pragma unroll
-    for (int k = 0; k < PER; ++k)
-      if (rank[k] < g.top) {
-        chosen[rank[k]] = tid + k * THREADS;
-        weights[rank[k]] = p[k] / sum * g.scale;
-      }
-  }
-  if (g.shared && store && tid == 0) {
-    chosen[g.top] = E;
-    weights[g.top] = shared;
-  }
-}
 
 // Many rows (bf16): sixteen of them per workgroup, whose waves share the features; BLOCKS * 16 logits of each at a time.
 constexpr int RR_WAVES = 8;
@@ -118,7 +64,7 @@ __global__ __launch_bounds__(RR_WAVES * 64) void route_rows_kernel(const bf16* h
 }
 
 __global__ __launch_bounds__(64) void route_kernel(const float* logits, pta_routing g) {
-  __shared__ float z[PTA_MAX_EXPERTS + 1];
+  __shared__ float z[ROUTE_FLOATS];
   const int n = g.experts + g.shared;
   for (int c = threadIdx.x; c < n; c += 64) z[c] = logits[(size_t)blockIdx.x * n + c];
   __syncthreads();
@@ -134,7 +80,7 @@ __global__ __launch_bounds__(THREADS) void result_norm_kernel(RN a) {
   constexpr int WAVES = THREADS / 64;
   extern __shared__ __align__(16) float u_row[];             // the result, then what h holds
   __shared__ float red[2][WAVES];
-  __shared__ float z[PTA_MAX_EXPERTS + 1];
+  __shared__ float z[ROUTE_FLOATS];
   __shared__ float pw[64];
   const int r = blockIdx.x, d = a.width;
   float* x = a.x + (size_t)r * d;
@@ -252,32 +198,8 @@ __global__ __launch_bounds__(THREADS) void result_norm_kernel(RN a) {
   }
   for (int c = d + threadIdx.x; c < a.h_ld; c += THREADS) h[c] = (T)0.0f;
   if (!a.router) return;
-  // one wave per expert at a time
-  for (int c = d + threadIdx.x; c < a.h_ld; c += THREADS) u_row[c] = 0.f;
-  __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, n = a.routing.experts + a.routing.shared;
-  for (int e = wave; e < n; e += WAVES) {
-    const T* w = reinterpret_cast<const T*>(a.router) + (size_t)e * a.h_ld;
-    float s = 0.f;
-#pragma unroll 4
-    for (int c = lane * 8; c < a.h_ld; c += 512) {
-      float t[8];
-      load8(w + c, true, 8, t);
-#pragma unroll
-      for (int k = 0; k < 8; ++k) s = __builtin_fmaf(t[k], u_row[c + k], s);
-    }
-    s = wave_total_dpp(s);
-    if (lane == 0) z[e] = s;
-  }
-  __syncthreads();
+  router_logits<T, WAVES>(a.router, a.h_ld, d, u_row, a.routing, z);
   route_row<THREADS>(a.routing, z, r, threadIdx.x, true);
-}
-
-static int check_routing(const pta_routing& g, const char* name) {
-  PTA_REQUIRE(g.experts >= 1 && g.experts <= PTA_MAX_EXPERTS && g.top >= 1 && g.top <= g.experts && (g.shared == 0 || g.shared == 1),
-              "%s: top %d of %d experts (at most %d)", name, g.top, g.experts, PTA_MAX_EXPERTS);
-  PTA_REQUIRE(g.chosen && g.weights, "%s: the routing has nowhere to go", name);
-  return PTA_OK;
 }
 
 extern "C" int pta_route(const float* logits, int rows, const pta_routing* routing, pta_stream_t stream) {
@@ -295,7 +217,7 @@ extern "C" int pta_route_rows(const uint16_t* h, int ld, int rows, const void* r
   PTA_REQUIRE(ld > 0 && ld % 8 == 0 && pta_aligned(h, 16) && pta_aligned(router, 16), "%s: rows of %d, or unaligned operands", name, ld);
   const int rc = check_routing(*routing, name);
   if (rc) return rc;
-  const int z_ld = routing->experts + routing->shared + 1;
+  const int z_ld = route_floats(*routing);
   const size_t smem = (size_t)16 * z_ld * sizeof(float);
   auto launch = [&](auto blocks) {
     constexpr int B = decltype(blocks)::value;
@@ -305,7 +227,7 @@ extern "C" int pta_route_rows(const uint16_t* h, int ld, int rows, const void* r
                        reinterpret_cast<const bf16*>(h), ld, rows, reinterpret_cast<const bf16x8*>(router), *routing, z_ld);
     return PTA_OK;
   };
-  const int blocks = (z_ld + 14) / 16;
+  const int blocks = (routing->experts + routing->shared + 15) / 16;
   const int launched = blocks == 1   ? launch(std::integral_constant<int, 1>{})
                        : blocks == 2 ? launch(std::integral_constant<int, 2>{})
                        : blocks == 3 ? launch(std::integral_constant<int, 3>{})

@@ -266,7 +266,7 @@ def _executor_dtype():
 
 def _build_parallel(facts, topk=1):
     """As _build_hybrid, for layers with latent attention whose sublayers stand side by side."""
-    from .hybrid import BiasedSwiGLU, HybridLayer, HybridSpec, LatentMixer
+    from .hybrid import BiasedSwiGLU, HybridLayer, HybridSpec, LatentMixer, Rotation
     from .loader import parallel_weights
     from .parallel import ParallelDecoder
     const = _const_reader(facts)
@@ -278,8 +278,8 @@ def _build_parallel(facts, topk=1):
         uk, uv, uq = (_need(facts, mix + n) for n in ("uk", "uv", "uq"))
         dim = uk.shape[0] // heads
         mixer = LatentMixer(heads, dim, uq.shape[0] // heads - dim, uv.shape[0] // heads, uq.shape[1], uk.shape[1],
-                            float(const(f"l{i}.scale")), int(const(f"l{i}.window")) or None, float(const(f"l{i}.rot_base")),
-                            int(const(f"l{i}.rot_dims")), source if source != i else None)
+                            float(const(f"l{i}.scale")), int(const(f"l{i}.window")) or None,
+                            Rotation(float(const(f"l{i}.rot_base")), int(const(f"l{i}.rot_dims"))), source if source != i else None)
         ff = f"l{i}.mlp.gate"
         layers.append(HybridLayer(mixer, BiasedSwiGLU(_need(facts, ff).shape[0]) if facts.has(ff) else None, i, shift=True))
     if not layers:

@@ -1,6 +1,7 @@
 """Executor of decoders that mix windowed attention with recurrent (matrix memory) layers over fp32 residual streams; the
-mixers, feed-forwards and the row handling that `parallel` uses for layers whose sublayers stand side by side, and
-`result_norm` for layers whose residual takes the norms of their sublayers' results.
+mixers, feed-forwards and the row handling that `parallel` uses for layers whose sublayers stand side by side, `result_norm`
+for layers whose residual takes the norms of their sublayers' results, and `depth` for layers whose results are averaged over
+the depths.  The mixers that several of them run are in `mixers`.
 
 The model is a list of layers, each described by its mixer, its feed-forward (or none) and the layer whose tensors it
 uses.  One forward function serves everything: it takes the ROWS of a pass (row = one token of the sequence in a slot, at
@@ -72,8 +73,8 @@ class MemoryMixer:
 @dataclass
 class LatentMixer:
     """Attention over the last `window` positions (None: all) whose keys and values are made from a cached latent of kv_rank
-    and one rotated key part shared by the heads; queries through a latent of q_rank, one output gate per head.  `source`: the
-    layer whose cache is read (None: the layer's own)."""
+    and one key part shared by the heads, which `rot` turns (its first features, the rest of it passes as it is); queries through a
+    latent of q_rank, one output gate per "head" or "feature".  `source`: the layer whose cache is read (None: the layer's own)."""
     heads: int
     dim: int
     rot_dim: int
@@ -82,9 +83,9 @@ class LatentMixer:
     kv_rank: int
     scale: float
     window: Optional[int]
-    rot_base: float
-    rot_turned: int                  # rotated features of rot_dim; the rest of it passes as it is
+    rot: "Rotation"
     source: Optional[int] = None
+    gate: str = "head"
     kind = "latent"
 
     @property
@@ -103,17 +104,21 @@ class LatentMixer:
 
     def pairs(self):
         """Order of the rotated features in which the two of a pair follow each other."""
-        half = self.rot_turned // 2
-        turned = np.arange(self.rot_turned).reshape(2, half).T.reshape(-1)
-        return np.concatenate([turned, np.arange(self.rot_turned, self.rot_dim)])
+        return self.rot.pairs(self.rot_dim)
 
     def angles(self, positions):
         """[positions, P / 2, (cos, sin)] of those pairs."""
-        f = np.zeros(HK.pad32(self.rot_dim) // 2)
-        half = self.rot_turned // 2
-        f[:half] = float(self.rot_base) ** (-2.0 * np.arange(half) / self.rot_turned)
-        a = np.arange(positions)[:, None] * f
-        return np.stack([np.cos(a), np.sin(a)], -1).astype(np.float32)
+        return self.rot.angles(positions, HK.pad32(self.rot_dim) // 2)
+
+    def numbers(self):
+        """What the tensors' shapes do not tell but the rotation, as a flat list, which `LatentMixer.of` reads."""
+        return [self.heads, self.scale, self.window or 0, -1 if self.source is None else self.source, ("head", "feature").index(self.gate)]
+
+    @staticmethod
+    def of(numbers, dim, rot_dim, vdim, q_rank, kv_rank, rot):
+        heads, scale, window, source, gate = (float(v) for v in numbers)
+        return LatentMixer(int(heads), dim, rot_dim, vdim, q_rank, kv_rank, scale, int(window) or None, rot, int(source) if source >= 0 else None,
+                           ("head", "feature")[int(gate)])
 
 
 @dataclass
@@ -157,11 +162,12 @@ class Rotation:
             turned = turned.reshape(2, -1).T.reshape(-1)
         return np.concatenate([turned, np.arange(self.dims, size)])
 
-    def angles(self, positions):
-        """fp32 [positions, pairs, (cos, sin)] of those pairs; whole pieces of eight features, the ones past `dims` stay as they are."""
+    def angles(self, positions, pairs=None):
+        """fp32 [positions, pairs, (cos, sin)] of those pairs, by default of whole pieces of eight features; the ones past `dims` stay
+        as they are."""
         f, amplitude = self.frequencies()
         a = np.arange(positions)[:, None] * f
-        out = np.zeros((positions, HK.pad8(self.dims) // 2, 2), np.float32)
+        out = np.zeros((positions, HK.pad8(self.dims) // 2 if pairs is None else pairs, 2), np.float32)
         out[..., 0] = 1.0
         out[:, :len(f), 0], out[:, :len(f), 1] = np.cos(a) * amplitude, np.sin(a) * amplitude
         return out
@@ -185,18 +191,22 @@ class HeadMixer:
     sink: bool = False               # a learned score per head in the softmax's denominator
     gate: Optional[str] = None       # sigmoid gate of the result, one number per "head" or per "feature"
     diff: Optional[float] = None     # two maps per head, the second subtracted; part of their weight, and 1 - diff of the result
+    norms: bool = True               # RMS norms of queries and keys, per head
+    far: bool = False                # far1 ln(1 + far2 distance) is taken off the scores, with two numbers per head
+    taps: int = 0                    # queries, keys and values pass a short convolution over so many tokens (0: none)
     kind = "heads"
 
     def numbers(self):
         """Everything but the feature sizes, the biases and the rotation as a flat list, which `HeadMixer.of` reads."""
         return [self.heads, self.kv_heads, self.scale, self.window or 0, self.keep, self.chunk or 0, self.keys_are_values, self.sink,
-                (None, "head", "feature").index(self.gate), *(() if self.diff is None else (self.diff,))]
+                (None, "head", "feature").index(self.gate), self.norms, self.far, self.taps, *(() if self.diff is None else (self.diff,))]
 
     @staticmethod
     def of(numbers, dim, vdim, biases, rot):
-        heads, kv_heads, scale, window, keep, chunk, keys_are_values, sink, gate, *diff = (float(v) for v in numbers)
+        heads, kv_heads, scale, window, keep, chunk, keys_are_values, sink, gate, norms, far, taps, *diff = (float(v) for v in numbers)
         return HeadMixer(int(heads), int(kv_heads), dim, vdim, scale, rot, int(window) or None, int(keep), int(chunk) or None,
-                         bool(keys_are_values), biases, bool(sink), (None, "head", "feature")[int(gate)], diff[0] if diff else None)
+                         bool(keys_are_values), biases, bool(sink), (None, "head", "feature")[int(gate)], diff[0] if diff else None, bool(norms),
+                         bool(far), int(taps))
 
     def visible(self, positions):
         """bool [position of the query, distance back to the key]."""
@@ -222,6 +232,11 @@ class HeadMixer:
         return HK.pad8(self.vdim)
 
     @property
+    def conv_channels(self):
+        """Channels of the convolution: queries, keys and values, as stored."""
+        return (self.heads + self.kv_heads) * self.maps * self.stored_dim + self.kv_heads * self.stored_vdim
+
+    @property
     def span(self):
         """Most positions, besides the kept ones, that one sees."""
         return min(self.window or 1 << 30, self.chunk or 1 << 30)
@@ -229,6 +244,49 @@ class HeadMixer:
     @property
     def out_channels(self):
         return self.heads * self.stored_vdim
+
+
+@dataclass
+class StateSpaceMixer:
+    """Mamba-2: a state of dim x vdim per head, keys and queries (b and c) shared by the heads of a group; x, b and c pass a short
+    convolution over `taps` tokens with silu; the result times silu of a gate, normed in norm_parts equal parts."""
+    heads: int
+    groups: int
+    dim: int
+    vdim: int
+    taps: int
+    norm_parts: int
+    kind = "ssd"
+
+    def numbers(self):
+        """The fields as a flat list, which `StateSpaceMixer.of` reads."""
+        return [self.heads, self.groups, self.dim, self.vdim, self.taps, self.norm_parts]
+
+    @staticmethod
+    def of(numbers):
+        return StateSpaceMixer(*(int(v) for v in numbers))
+
+    @property
+    def stored_dim(self):
+        return HK.pad8(self.dim)
+
+    @property
+    def stored_vdim(self):
+        return HK.pad8(self.vdim)
+
+    @property
+    def out_channels(self):
+        return self.heads * self.stored_vdim
+
+    @property
+    def conv_channels(self):
+        return self.out_channels + 2 * self.groups * self.stored_dim
+
+
+@dataclass
+class SquaredReLU:
+    """relu(u)^2 between the up and the down projection."""
+    ff: int
 
 
 @dataclass
@@ -253,13 +311,33 @@ class ClampedGLU:
 
 @dataclass
 class Experts:
-    """Mixture of experts: of `count` feed-forwards every token has the `top` with the largest router softmax scores, weighted by
-    score * scale; `shared` runs for every token, weighted by a sigmoid of its own."""
+    """Mixture of experts: of `count` feed-forwards every token has the `top` with the largest router scores, weighted by
+    score * scale; `shared` runs for every token, weighted by a sigmoid of its own.  Scores are the router's "softmax" or "sigmoid";
+    sigmoid scores may be `corrected` for the choice, and experts be chosen from the `keep` best of equal `groups` of neighbours only."""
     count: int
     top: int
     scale: float
-    expert: ClampedGLU
+    expert: object                   # ClampedGLU or SwiGLU
     shared: Optional[ClampedGLU] = None
+    score: str = "softmax"
+    corrected: bool = False
+    groups: int = 1
+    keep: int = 1
+    share: bool = False              # weights are shares of the chosen scores' sum
+
+    @property
+    def routing_key(self):
+        return self.count, self.top, self.shared is not None, self.scale, self.score, self.groups, self.keep, self.share
+
+    def numbers(self):
+        """Everything but the feed-forwards as a flat list, which `Experts.of` reads."""
+        return [self.count, self.top, self.scale, ("softmax", "sigmoid").index(self.score), self.corrected, self.groups, self.keep, self.share]
+
+    @staticmethod
+    def of(numbers, expert, shared=None):
+        count, top, scale, score, corrected, groups, keep, share = (float(v) for v in numbers)
+        return Experts(int(count), int(top), scale, expert, shared, ("softmax", "sigmoid")[int(score)], bool(corrected), int(groups), int(keep),
+                       bool(share))
 
 
 @dataclass
@@ -290,6 +368,7 @@ class HybridSpec:
     dtype: str = "bfloat16"          # or float32: everything in true 32-bit
     norm_groups: int = 1             # parallel layers: equal parts of the width with a norm of their own
     positions: Optional[int] = None  # parallel layers: rows of the position table
+    side_dim: int = 0                # depth-averaged layers: features of the token's own part of every layer
 
 
 @dataclass

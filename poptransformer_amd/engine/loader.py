@@ -251,7 +251,7 @@ def hybrid_weights(tensors, spec, device="cuda"):
 # ----------------------------------------------------------------------------------- layers with sublayers side by side
 def latent_layers(layers):
     """The `layers` list of a configuration with latent attention -> [HybridLayer]."""
-    from .hybrid import BiasedSwiGLU, HybridLayer, LatentMixer
+    from .hybrid import BiasedSwiGLU, HybridLayer, LatentMixer, Rotation
     out = []
     for i, c in enumerate(layers):
         if c["type"] != "latent_attention":
@@ -261,12 +261,12 @@ def latent_layers(layers):
             raise ValueError(f"layer {i}: {rot['dims']} rotated features of {m['rot_dim']}")
         source = m.get("kv_from")
         mixer = LatentMixer(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["q_rank"], m["kv_rank"], float(m["scale"]),
-                            (m.get("mask") or {}).get("size"), float(rot["base"]), rot["dims"], source)
+                            (m.get("mask") or {}).get("size"), Rotation(float(rot["base"]), rot["dims"]), source)
         if source is not None:
             if not 0 <= source < i or out[source].mixer.source is not None:
                 raise ValueError(f"layer {i}: kv_from {source} names no earlier layer with a cache of its own")
             o = out[source].mixer
-            if (o.kv_rank, o.rot_dim, o.rot_base, o.rot_turned) != (mixer.kv_rank, mixer.rot_dim, mixer.rot_base, mixer.rot_turned):
+            if (o.kv_rank, o.rot_dim, o.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot):
                 raise ValueError(f"layer {i}: the latent or the rotation differs from layer {source}'s")
         f = c.get("mlp")
         if f is not None and f.get("kind", "dense") != "dense":
@@ -292,6 +292,26 @@ def _padded(t, *shape):
     return out
 
 
+def _latent_tensors(get, vec, mix, m, d, dtype, device):
+    """Of a layer with latent attention: the rows of its projection up to the gate, and the weights behind it."""
+    from .. import hybrid_kernels as HK
+    heads, D, P, E, R, q_rank, kv_rank = m.sizes
+    Qp, pairs = HK.pad8(q_rank), torch.from_numpy(m.pairs()).to(device)
+    parts = [_padded(get(mix + "dq", (q_rank, d)), Qp, d)]
+    if m.source is None:
+        dkv = get(mix + "dkv", (kv_rank + m.rot_dim, d))
+        parts += [_padded(dkv[:kv_rank], R, d), _padded(dkv[kv_rank:][pairs], P, d)]
+    uq = get(mix + "uq", (heads * (m.dim + m.rot_dim), q_rank)).view(heads, m.dim + m.rot_dim, q_rank)
+    uq = torch.cat([_padded(uq[:, :m.dim], heads, D, q_rank), _padded(uq[:, m.dim:][:, pairs], heads, P, q_rank)], 1)
+    uk = _padded(get(mix + "uk", (heads * m.dim, kv_rank)).view(heads, m.dim, kv_rank), heads, D, R)
+    uv = _padded(get(mix + "uv", (heads * m.vdim, kv_rank)).view(heads, m.vdim, kv_rank), heads, E, R)
+    o = _padded(get(mix + "o", (d, heads * m.vdim)).view(d, heads, m.vdim), d, heads, E)
+    kv = HK.WideWeight(torch.cat([uk.reshape(-1, R), uv.reshape(-1, R)]), dtype) if HK.latent_tiles_fit(dtype, D, P, E) else None
+    return parts, dict(q_norm=vec(mix + "dq.norm", q_rank), kv_norm=vec(mix + "dkv.norm", kv_rank) if m.source is None else None,
+                       uq=HK.WideWeight(uq.reshape(-1, q_rank), dtype), uk_t=uk.transpose(1, 2).to(dtype).contiguous(),
+                       uv=uv.to(dtype).contiguous(), kv=kv, out=HK.WideWeight(o.reshape(d, -1), dtype))
+
+
 def parallel_weights(tensors, spec, device="cuda"):
     """As hybrid_weights, for layers with latent attention whose sublayers stand side by side.  Every head size is rounded up to
     what the kernels take, with zeros; the two features of a rotated pair come to stand side by side, in queries and keys."""
@@ -304,25 +324,10 @@ def parallel_weights(tensors, spec, device="cuda"):
     for i, lay in enumerate(spec.layers):
         p, m = f"l{i}.", lay.mixer
         mix = p + "mix."
-        heads, D, P, E, R, q_rank, kv_rank = m.sizes
-        Qp, pairs = HK.pad8(q_rank), torch.from_numpy(m.pairs()).to(device)
-        parts = [_padded(get(mix + "dq", (q_rank, d)), Qp, d)]
-        if m.source is None:
-            dkv = get(mix + "dkv", (kv_rank + m.rot_dim, d))
-            parts += [_padded(dkv[:kv_rank], R, d), _padded(dkv[kv_rank:][pairs], P, d)]
-        parts.append(get(mix + "g", (heads, d)))
-        uq = get(mix + "uq", (heads * (m.dim + m.rot_dim), q_rank)).view(heads, m.dim + m.rot_dim, q_rank)
-        uq = torch.cat([_padded(uq[:, :m.dim], heads, D, q_rank), _padded(uq[:, m.dim:][:, pairs], heads, P, q_rank)], 1)
-        uk = _padded(get(mix + "uk", (heads * m.dim, kv_rank)).view(heads, m.dim, kv_rank), heads, D, R)
-        uv = _padded(get(mix + "uv", (heads * m.vdim, kv_rank)).view(heads, m.vdim, kv_rank), heads, E, R)
-        o = _padded(get(mix + "o", (d, heads * m.vdim)).view(d, heads, m.vdim), d, heads, E)
+        parts, latent = _latent_tensors(get, vec, mix, m, d, dtype, device)
+        parts.append(get(mix + "g", (m.heads, d)))
         lw = dict(norm1=vec(p + "norm1", d), shift=vec(p + "shift", d), gate1=HK.WideWeight(get(p + "rg1", (d, d)), dtype),
-                  gate1_bias=vec(p + "rg1.b", d), proj=HK.WideWeight(torch.cat(parts), dtype, tail=heads),
-                  q_norm=vec(mix + "dq.norm", q_rank), kv_norm=vec(mix + "dkv.norm", kv_rank) if m.source is None else None,
-                  uq=HK.WideWeight(uq.reshape(-1, q_rank), dtype), uk_t=uk.transpose(1, 2).to(dtype).contiguous(),
-                  uv=uv.to(dtype).contiguous(), kv=None, out=HK.WideWeight(o.reshape(d, -1), dtype))
-        if HK.latent_tiles_fit(dtype, D, P, E):
-            lw.update(kv=HK.WideWeight(torch.cat([uk.reshape(-1, R), uv.reshape(-1, R)]), dtype))
+                  gate1_bias=vec(p + "rg1.b", d), proj=HK.WideWeight(torch.cat(parts), dtype, tail=m.heads), **latent)
         if lay.mlp is not None:
             ff, mlp = lay.mlp.ff, p + "mlp."
             n = HK.pad8(ff)
@@ -393,21 +398,31 @@ def golapel_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dty
                       0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype)
 
 
+def _head_rows(t, heads, size, which, stored):
+    """[heads * size, ...] in the order `which` of every head's features, each head padded to `stored`"""
+    t = t.view(heads, size, -1)[:, which]
+    return _padded(t, heads, stored, t.shape[2]).reshape(heads * stored, -1)
+
+
+def _glu(get, make, names, ff, d, dtype):
+    """Gate, up and down of one feed-forward or of several alike.  make(tensors, dtype, further keywords) -> weight; names: prefixes of
+    their tensors"""
+    from .. import hybrid_kernels as HK
+    from .result_norm import FeedForwardWeights
+    n = HK.pad8(ff)
+    gate, up = (make([get(p + part, (ff, d)) for p in names], dtype, main_to=n) for part in ("gate", "up"))
+    return FeedForwardWeights(gate, up, make([get(p + "down", (d, ff)) for p in names], dtype))
+
+
 def result_norm_weights(tensors, spec, device="cuda"):
     """As hybrid_weights, for layers with attention by heads.  Head sizes are rounded up to whole pieces of eight features with
     zeros; the two features of a rotated pair come to stand side by side in queries and keys (and so in values that are keys)."""
     from .. import hybrid_kernels as HK
     from .hybrid import Experts
-    from .result_norm import FeedForwardWeights, ResultNormLayerWeights, ResultNormWeights
+    from .result_norm import ResultNormLayerWeights, ResultNormWeights
     dtype = HK.DTYPES[spec.dtype]
     get, vec = _lookup(tensors, device)
     d = spec.width
-
-    def feed_forward(make, names, ff):
-        """make(tensors of the experts, further keywords) -> weight; names: prefixes of the experts' tensors"""
-        n = HK.pad8(ff)
-        gate, up = (make([get(p + part, (ff, d)) for p in names], dtype, main_to=n) for part in ("gate", "up"))
-        return FeedForwardWeights(gate, up, make([get(p + "down", (d, ff)) for p in names], dtype))
 
     layers = []
     for i, lay in enumerate(spec.layers):
@@ -417,10 +432,7 @@ def result_norm_weights(tensors, spec, device="cuda"):
         pairs = torch.from_numpy(m.rot.pairs(m.dim) if m.rot is not None else np.arange(m.dim)).to(device)
         order = pairs if m.keys_are_values else torch.arange(m.vdim, device=device)
 
-        def rows(t, heads, size, which, stored):
-            """[heads * size, ...] in the order `which` of every head's features, each head padded to `stored`"""
-            t = t.view(heads, size, -1)[:, which]
-            return _padded(t, heads, stored, t.shape[2]).reshape(heads * stored, -1)
+        rows = _head_rows
         parts = [("q", H * M, m.dim, pairs, D), ("k", G * M, m.dim, pairs, D)]
         if not m.keys_are_values:
             parts.append(("v", G, m.vdim, order, E))
@@ -444,15 +456,134 @@ def result_norm_weights(tensors, spec, device="cuda"):
             lw.update(norm2=vec(p + "norm2", d))
         mp = p + "mlp."
         if isinstance(mlp, Experts):
-            lw.update(ff=feed_forward(HK.ExpertWeight, [f"{mp}e{e}." for e in range(mlp.count)], mlp.expert.ff), top=mlp.top)
+            lw.update(ff=_glu(get, HK.ExpertWeight, [f"{mp}e{e}." for e in range(mlp.count)], mlp.expert.ff, d, dtype), top=mlp.top)
             router = [get(mp + "router", (mlp.count, d))]
             if mlp.shared is not None:
-                lw.update(shared=feed_forward(HK.ExpertWeight, [mp + "shared."], mlp.shared.ff))
+                lw.update(shared=_glu(get, HK.ExpertWeight, [mp + "shared."], mlp.shared.ff, d, dtype))
                 router.append(get(mp + "shared.sg", (1, d)))
             router = torch.cat(router)
             lw.update(router=_padded(router, router.shape[0], HK.pad8(d)).to(dtype).contiguous(), router_linear=HK.WideWeight(router, dtype))
         elif mlp is not None:
-            lw.update(ff=feed_forward(lambda w, *a, **kw: HK.WideWeight(w[0], *a, **kw), [mp], mlp.ff))
+            lw.update(ff=_glu(get, lambda w, *a, **kw: HK.WideWeight(w[0], *a, **kw), [mp], mlp.ff, d, dtype))
         layers.append(ResultNormLayerWeights(**lw))
     embed = get("embed", (spec.vocab, d)).to(dtype).contiguous()
     return ResultNormWeights(embed, layers, vec("final.norm", d), HK.WideWeight(embed, dtype))
+
+
+# ----------------------------------------------------------------------------------- results averaged over the depths
+def depth_layers(layers):
+    """The `layers` list of a configuration with latent attention (an output gate per feature, neighbours rotated), attention by heads
+    (short convolutions, a penalty of the distance) and the state-space recurrence -> [HybridLayer]."""
+    from .hybrid import Experts, HeadMixer, HybridLayer, LatentMixer, SquaredReLU, StateSpaceMixer, SwiGLU
+    out = []
+    for i, c in enumerate(layers):
+        m, kind, where = c["mixer"], c["type"], f"layer {i}"
+        if kind == "latent_attention":
+            rot, source = _rotation(m["rot"], True, True, where), m.get("kv_from")
+            if rot.dims > m["rot_dim"]:
+                raise ValueError(f"{where}: {rot.dims} rotated features of {m['rot_dim']}")
+            mixer = LatentMixer(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["q_rank"], m["kv_rank"], float(m["scale"]), None, rot, source,
+                                "feature")
+            if source is not None:
+                o = out[source].mixer if 0 <= source < i else None
+                if getattr(o, "kind", None) != "latent" or o.source is not None:
+                    raise ValueError(f"{where}: kv_from {source} names no earlier layer with a cache of its own")
+                if (o.kv_rank, o.rot_dim, o.rot) != (mixer.kv_rank, mixer.rot_dim, rot):
+                    raise ValueError(f"{where}: the latent or the rotation differs from layer {source}'s")
+        elif kind == "attention":
+            mixer = HeadMixer(m["heads"], m["kv_heads"], m["dim"], m["vdim"], float(m["scale"]), biases="qkv", norms=False, far=True,
+                              taps=m["conv"])
+            if mixer.heads % mixer.kv_heads:
+                raise ValueError(f"{where}: {mixer.heads} heads on {mixer.kv_heads}")
+        elif kind == "mamba2":
+            mixer = StateSpaceMixer(m["heads"], m["groups"], m["state"], m["vdim"], m["conv"], m["norm_groups"])
+            if mixer.heads % mixer.groups or mixer.heads * mixer.vdim % mixer.norm_parts:
+                raise ValueError(f"{where}: {mixer.heads} heads of {mixer.vdim} in {mixer.groups} groups, normed in {mixer.norm_parts}")
+        else:
+            raise NotImplementedError(f"{where}: mixer {kind}")
+        f, mlp = c.get("mlp"), None
+        if f is not None and f.get("kind", "dense") == "dense":
+            mlp = SquaredReLU(f["ff"])
+        elif f is not None and f["kind"] == "moe":
+            r = f["router"]
+            g = r.get("groups") or {"count": 1, "keep": 1}
+            if r["experts"] % g["count"] or r["experts"] // g["count"] * g["keep"] < r["top"]:
+                raise ValueError(f"{where}: {r['top']} of {r['experts']} experts, {g['keep']} of {g['count']} groups")
+            mlp = Experts(r["experts"], r["top"], 1.0, SwiGLU(f["expert"]["ff"]), None, "sigmoid", True, g["count"], g["keep"], True)
+        elif f is not None:
+            raise NotImplementedError(f"{where}: feed-forward {f['kind']}")
+        out.append(HybridLayer(mixer, mlp, i))
+    return out
+
+
+def sabolorn_spec(cfg, max_len, batch, pad_id=0, eos_id=-1, early_stop=False, dtype="bfloat16", topk=1):
+    from .hybrid import HybridSpec
+    scale = (cfg.get("embedding") or {}).get("scale")
+    return HybridSpec("sabolorn", depth_layers(cfg["layers"]), cfg["width"], cfg["vocab"], 1, cfg["norm"]["eps"], 1.0, 1.0 if scale is None else scale,
+                      cfg.get("logit_softcap") or 0.0, max_len, batch, pad_id, eos_id, early_stop, topk, dtype, side_dim=cfg["token_side"]["dim"])
+
+
+def depth_weights(tensors, spec, device="cuda"):
+    """As hybrid_weights, for layers whose results are averaged over the depths.  Head and state sizes are rounded up to whole pieces of
+    eight features (latent ones as _latent_tensors does) with zeros."""
+    from .. import hybrid_kernels as HK
+    from .depth import DepthLayerWeights, DepthWeights
+    from .hybrid import Experts
+    dtype = HK.DTYPES[spec.dtype]
+    get, vec = _lookup(tensors, device)
+    d, n_side = spec.width, spec.side_dim
+
+    def by_heads(t, heads, size, stored):
+        return _head_rows(t, heads, size, slice(None), stored)
+
+    layers = []
+    for i, lay in enumerate(spec.layers):
+        p, m, mlp = f"l{i}.", lay.mixer, lay.mlp
+        mix = p + "mix."
+        side = HK.pad8(n_side)
+        lw = dict(norm=vec(p + "norm1", d), average=vec(p + "dwa", i + 2), side_norm=vec(p + "side.norm", d),
+                  side_gate=HK.WideWeight(get(p + "side.gate", (n_side, d)), dtype, main_to=side),
+                  side_proj=HK.WideWeight(get(p + "side.proj", (d, n_side)), dtype))
+        if m.kind == "latent":
+            parts, latent = _latent_tensors(get, vec, mix, m, d, dtype, device)
+            E = m.sizes[3]
+            parts.append(by_heads(get(mix + "g", (m.heads * m.vdim, d)), m.heads, m.vdim, E))
+            lw.update(latent, proj=HK.WideWeight(torch.cat(parts), dtype))
+        elif m.kind == "heads":
+            H, G, D, E = m.heads, m.kv_heads, m.stored_dim, m.stored_vdim
+            parts = [("q", H, m.dim, D), ("k", G, m.dim, D), ("v", G, m.vdim, E)]
+            lw.update(proj=HK.WideWeight(torch.cat([by_heads(get(mix + n, (h * s, d)), h, s, e) for n, h, s, e in parts]), dtype),
+                      proj_bias=torch.cat([by_heads(vec(mix + n + ".b", h * s), h, s, e).reshape(-1) for n, h, s, e in parts]).contiguous(),
+                      conv=HK.ShortConv(torch.cat([by_heads(get(mix + n + ".conv", (h * s, m.taps)).float(), h, s, e) for n, h, s, e in parts])
+                                        .t().contiguous()),
+                      far=(vec(mix + "r1", H), vec(mix + "r2", H)))
+        else:
+            H, G, D, E = m.heads, m.groups, m.stored_dim, m.stored_vdim
+            inner, states = H * m.vdim, G * m.dim
+            columns = [(inner, H, m.vdim, E), (states, G, m.dim, D), (states, G, m.dim, D)]                # x | b | c
+
+            def convolved(t):
+                return torch.cat([by_heads(u, h, s, e) for u, (_, h, s, e) in zip(torch.split(t, [c[0] for c in columns]), columns)])
+            w = get(mix + "in", (2 * inner + 2 * states + H, d))
+            lw.update(proj=HK.WideWeight(torch.cat([by_heads(w[:inner], H, m.vdim, E), convolved(w[inner:-H]), w[-H:]]), dtype, tail=H),
+                      conv=HK.ShortConv(convolved(get(mix + "conv", (inner + 2 * states, m.taps)).float()).t().contiguous(),
+                                        convolved(vec(mix + "conv.b", inner + 2 * states)).reshape(-1).contiguous(), silu=True),
+                      ssd=(vec(mix + "dt_bias", H), vec(mix + "A_log", H), vec(mix + "D", H)),
+                      head_norm=by_heads(vec(mix + "norm", inner), H, m.vdim, E).reshape(-1).contiguous())
+        if m.kind != "latent":
+            o = get(mix + "o", (d, m.heads * m.vdim)).view(d, m.heads, m.vdim)
+            lw.update(out=HK.WideWeight(_padded(o, d, m.heads, m.stored_vdim).reshape(d, -1), dtype))
+        mp = p + "mlp."
+        if isinstance(mlp, Experts):
+            router = get(mp + "router", (mlp.count, d))
+            lw.update(ff=_glu(get, HK.ExpertWeight, [f"{mp}e{e}." for e in range(mlp.count)], mlp.expert.ff, d, dtype), top=mlp.top,
+                      router=_padded(router, mlp.count, HK.pad8(d)).to(dtype).contiguous(), router_linear=HK.WideWeight(router, dtype),
+                      correction=vec(mp + "correction", mlp.count))
+        elif mlp is not None:
+            lw.update(up=HK.WideWeight(get(mp + "up", (mlp.ff, d)), dtype, main_to=HK.pad8(mlp.ff)),
+                      down=HK.WideWeight(get(mp + "down", (d, mlp.ff)), dtype))
+        layers.append(DepthLayerWeights(**lw))
+    embed = get("embed", (spec.vocab, d)).to(dtype).contiguous()
+    own = get("side.embed", (spec.vocab, len(layers) * n_side)).view(spec.vocab, len(layers), n_side)
+    own = _padded(own, spec.vocab, len(layers), HK.pad8(n_side)).to(dtype).contiguous()
+    return DepthWeights(embed, own, layers, vec("final.norm", d), HK.WideWeight(embed, dtype))

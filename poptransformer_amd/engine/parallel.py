@@ -13,12 +13,12 @@ every head instead of the middle three.
 from dataclasses import dataclass
 from typing import List, Optional
 
-import numpy as np
 import torch
 
 from .. import _hybrid_lib as H
 from .. import hybrid_kernels as HK
-from .hybrid import F32, I32, HybridDecoder
+from .hybrid import F32, HybridDecoder
+from .mixers import LatentBuffers, LatentMixing
 
 
 @dataclass
@@ -67,39 +67,27 @@ class ParallelWeights:
                                       for lay in self.layers)
 
 
-class ParallelBuffers:
+class ParallelBuffers(LatentBuffers):
     """Activations of up to `rows` rows."""
 
     def __init__(self, spec, weights, rows, dtype, device):
         def buf(*shape, dtype=dtype):
             return torch.zeros(shape, dtype=dtype, device=device)
         mixers, ld = [lay.mixer for lay in spec.layers], HK.pad8(spec.width)
-        self._buf = buf
         self.rows = rows
         self.x = buf(rows, spec.width, dtype=F32)
         self.h1, self.h2, self.hm = buf(rows, ld), buf(rows, ld), buf(rows, ld)
         self.gate1, self.gate2 = buf(rows, spec.width), buf(rows, spec.width)
         self.proj = {n: buf(rows, n) for n in {lw.proj.n_main for lw in weights.layers}}
         self.head_gates = {n: buf(rows, n, dtype=F32) for n in {m.heads for m in mixers}}
-        self.cq = {n: buf(rows, n) for n in {lw.uq.K for lw in weights.layers}}
-        self.q = {n: buf(rows, n) for n in {lw.uq.n_main for lw in weights.layers}}
+        self.latent_buffers(buf, mixers, weights.layers)
         self.ctx = {n: buf(rows, n) for n in {m.out_channels for m in mixers}}
         self.act = {n: buf(rows, n) for n in {lw.gate.n_main for lw in weights.layers if lw.gate is not None}}
         channels = max(w.N for lw in weights.layers for w in lw.linears())
         self.workspace = HK.linear_workspace(rows, channels, device) if rows > 16 else None
-        self._absorbed = {}
-
-    def absorbed(self, heads, R, P, splits):
-        """(queries against the latent, the parts' sums, their softmax states)"""
-        key = (heads, R, P, splits)
-        if key not in self._absorbed:
-            n = self.rows * heads
-            self._absorbed[key] = (self._buf(n, R + P), self._buf(n * splits, R, dtype=F32), self._buf(n * splits, 2, dtype=F32))
-        return self._absorbed[key]
 
 
-class ParallelDecoder(HybridDecoder):
-    absorbed_rows = 16               # sequences with up to this many rows in a pass work on the cached rows themselves
+class ParallelDecoder(LatentMixing, HybridDecoder):
     # passes of up to branch_rows single rows run a feed-forward of at least branch_bytes on a stream beside the mixer: what two
     # streams cost to part and meet (measured: feed-forwards of 80 MB lose 4 us per layer by it, of 300 MB gain 11)
     branch_rows = 16
@@ -107,9 +95,7 @@ class ParallelDecoder(HybridDecoder):
 
     def __init__(self, spec, weights, device="cuda", slots=None):
         super().__init__(spec, weights, device, slots)
-        self._angles = {}
         self._side = torch.cuda.Stream()
-        self._key_lists = None
 
     def _rows_buffers(self, rows):
         size = rows if rows <= 16 else max(64, 1 << (rows - 1).bit_length())
@@ -117,71 +103,19 @@ class ParallelDecoder(HybridDecoder):
             self._buffers[size] = ParallelBuffers(self.spec, self.w, size, self.dtype, self.dev)
         return self._buffers[size]
 
-    def _cos_sin(self, m):
-        key = (m.rot_base, m.rot_turned, m.rot_dim)
-        if key not in self._angles:
-            self._angles[key] = torch.from_numpy(m.angles(self.store.max_len)).to(self.dev)
-        return self._angles[key]
-
-    def _splits(self, rows, mixer):
-        """Parts of the window per row: enough workgroups to fill the machine, at least 64 keys per part.  Fixed per shape, since
-        the launch is replayed while the context grows."""
-        wgs = rows * (-(-mixer.heads // 16) if self.dtype == torch.bfloat16 else mixer.heads)
-        keys = min(mixer.window or self.store.max_len, self.store.max_len)
-        return max(1, min(256 // wgs, -(-keys // 64), 64))
-
-    def _keys(self, rows, window):
-        """Cache rows that a pass's rows look at, sequence after sequence: (slots, positions), and where position 0 of a tile's
-        sequence would lie among them.  One list per distinct window of a pass."""
-        if self._key_lists is None or self._key_lists[0] is not rows:
-            self._key_lists = (rows, {})
-        lists = self._key_lists[1]
-        if window not in lists:
-            slots, places, zero, at = [], [], [], 0
-            for slot, p0, count in rows.portions:
-                first = max(0, p0 - window + 1) if window is not None else 0
-                n = p0 + count - first
-                slots.append(np.full(n, slot, np.int32))
-                places.append(np.arange(first, first + n, dtype=np.int32))
-                zero += [at - first] * -(-count // H.LATENT_TILE)
-                at += n
-            flat = torch.from_numpy(np.concatenate(slots + places + [np.array(zero, np.int32)])).to(self.dev)
-            slot, pos, tile_key = torch.split(flat, [at, at, len(zero)])
-            lists[window] = ((slot, pos), (*rows.tiles[:2], tile_key))
-        return lists[window]
-
     def _mixer(self, i, b, rows):
         """The heads' gated results, before the output projection."""
-        m, lw, n = self.spec.layers[i].mixer, self.w.layers[i], rows.n
-        heads, D, P, E, R = m.sizes[:5]
-        proj, cq, q = b.proj[lw.proj.n_main], b.cq[lw.uq.K], b.q[lw.uq.n_main]
-        gates, ctx = b.head_gates[heads], b.ctx[m.out_channels]
-        ring, = self.store.stores[i if m.source is None else m.source]
-        att = HK.LatentAttention(m.sizes, m.scale, m.window, self.spec.eps, lw.q_norm, lw.kv_norm, self._cos_sin(m), ring, n, rows.slot, rows.pos)
-        att.append(proj, cq)
-        HK.linear(cq, lw.uq, q, n, workspace=b.workspace)
-        if lw.kv is None or rows.single or rows.longest <= self.absorbed_rows:
-            splits = self._splits(b.rows, m)
-            q_latent, part_o, part_ml = b.absorbed(heads, R, P, splits)
-            att.absorbed(q, lw.uk_t, q_latent, splits, part_o, part_ml, lw.uv, gates, ctx)
-        else:
-            keys, tiles = self._keys(rows, m.window)
-            count = keys[0].numel()
-            # latents, rotated parts, then keys and values of all heads
-            sizes = [count * R, count * P, count * lw.kv.n_main]
-            flat = self._scratch(2 * sum(sizes))[:2 * sum(sizes)].view(self.dtype)
-            latent, rot, kv = torch.split(flat, sizes)
-            att.over_heads(q, keys, latent.view(count, R), rot.view(count, P), lw.kv, kv.view(count, -1), tiles, gates, ctx)
-        return ctx
+        lw = self.w.layers[i]
+        return self._latent(i, lw, b, rows, b.proj[lw.proj.n_main], b.head_gates[self.spec.layers[i].mixer.heads])
 
     def _projections(self, i, b, n, mixer=True, ff=True):
         """The sublayers' residual gates, and the mixer's down-projections."""
         lw, ld, calls = self.w.layers[i], self.spec.width, []
         if mixer:
-            calls += [(b.h1, lw.gate1, b.gate1, dict(ld=ld, bias=lw.gate1_bias, sigmoid=True, workspace=b.workspace)),
+            calls += [(b.h1, lw.gate1, b.gate1, dict(ld=ld, bias=lw.gate1_bias, act=H.ACT_SIGMOID, workspace=b.workspace)),
                       (b.hm, lw.proj, b.proj[lw.proj.n_main], dict(tail=b.head_gates[self.spec.layers[i].mixer.heads], workspace=b.workspace))]
         if ff:
-            calls.append((b.h2, lw.gate2, b.gate2, dict(ld=ld, bias=lw.gate2_bias, sigmoid=True, workspace=b.workspace)))
+            calls.append((b.h2, lw.gate2, b.gate2, dict(ld=ld, bias=lw.gate2_bias, act=H.ACT_SIGMOID, workspace=b.workspace)))
         HK.linear_group(n, *calls)
 
     def _output(self, i, b, n, ctx):

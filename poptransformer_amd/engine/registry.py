@@ -26,6 +26,13 @@ def _golapel(cfg, path, max_len, batch, dtype, slots):
     return ResultNormDecoder(spec, loader.result_norm_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
 
 
+def _sabolorn(cfg, path, max_len, batch, dtype, slots):
+    from ..utils import checkpoint
+    from .depth import DepthDecoder
+    spec = loader.sabolorn_spec(cfg, max_len, batch, dtype=dtype)
+    return DepthDecoder(spec, loader.depth_weights(checkpoint.load_state_dict(path, floats="fp32"), spec), slots=slots)
+
+
 def _fused(spec_of, weights_of):
     def make(cfg, path, max_len, batch, dtype, slots):
         from ..utils import checkpoint
@@ -52,6 +59,7 @@ ARCHITECTURES = {
     "Zekilix": (("hybrid",), _zekilix),
     "Ruperax": (("hybrid",), _ruperax),
     "Golapel": (("hybrid",), _golapel),
+    "Sabolorn": (("hybrid",), _sabolorn),
     "GPT2LMHeadModel": (("hip", "hybrid"), _fused(loader.gpt2_spec, loader.gpt2_weights)),
     "LlamaForCausalLM": (("hip", "hybrid"), _fused(loader.llama2_spec, loader.llama2_weights)),
     "ChatGLMModel": (("hip", "hybrid"), _fused(loader.chatglm2_spec, loader.chatglm2_weights)),

@@ -15,9 +15,9 @@ from typing import List, Optional
 
 import torch
 
-from .. import _hybrid_lib as H
 from .. import hybrid_kernels as HK
 from .hybrid import F32, Experts, HybridDecoder
+from .mixers import ExpertBuffers, ExpertMixing, HeadMixing, glu_pair
 
 
 @dataclass
@@ -41,12 +41,15 @@ class ResultNormLayerWeights:
     k_norm: torch.Tensor
     sink: Optional[torch.Tensor] = None
     lam: float = 0.0                 # weight of the second map
+    far: Optional[tuple] = None      # (far1, far2) of the heads' distance penalty
+    conv: Optional[HK.ShortConv] = None
     norm2: Optional[torch.Tensor] = None
     ff: Optional[FeedForwardWeights] = None          # dense, or the routed experts
     shared: Optional[FeedForwardWeights] = None
     router: Optional[torch.Tensor] = None            # [experts (+ the shared one's gate), padded width]
     router_linear: Optional[HK.WideWeight] = None    # the same as a Linear
     top: int = 0
+    correction: Optional[torch.Tensor] = None        # of the router's scores
 
     def active_parameters(self):
         """Parameters of the products that one row goes through."""
@@ -78,7 +81,7 @@ class ResultNormWeights:
         return n
 
 
-class ResultNormBuffers:
+class ResultNormBuffers(ExpertBuffers):
     """Activations of up to `rows` rows."""
 
     def __init__(self, spec, weights, rows, direct, dtype, device):
@@ -91,141 +94,33 @@ class ResultNormBuffers:
         self.proj = {n: buf(rows, n) for n in {lw.proj.n_main for lw in weights.layers}}
         self.head_gates = {n: buf(rows, n, dtype=F32) for n in {lw.proj.tail for lw in weights.layers} if n}
         self.ctx = {n: buf(rows, n) for n in {lay.mixer.out_channels for lay in spec.layers}}
-        self.act, self.parts, self.routing, self.lists, self.logits = {}, {}, {}, {}, {}
-        for lay, lw in zip(spec.layers, weights.layers):
-            e = lay.mlp
-            if not isinstance(e, Experts):
-                if e is not None:
-                    self.act[lw.ff.gate.n_main] = buf(rows, lw.ff.gate.n_main)
-                continue
-            key, choices = (e.count, e.top, e.shared is not None, e.scale), e.top + (e.shared is not None)
-            if key not in self.routing:
-                self.routing[key] = HK.Routing(rows, e.count, e.top, e.shared is not None, e.scale, device)
-            n = lw.ff.gate.n_main
-            if lw.shared is not None:
-                self.act[lw.shared.gate.n_main] = buf(rows, lw.shared.gate.n_main)
-                n = max(n, lw.shared.gate.n_main) if direct else n
-            if (choices, n) not in self.act:
-                self.act[choices, n] = buf(rows * choices, n)
-            if choices not in self.parts:
-                self.parts[choices] = buf(rows * choices, spec.width, dtype=F32 if direct else dtype)
-            if dtype == F32:
-                self.logits[lw.router.shape[0]] = buf(rows, lw.router.shape[0], dtype=F32)
-            if not direct:
-                for t in (128, 256):
-                    self.lists[e.count, e.top, t] = HK.expert_lists(rows, e.top, e.count, t, device)
+        self.act = {lw.ff.gate.n_main: buf(rows, lw.ff.gate.n_main) for lay, lw in zip(spec.layers, weights.layers)
+                    if lay.mlp is not None and not isinstance(lay.mlp, Experts)}
+        self.expert_buffers(buf, spec, weights.layers, direct, dtype, device)
         channels = max([spec.width] + [lw.proj.N for lw in weights.layers])
         self.workspace = HK.linear_workspace(rows, channels, device) if rows > 16 else None
 
 
-class ResultNormDecoder(HybridDecoder):
-    direct_rows = 16                 # passes of up to this many bf16 rows find their experts' rows without lists
-    # routers up to this size are multiplied in the norm's launch by passes of up to so many rows (every row reads all of it: 2048
-    # rows of 4096 features and 33 logits take 43 us that way, 19 + 21 with a launch for the routing, 512 rows 16 against 10 + 15)
-    router_bytes, router_rows = 1 << 20, 512
-    tall_rows = 128                  # rows per expert, on average, above which their lists are cut into tiles of 256 (else 128)
-
-    def __init__(self, spec, weights, device="cuda", slots=None):
-        super().__init__(spec, weights, device, slots)
-        self._angles = {}
-
-    def _direct(self, rows):
-        return self.dtype == torch.bfloat16 and rows <= self.direct_rows
-
+class ResultNormDecoder(HeadMixing, ExpertMixing, HybridDecoder):
     def _rows_buffers(self, rows):
         size = rows if rows <= 16 else max(64, 1 << (rows - 1).bit_length())
         if size not in self._buffers:
             self._buffers[size] = ResultNormBuffers(self.spec, self.w, size, self._direct(size), self.dtype, self.dev)
         return self._buffers[size]
 
-    def _cos_sin(self, rot):
-        if rot is None:
-            return None
-        key = (rot.base, rot.dims, rot.neighbours, rot.factor, rot.yarn)
-        if key not in self._angles:
-            self._angles[key] = torch.from_numpy(rot.angles(self.store.max_len)).to(self.dev)
-        return self._angles[key]
-
-    def _splits(self, rows, mixer):
-        """Parts of the visible keys per (row, key head) of a decode pass, and the scratch they meet in: as HybridDecoder's."""
-        m = mixer
-        key = (rows, m.heads, m.kv_heads, m.stored_dim, m.stored_vdim, m.maps, m.keep, m.span)
-        if key not in self._splits_for:
-            group, most = m.heads // m.kv_heads, 4 // m.maps
-            wgs = rows * m.kv_heads * -(-group // (group if group <= 2 // m.maps else most))
-            keys = min(m.keep + m.span, self.store.max_len)
-            splits = max(1, min(768 // wgs, -(-keys // 64), 64)) if keys > 256 else 1
-            self._splits_for[key] = (splits, HK.head_workspace(rows, m, splits, self.dev) if splits > 1 else None)
-        return self._splits_for[key]
-
     def _mixer(self, i, b, rows):
-        spec, m, lw, n = self.spec, self.spec.layers[i].mixer, self.w.layers[i], rows.n
-        proj, ctx, gates = b.proj[lw.proj.n_main], b.ctx[m.out_channels], b.head_gates[lw.proj.tail] if lw.proj.tail else None
+        lw, n = self.w.layers[i], rows.n
+        proj, gates = b.proj[lw.proj.n_main], b.head_gates[lw.proj.tail] if lw.proj.tail else None
         HK.linear(b.h, lw.proj, proj, n, tail=gates, bias=lw.proj_bias, workspace=b.workspace)
-        att = HK.HeadAttention(m, spec.eps, lw.q_norm, lw.k_norm, self._cos_sin(m.rot), lw.sink, lw.lam, *self.store.stores[i], proj, n,
-                               rows.slot, rows.pos, gates, ctx)
-        if rows.single:
-            att.decode(*self._splits(n, m))
-        else:
-            att.prompt(rows.tiles)
-        HK.linear(ctx, lw.out, b.y, n, ld=spec.width, workspace=b.workspace)
-
-    def _routing(self, i, b):
-        e = self.spec.layers[i].mlp
-        return b.routing[e.count, e.top, e.shared is not None, e.scale]
-
-    def _routed_by_norm(self, i, b):
-        """What the norm's launch needs to route the rows to layer i's experts, where it does."""
-        lw = self.w.layers[i]
-        if lw.router is None or b.rows > self.router_rows or lw.router.numel() * lw.router.element_size() > self.router_bytes:
-            return {}
-        return dict(router=lw.router, routing=self._routing(i, b))
+        HK.linear(self._heads(i, lw, b, rows, proj, gates), lw.out, b.y, n, ld=self.spec.width, workspace=b.workspace)
 
     def _feed_forward(self, i, b, n):
         """The feed-forward's result, as arguments of result_norm."""
-        spec, mlp, lw = self.spec, self.spec.layers[i].mlp, self.w.layers[i]
-        if not isinstance(mlp, Experts):
-            self._dense(b, n, lw.ff, pair=H.PAIR_SWIGLU)
-            return dict(y=b.y)
-        r = self._routing(i, b)
-        if not self._routed_by_norm(i, b):
-            if self.dtype == torch.bfloat16:
-                r.by_product(b.h, lw.router_linear, n)
-            else:
-                logits = b.logits[lw.router.shape[0]]
-                HK.linear(b.h, lw.router_linear, logits, n)
-                r(logits, n)
-
-        def clamped(glu):
-            return dict(pair=H.PAIR_CLAMPED, limit=glu.limit, slope=glu.slope)
-        parts = b.parts[r.choices]
-        result = dict(parts=parts, parts_ld=r.choices, part_weight=r.weights)
-        pair, down = dict(w=lw.ff.gate, up=lw.ff.up, **clamped(mlp.expert)), dict(w=lw.ff.down)
-        if self._direct(b.rows):
-            shared_pair = shared_down = None
-            act_ld = lw.ff.gate.n_main
-            if mlp.shared is not None:
-                shared_pair, shared_down = dict(w=lw.shared.gate, up=lw.shared.up, **clamped(mlp.shared)), dict(w=lw.shared.down)
-                act_ld = max(act_ld, lw.shared.gate.n_main)
-            act = b.act[r.choices, act_ld]
-            HK.experts(b.h, r, n, pair, act, shared_pair)
-            HK.experts(act, r, n, down, parts, shared_down)
-            return dict(result, n_parts=r.choices)
-        tile = 256 if n * mlp.top > self.tall_rows * mlp.count else 128
-        lists, act = b.lists[mlp.count, mlp.top, tile], b.act[r.choices, lw.ff.gate.n_main]
-        HK.group_experts(r, n, tile, lists)
-        HK.experts(b.h, r, n, pair, act, lists=lists, tile_rows=tile)
-        HK.experts(act, r, n, down, parts, lists=lists, tile_rows=tile)
-        result.update(n_parts=mlp.top)
-        if mlp.shared is not None:
-            self._dense(b, n, lw.shared, **clamped(mlp.shared))
-            result.update(y=b.y, y_weight=(r.weights, mlp.top))
-        return result
-
-    def _dense(self, b, n, ff, **pair):
-        act = b.act[ff.gate.n_main]
-        HK.linear(b.h, ff.gate, act, n, up=ff.up, **pair)
-        HK.linear(act, ff.down, b.y, n, ld=self.spec.width, workspace=b.workspace)
+        mlp = self.spec.layers[i].mlp
+        if isinstance(mlp, Experts):
+            return self._mixture(i, b, n)
+        self._dense(b, n, self.w.layers[i].ff, **glu_pair(mlp))
+        return dict(y=b.y)
 
     def _layers(self, rows, pos_out=None):
         """All layers over the rows; h holds the model's norm of them."""

@@ -6,7 +6,8 @@ own) a slot is
   * for attention by heads: rings of keys (normed, rotated) and values, the first `keep` positions in rows of their own before
     the ring of the others;
   * for latent attention: a ring of latents with their rotated key part - a layer that reads another one's cache has none;
-  * for matrix memory: the fp32 state, zero before the first token;
+  * for matrix memory and the state-space recurrence: the fp32 state, zero before the first token;
+  * for a short convolution: a ring of its newest rows as they were projected;
 and with a token shift per layer the normed fp32 row of the newest token.
 Ring rows need no clearing: a position is only looked at once its own sequence has written it; nor does the shift's row,
 which position 0 does not look at.
@@ -26,6 +27,7 @@ class SequenceStore:
         self.capacity = 0
         self.stores = [None] * len(spec.layers)
         self.shifted = [None] * len(spec.layers)      # fp32 [slots, width] per layer with a token shift
+        self.recent = [None] * len(spec.layers)       # [slots, taps, channels] per layer with a short convolution
         self.length = []                      # tokens each slot holds, -1: free
         self._grow(slots)
 
@@ -62,9 +64,14 @@ class SequenceStore:
                 new = (zeros(slots, m.kv_heads, m.maps, n, m.stored_dim), zeros(slots, m.kv_heads, n, m.stored_vdim))
             elif m.kind == "latent":
                 new = (zeros(slots, self.ring_len(i), m.cache_row),) if m.source is None else ()
+            elif m.kind == "ssd":
+                new = (HK.ssd_state(slots, m.heads, m.stored_dim, m.stored_vdim, self.dev),)
             else:
                 new = (HK.mlstm_state(slots, m.heads, m.dim, m.vdim, self.dev),)
             self.stores[i] = moved(self.stores[i], new)
+            if getattr(m, "taps", 0):
+                old = self.recent[i]
+                self.recent[i], = moved(old if old is None else (old,), (zeros(slots, m.taps, m.conv_channels),))
             if layer.shift:
                 old = self.shifted[i]
                 self.shifted[i], = moved(old if old is None else (old,), (zeros(slots, self.spec.width, dtype=torch.float32),))
@@ -87,7 +94,7 @@ class SequenceStore:
     def restart(self, slots):
         """The given slots hold a sequence without tokens."""
         for layer, store in zip(self.spec.layers, self.stores):
-            if layer.mixer.kind == "mlstm":
+            if layer.mixer.kind in ("mlstm", "ssd"):
                 for slot in slots:
                     store[0][slot].zero_()
         for slot in slots:
@@ -95,4 +102,5 @@ class SequenceStore:
 
     @property
     def nbytes(self):
-        return sum(t.numel() * t.element_size() for store in self.stores + [[s] for s in self.shifted if s is not None] for t in store)
+        rest = [[t] for t in self.shifted + self.recent if t is not None]
+        return sum(t.numel() * t.element_size() for store in self.stores + rest for t in store)

@@ -67,7 +67,7 @@ def linear_workspace(rows, channels, device):
 
 
 def _linear_args(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.PAIR_NONE, limit=0.0, slope=0.0, workspace=None, bias=None,
-                 bias2=None, sigmoid=False, mul=None, accumulate=False):
+                 bias2=None, act=H.ACT_NONE, mul=None, accumulate=False):
     _need(x, w.dtype, "x", rows * w.K)
     ld = w.n_main if ld is None else ld
     if out.dtype not in (w.dtype, F32):
@@ -86,7 +86,7 @@ def _linear_args(x, w, out, rows, ld=None, tail=None, cap=0.0, up=None, pair=H.P
         _need(mul, w.dtype, "mul", rows * ld)
     return H.WideLinearArgs(_CODE[w.dtype], _p(x), rows, w.K, w.N, _p(w.data), _p(up.data) if up is not None else None, pair, limit, slope,
                             cap, _p(out), ld, w.n_main, int(out.dtype == F32), _p(tail) if w.tail else None, w.tail, _p(w.tail_bias),
-                            _p(workspace), workspace.numel() if workspace is not None else 0, _p(bias), _p(bias2), int(sigmoid), _p(mul),
+                            _p(workspace), workspace.numel() if workspace is not None else 0, _p(bias), _p(bias2), act, _p(mul),
                             int(accumulate))
 
 
@@ -202,6 +202,39 @@ def shift_norm(x, rows, groups, eps, w1, h1, w2=None, h2=None, shift=None, hm=No
     H.check(H.load().pta_shift_norm(ctypes.byref(a), _stream()))
 
 
+class ShortConv:
+    """A short causal convolution over `channels` channels: weight [taps, channels] (the last row is the current token's), bias
+    [channels] or None.  ring [slots, taps, channels] holds the newest rows of every sequence as they were projected."""
+
+    def __init__(self, weight, bias=None, silu=False):
+        _need(weight, F32, "weight")
+        self.weight, self.bias, self.silu = weight, bias, bool(silu)
+        self.taps, self.channels = weight.shape
+        if bias is not None:
+            _need(bias, F32, "bias", self.channels)
+
+    def args(self, ring):
+        _need(ring, ring.dtype, "ring")
+        if tuple(ring.shape[1:]) != (self.taps, self.channels):
+            raise ValueError(f"ring must be [slots, {self.taps}, {self.channels}], got {tuple(ring.shape)}")
+        return H.Conv(self.channels, self.taps, _p(self.weight), _p(self.bias), int(self.silu), _p(ring))
+
+    def __call__(self, x, x_at, y, ring, rows, slot, pos, last, tiles):
+        """y[:, :channels] = the convolved columns x_at .. of x, for rows of a pass; tiles = (first rows, row counts, how many)."""
+        _need(x, ring.dtype, "x", rows * x.shape[-1])
+        _need(y, ring.dtype, "y", rows * y.shape[-1])
+        if x.shape[-1] < x_at + self.channels or x_at % 8:
+            raise ValueError("the rows do not hold the channels")
+        for t in (slot, pos, last):
+            _need(t, I32, "rows' places", rows)
+        tr, tc, n = tiles
+        _need(tr, I32, "tiles", n)
+        _need(tc, I32, "tiles", n)
+        a = H.ShortConvArgs(_CODE[ring.dtype], self.args(ring), x.data_ptr() + x_at * x.element_size(), x.shape[-1], _p(y), y.shape[-1],
+                            _p(slot), _p(pos), _p(last), _p(tr), _p(tc), n)
+        H.check(H.load().pta_short_conv(ctypes.byref(a), _stream()))
+
+
 def pad32(n):
     return (n + 31) // 32 * 32
 
@@ -241,10 +274,19 @@ class LatentAttention:
         self._call("append")
 
     def _result(self, q, gate, out):
+        """gate: fp32 [rows, H] per head, or (rows of a projection, first column) per feature"""
         _need(q, self.dtype, "q", self.rows * self.H * (self.D + self.P))
-        _need(gate, F32, "gate", self.rows * self.H)
         _need(out, self.dtype, "out", self.rows * self.H * self.E)
-        self.a.q, self.a.gate, self.a.out = _p(q), _p(gate), _p(out)
+        self.a.q, self.a.out = _p(q), _p(out)
+        if isinstance(gate, tuple):
+            proj, at = gate
+            _need(proj, self.dtype, "gate", self.rows * proj.shape[-1])
+            if proj.shape[-1] < at + self.H * self.E:
+                raise ValueError("the projection does not hold the gate")
+            self.a.feature_gate, self.a.gate_ld = proj.data_ptr() + at * proj.element_size(), proj.shape[-1]
+        else:
+            _need(gate, F32, "gate", self.rows * self.H)
+            self.a.gate = _p(gate)
 
     def absorbed(self, q, uk_t, q_latent, splits, part_o, part_ml, uv, gate, out):
         """Every row over the cache itself, its window in `splits` parts."""
@@ -291,7 +333,7 @@ class HeadAttention:
     result goes through (engine/hybrid.py HeadMixer); proj rows hold q | k | v (none where the values are the keys) | gate per
     feature (where there is one)."""
 
-    def __init__(self, mixer, eps, q_norm, k_norm, cos_sin, sink, lam, keys, values, proj, rows, slot, pos, head_gate, out):
+    def __init__(self, mixer, eps, q_norm, k_norm, cos_sin, sink, lam, keys, values, proj, rows, slot, pos, head_gate, out, far=None):
         m = mixer
         heads, G, M, D, E = m.heads, m.kv_heads, m.maps, m.stored_dim, m.stored_vdim
         es, ld = proj.element_size(), proj.shape[-1]
@@ -322,10 +364,17 @@ class HeadAttention:
         a.lambda_, a.diff, a.out, a.splits = lam, m.diff or 0.0, _p(out), 1
         a.head_gate = _p(head_gate)
         a.gate = base + at_gate * es if m.gate == "feature" else None
+        if far is not None:
+            for t in far:
+                _need(t, F32, "far", heads)
+            a.far1, a.far2 = (_p(t) for t in far)
 
-    def decode(self, splits, workspace):
-        """One row per sequence: norms, rotation, append and attention."""
+    def decode(self, splits, workspace, conv=None):
+        """One row per sequence: norms, rotation, append and attention; conv = (ShortConv, ring): queries, keys and values go
+        through it first."""
         a = self.a
+        if conv is not None:
+            a.conv = conv[0].args(conv[1])
         a.splits, a.workspace, a.workspace_bytes = splits, _p(workspace), workspace.numel() if workspace is not None else 0
         H.check(H.load().pta_head_decode(ctypes.byref(a), _stream()))
 
@@ -348,27 +397,31 @@ def head_workspace(rows, mixer, splits, device):
 class Routing:
     """Where the routing of up to `rows` rows goes: choice c of row r in chosen[r, c], its weight beside it."""
 
-    def __init__(self, rows, experts, top, shared, scale, device):
+    def __init__(self, rows, experts, top, shared, scale, device, score=H.SCORE_SOFTMAX, groups=1, keep=1, share=False):
+        self.score, self.groups, self.keep, self.share = score, groups, keep, bool(share)
         self.experts, self.top, self.shared, self.scale, self.choices = experts, top, bool(shared), scale, top + bool(shared)
         self.chosen = torch.zeros((rows, self.choices), dtype=I32, device=device)
         self.weights = torch.zeros((rows, self.choices), dtype=F32, device=device)
 
-    def args(self, rows):
+    def args(self, rows, correction=None):
         _need(self.chosen, I32, "routing", rows * self.choices)
-        return H.Routing(self.experts, self.top, int(self.shared), self.scale, _p(self.chosen), _p(self.weights))
+        if correction is not None:
+            _need(correction, F32, "correction", self.experts)
+        return H.Routing(self.experts, self.top, int(self.shared), self.scale, _p(self.chosen), _p(self.weights), self.score, _p(correction),
+                         self.groups, self.keep, int(self.share))
 
-    def __call__(self, logits, rows):
+    def __call__(self, logits, rows, correction=None):
         """Routes rows by their logits fp32 [rows, experts + shared]."""
         _need(logits, F32, "router logits", rows * (self.experts + self.shared))
-        a = self.args(rows)
+        a = self.args(rows, correction)
         H.check(H.load().pta_route(_p(logits), rows, ctypes.byref(a), _stream()))
 
-    def by_product(self, h, router, rows):
+    def by_product(self, h, router, rows, correction=None):
         """Routes bf16 rows by their products with the router, a WideWeight."""
         _need(h, torch.bfloat16, "rows", rows * h.shape[-1])
         if (router.dtype, router.K, router.n_main) != (torch.bfloat16, h.shape[-1], self.experts + self.shared):
             raise ValueError("the router does not fit the rows or the routing")
-        a = self.args(rows)
+        a = self.args(rows, correction)
         H.check(H.load().pta_route_rows(_p(h), h.shape[-1], rows, _p(router.data), ctypes.byref(a), _stream()))
 
 
@@ -410,6 +463,62 @@ def result_norm(x, rows, eps, h, weight=None, table=None, embed_scale=1.0, ids=N
         _need(router, h.dtype, "router", (routing.experts + routing.shared) * h.shape[-1])
         a.router, a.routing = _p(router), routing.args(rows)
     H.check(H.load().pta_result_norm(ctypes.byref(a), _stream()))
+
+
+def depth_norm(history, depth, rows, eps, h, norm_weight, centred=True, weights=None, y=None, y_weight=None, next=None, table=None, embed_scale=1.0,
+               ids=None, ids_index=None, pos_out=None, side_table=None, side=None, router=None, routing=None, correction=None):
+    """The end of a layer (pta_depth_norm).  history fp32 [depths, R, width], of which the first `depth` count; next: the index in it
+    that gets the average; side_table [vocab, layers, ld], side [layers, R, ld]."""
+    width = history.shape[-1]
+    _need(history, F32, "history")
+    if history.shape[1] < rows or depth > history.shape[0] or (next is not None and not depth <= next < history.shape[0]):
+        raise ValueError(f"a history of {tuple(history.shape)} for {rows} rows at depth {depth}")
+    _need(h, h.dtype, "h", rows * h.shape[-1])
+    _need(norm_weight, F32, "norm_weight", width)
+    a = H.DepthNormArgs(_CODE[h.dtype], rows, width, _p(history), history.shape[1] * width, depth)
+    if weights is not None:
+        _need(weights, F32, "weights", depth)
+        a.weights = _p(weights)
+    if y is not None:
+        _need(y, F32, "y", rows * width)
+        _need(y_weight, F32, "y_weight", width)
+        a.y, a.y_weight = _p(y), _p(y_weight)
+    if next is not None:
+        a.next = history[next].data_ptr()
+    a.centred, a.norm_weight, a.eps, a.h, a.h_ld = int(centred), _p(norm_weight), eps, _p(h), h.shape[-1]
+    if table is not None:
+        _need(table, h.dtype, "table")
+        _need(ids, I32, "ids")
+        a.table, a.vocab, a.embed_scale, a.ids = _p(table), table.shape[0], embed_scale, _p(ids)
+        a.ids_stride, a.ids_index, a.pos_out = ids.shape[-1] if ids.dim() == 2 else 1, _p(ids_index), _p(pos_out)
+        if side is not None:
+            _need(side_table, h.dtype, "side_table")
+            _need(side, h.dtype, "side")
+            if side_table.shape != (table.shape[0], side.shape[0], side.shape[2]) or side.shape[1] < rows:
+                raise ValueError(f"the tokens' own parts {tuple(side_table.shape)} do not fit {tuple(side.shape)}")
+            a.side_table, a.side, a.side_layers, a.side_ld, a.side_stride = _p(side_table), _p(side), side.shape[0], side.shape[2], side[0].numel()
+    if router is not None:
+        _need(router, h.dtype, "router", (routing.experts + routing.shared) * h.shape[-1])
+        a.router, a.routing = _p(router), routing.args(rows, correction)
+    H.check(H.load().pta_depth_norm(ctypes.byref(a), _stream()))
+
+
+def add_parts(x, rows, h, parts=None, n_parts=0, parts_ld=None, part_weight=None):
+    """x [R, width] fp32 += the weighted parts [rows, parts_ld, width]; h = x (pta_add_parts)."""
+    width = x.shape[-1]
+    _need(x, F32, "x", rows * width)
+    _need(h, h.dtype, "h", rows * h.shape[-1])
+    a = H.AddPartsArgs(_CODE[h.dtype], rows, width, _p(x))
+    if parts is not None:
+        parts_ld = parts_ld or n_parts
+        if parts.dtype not in (F32, h.dtype):
+            raise ValueError(f"parts must be float32 or {h.dtype}")
+        _need(parts, parts.dtype, "parts", rows * parts_ld * width)
+        _need(part_weight, F32, "part_weight", rows * part_weight.shape[-1])
+        a.parts, a.n_parts, a.parts_ld, a.part_f32 = _p(parts), n_parts, parts_ld, int(parts.dtype == F32)
+        a.part_weight, a.weights_ld = _p(part_weight), part_weight.shape[-1]
+    a.h, a.h_ld = _p(h), h.shape[-1]
+    H.check(H.load().pta_add_parts(ctypes.byref(a), _stream()))
 
 
 class ExpertWeight:
@@ -512,6 +621,49 @@ def head_norm_gate(o, weight, proj, gate_at, out, rows, heads, vdim, eps):
         raise ValueError("the projection does not hold the gate")
     H.check(H.load().pta_head_norm_gate(_CODE[proj.dtype], _p(o), _p(weight), proj.data_ptr() + gate_at * proj.element_size(),
                                         proj.shape[-1], _p(out), out.shape[-1], rows, heads, vdim, eps, _stream()))
+
+
+def ssd_state(slots, heads, dim, vdim, device):
+    return torch.zeros((slots, H.load().pta_ssd_state_floats(heads, dim, vdim)), dtype=F32, device=device)
+
+
+def ssd(x, x_at, rows, heads, groups, dim, vdim, dt, constants, state, slot, seqs, longest, y, chunked=False, scratch=None, pos=None, conv=None):
+    """State-space recurrence (pta_ssd) over columns x_at .. of x, which hold x | b | c; sizes as stored.  dt fp32 [rows, heads];
+    constants = (dt_bias, a_log, skip); seqs = (first rows, row counts, how many); y fp32 [rows, heads * vdim].  conv = (ShortConv, ring):
+    every sequence has one row, its columns as projected."""
+    es, at_b, at_c = x.element_size(), heads * vdim, heads * vdim + groups * dim
+    _need(x, x.dtype, "x", rows * x.shape[-1])
+    _need(dt, F32, "dt", rows * heads)
+    for t in constants:
+        _need(t, F32, "dt_bias, a_log and skip", heads)
+    _need(state, F32, "state")
+    _need(slot, I32, "slot", rows)
+    _need(y, F32, "y", rows * heads * vdim)
+    if state.shape[1] != H.load().pta_ssd_state_floats(heads, dim, vdim) or x.shape[-1] < x_at + at_c + groups * dim or x_at % 8:
+        raise ValueError("ssd: the state or the rows do not fit the sizes")
+    base, (seq_row, seq_count, n) = x.data_ptr() + x_at * es, seqs
+    a = H.SsdArgs(_CODE[x.dtype], rows, heads, groups, dim, vdim, base, base + at_b * es, base + at_c * es, x.shape[-1], _p(dt),
+                  *(_p(t) for t in constants), _p(state), _p(slot), _p(pos), _p(seq_row), _p(seq_count), n, longest, int(chunked), _p(y))
+    if conv is not None:
+        _need(pos, I32, "pos", rows)
+        a.conv = conv[0].args(conv[1])
+    else:
+        need = H.load().pta_ssd_workspace_bytes(ctypes.byref(a))
+        if need:
+            ws = scratch(need) if scratch is not None else torch.empty(need, dtype=torch.uint8, device=x.device)
+            a.workspace, a.workspace_bytes = _p(ws), ws.numel()
+    H.check(H.load().pta_ssd(ctypes.byref(a), _stream()))
+
+
+def gated_norm(y, z, weight, out, rows, heads, stored, vdim, parts, eps):
+    """out = norm in `parts` equal parts of y silu(z), times weight (pta_gated_norm); z: rows whose first columns are the gate."""
+    n = heads * stored
+    _need(y, F32, "y", rows * n)
+    _need(z, z.dtype, "z", rows * z.shape[-1])
+    _need(weight, F32, "weight", n)
+    _need(out, z.dtype, "out", rows * n)
+    a = H.GatedNormArgs(_CODE[z.dtype], rows, heads, stored, vdim, parts, _p(y), _p(z), z.shape[-1], _p(weight), eps, _p(out))
+    H.check(H.load().pta_gated_norm(ctypes.byref(a), _stream()))
 
 
 def argmax(logits, ids):

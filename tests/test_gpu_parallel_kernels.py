@@ -4,6 +4,7 @@ import pytest
 import torch
 
 from oracle import ruperax as R
+from poptransformer_amd import _hybrid_lib as H
 
 pytestmark = pytest.mark.gpu
 
@@ -46,7 +47,7 @@ def test_linear_bias_gate_and_accumulation(dtype, rows):
         HK.linear(x, ww, y, rows, ld=n, bias=bias, mul=mul, accumulate=True, workspace=HK.linear_workspace(rows, ww.N, "cuda"))
         assert _rel(_np(y), want) < 1e-5
         out = torch.empty((rows, n), dtype=T[dtype], device="cuda")
-        HK.linear(x, ww, out, rows, ld=n, bias=bias, sigmoid=True)
+        HK.linear(x, ww, out, rows, ld=n, bias=bias, act=H.ACT_SIGMOID)
         assert _rel(_np(out), R.sigmoid(z)) < (1e-5 if dtype == "float32" else 6e-3)
 
 
@@ -62,7 +63,7 @@ def test_linears_with_inputs_of_their_own(dtype, rows):
             w, x = _dev(rng.standard_normal((n, k)) / np.sqrt(k)).to(T[dtype]), _dev(rng.standard_normal((rows, k)), T[dtype])
             ww = HK.WideWeight(w.float(), T[dtype], tail=5 if i == 1 else 0)
             out = torch.full((rows, ww.n_main), 7.0, dtype=T[dtype], device="cuda")
-            calls.append((x, ww, out, dict(tail=tail if i == 1 else None, sigmoid=i == 2)))
+            calls.append((x, ww, out, dict(tail=tail if i == 1 else None, act=H.ACT_SIGMOID if i == 2 else H.ACT_NONE)))
             want.append(_np(x) @ _np(w).T)
         HK.linear_group(rows, *calls)
         tol = 1e-5 if dtype == "float32" else 6e-3
@@ -167,11 +168,11 @@ class Case:
     sequence holds."""
 
     def __init__(self, dtype, heads, dim, rot, vdim, kv_rank, window, ring_len, lens, seed=0, plant=()):
-        from poptransformer_amd.engine.hybrid import LatentMixer
+        from poptransformer_amd.engine.hybrid import LatentMixer, Rotation
         self.HK, self.T = _hk()
         T = self.dtype = self.T[dtype]
         rng = np.random.default_rng(seed)
-        self.m = m = LatentMixer(heads, dim, rot, vdim, 24, kv_rank, (dim + rot) ** -0.5 * 2, window, 20.0, rot)
+        self.m = m = LatentMixer(heads, dim, rot, vdim, 24, kv_rank, (dim + rot) ** -0.5 * 2, window, Rotation(20.0, rot))
         _, D, P, E, Rp, _, _ = m.sizes
         self.lens, self.ring_len, self.slots = lens, ring_len, [2 * i + 1 for i in range(len(lens))]
         total = max(lens)
@@ -296,11 +297,11 @@ def test_one_key_at_the_edge_of_the_window(window, dtype, absorbed):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("own", [True, False])
 def test_latent_norms_and_cache_entries(dtype, own):
-    from poptransformer_amd.engine.hybrid import LatentMixer
+    from poptransformer_amd.engine.hybrid import LatentMixer, Rotation
     HK, T = _hk()
     rng = np.random.default_rng(0)
     for q_rank, kv_rank, rot in ((30, 44, 6), (300, 512, 64), (9, 32, 32)):
-        m = LatentMixer(2, 16, rot, 16, q_rank, kv_rank, 1.0, 10, 7.0, rot)
+        m = LatentMixer(2, 16, rot, 16, q_rank, kv_rank, 1.0, 10, Rotation(7.0, rot))
         _, D, P, E, Rp, _, _ = m.sizes
         Qp, pairs, n, slots, ring_len = HK.pad8(q_rank), m.pairs(), 40, 3, 64
         cq, c, k = (rng.standard_normal((n, w)) for w in (q_rank, kv_rank, rot))
