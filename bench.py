@@ -27,8 +27,8 @@ Other workloads (``--workload``), each printing one line of the same form: ``gem
 weight-only operator X[M, 4096] by W[4096, 11008] at M = ``--batch``; ``chatglm2`` = ChatGLM2-6B-shape FP8
 decode; ``rwkv`` = RWKV-4-7B-shape INT4 recurrent decode; ``prompt`` = the prompt of the headline model taken in
 passes of ``--rows-per-pass`` rows (a step is one pass) instead of one position per loop iteration; ``zekilix``,
-``ruperax`` and ``golapel`` = these designs (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights (and, for
-Ruperax and Golapel, the Zekilix design) at the same sizes: decode at batch 1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
+``ruperax``, ``golapel`` and ``sabolorn`` = these designs (bf16) at two layer sizes beside the Llama-2 executor with fp16 weights (and, for
+Ruperax, Golapel and Sabolorn, the Zekilix design) at the same sizes: decode at batch 1 and 16, and prompt passes.  ``--copy-calibration`` and ``--summarize-pmc``
 serve the hardware-counter measurement of the HBM traffic (see their help).
 """
 import argparse
@@ -460,14 +460,38 @@ def golapel_config(width, ff, layers):
             "norm": {"eps": 1e-5}, "vocab": 32000, "width": width}
 
 
+def sabolorn_config(width, ff, layers):
+    """Two state-space layers (inner size twice the width, heads of 64, states of 128) to one with latent attention and one with attention
+    by heads; every second layer has a mixture of experts: 6 of 64 in 8 groups, of which 4 are kept, with half the dense feed-forward's
+    parameters per token."""
+    scale = 128 ** -0.5
+    dense = {"kind": "dense", "ff": ff * 3 // 2}
+    moe = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 64, "top": 6, "groups": {"count": 8, "keep": 4}}}
+    space = {"heads": width // 32, "groups": 8, "state": 128, "vdim": 64, "conv": 4, "norm_groups": 8}
+    rot = {"base": 1e4, "dims": 64, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}
+    low = {"heads": width // 128, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": width * 3 // 8, "kv_rank": 512, "scale": 192 ** -0.5, "rot": rot}
+    heads = {"heads": width // 128, "kv_heads": width // 512, "dim": 128, "vdim": 128, "conv": 4, "scale": scale}
+    period = [{"type": "mamba2", "mixer": space, "mlp": dense}, {"type": "latent_attention", "mixer": low, "mlp": moe},
+              {"type": "mamba2", "mixer": space, "mlp": moe}, {"type": "attention", "mixer": heads, "mlp": dense}]
+    return {"architecture": "Sabolorn", "embedding": {"scale": 16.0}, "layers": (period * layers)[:layers], "logit_softcap": 30.0,
+            "norm": {"eps": 1e-5}, "token_side": {"dim": 256}, "vocab": 32000, "width": width}
+
+
 def hybrid_step_bytes(spec, weights, B, t):
     """Bytes one decode iteration of a hybrid decoder must move at context t: the weights of every layer run (of a mixture the
     experts that the rows choose on average), the key rows that are seen, the memories (read and written), the head."""
-    n = weights.head.nbytes if spec.family != "golapel" else weights.nbytes(B)
+    n = weights.head.nbytes if spec.family not in ("golapel", "sabolorn") else weights.nbytes(B)
     for lay in spec.layers:
         m = lay.mixer
         if m.kind == "heads":
-            n += B * m.kv_heads * 2 * (m.maps * m.dim + m.vdim) * (min(t + 1, m.keep + m.window) if m.window else t % m.chunk + 1)
+            seen = min(t + 1, m.keep + m.window) if m.window else t % m.chunk + 1 if m.chunk else t + 1
+            n += B * m.kv_heads * 2 * (m.maps * m.dim + m.vdim) * seen
+            continue
+        if m.kind == "ssd":
+            n += B * 2 * 4 * m.heads * m.dim * m.vdim
+            continue
+        if spec.family == "sabolorn":
+            n += B * 2 * (m.kv_rank + m.rot_dim) * (t + 1)
             continue
         n += sum(w.nbytes for w in weights.layers[lay.source].linears())
         seen = min(t + 1, getattr(m, "window", None) or t + 1)
@@ -486,7 +510,7 @@ def design_workload(args, design):
     Zekilix) at equal width, feed-forward size, layer count, vocabulary and head size.  --layers shortens all of them (for
     profiles)."""
     import torch
-    from poptransformer_amd.engine import fused, hybrid, loader, parallel, result_norm, synthetic
+    from poptransformer_amd.engine import depth, fused, hybrid, loader, parallel, result_norm, synthetic
     rng = np.random.Generator(np.random.PCG64(1234))
     first, steps, max_len = 1024, args.steps, 2048
     results = []
@@ -516,12 +540,15 @@ def design_workload(args, design):
         elif name == "golapel":
             cfg, spec_of, tensors, weights_of, decoder = (golapel_config(width, ff, layers), loader.golapel_spec, synthetic.HeadTensors,
                                                           loader.result_norm_weights, result_norm.ResultNormDecoder)
+        elif name == "sabolorn":
+            cfg, spec_of, tensors, weights_of, decoder = (sabolorn_config(width, ff, layers), loader.sabolorn_spec, synthetic.DepthTensors,
+                                                          loader.depth_weights, depth.DepthDecoder)
         else:
             cfg, spec_of, tensors, weights_of, decoder = (ruperax_config(width, ff, layers), loader.ruperax_spec, synthetic.ParallelTensors,
                                                           loader.parallel_weights, parallel.ParallelDecoder)
         spec = spec_of(cfg, max_len, 1)
         w = weights_of(tensors(cfg), spec)
-        if name == "golapel":
+        if name in ("golapel", "sabolorn"):
             params = sum(lw.active_parameters() for lw in w.layers)
             return lambda B, L: decoder(spec_of(cfg, L, B), w), lambda B, t: hybrid_step_bytes(spec, w, B, t), params
         params = sum(x.n_main * x.K for lay in spec.layers for x in w.layers[lay.source].linears())
@@ -595,15 +622,15 @@ def main():
     ap.add_argument("--batch", type=int, default=1)
     ap.add_argument("--executor", choices=["persistent", "operators"], default=None,
                     help="default: persistent when the batch fits it (<= 16, fp16 cache), else operators")
-    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix", "ruperax", "golapel"], default="decode",
+    ap.add_argument("--workload", choices=["decode", "gemm", "chatglm2", "rwkv", "prompt", "zekilix", "ruperax", "golapel", "sabolorn"], default="decode",
                     help="decode: the Llama2-7B-shape INT4 decode loop (the headline); gemm: the single INT4 "
                          "weight-only operator at M = --batch rows; chatglm2: ChatGLM2-6B-shape FP8 decode; "
                          "rwkv: RWKV-4-7B-shape INT4 recurrent decode; prompt: the headline model's prompt in passes "
-                         "of --rows-per-pass rows (--steps passes); zekilix, ruperax, golapel: that design beside Llama-2 with fp16 "
+                         "of --rows-per-pass rows (--steps passes); zekilix, ruperax, golapel, sabolorn: that design beside Llama-2 with fp16 "
                          "weights (the latter two: and Zekilix) at equal sizes, decode and prompts")
     ap.add_argument("--width", type=int, default=0, help="workloads of a design: only this width")
     ap.add_argument("--layers", type=int, default=0, help="workloads of a design: layers of the models (even)")
-    ap.add_argument("--only", choices=["zekilix", "ruperax", "golapel", "llama2"], default=None, help="workloads of a design: one of the models")
+    ap.add_argument("--only", choices=["zekilix", "ruperax", "golapel", "sabolorn", "llama2"], default=None, help="workloads of a design: one of the models")
     ap.add_argument("--decode-only", action="store_true", help="workloads of a design: no prompts")
     ap.add_argument("--rows-only", action="store_true", help="workloads of a design: prompts only")
     ap.add_argument("--one-stream", action="store_true", help="ruperax workload: no feed-forward on a stream beside the mixer (for profiles)")
@@ -655,7 +682,7 @@ def main():
     if args.workload == "prompt":
         print(json.dumps(prompt_workload(args)))
         return
-    if args.workload in ("zekilix", "ruperax", "golapel"):
+    if args.workload in ("zekilix", "ruperax", "golapel", "sabolorn"):
         print(json.dumps(design_workload(args, args.workload)))
         return
     B, cfg = args.batch, LLAMA2_7B

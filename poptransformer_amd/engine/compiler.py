@@ -1,8 +1,8 @@
 """From a recorded graph to something that runs: `Session.compile` ends here.
 
 Every graph can run op by op (engine/interpreter.py).  A graph that is one of the decoder loops
-this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix, Ruperax, Golapel as the models build them through the operator
-API - is additionally mapped onto the fused executor for its family: the family is read off the
+this package knows - GPT-2, Llama 2, ChatGLM2, RWKV, Zekilix, Ruperax, Golapel, Sabolorn as the models build them through
+the operator API - is additionally mapped onto the fused executor for its family: the family is read off the
 state-dict keys the layers registered as initializer names, the shapes off a one-iteration probe of
 the interpreter, and the weights off the initializers.  The fused executor is then VALIDATED: it
 must generate the same token ids as the interpreter on a probe prompt (for a sampling graph: the same top-k candidates), otherwise
@@ -264,24 +264,76 @@ def _executor_dtype():
     return {"bf16": "bfloat16", "fp32": "float32"}[REGISTRY.get("tensor_type").precision]
 
 
+def _latent_mixer(facts, const, i):
+    from .hybrid import LatentMixer, Rotation
+    numbers = const(f"l{i}.mixer")
+    uk, uv, uq = (_need(facts, f"l{i}.mix.{n}") for n in ("uk", "uv", "uq"))
+    heads = int(numbers[0])
+    dim = uk.shape[0] // heads
+    return LatentMixer.of(numbers, dim, uq.shape[0] // heads - dim, uv.shape[0] // heads, uq.shape[1], uk.shape[1],
+                          Rotation.of(const(f"l{i}.rotation")))
+
+
+def _head_mixer(facts, const, i):
+    from .hybrid import HeadMixer, Rotation
+    mix, numbers, rot = f"l{i}.mix.", const(f"l{i}.mixer"), const(f"l{i}.rotation", False)
+    dim = HeadMixer.of(numbers, 1, 1, "", None)
+    dim = _need(facts, mix + "q").shape[0] // (dim.heads * dim.maps)
+    vdim = facts.init[mix + "v"].shape[0] // int(numbers[1]) if facts.has(mix + "v") else dim
+    return HeadMixer.of(numbers, dim, vdim, "".join(n for n in "qkv" if facts.has(mix + n + ".b")), Rotation.of(rot) if rot is not None else None)
+
+
+def _experts(facts, const, i):
+    """The mixture of experts of layer i, or None."""
+    from .hybrid import ClampedGLU, Experts, SwiGLU
+    numbers, limits, mlp = const(f"l{i}.experts", False), const(f"l{i}.limits", False), f"l{i}.mlp."
+    if numbers is None:
+        return None
+    parts = [_need(facts, mlp + n + ".gate").shape[0] for n in ("e0", "shared") if facts.has(mlp + n + ".gate")]
+    return Experts.of(numbers, *(SwiGLU(ff) if limits is None else ClampedGLU(ff, float(limits[k])) for k, ff in enumerate(parts)))
+
+
+def _build_depth(facts, topk=1):
+    """As _build_result_norm, for layers whose results are averaged over the depths."""
+    from .depth import DepthDecoder
+    from .hybrid import HybridLayer, HybridSpec, SquaredReLU, StateSpaceMixer
+    from .loader import depth_weights
+    const = _const_reader(facts)
+    layers = []
+    while const(f"l{len(layers)}.mixer", False) is not None:
+        i = len(layers)
+        mix, up = f"l{i}.mix.", f"l{i}.mlp.up"
+        if facts.has(mix + "uk"):
+            mixer = _latent_mixer(facts, const, i)
+        elif facts.has(mix + "A_log"):
+            mixer = StateSpaceMixer.of(const(f"l{i}.mixer"))
+        else:
+            mixer = _head_mixer(facts, const, i)
+        ff = _experts(facts, const, i)
+        if ff is None and facts.has(up):
+            ff = SquaredReLU(facts.init[up].shape[0])
+        layers.append(HybridLayer(mixer, ff, i))
+    if not layers:
+        raise ValueError("no layers found among the graph's constants")
+    vocab, width = _need(facts, "embed").shape
+    cap = const("logit_softcap", False)
+    spec = HybridSpec("sabolorn", layers, width, vocab, 1, float(const("eps")), 1.0, float(const("embedding_scale")),
+                      float(cap) if cap is not None else 0.0, facts.max_len, facts.batch, facts.pad_id, facts.eos_id, facts.early_stop, topk,
+                      _executor_dtype(), side_dim=_need(facts, "side.embed").shape[1] // len(layers))
+    return DepthDecoder(spec, depth_weights(facts.init, spec))
+
+
 def _build_parallel(facts, topk=1):
     """As _build_hybrid, for layers with latent attention whose sublayers stand side by side."""
-    from .hybrid import BiasedSwiGLU, HybridLayer, HybridSpec, LatentMixer, Rotation
+    from .hybrid import BiasedSwiGLU, HybridLayer, HybridSpec
     from .loader import parallel_weights
     from .parallel import ParallelDecoder
     const = _const_reader(facts)
     layers = []
-    while const(f"l{len(layers)}.cache_of", False) is not None:
+    while const(f"l{len(layers)}.mixer", False) is not None:
         i = len(layers)
-        mix = f"l{i}.mix."
-        heads, source = int(const(f"l{i}.heads")), int(const(f"l{i}.cache_of"))
-        uk, uv, uq = (_need(facts, mix + n) for n in ("uk", "uv", "uq"))
-        dim = uk.shape[0] // heads
-        mixer = LatentMixer(heads, dim, uq.shape[0] // heads - dim, uv.shape[0] // heads, uq.shape[1], uk.shape[1],
-                            float(const(f"l{i}.scale")), int(const(f"l{i}.window")) or None,
-                            Rotation(float(const(f"l{i}.rot_base")), int(const(f"l{i}.rot_dims"))), source if source != i else None)
         ff = f"l{i}.mlp.gate"
-        layers.append(HybridLayer(mixer, BiasedSwiGLU(_need(facts, ff).shape[0]) if facts.has(ff) else None, i, shift=True))
+        layers.append(HybridLayer(_latent_mixer(facts, const, i), BiasedSwiGLU(_need(facts, ff).shape[0]) if facts.has(ff) else None, i, shift=True))
     if not layers:
         raise ValueError("no layers found among the graph's constants")
     vocab, width = _need(facts, "embed").shape
@@ -294,26 +346,18 @@ def _build_parallel(facts, topk=1):
 def _build_result_norm(facts, topk=1):
     """As _build_hybrid, for layers with attention by heads whose results are normed: the layers recorded the numbers of their
     mixers, rotations and mixtures of experts as one constant each."""
-    from .hybrid import ClampedGLU, Experts, HeadMixer, HybridLayer, HybridSpec, Rotation, SwiGLU
+    from .hybrid import HybridLayer, HybridSpec, SwiGLU
     from .loader import result_norm_weights
     from .result_norm import ResultNormDecoder
     const = _const_reader(facts)
     layers = []
     while const(f"l{len(layers)}.mixer", False) is not None:
         i = len(layers)
-        mix, mlp = f"l{i}.mix.", f"l{i}.mlp."
-        numbers, rot = const(f"l{i}.mixer"), const(f"l{i}.rotation", False)
-        dim = _need(facts, mix + "q.norm").shape[0]
-        vdim = facts.init[mix + "v"].shape[0] // int(numbers[1]) if facts.has(mix + "v") else dim
-        mixer = HeadMixer.of(numbers, dim, vdim, "".join(n for n in "qkv" if facts.has(mix + n + ".b")), Rotation.of(rot) if rot is not None else None)
-        experts, ff = const(f"l{i}.experts", False), None
-        if experts is not None:
-            count, top, scale, limit, *shared = (float(v) for v in experts)
-            ff = Experts(int(count), int(top), scale, ClampedGLU(_need(facts, mlp + "e0.gate").shape[0], limit),
-                         ClampedGLU(_need(facts, mlp + "shared.gate").shape[0], shared[0]) if shared else None)
-        elif facts.has(mlp + "gate"):
-            ff = SwiGLU(facts.init[mlp + "gate"].shape[0])
-        layers.append(HybridLayer(mixer, ff, i))
+        gate = f"l{i}.mlp.gate"
+        ff = _experts(facts, const, i)
+        if ff is None and facts.has(gate):
+            ff = SwiGLU(facts.init[gate].shape[0])
+        layers.append(HybridLayer(_head_mixer(facts, const, i), ff, i))
     if not layers:
         raise ValueError("no layers found among the graph's constants")
     vocab, width = _need(facts, "embed").shape
@@ -365,6 +409,8 @@ def _family(facts):
         return "gpt2"
     if facts.has("rwkv.blocks.0.attention.key.weight"):
         return "rwkv"
+    if facts.has("l0.dwa"):
+        return "sabolorn"
     if facts.has("l0.mix.q") and facts.has("l0.norm1") and facts.has("head"):
         return "zekilix"
     if facts.has("l0.mix.q.norm") and facts.has("l0.norm1"):          # the embedding is the head
@@ -566,7 +612,7 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
         prog.interp_outputs = list(graph.outputs)
         k = _sampling_k(facts)
         use_fp8_cache = _fp8_cache_of(facts, fp8_cache)
-        if use_fp8_cache and family in ("rwkv", "zekilix", "ruperax", "golapel"):
+        if use_fp8_cache and family in ("rwkv", "zekilix", "ruperax", "golapel", "sabolorn"):
             raise ValueError(f"fp8_cache: the {family} executor has no FP8 KV cache")
         steps = min(PROBE_STEPS, facts.max_loop)
         # one-iteration probe: operand shapes of the native operators
@@ -583,6 +629,8 @@ def compile_graph(graph, anchors, batches_per_step=1, allow_fused=True, strict=F
             decoder = _build_parallel(facts, k)
         elif family == "golapel":
             decoder = _build_result_norm(facts, k)
+        elif family == "sabolorn":
+            decoder = _build_depth(facts, k)
         else:
             spec, weights = _build_transformer(facts, shapes, family, k, use_fp8_cache)
             decoder = fused.FusedDecoder(spec, weights)

@@ -116,6 +116,7 @@ class Interpreter:
     def _aiOnnx_relu(self, n, env, x): return torch.relu(x)
     def _aiOnnx_sigmoid(self, n, env, x): return torch.sigmoid(x)
     def _aiOnnx_exp(self, n, env, x): return torch.exp(x)
+    def _aiOnnx_log(self, n, env, x): return torch.log(x)
     def _aiOnnx_abs(self, n, env, x): return torch.abs(x)
     def _aiOnnx_softplus(self, n, env, x): return torch.nn.functional.softplus(x)
     def _aiOnnx_sqrt(self, n, env, x): return torch.sqrt(x)

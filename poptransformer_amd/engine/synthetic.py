@@ -280,3 +280,49 @@ class HeadTensors(HybridTensors):
         if len(shape) == 1 and (name.endswith(".b") or name.split(".")[-1] in ("sink", "lq1", "lk1", "lq2", "lk2")):
             return torch.zeros(shape, device=self.dev)
         return super().__getitem__(name)
+
+
+class DepthTensors(HybridTensors):
+    """As HybridTensors, for a configuration whose results are averaged over the depths."""
+
+    def __init__(self, cfg, seed=0, device="cuda"):
+        super().__init__(dict(cfg, layers=[], streams=None), seed, device)
+        d, n = cfg["width"], cfg["token_side"]["dim"]
+        del self.shapes["head"]
+        self.shapes["side.embed"] = (cfg["vocab"], len(cfg["layers"]) * n)
+        for i, lay in enumerate(cfg["layers"]):
+            p, m, f, kind = f"l{i}.", lay["mixer"], lay["mlp"], lay["type"]
+            H, E = m["heads"], m["vdim"]
+            mix = {"o": (d, H * E)}
+            if kind == "latent_attention":
+                D, P, R, Q = m["dim"], m["rot_dim"], m["kv_rank"], m["q_rank"]
+                mix.update({"dq": (Q, d), "dq.norm": (Q,), "uq": (H * (D + P), Q), "uk": (H * D, R), "uv": (H * E, R), "g": (H * E, d)})
+                if m.get("kv_from") is None:
+                    mix.update({"dkv": (R + P, d), "dkv.norm": (R,)})
+            elif kind == "attention":
+                for name, c in (("q", H * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * E)):
+                    mix.update({name: (c, d), name + ".b": (c,), name + ".conv": (c, m["conv"])})
+                mix.update({"r1": (H,), "r2": (H,)})
+            else:
+                inner, states = H * E, m["groups"] * m["state"]
+                mix.update({"in": (2 * inner + 2 * states + H, d), "conv": (inner + 2 * states, m["conv"]), "conv.b": (inner + 2 * states,),
+                            "dt_bias": (H,), "A_log": (H,), "D": (H,), "norm": (inner,)})
+            mlp = {}
+            if f["kind"] == "dense":
+                mlp = {"up": (f["ff"], d), "down": (d, f["ff"])}
+            else:
+                count, ff = f["router"]["experts"], f["expert"]["ff"]
+                mlp = {"router": (count, d), "correction": (count,)}
+                for e in range(count):
+                    mlp.update({f"e{e}.gate": (ff, d), f"e{e}.up": (ff, d), f"e{e}.down": (d, ff)})
+            rest = {"norm1": (d,), "dwa": (i + 2,), "side.gate": (n, d), "side.proj": (d, n), "side.norm": (d,)}
+            for group, names in (("mix.", mix), ("mlp.", mlp), ("", rest)):
+                self.shapes.update({p + group + name: shape for name, shape in names.items()})
+
+    def __getitem__(self, name):
+        shape, last = self.shapes[name], name.split(".")[-1]
+        if len(shape) == 1 and last in ("b", "correction", "A_log"):
+            return torch.zeros(shape, device=self.dev)
+        if last in ("dt_bias", "dwa", "r1", "r2"):
+            return torch.full(shape, {"dt_bias": -3.0, "dwa": 1.0 / shape[0], "r1": 0.5, "r2": 0.1}[last], device=self.dev)
+        return super().__getitem__(name)

@@ -11,7 +11,10 @@ from .lm_head import LMHead
 from .streams import NamedLinear, StreamConnection, WeightNorm
 from .parallel import BiasedSwiGLU, GroupedRMSNorm, ResultGate, RotaryTable, TokenShift
 from .heads import ExpertMixture, HeadAttention, SwiGLU
+from .latent import LatentAttention
+from .state_space import ShortConvolution, StateSpace
+from .depth import DepthAverage, SquaredReLU, TokenInput
 
 __all__ = ["BaseLayer", "Linear", "LayerNorm", "RMSLayerNorm", "Embedding", "MLP", "LMHead", "NamedLinear", "StreamConnection",
            "WeightNorm", "BiasedSwiGLU", "GroupedRMSNorm", "ResultGate", "RotaryTable", "TokenShift", "HeadAttention",
-           "SwiGLU", "ExpertMixture"]
+           "SwiGLU", "ExpertMixture", "LatentAttention", "ShortConvolution", "StateSpace", "DepthAverage", "SquaredReLU", "TokenInput"]

@@ -2,66 +2,18 @@
 
 hf_config: the design's config.json (keys architecture, embedding, layers, max_positions, norm, vocab, width).  Layer i's
 tensors start with `l<i>.`; a layer whose mixer has `kv_from` reads another layer's cache.  The model is recorded one token
-per loop iteration, as the other decoders are; the constants a fused executor needs are recorded under names of their own
-(`l<i>.window` and so on).
+per loop iteration, as the other decoders are; what a fused executor needs is recorded in constants of the layers (`l<i>.mixer`,
+`l<i>.rotation`).
 """
 import numpy as np
 
 from ... import ops
+from ...engine.loader import latent_layers
 from ...layers import BaseLayer
+from ...layers.latent import LatentAttention
 from ...layers.parallel import BiasedSwiGLU, GroupedRMSNorm, ResultGate, RotaryTable, TokenShift
 from ...layers.streams import NamedLinear, WeightNorm, scalar
 from ..base_model import HFDecBaseModel
-
-
-class LatentAttention(BaseLayer):
-    """Attention over the newest `window` positions with keys and values made from a cached latent and one rotated key part
-    that the heads share; queries through a latent of their own, a sigmoid gate per head."""
-
-    def __init__(self, context, name, width, eps, max_length, rotation, heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot, mask=None,
-                 kv_from=None):
-        super().__init__(context, name)
-        self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.scale = heads, dim, rot_dim, vdim, kv_rank, scale
-        self.rot, self.rotation, self.kv_from = rot, rotation, kv_from
-        self.window = (mask or {}).get("size")
-        self.rows = min(self.window or max_length, max_length)
-        self.dq = NamedLinear(self.context, "dq", width, q_rank)
-        self.q_norm = WeightNorm(self.context, "dq.norm", q_rank, eps, centred=False)
-        self.uq = NamedLinear(self.context, "uq", q_rank, heads * (dim + rot_dim))
-        if kv_from is None:
-            self.dkv = NamedLinear(self.context, "dkv", width, kv_rank + rot_dim)
-            self.kv_norm = WeightNorm(self.context, "dkv.norm", kv_rank, eps, centred=False)
-        self.uk, self.uv = (NamedLinear(self.context, n, kv_rank, heads * c) for n, c in (("uk", dim), ("uv", vdim)))
-        self.g, self.o = NamedLinear(self.context, "g", width, heads), NamedLinear(self.context, "o", heads * vdim, width)
-
-    def cache(self, graph, h, step, rows):
-        """The newest `rows` cache entries [B, rows, kv_rank + rot_dim], newest first."""
-        B, R, P = self.batch_size, self.kv_rank, self.rot_dim
-        c, k = ops.split(graph, self.dkv(graph, h), 2, axis=2, splits=[R, P], name="split_latent")
-        entry = ops.concat(graph, self.kv_norm(graph, c), self.rotation(graph, k, step, P), 2)
-        past = ops.kv_cache(graph, step, ops.reshape(graph, entry, [B, 1, 1, R + P]), rows, 2, 1)
-        return ops.reshape(graph, past, [B, rows, R + P])
-
-    def __call__(self, graph, h, layer_id, step, attention_mask, cache):
-        B, H, D, P, E, R, W = self.batch_size, self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank, self.rows
-        with graph.nameScope(self.context):
-            for fact, value in (("window", self.window or 0), ("heads", H), ("rot_dims", self.rot["dims"])):
-                ops.constant(graph, np.array(value).astype(np.int32), f"l{layer_id}.{fact}")
-            ops.constant(graph, np.array(self.rot["base"], np.float64), f"l{layer_id}.rot_base")     # (fp32 would move far angles)
-            q = self.uq(graph, self.q_norm(graph, self.dq(graph, h)))
-            q, q_rot = ops.split(graph, ops.reshape(graph, q, [B, H, D + P]), 2, axis=2, splits=[D, P], name="split_query")
-            q = ops.concat(graph, q, self.rotation(graph, q_rot, step, P), 2)
-            past = ops.static_slice(graph, cache, [0], [W], [1])
-            c, k_rot = ops.split(graph, past, 2, axis=2, splits=[R, P], name="split_cache")
-            k = ops.transpose(graph, ops.reshape(graph, self.uk(graph, c), [B, W, H, D]), [0, 2, 3, 1])
-            k_rot = ops.tile(graph, ops.transpose(graph, ops.reshape(graph, k_rot, [B, W, 1, P]), [0, 2, 3, 1]), [1, H, 1, 1])
-            v = ops.transpose(graph, ops.reshape(graph, self.uv(graph, c), [B, W, H, E]), [0, 2, 1, 3])
-            s = ops.matmul(graph, ops.reshape(graph, q, [B, H, 1, D + P]), ops.concat(graph, k, k_rot, 2))
-            s = ops.mul(graph, s, scalar(graph, self.scale, f"l{layer_id}.scale"))
-            s = ops.add(graph, s, ops.static_slice(graph, attention_mask, [0], [W], [3]))
-            o = ops.matmul(graph, ops.softmax_ce(graph, s, -1, stable_mode=True), v)
-            o = ops.mul(graph, o, ops.reshape(graph, ops.sigmoid(graph, self.g(graph, h)), [B, H, 1, 1]))
-            return self.o(graph, ops.reshape(graph, o, [B, 1, H * E]))
 
 
 class Block(BaseLayer):
@@ -69,26 +21,22 @@ class Block(BaseLayer):
 
     def __init__(self, context, layer, width, eps, groups, max_length, rotation):
         super().__init__(None, context)
-        if layer["type"] != "latent_attention":
-            raise ValueError(f"Invalid mixer {layer['type']}, options: ['latent_attention']")
         self.norm1 = GroupedRMSNorm(self.context, "norm1", width, eps, groups)
         self.shift = TokenShift(self.context, "shift", width)
-        self.mixer = LatentAttention(self.context, "mix", width, eps, max_length, rotation, **layer["mixer"])
+        self.mixer = LatentAttention(self.context, "mix", width, eps, max_length, layer.mixer, rotation)
         self.gate1 = ResultGate(self.context, "rg1", width)
         self.mlp = None
-        if layer.get("mlp") is not None:
+        if layer.mlp is not None:
             self.norm2 = GroupedRMSNorm(self.context, "norm2", width, eps, groups)
-            self.mlp = BiasedSwiGLU(self.context, "mlp", width, **layer["mlp"])
+            self.mlp = BiasedSwiGLU(self.context, "mlp", width, layer.mlp.ff)
             self.gate2 = ResultGate(self.context, "rg2", width)
 
     def __call__(self, graph, x, layer_id, step, attention_mask, before, caches, cache_rows):
         h1 = self.norm1(graph, x)
         h, before = self.shift(graph, h1, before)
-        if self.mixer.kv_from is None:
-            with graph.nameScope(self.mixer.context):
-                caches[layer_id] = self.mixer.cache(graph, h, step, cache_rows)
-        source = layer_id if self.mixer.kv_from is None else self.mixer.kv_from
-        ops.constant(graph, np.array(source).astype(np.int32), f"l{layer_id}.cache_of")
+        source = self.mixer.mixer.source
+        if source is None:
+            source, caches[layer_id] = layer_id, self.mixer.cache(graph, h, step, cache_rows)
         y = self.gate1(graph, h1, self.mixer(graph, h, layer_id, step, attention_mask, caches[source]))
         if self.mlp is not None:
             h2 = self.norm2(graph, x)
@@ -112,16 +60,16 @@ class RuperaxDecModel(HFDecBaseModel):
         self.pos_id = self._tensor("pos", [c.max_positions, c.width])
         rotations = {}
         self.blocks = []
-        for i, layer in enumerate(c.layers):
-            rot = layer["mixer"]["rot"]
-            key = (rot["base"], rot["dims"])
+        for i, layer in enumerate(latent_layers(c.layers)):
+            rot = layer.mixer.rot
+            key = (rot.base, rot.dims)
             if key not in rotations:
                 rotations[key] = RotaryTable(f"rotary{len(rotations)}", self.max_length, *key)
             self.blocks.append(Block(f"l{i}", layer, c.width, eps, groups, self.max_length, rotations[key]))
         self.final_norm = GroupedRMSNorm(None, "final.norm", c.width, eps, groups)
         self.head = NamedLinear(None, "head", c.width, c.vocab)
         # a cache holds what the widest window over it sees
-        self.cache_rows = [max(b.mixer.rows for j, b in enumerate(self.blocks) if i in (j, b.mixer.kv_from)) for i in range(len(self.blocks))]
+        self.cache_rows = [max(b.mixer.rows for j, b in enumerate(self.blocks) if i in (j, b.mixer.mixer.source)) for i in range(len(self.blocks))]
 
     def _tensor(self, key, shape):
         value = self.state_dict.get(key)
