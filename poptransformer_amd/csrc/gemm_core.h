@@ -1995,7 +1995,8 @@ template <class Fmt, bool PAIR>
 static int dispatch_many_rows(const GemmArgs& a, int total_nb, hipStream_t s, const char* name) {
   const int cus = device_compute_units();
   const int per_wg = PAIR ? 4 : 8;
-  const bool tiles = a.epi.norm == PTA_NORM_NONE && tile_fits(a, per_wg, 2, PAIR);
+  // (few features: the wide formats only, whose other path would take 64 rows per launch)
+  const bool tiles = a.epi.norm == PTA_NORM_NONE && tile_fits(a, per_wg, Fmt::kWide ? 0 : 2, PAIR);
   // More than 128 rows (measured on whole prompt passes of the 7B shape, gemm_rows_kernel against this: 6.5 against
   // 7.2 ms at 128 rows, 7.7 against 7.3 at 192, 8.1 against 7.5 at 256): 128-row panels through LDS, the weights
   // straight into registers.  Formats of up to two vectors per tile only - with four (fp16) two tiles of four

@@ -131,6 +131,7 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
   __shared__ float sm[NG][NQ], sl[NG][NQ], inv_s[NQ];
   __shared__ __align__(16) float so[NG * NQ * DL];
   __shared__ float res[NQ * DL];
+  __shared__ __align__(16) float s_conv[MAPS == 1 ? (RG + 2) * DL : 8];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int D = a.D, E = a.E, R = a.H / a.G;
   int b = blockIdx.x;
@@ -177,12 +178,24 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     for (int t = 0; t < MAPS; ++t) load8(proj_q + (head * MAPS + t) * D + (dk ? d0 : 0), true, 8, qv[h * MAPS + t]);
     far1[h] = a.far1 ? a.far1[head] : 0.f;
     far2[h] = a.far1 ? a.far2[head] : 0.f;
-    if constexpr (MAPS == 1) {
-      if (a.conv.ring && fused) {
-        const int c0 = head * D + (dk ? d0 : 0);
-        if (split == 0 && grp == 0 && dk && hg * RG + h < R) store8(conv_place<T>(a.conv, slot, i, c0), qv[h]);
-        conv8<T>(a.conv, slot, i, c0, qv[h]);
+  }
+  const bool convolved = MAPS == 1 && fused && a.conv.ring;
+  if constexpr (MAPS == 1) {
+    if (convolved) {                                      // the workgroup's queries, and the row's own key and value: a thread per piece
+      for (int p = threadIdx.x; p < (RG + 2) * LPK; p += 256) {
+        const int which = p / LPK, d = p % LPK * 8;
+        if (d >= (which <= RG ? D : E) || (which >= RG && !own)) continue;
+        const int hr = hg * RG + which < R ? hg * RG + which : R - 1;
+        const int c0 = (which < RG ? (g * R + hr) * D : which == RG ? (a.H + g) * D : (a.H + a.G) * D + g * E) + d;
+        float v[8];
+        load8(proj_q + c0, true, 8, v);
+        if (which < RG ? split == 0 && hg * RG + which < R : hg == 0) store8(conv_place<T>(a.conv, slot, i, c0), v);
+        conv8<T>(a.conv, slot, i, c0, v);
+        store8(s_conv + p * 8, v);
       }
+      __syncthreads();
+#pragma unroll
+      for (int h = 0; h < RG; ++h) load8(s_conv + (h * LPK + sub) * 8, true, 8, qv[h]);
     }
   }
 #pragma unroll
@@ -254,23 +267,14 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     load8(reinterpret_cast<const T*>(a.v) + (size_t)r * a.ld + g * E + (dv ? d0 : 0), true, 8, vv[0]);
     const bool put = hg == 0 && grp == 0;
     const int row = ring_row(a, i);
-    if constexpr (MAPS == 1) {
-      if (a.conv.ring) {
-        const int c0 = (a.H + a.G) * D + g * E + (dv ? d0 : 0);
-        if (put && dv) store8(conv_place<T>(a.conv, slot, i, c0), vv[0]);
-        conv8<T>(a.conv, slot, i, c0, vv[0]);
-      }
+    if (convolved) {
+      load8(s_conv + ((RG + 1) * LPK + sub) * 8, true, 8, vv[0]);
+      zero_past(dv, vv[0]);
     }
 #pragma unroll
     for (int t = 0; t < MAPS; ++t) {
       load8(pk + t * D, true, 8, kv[0][t]);
-      if constexpr (MAPS == 1) {
-        if (a.conv.ring) {
-          const int c0 = (a.H + g) * D + (dk ? d0 : 0);
-          if (put && dk) store8(conv_place<T>(a.conv, slot, i, c0), kv[0][t]);
-          conv8<T>(a.conv, slot, i, c0, kv[0][t]);
-        }
-      }
+      if (convolved) load8(s_conv + (RG * LPK + sub) * 8, true, 8, kv[0][t]);
       zero_past(dk, kv[0][t]);
       norm_rotate<LPK>(a, wn, a.k_norm != nullptr, d0, cs, kv[0][t]);
       if (put && dk) store8(const_cast<T*>(kring) + ((size_t)t * a.ring_len + row) * D, kv[0][t]);

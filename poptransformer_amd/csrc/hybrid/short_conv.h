@@ -14,23 +14,41 @@ __device__ __forceinline__ void conv_ring8(const T* ring, int channels, int taps
 }
 
 // Eight channels from c0 on of one row at position pos: v holds the row's own values and becomes the rounded result.
+// What the three rows before it need is requested at once.
 template <typename T>
 __device__ __forceinline__ void conv8(const pta_conv& c, int slot, int pos, int c0, float (&v)[8]) {
+  constexpr int NEAR = 3;
   const T* ring = reinterpret_cast<const T*>(c.ring) + (size_t)slot * c.taps * c.channels + c0;
-  float s[8], w[8];
+  const float* weight = c.weight + c0;
+  const int own = (int)((unsigned)pos % (unsigned)c.taps);
+  float s[8], w[NEAR + 1][8];
+  Raw8<T> u[NEAR + 1];
   load8(c.bias ? c.bias + c0 : nullptr, c.bias != nullptr, 0, s);
-#pragma unroll 4
-  for (int j = 0; j + 1 < c.taps; ++j) {
-    float u[8];
-    conv_ring8(ring, c.channels, c.taps, pos - (c.taps - 1 - j), u);
-    load8(c.weight + (size_t)j * c.channels + c0, true, 8, w);
+  load8(weight + (size_t)(c.taps - 1) * c.channels, true, 8, w[0]);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) s[e] = __builtin_fmaf(w[e], u[e], s[e]);
+  for (int b = 1; b <= NEAR; ++b) {
+    const int back = b < c.taps ? b : 0, row = own - back;
+    u[b].load(ring + (size_t)(row < 0 ? row + c.taps : row) * c.channels, true, 8);
+    load8(weight + (size_t)(c.taps - 1 - back) * c.channels, true, 8, w[b]);
   }
-  load8(c.weight + (size_t)(c.taps - 1) * c.channels + c0, true, 8, w);
+  for (int back = c.taps - 1; back > NEAR; --back) {
+    float x[8], f[8];
+    conv_ring8(ring, c.channels, c.taps, pos - back, x);
+    load8(weight + (size_t)(c.taps - 1 - back) * c.channels, true, 8, f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s[e] = __builtin_fmaf(f[e], x[e], s[e]);
+  }
+#pragma unroll
+  for (int b = NEAR; b >= 1; --b) {
+    float x[8];
+    u[b].unpack(x);
+    const bool there = b < c.taps && b <= pos;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s[e] = __builtin_fmaf(there ? w[b][e] : 0.f, there ? x[e] : 0.f, s[e]);
+  }
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
-    s[e] = __builtin_fmaf(w[e], v[e], s[e]);
+    s[e] = __builtin_fmaf(w[0][e], v[e], s[e]);
     v[e] = (float)(T)(c.silu ? silu_f32(s[e]) : s[e]);
   }
 }

@@ -41,23 +41,35 @@ __global__ __launch_bounds__(64) void short_conv_kernel(SC a, int each, int part
       load8(a.c.weight + (size_t)j * a.c.channels + c0, true, 8, w[j]);
       if (j > 0) before(r0, TAPS - j, u[j]);
     }
-    Raw8<T> next;
-    next.load(x + (size_t)r0 * a.ld_x, true, 8);
-    for (int r = r0; r < r1; ++r) {
+    constexpr int AHEAD = 4;                                  // rows requested together
+    Raw8<T> next[AHEAD];
+    auto fetch = [&](int r) {
 #pragma unroll
-      for (int j = 0; j + 1 < TAPS; ++j)
+      for (int k = 0; k < AHEAD; ++k) next[k].load(x + (size_t)(r + k < r1 ? r + k : r1 - 1) * a.ld_x, true, 8);
+    };
+    fetch(r0);
+    for (int r = r0; r < r1; r += AHEAD) {
+      Raw8<T> now[AHEAD];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) u[j][e] = u[j + 1][e];
-      next.unpack(u[TAPS - 1]);
-      next.load(x + (size_t)(r + 1 < r1 ? r + 1 : r) * a.ld_x, true, 8);
-      float s[8];
+      for (int k = 0; k < AHEAD; ++k) now[k] = next[k];
+      fetch(r + AHEAD < r1 ? r + AHEAD : r);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        s[e] = bias[e];
+      for (int k = 0; k < AHEAD; ++k) {
+        if (r + k >= r1) break;
 #pragma unroll
-        for (int j = 0; j < TAPS; ++j) s[e] = __builtin_fmaf(w[j][e], u[j][e], s[e]);
+        for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) u[j][e] = u[j + 1][e];
+        now[k].unpack(u[TAPS - 1]);
+        float s[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          s[e] = bias[e];
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) s[e] = __builtin_fmaf(w[j][e], u[j][e], s[e]);
+        }
+        put(r + k, s);
       }
-      put(r, s);
     }
   } else {
     for (int r = r0; r < r1; ++r) {

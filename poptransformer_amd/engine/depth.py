@@ -6,7 +6,7 @@ token's own part of the layer, and go on from an average over all depths:
 Layers mix attention over latents, attention by heads and the state-space recurrence; feed-forwards are squared ReLU or mixtures of
 experts.  Rows, sequences, sampling and the decode loop are HybridDecoder's.
 
-Launches of a layer in a decode iteration: the mixer's projections, with the dense feed-forward's; the mixer's own (attention
+Launches of a layer in a decode iteration: the mixer's projections, with the dense feed-forward's or a large router's; the mixer's own (attention
 with its cache entries, or the recurrence; a short convolution is part of them; passes of many rows run it in a launch of its own);
 output projection and the feed-forward's, whose epilogues add to the residual (of a mixture: pairs and downs of the chosen experts);
 the experts' weighted sum, rounding; the token's gate; its projection; the end of the layer, which adds, averages, norms and routes.
@@ -113,11 +113,16 @@ class DepthBuffers(LatentBuffers, ExpertBuffers):
         self.act = {lw.up.n_main: buf(rows, lw.up.n_main) for lw in layers if lw.up is not None}
         self.latent_buffers(buf, mixers, layers)
         self.expert_buffers(buf, spec, layers, direct, dtype, device)
+        self.logits = {n: buf(rows, n, dtype=F32) for n in {lw.router.shape[0] for lw in layers if lw.router is not None}}
         channels = max([spec.width] + [w.N for lw in layers for w in lw.linears()])
         self.workspace = HK.linear_workspace(rows, channels, device) if rows > 16 else None
 
 
 class DepthDecoder(HeadMixing, LatentMixing, StateSpaceMixing, ExpertMixing, HybridDecoder):
+    # larger routers are multiplied beside the mixer's projections, with a launch for the choice (64 logits of 4096 features in the
+    # norm's launch cost one row 10 us, the launch 4)
+    router_bytes = 128 << 10
+
     def _rows_buffers(self, rows):
         size = rows if rows <= 16 else max(64, 1 << (rows - 1).bit_length())
         if size not in self._buffers:
@@ -125,15 +130,20 @@ class DepthDecoder(HeadMixing, LatentMixing, StateSpaceMixing, ExpertMixing, Hyb
         return self._buffers[size]
 
     def _projections(self, i, b, n):
-        """What the mixer and a dense feed-forward make of the normed rows.  Returns the mixer's."""
+        """What the mixer, a dense feed-forward and a router make of the normed rows.  Returns the mixer's, and the router's logits (None:
+        the norm's launch has routed the rows)."""
         m, lw = self.spec.layers[i].mixer, self.w.layers[i]
         proj = b.proj[lw.proj.n_main]
         dt = b.dt[:n * m.heads] if m.kind == "ssd" else None
         calls = [(b.h, lw.proj, proj, dict(tail=dt, bias=lw.proj_bias, workspace=b.workspace))]
         if lw.up is not None:
             calls.append((b.h, lw.up, b.act[lw.up.n_main], dict(act=H.ACT_RELU_SQUARE, workspace=b.workspace)))
+        logits = None
+        if lw.router is not None and not self._routed_by_norm(i, b):
+            logits = b.logits[lw.router_linear.n_main]
+            calls.append((b.h, lw.router_linear, logits, dict(workspace=b.workspace)))
         HK.linear_group(n, *calls)
-        return proj, dt
+        return proj, dt, logits
 
     def _mixer(self, i, b, rows, proj, dt):
         """The heads' results, before the output projection."""
@@ -148,6 +158,7 @@ class DepthDecoder(HeadMixing, LatentMixing, StateSpaceMixing, ExpertMixing, Hyb
         """All layers over the rows; h holds the model's norm of them."""
         spec, w, n = self.spec, self.w, rows.n
         b, depths = self._rows_buffers(n), len(spec.layers)
+        self._lists_ahead(rows)
 
         def ahead(i):
             """the norm in front of layer i, and its routing"""
@@ -160,11 +171,11 @@ class DepthDecoder(HeadMixing, LatentMixing, StateSpaceMixing, ExpertMixing, Hyb
         for i, layer in enumerate(spec.layers):
             lw, x = w.layers[i], b.history[i + 1]
             add = dict(ld=spec.width, accumulate=True, workspace=b.workspace)
-            proj, dt = self._projections(i, b, n)
+            proj, dt, logits = self._projections(i, b, n)
             HK.linear(self._mixer(i, b, rows, proj, dt), lw.out, x, n, **add)
             parts = {}
             if isinstance(layer.mlp, Experts):
-                parts = self._mixture(i, b, n)
+                parts = self._mixture(i, b, n, logits)
             elif layer.mlp is not None:
                 HK.linear(b.act[lw.up.n_main], lw.down, x, n, **add)
             HK.add_parts(x, n, b.rounded, **parts)

@@ -577,7 +577,7 @@ def depth_weights(tensors, spec, device="cuda"):
         if isinstance(mlp, Experts):
             router = get(mp + "router", (mlp.count, d))
             lw.update(ff=_glu(get, HK.ExpertWeight, [f"{mp}e{e}." for e in range(mlp.count)], mlp.expert.ff, d, dtype), top=mlp.top,
-                      router=_padded(router, mlp.count, HK.pad8(d)).to(dtype).contiguous(), router_linear=HK.WideWeight(router, dtype),
+                      router=_padded(router, mlp.count, HK.pad8(d)).to(dtype).contiguous(), router_linear=HK.WideWeight(router, dtype, whole=True),
                       correction=vec(mp + "correction", mlp.count))
         elif mlp is not None:
             lw.update(up=HK.WideWeight(get(mp + "up", (mlp.ff, d)), dtype, main_to=HK.pad8(mlp.ff)),

@@ -75,6 +75,16 @@ class LatentMixing(Angles):
             lists[window] = ((slot, pos), (*rows.tiles[:2], tile_key))
         return lists[window]
 
+    def _takes_heads(self, i, rows):
+        """Whether the pass makes keys and values of all heads for layer i (else it works on the cached rows themselves)."""
+        return self.w.layers[i].kv is not None and not rows.single and rows.longest > self.absorbed_rows
+
+    def _lists_ahead(self, rows):
+        """Makes the key lists of a pass before its first launch: the copy to the device would wait for those ahead of it."""
+        for i, lay in enumerate(self.spec.layers):
+            if lay.mixer.kind == "latent" and self._takes_heads(i, rows):
+                self._keys(rows, lay.mixer.window)
+
     def _latent(self, i, lw, b, rows, proj, gates):
         """The heads' gated results of layer i, before the output projection; gates: as LatentAttention takes them."""
         m, n = self.spec.layers[i].mixer, rows.n
@@ -85,7 +95,7 @@ class LatentMixing(Angles):
                                  rows.slot, rows.pos)
         att.append(proj, cq)
         HK.linear(cq, lw.uq, q, n, workspace=b.workspace)
-        if lw.kv is None or rows.single or rows.longest <= self.absorbed_rows:
+        if not self._takes_heads(i, rows):
             splits = self._latent_splits(b.rows, m)
             q_latent, part_o, part_ml = b.absorbed(heads, R, P, splits)
             att.absorbed(q, lw.uk_t, q_latent, splits, part_o, part_ml, lw.uv, gates, ctx)
@@ -210,11 +220,14 @@ class ExpertMixing:
         out = dict(router=lw.router, routing=self._routing(i, b))
         return out if lw.correction is None else dict(out, correction=lw.correction)
 
-    def _mixture(self, i, b, n):
-        """The results of layer i's experts over the rows of b.h, as arguments of what adds them up."""
+    def _mixture(self, i, b, n, logits=None):
+        """The results of layer i's experts over the rows of b.h, as arguments of what adds them up; logits: the router's, where they
+        are there already."""
         mlp, lw = self.spec.layers[i].mlp, self.w.layers[i]
         r = self._routing(i, b)
-        if not self._routed_by_norm(i, b):
+        if logits is not None:
+            r(logits, n, lw.correction)
+        elif not self._routed_by_norm(i, b):
             if self.dtype == torch.bfloat16:
                 r.by_product(b.h, lw.router_linear, n, lw.correction)
             else:

@@ -133,6 +133,7 @@ class ParallelDecoder(LatentMixing, HybridDecoder):
         spec, w, store, n = self.spec, self.w, self.store, rows.n
         b = self._rows_buffers(n)
         last = None if rows.single else rows.last
+        self._lists_ahead(rows)
         for i, layer in enumerate(spec.layers):
             lw, ff = w.layers[i], layer.mlp is not None
             first = dict(table=w.embed, pos_table=w.pos, embed_scale=spec.embed_scale, ids=rows.ids, ids_index=rows.ids_index,

@@ -34,9 +34,10 @@ def pad8(n):
 class WideWeight:
     """A Linear weight [N, K] in bf16 (tiled for the matrix unit) or fp32 (as it is).  K is padded with zeros to a multiple
     of 8.  The last `tail` channels may go to an fp32 buffer of their own, with a bias.  `main_to`: further zero channels
-    after the main ones (results 0) up to that count, so that the result can be the padded input of another Linear."""
+    after the main ones (results 0) up to that count, so that the result can be the padded input of another Linear.  `whole`: whole
+    workgroup tiles of channels also where there are few, for launches of many rows that it shares with larger weights."""
 
-    def __init__(self, w, dtype, tail=0, tail_bias=None, main_to=None):
+    def __init__(self, w, dtype, tail=0, tail_bias=None, main_to=None, whole=False):
         n, k = w.shape
         main = n - tail
         self.n_main = main if main_to is None else main_to
@@ -45,7 +46,7 @@ class WideWeight:
             raise ValueError("a weight with a tail takes no further channels")
         total = self.n_main + tail
         # many channels: whole workgroup tiles of 128 (the padding goes nowhere)
-        self.N = (total + 127) // 128 * 128 if dtype == torch.bfloat16 and total >= 1024 else total
+        self.N = (total + 127) // 128 * 128 if dtype == torch.bfloat16 and (whole or total >= 1024) else total
         full = torch.zeros((self.N, self.K), dtype=dtype, device=w.device)
         full[:n, :k] = w.to(dtype)
         self.tail_bias = tail_bias.to(F32).contiguous() if tail_bias is not None else None
