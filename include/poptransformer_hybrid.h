@@ -329,7 +329,7 @@ typedef struct pta_head_attention_args {
   void* workspace;        /* decode with splits > 1: pta_head_attention_workspace_bytes                            */
   size_t workspace_bytes;
   void* out;              /* [rows, H * E]                                                                         */
-  const float* far1;      /* [H] or NULL: far1 ln(1 + far2 (i - j)) is taken off the scores (with keep = 0 only)   */
+  const float* far1;      /* [H] or NULL: far1 ln(1 + far2 (i - j)) is taken off the scores (keep = 0, maps = 1)   */
   const float* far2;      /* [H], not negative                                                                     */
   pta_conv conv;          /* decode: q | k | v, one behind the other, go through it first (maps = 1)               */
 } pta_head_attention_args;

@@ -121,17 +121,17 @@ __device__ __forceinline__ void finish_head(const HA& a, int r, int head, int la
 // ------------------------------------------------------------------------------------------
 // Row by row on the vector unit: a workgroup per (row, key head, RG of its query heads, part of the visible keys).  LPK lanes
 // share a key (eight features each) and its value, for the RG heads and the maps.  `fused`: the row's own key and value come
-// from the projection and are put into the cache by this launch.
+// from the projection and are put into the cache by this launch.  FAR: there may be a penalty of the distance, or convolutions.
 // ------------------------------------------------------------------------------------------
 constexpr int HR_KEYS = 4;               // keys a lane group takes per step
 
-template <typename T, int RG, int MAPS, int LPK>
+template <typename T, int RG, int MAPS, int LPK, bool FAR>
 __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int groups, float* part_o, float* part_ml) {
   constexpr int NG = 256 / LPK, DL = LPK * 8, NQ = RG * MAPS;
   __shared__ float sm[NG][NQ], sl[NG][NQ], inv_s[NQ];
   __shared__ __align__(16) float so[NG * NQ * DL];
   __shared__ float res[NQ * DL];
-  __shared__ __align__(16) float s_conv[MAPS == 1 ? (RG + 2) * DL : 8];
+  __shared__ __align__(16) float s_conv[FAR ? (RG + 2) * DL : 8];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int D = a.D, E = a.E, R = a.H / a.G;
   int b = blockIdx.x;
@@ -176,11 +176,11 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     const int head = g * R + (hg * RG + h < R ? hg * RG + h : R - 1);               // (a duplicate that is not stored)
 #pragma unroll
     for (int t = 0; t < MAPS; ++t) load8(proj_q + (head * MAPS + t) * D + (dk ? d0 : 0), true, 8, qv[h * MAPS + t]);
-    far1[h] = a.far1 ? a.far1[head] : 0.f;
-    far2[h] = a.far1 ? a.far2[head] : 0.f;
+    far1[h] = FAR && a.far1 ? a.far1[head] : 0.f;
+    far2[h] = FAR && a.far1 ? a.far2[head] : 0.f;
   }
-  const bool convolved = MAPS == 1 && fused && a.conv.ring;
-  if constexpr (MAPS == 1) {
+  const bool convolved = FAR && fused && a.conv.ring;
+  if constexpr (FAR) {
     if (convolved) {                                      // the workgroup's queries, and the row's own key and value: a thread per piece
       for (int p = threadIdx.x; p < (RG + 2) * LPK; p += 256) {
         const int which = p / LPK, d = p % LPK * 8;
@@ -226,7 +226,7 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
 #pragma unroll
         for (int e = 0; e < 8; ++e) t = __builtin_fmaf(qv[q][e], kv[u][q % MAPS][e], t);
         t = group_sum<LPK>(t);
-        if (a.far1) t -= far1[q / MAPS] * log_of<T>(1.0f + far2[q / MAPS] * back[u]);
+        if constexpr (FAR) t -= far1[q / MAPS] * log_of<T>(1.0f + far2[q / MAPS] * back[u]);
         s[u] = seen[u] ? t : -INFINITY;
         top = fmaxf(top, s[u]);
       }
@@ -252,7 +252,7 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HA a, int fused, int gro
     for (int u = 0; u < HR_KEYS; ++u) {
       const int n = nb + u * NG + grp;
       seen[u] = n < n_end;
-      back[u] = seen[u] ? (float)(i - keys.position(n)) : 0.f;
+      back[u] = FAR && seen[u] ? (float)(i - keys.position(n)) : 0.f;
 #pragma unroll
       for (int t = 0; t < MAPS; ++t) kr[u][t].unpack(kv[u][t]);
       vr[u].unpack(vv[u]);
@@ -491,7 +491,7 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
       for (int m = 0; m < DKT; ++m) *reinterpret_cast<u32x4*>(sk + (t * HT_KEYS + my_key) * KS + m * 32 + my_piece) = kf[t][m];
 #pragma unroll
     for (int m = 0; m < VIT; ++m) *reinterpret_cast<u32x4*>(sv + my_key * VS + m * 32 + my_piece) = vf[m];
-    if (a.far1 && (int)threadIdx.x < HT_KEYS + 4 * RW - 1) {           // (positions follow each other: keep = 0)
+    if (MAPS == 1 && a.far1 && (int)threadIdx.x < HT_KEYS + 4 * RW - 1) {           // (positions follow each other: keep = 0)
       const int back = p0 + 4 * RW - 1 - keys.position(nt) - (int)threadIdx.x;
       far[threadIdx.x] = far1 * __log2f(1.0f + far2 * (float)(back > 0 ? back : 0));
     }
@@ -514,10 +514,10 @@ __global__ __launch_bounds__(256) void head_tile_kernel(HA a) {
         for (int w = 0; w < QW; ++w) s[w][t] = mma(kv[MAPS == 2 ? w : 0], qf[w][c], s[w][t]);
       }
     }
-    if (a.far1) {
+    if (MAPS == 1 && a.far1) {
 #pragma unroll
       for (int w = 0; w < QW; ++w) {
-        const float* f = far + lg * 4 + 4 * RW - 1 - (MAPS == 2 ? wave * 16 + lc : (wave * QW + w) * 16 + lc);
+        const float* f = far + lg * 4 + 4 * RW - 1 - ((wave * QW + w) * 16 + lc);
 #pragma unroll
         for (int t = 0; t < 4; ++t)
 #pragma unroll
@@ -635,7 +635,8 @@ static int check_head(const HA* args, const char* name) {
   PTA_REQUIRE(a.rot == 0 || (a.rot > 0 && a.rot % 8 == 0 && a.rot <= a.D && a.cos_sin && a.positions > 0), "%s: %d rotated features", name, a.rot);
   PTA_REQUIRE(a.window > 0 && a.keep >= 0 && a.chunk >= 0 && (a.chunk == 0 || a.keep == 0), "%s: window %d, keep %d, chunk %d", name, a.window,
               a.keep, a.chunk);
-  PTA_REQUIRE(!a.far1 || (a.far2 && a.keep == 0), "%s: a penalty of the distance needs both of its numbers, and no kept positions", name);
+  PTA_REQUIRE(!a.far1 || (a.far2 && a.keep == 0 && a.maps == 1), "%s: a penalty of the distance needs both of its numbers, single maps and no kept positions",
+              name);
   PTA_REQUIRE(a.keys && a.values && pta_aligned(a.keys, 16) && pta_aligned(a.values, 16) && a.ring_len > a.keep && a.slot && a.pos,
               "%s: the cache (%d rows) or the rows' places are missing", name, a.ring_len);
   return PTA_OK;
@@ -659,7 +660,14 @@ static void launch_rows_for(const HA& a, int fused, float* po, float* pml, hipSt
   const int groups = (a.H / a.G + RG - 1) / RG;
   const dim3 grid((unsigned)((size_t)a.rows * a.G * groups * a.splits));
   with_lanes(a.D > a.E ? a.D : a.E, [&](auto lanes) {
-    hipLaunchKernelGGL((head_rows_kernel<T, RG, MAPS, decltype(lanes)::value>), grid, dim3(256), 0, s, a, fused, groups, po, pml);
+    constexpr int L = decltype(lanes)::value;
+    if constexpr (MAPS == 1) {
+      if (a.far1 || a.conv.ring) {
+        hipLaunchKernelGGL((head_rows_kernel<T, RG, MAPS, L, true>), grid, dim3(256), 0, s, a, fused, groups, po, pml);
+        return;
+      }
+    }
+    hipLaunchKernelGGL((head_rows_kernel<T, RG, MAPS, L, false>), grid, dim3(256), 0, s, a, fused, groups, po, pml);
   });
 }
 

@@ -63,12 +63,13 @@ __global__ __launch_bounds__(RR_WAVES * 64) void route_rows_kernel(const bf16* h
   for (int m = wave; m < 16; m += RR_WAVES) route_row<64>(g, z_rows + m * z_ld, row0 + m, lane, row0 + m < rows);
 }
 
+template <int PER>
 __global__ __launch_bounds__(64) void route_kernel(const float* logits, pta_routing g) {
   __shared__ float z[ROUTE_FLOATS];
   const int n = g.experts + g.shared;
   for (int c = threadIdx.x; c < n; c += 64) z[c] = logits[(size_t)blockIdx.x * n + c];
   __syncthreads();
-  route_row<64>(g, z, blockIdx.x, threadIdx.x, true);
+  route_row<64, PER>(g, z, blockIdx.x, threadIdx.x, true);
 }
 
 __device__ __forceinline__ float rounded(float v, bf16) { return (float)(bf16)v; }
@@ -206,7 +207,10 @@ extern "C" int pta_route(const float* logits, int rows, const pta_routing* routi
   PTA_REQUIRE(logits && routing && rows > 0, "pta_route: null pointer, or %d rows", rows);
   const int rc = check_routing(*routing, "pta_route");
   if (rc) return rc;
-  hipLaunchKernelGGL(route_kernel, dim3(rows), dim3(64), 0, (hipStream_t)stream, logits, *routing);
+  hipStream_t s = (hipStream_t)stream;
+  if (routing->experts <= 64) hipLaunchKernelGGL((route_kernel<1>), dim3(rows), dim3(64), 0, s, logits, *routing);
+  else if (routing->experts <= 256) hipLaunchKernelGGL((route_kernel<4>), dim3(rows), dim3(64), 0, s, logits, *routing);
+  else hipLaunchKernelGGL((route_kernel<16>), dim3(rows), dim3(64), 0, s, logits, *routing);
   PTA_CHECK_LAUNCH("pta_route");
   return PTA_OK;
 }

@@ -8,27 +8,24 @@ static inline int route_floats(const pta_routing& g) { return g.experts + 1 + g.
 
 // Routing of row r by THREADS threads, of which this is `tid`: z (route_floats) holds the logits (in LDS, visible to all; overwritten).  Expert e's
 // place among the chosen is the number of larger choice scores (of equal ones the first comes first), so no choice waits for another.
-// The whole workgroup calls it, each group of THREADS for a row of its own; with `store` unset nothing is kept.
-template <int THREADS>
+// The whole workgroup calls it, each group of THREADS for a row of its own; with `store` unset nothing is kept.  PER: experts of a
+// thread, at most (fewer make for less code, whose first fetch is much of a short launch).
+template <int THREADS, int PER = (PTA_MAX_EXPERTS + THREADS - 1) / THREADS>
 __device__ __forceinline__ void route_row(const pta_routing& g, float* z, int r, int tid, bool store) {
   const int E = g.experts, choices = g.top + g.shared;
   int32_t* chosen = g.chosen + (size_t)r * choices;
   float* weights = g.weights + (size_t)r * choices;
-  constexpr int PER = (PTA_MAX_EXPERTS + THREADS - 1) / THREADS;
   int rank[PER];
   float p[PER];
   const float shared = g.shared && tid == 0 ? sigmoid_f32(z[E]) : 0.f;
-  if (g.score == PTA_SCORE_SIGMOID) {                        // z becomes the choice scores
+  if (g.score == PTA_SCORE_SIGMOID) {                        // z becomes the choice scores (a thread's own logits only)
 #pragma unroll
     for (int k = 0; k < PER; ++k) {
       const int e = tid + k * THREADS;
-      p[k] = e < E ? sigmoid_f32(z[e]) : 0.f;
-    }
-    __syncthreads();
-#pragma unroll
-    for (int k = 0; k < PER; ++k) {
-      const int e = tid + k * THREADS;
-      if (e < E) z[e] = p[k] + (g.correction ? g.correction[e] : 0.f);
+      p[k] = 0.f;
+      if (e >= E) continue;
+      p[k] = sigmoid_f32(z[e]);
+      z[e] = p[k] + (g.correction ? g.correction[e] : 0.f);
     }
     __syncthreads();
   }

@@ -3,7 +3,10 @@
 #pragma once
 #include "attention.h"
 
-__device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+// silu in fp32; for results that are rounded to bf16 by the hardware's exponential and reciprocal (a few units in the last place)
+template <typename T> __device__ __forceinline__ float silu_of(float z);
+template <> __device__ __forceinline__ float silu_of<float>(float z) { return z / (1.0f + expf(-z)); }
+template <> __device__ __forceinline__ float silu_of<bf16>(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
 
 // eight channels of position p as the ring holds them (zeros before the start)
 template <typename T>
@@ -49,7 +52,7 @@ __device__ __forceinline__ void conv8(const pta_conv& c, int slot, int pos, int 
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
     s[e] = __builtin_fmaf(w[0][e], v[e], s[e]);
-    v[e] = (float)(T)(c.silu ? silu_f32(s[e]) : s[e]);
+    v[e] = (float)(T)(c.silu ? silu_of<T>(s[e]) : s[e]);
   }
 }
 

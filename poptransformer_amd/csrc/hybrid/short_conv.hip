@@ -31,7 +31,7 @@ __global__ __launch_bounds__(64) void short_conv_kernel(SC a, int each, int part
   auto put = [&](int r, float (&s)[8]) {
     if (a.c.silu)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) s[e] = silu_f32(s[e]);
+      for (int e = 0; e < 8; ++e) s[e] = silu_of<T>(s[e]);
     store8(y + (size_t)r * a.ld_y, s);
   };
   if constexpr (TAPS > 0) {

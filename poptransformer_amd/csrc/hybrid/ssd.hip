@@ -182,7 +182,7 @@ __global__ __launch_bounds__(THREADS) void gated_norm_kernel(pta_gated_norm_args
     load8(y + c, true, 8, v);
     load8(z + c, true, 8, g);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = whole || (c + e >= c_lo && c + e < c_hi) ? v[e] * silu_f32(g[e]) : 0.f;
+    for (int e = 0; e < 8; ++e) v[e] = whole || (c + e >= c_lo && c + e < c_hi) ? v[e] * silu_of<T>(g[e]) : 0.f;
   };
   float v[KEEP][8], w[KEEP][8], sq = 0.f;
 #pragma unroll
