@@ -6,11 +6,11 @@ token's own part of the layer, and go on from an average over all depths:
 Layers mix attention over latents, attention by heads and the state-space recurrence; feed-forwards are squared ReLU or mixtures of
 experts.  Rows, sequences, sampling and the decode loop are HybridDecoder's.
 
-Launches of a layer in a decode iteration: the mixer's projections, with the dense feed-forward's or a large router's; the mixer's own (attention
-with its cache entries, or the recurrence; a short convolution is part of them; passes of many rows run it in a launch of its own);
-output projection and the feed-forward's, whose epilogues add to the residual (of a mixture: pairs and downs of the chosen experts);
-the experts' weighted sum, rounding; the token's gate; its projection; the end of the layer, which adds, averages, norms and routes.
-The residuals of all depths stay in the row buffers: the mean of a pass reads them once per layer.
+Launches of a layer in a decode iteration: the mixer's projections, with the dense feed-forward's or a large router's; the mixer's
+own (attention with its cache entries, or the recurrence; a short convolution is part of them, passes of many rows run it in a launch
+of its own); output projection and the feed-forward's, whose epilogues add to the residual (of a mixture: pairs and downs of the chosen
+experts); the experts' weighted sum, rounding; the token's gate; its projection; the end of the layer, which adds, averages, norms and
+routes.  The residuals of all depths stay in the row buffers: the mean of a pass reads them once per layer.
 """
 from dataclasses import dataclass
 from typing import List, Optional
